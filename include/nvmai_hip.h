@@ -23,7 +23,7 @@
  *     nibble of byte k) or 8 bit, plus one BF16 scale and one BF16 bias per group
  *     (nvmai_kernels.h:10-21, Quantization.swift:32-38).  Code rows must be
  *     16-byte aligned.
- *   - activations: 16-bit, BF16 or FP16 chosen at ctx creation.
+ *   - activations: 16-bit, BF16 or FP16 chosen at ctx creation (or 32-bit, for the dense models).
  *   - routing weights, softmax probabilities, KV scale/bias: FP16.
  */
 #ifndef NVMAI_HIP_H
@@ -49,7 +49,9 @@ typedef enum {
     NVMAI_ERR_NO_DEVICE = -6
 } nvmai_status;
 
-enum { NVMAI_ACT_BF16 = 0, NVMAI_ACT_FP16 = 1 };
+/* NVMAI_ACT_FP32: activations are floats.  Taken by the entry points of the dense models at the end of this
+ * header and by the softmax and the samplers; every other entry point returns NVMAI_ERR_INVALID_ARG. */
+enum { NVMAI_ACT_BF16 = 0, NVMAI_ACT_FP16 = 1, NVMAI_ACT_FP32 = 2 };
 
 /* Rows in "router format": kind 4 / 8 = affine codes with BF16 scale/bias per
  * group of 64; kind 16 = dense BF16 (scales/biases unused); kind 0 = absent. */
@@ -742,6 +744,95 @@ int nvmai_hip_affine_gemv_fused(nvmai_hip_ctx* ctx, nvmai_stream stream, const n
 
 /* Sampler.seedFor (Sampler.swift:304-325): splitmix64(seed + position), 0 mapped away. */
 uint64_t nvmai_sampler_seed_for(uint64_t seed, int64_t position);
+
+/* ---- dense models: BF16 weights, a 32-bit residual stream, gated linear and latent attention --------- *
+ * No counterpart in the reference.  Contexts: BF16 or FP32 (everything in 32 bits; the weights stay BF16).  Matrices
+ * are [n, k] BF16 rows with k a multiple of 64; a model whose sizes are not multiples of 64 (rows of a matrix
+ * product) or 16 (head sizes) is padded with zero weights when it is loaded, and the counts below that are called
+ * `..._count` say how many of the elements are real where a mean is taken over them. */
+enum { NVMAI_LINEAR_NONE = 0, NVMAI_LINEAR_GELU_ERF = 1 };
+enum { NVMAI_FORM_AUTO = 0, NVMAI_GLA_RECURRENT = 1, NVMAI_GLA_CHUNKED = 2, NVMAI_LATENT_ABSORBED = 1, NVMAI_LATENT_EXPANDED = 2 };
+
+/* y[t, :] = act(W x[t, :]) for any number of rows: a wave per weight row up to 4 rows, split-k matrix-core products
+ * up to 64, LDS-tiled matrix-core products above; fp32 FMA in a 32-bit context.  y (activations) and / or y_f32, one
+ * row stride for both. */
+int nvmai_hip_dense_linear(nvmai_hip_ctx* ctx, nvmai_stream stream, const uint16_t* w, uint32_t w_stride, const void* x,
+                           uint32_t x_stride, uint32_t rows, uint32_t n, uint32_t k, void* y, float* y_f32, uint32_t y_stride,
+                           int activation);
+
+/* The end of one sublayer and the start of the next over the 32-bit residual:
+ *   x   += mult * LN(delta) * post_weight + post_bias   (post_weight NULL: x += mult * delta; delta NULL: x as it is)
+ *   out  = LN(x) * next_weight + next_bias              (next_weight NULL: not computed)
+ * LN(v) = (v - mean) / sqrt(mean((v - mean)^2) + eps).  d <= 16384. */
+int nvmai_hip_norm_residual(nvmai_hip_ctx* ctx, nvmai_stream stream, float* x, uint32_t x_stride, const float* delta,
+                            uint32_t delta_stride, const uint16_t* post_weight, const uint16_t* post_bias, float mult,
+                            const uint16_t* next_weight, const uint16_t* next_bias, void* out, uint32_t out_stride, uint32_t rows,
+                            uint32_t d, float eps);
+
+/* out[t, :] = row token_ids[t] of a BF16 table, as floats; an id >= vocab gives zeros. */
+int nvmai_hip_embed_rows(nvmai_hip_ctx* ctx, nvmai_stream stream, const uint16_t* table, uint32_t table_stride,
+                         const uint32_t* token_ids, uint32_t n_tokens, float* out, uint32_t out_stride, uint32_t d, uint32_t vocab);
+
+/* Index of the largest finite value of each row, ties to the lower index, 0 when none is finite. */
+int nvmai_hip_argmax_rows(nvmai_hip_ctx* ctx, nvmai_stream stream, const float* x, uint32_t x_stride, uint32_t rows, uint32_t n,
+                          uint32_t* out_index);
+
+/* Which sequence (slot of a cache or state array) and position each row of a call is: two device arrays (a decode
+ * batch), or NULL, NULL: row r is position `position` + r of `slot` (a portion of one prompt). */
+typedef struct {
+    const uint32_t* slots;
+    const uint32_t* positions;
+    uint32_t slot, position;
+} nvmai_row_map;
+
+/* Gated linear attention with a decay per key channel: z = W_a2 a1 + b, alpha = sigmoid(z)^(1/tau),
+ *   S_t = diag(alpha_t) S_(t-1) + k_t v_t^T,  o_t = S_t^T (q_scale q_t),  out = rmsnorm(o) * norm_weight * silu(g)
+ * per head.  q, k [.., heads * key_dim], v, g [.., heads * value_dim], a1 [.., rank] are columns of projected rows
+ * with one row stride; a2 [heads * key_dim, rank] and a2_bias BF16; norm_weight BF16 [value_dim]; state
+ * [slots, heads, key_dim, value_dim] floats, updated in place.  `batch` sequences of `rows` rows each: sequence b
+ * uses slot slots[b] (device array), or slot + b when slots is NULL.  key_dim, value_dim multiples of 16, rank of 8,
+ * value_dim <= 512.  The chunked form (one sequence, NULL slots, key_dim and value_dim <= 256) takes workspace. */
+typedef struct {
+    uint32_t heads, key_dim, value_dim, value_count, rank;
+    float tau, q_scale, eps;
+} nvmai_gla_config;
+int nvmai_hip_gla(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_gla_config* config, const void* q, const void* k,
+                  const void* v, const void* g, const void* a1, uint32_t proj_stride, const uint16_t* a2, const uint16_t* a2_bias,
+                  const uint16_t* norm_weight, float* state, const uint32_t* slots, uint32_t slot, void* out, uint32_t out_stride,
+                  uint32_t rows, uint32_t batch, int form);
+
+/* Latent attention.  window: position i sees j with 0 <= i - j < window, 0 = every j <= i.  inv_freq: device array of
+ * rotary_dims / 2 doubles; entries i and i + rotary_dims / 2 of the rope part turn by position * inv_freq[i]. */
+typedef struct {
+    uint32_t heads, nope_dim, rope_dim, value_dim, rank, rank_count, rotary_dims, window;
+    float scale, eps;
+    const double* inv_freq;
+} nvmai_latent_config;
+/* Rows [latent: rank | rope part: rope_dim | zeros] of activations; position p of a slot lies at row p % capacity.
+ * Elements a model's counts leave out are zero and stay so (the caller clears the array once). */
+typedef struct {
+    void* base;
+    uint64_t slot_stride;      /* elements */
+    uint32_t row_stride;       /* elements, a multiple of 32 */
+    uint32_t capacity;         /* rows per slot, at least 64 */
+} nvmai_latent_cache;
+
+/* From the down projections proj[t] = [.. c_q at q_at .. c_kv at kv_at .. rope part at rope_at ..]:
+ * cq[t] = rmsnorm(c_q) * q_norm, and the token's cache row = [rmsnorm(c_kv) * kv_norm | rotated rope part]. */
+int nvmai_hip_latent_epilogue(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_latent_config* config, const void* proj,
+                              uint32_t proj_stride, uint32_t q_at, uint32_t q_count, const uint16_t* q_norm, uint32_t kv_at,
+                              uint32_t rope_at, const uint16_t* kv_norm, void* cq, uint32_t cq_stride,
+                              const nvmai_latent_cache* cache, const nvmai_row_map* map, uint32_t rows);
+
+/* q [rows, heads * (nope_dim + rope_dim)] head by head, not yet rotated (the expanded form rotates it in place);
+ * gate [rows, gate_stride]: one logit per head, out *= sigmoid, NULL = none; uk [heads * nope_dim, rank],
+ * uv [heads * value_dim, rank] BF16.  out [rows, heads * value_dim].  The rows' own cache rows must have been
+ * written.  The ring has to hold what the rows look at: window + rows - 1 positions for (slot, position) rows, the
+ * window (or every position, when the positions stay below the capacity) for rows by arrays.  Takes workspace. */
+int nvmai_hip_latent_attention(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_latent_config* config, void* q,
+                               uint32_t q_stride, const void* gate, uint32_t gate_stride, const uint16_t* uk, const uint16_t* uv,
+                               const nvmai_latent_cache* cache, const nvmai_row_map* map, void* out, uint32_t out_stride,
+                               uint32_t rows, int form);
 
 #ifdef __cplusplus
 }

@@ -1,10 +1,14 @@
 """ctypes view of libnvmai_hip.so (the C ABI declared in include/nvmai_hip.h).
 
 The library is the product; there is no fallback.  If it has not been built the
-import fails loudly.
+import fails loudly.  A part library (build.PARTS: the entry points one family of models needs) serves where the
+whole one has not been built; an entry point it does not hold fails when it is called.
 """
 import ctypes as C
+import glob
 import os
+
+import torch  # noqa: F401  -- before the library: the process then has one HIP runtime, torch's
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libnvmai_hip.so")
@@ -15,10 +19,13 @@ class NvmaiLibraryMissing(ImportError):
 
 
 def load():
-    if not os.path.exists(LIB_PATH):
+    if os.path.exists(LIB_PATH):
+        return C.CDLL(LIB_PATH)
+    parts = sorted(glob.glob(LIB_PATH[:-3] + ".*.so"))
+    if not parts:
         raise NvmaiLibraryMissing(
             "%s is missing: run `python -m nvmai_amd.build` (hipcc, gfx950) first" % LIB_PATH)
-    return C.CDLL(LIB_PATH)
+    return C.CDLL(parts[0])
 
 
 lib = load()
@@ -64,6 +71,28 @@ class GdnConfig(C.Structure):
 class GemvPart(C.Structure):
     """nvmai_gemv_part"""
     _fields_ = [("weights", vp), ("scales", vp), ("biases", vp), ("rows", u32), ("y", vp), ("y_stride", u32)]
+
+
+class RowMap(C.Structure):
+    """nvmai_row_map"""
+    _fields_ = [("slots", vp), ("positions", vp), ("slot", u32), ("position", u32)]
+
+
+class GlaConfig(C.Structure):
+    """nvmai_gla_config"""
+    _fields_ = ([(n, u32) for n in ("heads", "key_dim", "value_dim", "value_count", "rank")] +
+                [(n, C.c_float) for n in ("tau", "q_scale", "eps")])
+
+
+class LatentConfig(C.Structure):
+    """nvmai_latent_config"""
+    _fields_ = ([(n, u32) for n in ("heads", "nope_dim", "rope_dim", "value_dim", "rank", "rank_count", "rotary_dims", "window")] +
+                [("scale", C.c_float), ("eps", C.c_float), ("inv_freq", vp)])
+
+
+class LatentCacheView(C.Structure):
+    """nvmai_latent_cache"""
+    _fields_ = [("base", vp), ("slot_stride", u64), ("row_stride", u32), ("capacity", u32)]
 
 
 class PrefillStreamedParams(C.Structure):
@@ -157,6 +186,15 @@ SIGNATURES = {
     "nvmai_hip_gdn_delta_gated_norm": [vp, vp, C.POINTER(GdnConfig), vp, u32, vp, vp, u32, vp, vp, vp, C.c_int, vp, u32,
                                        vp, vp, u32, u32, u32],
     "nvmai_hip_affine_gemv_fused": [vp, vp, C.POINTER(GemvPart), u32, u32, vp, u32, u32, u32],
+    "nvmai_hip_dense_linear": [vp, vp, vp, u32, vp, u32, u32, u32, u32, vp, vp, u32, C.c_int],
+    "nvmai_hip_norm_residual": [vp, vp, vp, u32, vp, u32, vp, vp, C.c_float, vp, vp, vp, u32, u32, u32, C.c_float],
+    "nvmai_hip_embed_rows": [vp, vp, vp, u32, vp, u32, vp, u32, u32, u32],
+    "nvmai_hip_argmax_rows": [vp, vp, vp, u32, u32, u32, vp],
+    "nvmai_hip_gla": [vp, vp, C.POINTER(GlaConfig), vp, vp, vp, vp, vp, u32, vp, vp, vp, vp, vp, u32, vp, u32, u32, u32, C.c_int],
+    "nvmai_hip_latent_epilogue": [vp, vp, C.POINTER(LatentConfig), vp, u32, u32, u32, vp, u32, u32, vp, vp, u32,
+                                  C.POINTER(LatentCacheView), C.POINTER(RowMap), u32],
+    "nvmai_hip_latent_attention": [vp, vp, C.POINTER(LatentConfig), vp, u32, vp, u32, vp, vp, C.POINTER(LatentCacheView),
+                                   C.POINTER(RowMap), vp, u32, u32, C.c_int],
     "nvmai_hip_sample": [vp, vp, vp, u32, u32, u32, C.c_float, u32, C.c_float, C.POINTER(u64), C.POINTER(u32), vp],
 }
 _OTHER = {
@@ -170,11 +208,10 @@ _OTHER = {
 
 
 def _declare():
-    for name, args in SIGNATURES.items():
-        fn = getattr(lib, name)
-        fn.restype = C.c_int
-        fn.argtypes = args
-    for name, (res, args) in _OTHER.items():
+    whole = lib._name == LIB_PATH
+    for name, (res, args) in [(n, (C.c_int, a)) for n, a in SIGNATURES.items()] + list(_OTHER.items()):
+        if not whole and not hasattr(lib, name):
+            continue                     # not in this part: the attribute stays missing
         fn = getattr(lib, name)
         fn.restype = res
         fn.argtypes = args

@@ -16,9 +16,15 @@ FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=o
          "-Wno-pass-failed"]
 
 
-def build(verbose=False, jobs=8):
-    """Compile every .hip file under csrc/ and link them into one shared library."""
-    srcs = sorted(glob.glob(os.path.join(CSRC, "*.hip")))
+# Part libraries: the sources that one family of models needs, for a run that must not wait for the rest.
+PARTS = {"dense": ["ctx_api", "dense_api", "gla_api", "latent_api", "sample_api"]}
+
+
+def part_path(part):
+    return LIB[:-3] + "." + part + ".so"
+
+
+def _compile(srcs, out, verbose, jobs):
     objs, procs = [], []
     for src in srcs:
         obj = src[:-4] + ".o"
@@ -30,9 +36,23 @@ def build(verbose=False, jobs=8):
         if len(procs) >= jobs:
             _wait(procs)
     _wait(procs)
-    cmd = ["hipcc", "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB, *objs]
-    subprocess.run(cmd, check=True)
-    return LIB
+    tmp = "%s.%d.tmp" % (out, os.getpid())
+    subprocess.run(["hipcc", "--offload-arch=gfx950", "-shared", "-fPIC", "-o", tmp, *objs], check=True)
+    os.replace(tmp, out)                 # a library is there whole or not at all
+    return out
+
+
+def build(verbose=False, jobs=8):
+    """Compile every .hip file under csrc/ and link them into one shared library."""
+    return _compile(sorted(glob.glob(os.path.join(CSRC, "*.hip"))), LIB, verbose, jobs)
+
+
+def ensure(part, verbose=False, jobs=8):
+    """The library if it is built, else the part library, built now if it is not there either."""
+    for path in (LIB, part_path(part)):
+        if os.path.exists(path):
+            return path
+    return _compile([os.path.join(CSRC, n + ".hip") for n in PARTS[part]], part_path(part), verbose, jobs)
 
 
 def _wait(procs):

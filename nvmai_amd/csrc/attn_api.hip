@@ -55,7 +55,7 @@ int check_view(const nvmai_kv_view* v, uint32_t elements) {
 extern "C" int nvmai_hip_kv_quantize_affine(nvmai_hip_ctx* ctx, nvmai_stream stream, const void* source,
                                             uint32_t source_stride, const nvmai_kv_view* dst,
                                             uint32_t token_count, uint32_t element_count) {
-    if (!ctx || !source || element_count == 0 || source_stride < element_count) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !source || element_count == 0 || source_stride < element_count) return NVMAI_ERR_INVALID_ARG;
     int rc = check_view(dst, element_count);
     if (rc) return rc;
     if (dst->bits == 16) return NVMAI_ERR_UNSUPPORTED;        // "KV quantizer requires 4-bit or 8-bit destination"
@@ -84,7 +84,7 @@ extern "C" int nvmai_hip_kv_quantize_affine(nvmai_hip_ctx* ctx, nvmai_stream str
 extern "C" int nvmai_hip_rope_neox_subdim(nvmai_hip_ctx* ctx, nvmai_stream stream, void* data, uint32_t tokens,
                                           uint32_t heads, uint32_t head_dim, uint32_t rotary_dim,
                                           const uint32_t* positions, uint32_t position, float theta) {
-    if (!ctx || !data || rotary_dim > head_dim || (rotary_dim & 1u) || heads == 0 || head_dim == 0)
+    if (!act16(ctx) || !data || rotary_dim > head_dim || (rotary_dim & 1u) || heads == 0 || head_dim == 0)
         return NVMAI_ERR_INVALID_ARG;
     const uint64_t n = (uint64_t)tokens * heads * (rotary_dim / 2);
     if (n == 0) return NVMAI_OK;
@@ -165,7 +165,7 @@ int run_attention(nvmai_hip_ctx* ctx, nvmai_stream stream, AttnParams p, const n
 int attention_setup(nvmai_hip_ctx* ctx, const void* q, const nvmai_kv_view* k, const nvmai_kv_view* v, void* out,
                     uint32_t batch, uint32_t head_dim, uint32_t num_q_heads, uint32_t num_kv_heads, float scale,
                     AttnParams& p) {
-    if (!ctx || !q || !out || batch == 0 || head_dim == 0 || num_kv_heads == 0 || num_q_heads == 0) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !q || !out || batch == 0 || head_dim == 0 || num_kv_heads == 0 || num_q_heads == 0) return NVMAI_ERR_INVALID_ARG;
     if (num_q_heads % num_kv_heads) return NVMAI_ERR_INVALID_ARG;      // Attention.swift:221-222
     if (head_dim > 512) return NVMAI_ERR_INVALID_ARG;                  // Attention.swift:223-224
     const uint32_t elements = num_kv_heads * head_dim;

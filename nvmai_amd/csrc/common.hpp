@@ -12,8 +12,12 @@
 namespace nvmai {
 
 // ---- 16-bit activations ---------------------------------------------------
-// Activations are stored as raw 16-bit patterns; ACT selects the format.
-enum ActType : int { ACT_BF16 = 0, ACT_FP16 = 1 };
+// Activations are stored as raw 16-bit patterns, or as floats in a 32-bit context; ACT selects the format.
+enum ActType : int { ACT_BF16 = 0, ACT_FP16 = 1, ACT_FP32 = 2 };
+
+// Storage of one activation.
+template <int ACT>
+using act_t = std::conditional_t<ACT == ACT_FP32, float, uint16_t>;
 
 __device__ __forceinline__ float bf16_to_f32(uint16_t b) {
     return __uint_as_float(((uint32_t)b) << 16);
@@ -42,13 +46,15 @@ __device__ __forceinline__ uint16_t f32_to_f16(float x) {
 }
 
 template <int ACT>
-__device__ __forceinline__ float act_to_f32(uint16_t v) {
-    return ACT == ACT_BF16 ? bf16_to_f32(v) : f16_to_f32(v);
+__device__ __forceinline__ float act_to_f32(act_t<ACT> v) {
+    if constexpr (ACT == ACT_FP32) return v;
+    else return ACT == ACT_BF16 ? bf16_to_f32(v) : f16_to_f32(v);
 }
 
 template <int ACT>
-__device__ __forceinline__ uint16_t f32_to_act(float v) {
-    return ACT == ACT_BF16 ? f32_to_bf16(v) : f32_to_f16(v);
+__device__ __forceinline__ act_t<ACT> f32_to_act(float v) {
+    if constexpr (ACT == ACT_FP32) return v;
+    else return ACT == ACT_BF16 ? f32_to_bf16(v) : f32_to_f16(v);
 }
 
 // Two packed activations in one dword -> two floats (low half first).

@@ -11,7 +11,7 @@
 struct nvmai_hip_ctx {
     int device;
     int compute_units;       // of the device (persistent grids are sized from it)
-    int act;                 // NVMAI_ACT_BF16 / NVMAI_ACT_FP16
+    int act;                 // NVMAI_ACT_BF16 / NVMAI_ACT_FP16 / NVMAI_ACT_FP32
     // Workspace: one device buffer carved by a bump pointer inside each entry
     // point.  Work on one stream is ordered, so consecutive calls may reuse it.
     uint8_t* ws;
@@ -21,7 +21,7 @@ struct nvmai_hip_ctx {
     // captured graph keeps the addresses it was recorded with, and replaying it must stay valid
     // after a later, larger call has moved the workspace.
     std::vector<void*> ws_retired;
-    uint8_t* static_scratch; // device address of the library's static scratch array on this device (moe_api.hip)
+    uint8_t* static_scratch; // device address of the library's static scratch array on this device (ctx_api.hip)
     uint32_t* tickets;       // zero-initialised device words for last-block-done kernels (TICKET_WORDS)
     // Optional per-kernel timing: event pairs recorded around tagged launches.
     bool prof_on;
@@ -36,6 +36,12 @@ namespace nvmai {
 // [16, 48) sampler block counters, [TICKET_GROUPS, TICKET_WORDS) router token-group tickets.
 constexpr uint32_t TICKET_WORDS = 2048;
 constexpr uint32_t TICKET_GROUPS = 64;
+
+// The static device array of the allocation-free decode entry point (ctx_api.hip).
+constexpr size_t STATIC_SCRATCH_BYTES = (size_t)4 << 20;
+
+// A context of 16-bit activations: what every entry point takes that has no 32-bit form.
+inline bool act16(const nvmai_hip_ctx* ctx) { return ctx && ctx->act != NVMAI_ACT_FP32; }
 
 #define NVMAI_HIP_TRY(expr)                         \
     do {                                            \

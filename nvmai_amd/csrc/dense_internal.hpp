@@ -1,0 +1,20 @@
+// The dense product, callable from other entry-point files.
+#pragma once
+
+#include "ctx.hpp"
+
+namespace nvmai {
+
+struct DenseLinearParams {
+    const uint16_t* w;      // [n, w_stride] BF16
+    const void* x;          // [rows, x_stride] activations
+    void* y;                // activations, or nullptr
+    float* y_f32;           // floats, or nullptr
+    uint32_t w_stride, x_stride, y_stride, rows, n, k;
+    int activation;         // NVMAI_LINEAR_*
+};
+
+int dense_linear_check(const nvmai_hip_ctx* ctx, const DenseLinearParams& p);
+int dense_linear(nvmai_hip_ctx* ctx, hipStream_t s, const DenseLinearParams& p);
+
+}  // namespace nvmai

@@ -1,0 +1,384 @@
+// Kernels of the dense models (BF16 weights; 16-bit BF16 or 32-bit activations; a 32-bit residual stream):
+// the matrix products, layer norm with bias, the norm-scale-add that closes a sublayer, embedding rows, argmax.
+// gfx950, wave64.
+#pragma once
+
+#include "common.hpp"
+#include "dense_internal.hpp"
+
+namespace nvmai {
+
+typedef __bf16 dn_b8 __attribute__((ext_vector_type(8)));
+typedef float dn_f4 __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ dn_f4 dn_mfma(const uint4& a, const uint4& b, dn_f4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(dn_b8, a), __builtin_bit_cast(dn_b8, b), c, 0, 0, 0);
+}
+
+// z/2 (1 + erf(z / sqrt 2))
+__device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
+
+__device__ __forceinline__ float dense_act(float v, int activation) { return activation == 1 ? gelu_erf(v) : v; }
+
+template <int ACT>
+__device__ __forceinline__ void dense_store(const DenseLinearParams& p, uint32_t t, uint32_t r, float v) {
+    v = dense_act(v, p.activation);
+    if (p.y) static_cast<act_t<ACT>*>(p.y)[(size_t)t * p.y_stride + r] = f32_to_act<ACT>(v);
+    if (p.y_f32) p.y_f32[(size_t)t * p.y_stride + r] = v;
+}
+
+// Four neighbouring outputs of one token (r0 a multiple of 4).
+__device__ __forceinline__ void dense_store4_bf16(const DenseLinearParams& p, uint32_t t, uint32_t r0, dn_f4 v) {
+    if (r0 + 4u <= p.n && (p.y_stride & 3u) == 0) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] = dense_act(v[j], p.activation);
+        if (p.y) {
+            uint2 q;
+            q.x = f32_to_bf16(v[0]) | ((uint32_t)f32_to_bf16(v[1]) << 16);
+            q.y = f32_to_bf16(v[2]) | ((uint32_t)f32_to_bf16(v[3]) << 16);
+            *reinterpret_cast<uint2*>(static_cast<uint16_t*>(p.y) + (size_t)t * p.y_stride + r0) = q;
+        }
+        if (p.y_f32) *reinterpret_cast<dn_f4*>(p.y_f32 + (size_t)t * p.y_stride + r0) = v;
+    } else {
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+            if (r0 + j < p.n) dense_store<ACT_BF16>(p, t, r0 + j, v[j]);
+    }
+}
+
+// ---- 1 .. 4 input rows: a wave owns RW weight rows, its lanes split k in 16-byte pieces -------------
+// Bound by the matrix's bytes.  The inputs are read from L1 / L2 beside the weights (no LDS, no barrier): every
+// load of a k step is independent of the others, so a wave has RW + NT 16-byte loads per lane in flight.
+template <int NT, int RW>
+__global__ __launch_bounds__(256) void dense_gemv_kernel(DenseLinearParams p) {
+    const uint32_t lane = threadIdx.x & 63u, wave = threadIdx.x >> 6;
+    const uint32_t r0 = (blockIdx.x * 4u + wave) * RW;
+    if (r0 >= p.n) return;
+    const uint16_t* wp[RW];
+#pragma unroll
+    for (int r = 0; r < RW; ++r) wp[r] = p.w + (size_t)min(r0 + r, p.n - 1u) * p.w_stride;
+    const uint16_t* x = static_cast<const uint16_t*>(p.x);
+    float acc[NT][RW];
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+#pragma unroll
+        for (int r = 0; r < RW; ++r) acc[t][r] = 0.0f;
+#pragma unroll 4
+    for (uint32_t k0 = 0; k0 < p.k; k0 += 512u) {
+        const uint32_t k = k0 + lane * 8u;
+        const bool live = k < p.k;
+        const uint32_t at = live ? k : p.k - 8u;             // past the end: reload the last piece, multiply by zero
+        uint4 wv[RW], xv[NT];
+#pragma unroll
+        for (int r = 0; r < RW; ++r) wv[r] = *reinterpret_cast<const uint4*>(wp[r] + at);
+#pragma unroll
+        for (int t = 0; t < NT; ++t) xv[t] = *reinterpret_cast<const uint4*>(x + (size_t)t * p.x_stride + at);
+        float wf[RW][8];
+#pragma unroll
+        for (int r = 0; r < RW; ++r) {
+            act2_to_f32<ACT_BF16>(wv[r].x, wf[r][0], wf[r][1]);
+            act2_to_f32<ACT_BF16>(wv[r].y, wf[r][2], wf[r][3]);
+            act2_to_f32<ACT_BF16>(wv[r].z, wf[r][4], wf[r][5]);
+            act2_to_f32<ACT_BF16>(wv[r].w, wf[r][6], wf[r][7]);
+        }
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            const uint4 q = live ? xv[t] : make_uint4(0u, 0u, 0u, 0u);
+            float xf[8];
+            act2_to_f32<ACT_BF16>(q.x, xf[0], xf[1]);
+            act2_to_f32<ACT_BF16>(q.y, xf[2], xf[3]);
+            act2_to_f32<ACT_BF16>(q.z, xf[4], xf[5]);
+            act2_to_f32<ACT_BF16>(q.w, xf[6], xf[7]);
+#pragma unroll
+            for (int r = 0; r < RW; ++r)
+#pragma unroll
+                for (int j = 0; j < 8; ++j) acc[t][r] = fmaf(wf[r][j], xf[j], acc[t][r]);
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+#pragma unroll
+        for (int r = 0; r < RW; ++r) {
+            const float v = wave_sum_bcast(acc[t][r]);
+            if (lane == (uint32_t)(t * RW + r) && r0 + r < p.n && (uint32_t)t < p.rows) dense_store<ACT_BF16>(p, t, r0 + r, v);
+        }
+}
+
+// ---- 5 .. 64 input rows: 16 weight rows per block, the waves split k, MFMA, sums through LDS ---------
+// Weight rows are the A operand as they lie in memory: lane (i = lane % 16, g = lane / 16) loads the 32 bytes
+// W[r0 + i, k + 16 g .. + 16), four lanes cover 128 contiguous bytes of a row; the inputs are the B operand in
+// the same order of k.
+template <int TT>
+__global__ __launch_bounds__(256) void dense_skinny_kernel(DenseLinearParams p) {
+    __shared__ __attribute__((aligned(16))) float part[3][64][TT * 4];
+    const uint32_t lane = threadIdx.x & 63u, wave = threadIdx.x >> 6, i = lane & 15u, g = lane >> 4;
+    const uint32_t r0 = blockIdx.x * 16u;
+    const uint16_t* wp = p.w + (size_t)min(r0 + i, p.n - 1u) * p.w_stride + g * 16u;
+    const uint16_t* x = static_cast<const uint16_t*>(p.x);
+    const uint16_t* xp[TT];
+#pragma unroll
+    for (int t = 0; t < TT; ++t) xp[t] = x + (size_t)min(16u * t + i, p.rows - 1u) * p.x_stride + g * 16u;
+    dn_f4 acc[TT];
+#pragma unroll
+    for (int t = 0; t < TT; ++t) acc[t] = dn_f4{0.0f, 0.0f, 0.0f, 0.0f};
+    const uint32_t steps = p.k / 64u;
+#pragma unroll 4
+    for (uint32_t st = wave; st < steps; st += 4u) {
+        const uint4 a0 = *reinterpret_cast<const uint4*>(wp + st * 64u), a1 = *reinterpret_cast<const uint4*>(wp + st * 64u + 8u);
+        uint4 b0[TT], b1[TT];
+#pragma unroll
+        for (int t = 0; t < TT; ++t) {
+            b0[t] = *reinterpret_cast<const uint4*>(xp[t] + st * 64u);
+            b1[t] = *reinterpret_cast<const uint4*>(xp[t] + st * 64u + 8u);
+        }
+#pragma unroll
+        for (int t = 0; t < TT; ++t) {
+            acc[t] = dn_mfma(a0, b0[t], acc[t]);
+            acc[t] = dn_mfma(a1, b1[t], acc[t]);
+        }
+    }
+    if (wave != 0) {
+#pragma unroll
+        for (int t = 0; t < TT; ++t) *reinterpret_cast<dn_f4*>(&part[wave - 1][lane][4 * t]) = acc[t];
+    }
+    __syncthreads();
+    if (wave != 0) return;
+#pragma unroll
+    for (int t = 0; t < TT; ++t) {
+#pragma unroll
+        for (int w = 0; w < 3; ++w) acc[t] += *reinterpret_cast<const dn_f4*>(&part[w][lane][4 * t]);
+        // acc[t][j] = y[token 16 t + i, row r0 + 4 g + j]
+        if (16u * t + i < p.rows) dense_store4_bf16(p, 16u * t + i, r0 + 4u * g, acc[t]);
+    }
+}
+
+// ---- many input rows: tiles of BN weight rows x BM tokens, k in steps of 64 through double-buffered LDS --------
+// Four waves, each a quarter of the tile (BN / 2 x BM / 2) in 16 x 16 x 32 products.  A tile's rows are 128 bytes
+// of LDS; the eight 16-byte pieces of row r lie in the order piece ^ (r % 8), so that the sixteen rows of an
+// operand read fall into different banks.  Loads go straight from memory into LDS.
+template <int BN, int BM>
+__global__ __launch_bounds__(256) void dense_gemm_kernel(DenseLinearParams p, uint32_t tiles_n, uint32_t tiles_m) {
+    constexpr int LA = BN / 32, LB = BM / 32;                // 1 KB pieces per wave
+    constexpr int TN = BN / 32, TM = BM / 32;                // 16 x 16 tiles per wave
+    constexpr uint32_t STAGE = (BN + BM) * 128u;
+    __shared__ __attribute__((aligned(16))) uint8_t lds[2 * STAGE];
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    // blocks are dealt to the eight XCDs in turn: give each XCD a run of neighbouring tiles (shared L2 lines)
+    const uint32_t total = tiles_n * tiles_m, xcd = blockIdx.x & 7u, nth = blockIdx.x >> 3;
+    const uint32_t base = total / 8u, extra = total % 8u;
+    const uint32_t tile = xcd * base + min(xcd, extra) + nth;
+    // in bands of eight token tiles, weight tiles outermost within the band
+    const uint32_t band = tile / (8u * tiles_n), in_band = tile % (8u * tiles_n);
+    const uint32_t band_m = min(8u, tiles_m - band * 8u);
+    const uint32_t m0 = (band * 8u + in_band % band_m) * BM, n0 = (in_band / band_m) * BN;
+
+    [[maybe_unused]] const __amdgpu_buffer_rsrc_t wrs = __builtin_amdgcn_make_buffer_rsrc(
+        const_cast<uint16_t*>(p.w), 0, (int)(uint32_t)((size_t)(p.n - 1u) * p.w_stride * 2u + p.k * 2u), 0x00020000);
+    [[maybe_unused]] const __amdgpu_buffer_rsrc_t xrs = __builtin_amdgcn_make_buffer_rsrc(
+        const_cast<void*>(p.x), 0, (int)(uint32_t)((size_t)(p.rows - 1u) * p.x_stride * 2u + p.k * 2u), 0x00020000);
+    uint32_t aoff[LA], boff[LB];
+    const uint32_t lr = lane >> 3, piece = (lane & 7u) ^ (lr & 7u);
+#pragma unroll
+    for (int j = 0; j < LA; ++j) aoff[j] = min(n0 + (wave * LA + j) * 8u + lr, p.n - 1u) * p.w_stride * 2u + piece * 16u;
+#pragma unroll
+    for (int j = 0; j < LB; ++j) boff[j] = min(m0 + (wave * LB + j) * 8u + lr, p.rows - 1u) * p.x_stride * 2u + piece * 16u;
+    auto issue = [&](uint32_t st, uint8_t* dst) {
+#if defined(__HIP_DEVICE_COMPILE__)     // the host pass rejects the 16-byte form of the load
+#pragma unroll
+        for (int j = 0; j < LA; ++j)
+            __builtin_amdgcn_raw_ptr_buffer_load_lds(wrs, (__attribute__((address_space(3))) void*)(dst + (wave * LA + j) * 1024u), 16, aoff[j], st * 128u, 0, 0);
+#pragma unroll
+        for (int j = 0; j < LB; ++j)
+            __builtin_amdgcn_raw_ptr_buffer_load_lds(xrs, (__attribute__((address_space(3))) void*)(dst + BN * 128u + (wave * LB + j) * 1024u), 16, boff[j], st * 128u, 0, 0);
+#endif
+    };
+    dn_f4 acc[TN][TM];
+#pragma unroll
+    for (int a = 0; a < TN; ++a)
+#pragma unroll
+        for (int b = 0; b < TM; ++b) acc[a][b] = dn_f4{0.0f, 0.0f, 0.0f, 0.0f};
+    const uint32_t i = lane & 15u, g = lane >> 4;
+    const uint32_t wn = (wave >> 1) * (BN / 2), wm = (wave & 1u) * (BM / 2);
+    const uint32_t steps = p.k / 64u;
+    issue(0, lds);
+    __syncthreads();
+    for (uint32_t st = 0; st < steps; ++st) {
+        uint8_t* cur = lds + (st & 1u) * STAGE;
+        if (st + 1u < steps) issue(st + 1u, lds + ((st + 1u) & 1u) * STAGE);
+#pragma unroll
+        for (uint32_t ks = 0; ks < 2; ++ks) {
+            const uint32_t sw = ((ks * 4u + g) ^ (i & 7u)) * 16u;
+            uint4 af[TN], bf[TM];
+#pragma unroll
+            for (int a = 0; a < TN; ++a) af[a] = *reinterpret_cast<const uint4*>(cur + (wn + 16 * a + i) * 128u + sw);
+#pragma unroll
+            for (int b = 0; b < TM; ++b) bf[b] = *reinterpret_cast<const uint4*>(cur + BN * 128u + (wm + 16 * b + i) * 128u + sw);
+#pragma unroll
+            for (int a = 0; a < TN; ++a)
+#pragma unroll
+                for (int b = 0; b < TM; ++b) acc[a][b] = dn_mfma(af[a], bf[b], acc[a][b]);
+        }
+        __syncthreads();                 // the next stage has landed, this one may be overwritten
+    }
+#pragma unroll
+    for (int b = 0; b < TM; ++b) {
+        const uint32_t t = m0 + wm + 16 * b + i;
+        if (t >= p.rows) continue;
+#pragma unroll
+        for (int a = 0; a < TN; ++a) {
+            const uint32_t r = n0 + wn + 16 * a + 4u * g;
+            if (r < p.n) dense_store4_bf16(p, t, r, acc[a][b]);
+        }
+    }
+}
+
+// ---- 32-bit activations: 64 x 64 tiles on the vector pipe, BF16 weights widened, fp32 FMA ------------
+// Sums are two-level (a step of 16 k, then the running total), which keeps the rounding error of a long k small.
+__global__ __launch_bounds__(256) void dense_f32_kernel(DenseLinearParams p) {
+    __shared__ float ws[16][65], xs[16][65];
+    const uint32_t tid = threadIdx.x, tx = tid & 15u, ty = tid >> 4;
+    const uint32_t n0 = blockIdx.x * 64u, m0 = blockIdx.y * 64u;
+    const float* x = static_cast<const float*>(p.x);
+    float acc[4][4] = {};
+    for (uint32_t k0 = 0; k0 < p.k; k0 += 16u) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const uint32_t r = (tid >> 4) + 16u * j, k = tid & 15u;
+            ws[k][r] = bf16_to_f32(p.w[(size_t)min(n0 + r, p.n - 1u) * p.w_stride + k0 + k]);
+            xs[k][r] = x[(size_t)min(m0 + r, p.rows - 1u) * p.x_stride + k0 + k];
+        }
+        __syncthreads();
+        float part[4][4] = {};
+#pragma unroll
+        for (int k = 0; k < 16; ++k) {
+            float a[4], b[4];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) { a[j] = xs[k][ty + 16 * j]; b[j] = ws[k][tx + 16 * j]; }
+#pragma unroll
+            for (int m = 0; m < 4; ++m)
+#pragma unroll
+                for (int n = 0; n < 4; ++n) part[m][n] = fmaf(a[m], b[n], part[m][n]);
+        }
+#pragma unroll
+        for (int m = 0; m < 4; ++m)
+#pragma unroll
+            for (int n = 0; n < 4; ++n) acc[m][n] += part[m][n];
+        __syncthreads();
+    }
+#pragma unroll
+    for (int m = 0; m < 4; ++m)
+#pragma unroll
+        for (int n = 0; n < 4; ++n) {
+            const uint32_t t = m0 + ty + 16u * m, r = n0 + tx + 16u * n;
+            if (t < p.rows && r < p.n) dense_store<ACT_FP32>(p, t, r, acc[m][n]);
+        }
+}
+
+// ---- norms over the 32-bit residual -----------------------------------------------------------------
+// Sum over the 256 threads of a block, every thread gets it.  `lds` holds four floats per call site.
+__device__ __forceinline__ float block_sum256(float v, float* lds) {
+    v = wave_sum_bcast(v);
+    if ((threadIdx.x & 63u) == 0) lds[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return (lds[0] + lds[1]) + (lds[2] + lds[3]);
+}
+
+// (v - mean) / sqrt(mean((v - mean)^2) + eps) over the d elements tid, tid + 256, ... held in v; dead slots are zero.
+template <int VPT>
+__device__ __forceinline__ void block_layernorm(float (&v)[VPT], uint32_t d, float eps, float* lds) {
+    float s = 0.0f;
+#pragma unroll
+    for (int j = 0; j < VPT; ++j) s += v[j];
+    const float mean = block_sum256(s, lds) / (float)d;
+    float q = 0.0f;
+#pragma unroll
+    for (int j = 0; j < VPT; ++j) {
+        const bool live = threadIdx.x + 256u * j < d;
+        v[j] = live ? v[j] - mean : 0.0f;
+        q = fmaf(v[j], v[j], q);
+    }
+    const float inv = 1.0f / sqrtf(block_sum256(q, lds + 4) / (float)d + eps);
+#pragma unroll
+    for (int j = 0; j < VPT; ++j) v[j] *= inv;
+}
+
+struct NormResidualParams {
+    float* x;                        // [rows, x_stride] residual stream
+    const float* delta;              // sublayer output, nullptr = none
+    const uint16_t *post_w, *post_b; // norm of delta, nullptr = delta is added as it is
+    const uint16_t *next_w, *next_b; // norm that opens the next sublayer, nullptr = no output
+    void* out;
+    uint32_t x_stride, delta_stride, out_stride, d;
+    float mult, eps;
+};
+
+// x += mult * LN(delta); out = LN(x): one block per row, the row in registers.
+template <int ACT, int VPT>
+__global__ __launch_bounds__(256) void norm_residual_kernel(NormResidualParams p) {
+    __shared__ float lds[16];
+    const uint32_t row = blockIdx.x, tid = threadIdx.x;
+    float* x = p.x + (size_t)row * p.x_stride;
+    float xv[VPT], dv[VPT], pw[VPT], pb[VPT], nw[VPT], nb[VPT];
+#pragma unroll
+    for (int j = 0; j < VPT; ++j) {          // every operand requested up front, dead slots reread the last element
+        const uint32_t at = min(tid + 256u * j, p.d - 1u);
+        xv[j] = x[at];
+        dv[j] = p.delta ? p.delta[(size_t)row * p.delta_stride + at] : 0.0f;
+        pw[j] = p.post_w ? bf16_to_f32(p.post_w[at]) : 1.0f;
+        pb[j] = p.post_b ? bf16_to_f32(p.post_b[at]) : 0.0f;
+        nw[j] = p.next_w ? bf16_to_f32(p.next_w[at]) : 1.0f;
+        nb[j] = p.next_b ? bf16_to_f32(p.next_b[at]) : 0.0f;
+    }
+#pragma unroll
+    for (int j = 0; j < VPT; ++j)
+        if (tid + 256u * j >= p.d) { xv[j] = 0.0f; dv[j] = 0.0f; }
+    if (p.delta) {
+        if (p.post_w) block_layernorm<VPT>(dv, p.d, p.eps, lds);
+#pragma unroll
+        for (int j = 0; j < VPT; ++j) {
+            const bool live = tid + 256u * j < p.d;
+            const float add = p.post_w ? fmaf(dv[j], pw[j], pb[j]) : dv[j];
+            xv[j] = live ? fmaf(p.mult, add, xv[j]) : 0.0f;
+            if (live) x[tid + 256u * j] = xv[j];
+        }
+    }
+    if (!p.next_w) return;
+    block_layernorm<VPT>(xv, p.d, p.eps, lds + 8);
+    act_t<ACT>* out = static_cast<act_t<ACT>*>(p.out) + (size_t)row * p.out_stride;
+#pragma unroll
+    for (int j = 0; j < VPT; ++j)
+        if (tid + 256u * j < p.d) out[tid + 256u * j] = f32_to_act<ACT>(fmaf(xv[j], nw[j], nb[j]));
+}
+
+// Rows of a BF16 table as 32-bit residual rows; an id past the table gives zeros.
+__global__ __launch_bounds__(256) void embed_rows_kernel(const uint16_t* table, uint32_t table_stride, const uint32_t* ids,
+                                                        float* out, uint32_t out_stride, uint32_t d, uint32_t vocab) {
+    const uint32_t row = blockIdx.y, j = blockIdx.x * 256u + threadIdx.x;
+    if (j >= d) return;
+    const uint32_t id = ids[row];
+    out[(size_t)row * out_stride + j] = id < vocab ? bf16_to_f32(table[(size_t)id * table_stride + j]) : 0.0f;
+}
+
+// Index of the largest finite value of each row, ties to the lower index, 0 when none is finite.
+__global__ __launch_bounds__(1024) void argmax_rows_kernel(const float* x, uint32_t x_stride, uint32_t n, uint32_t* out) {
+    __shared__ float bv[16];
+    __shared__ uint32_t bi[16];
+    const float* row = x + (size_t)blockIdx.x * x_stride;
+    float v = -INFINITY;
+    uint32_t at = 0xFFFFFFFFu;
+    for (uint32_t j = threadIdx.x; j < n; j += 1024u) {
+        const float c = row[j];
+        if (c > v && c < INFINITY) { v = c; at = j; }
+    }
+    const float wm = wave_max_f32(v);
+    const uint32_t wi = wave_min_u32(v == wm ? at : 0xFFFFFFFFu);
+    if ((threadIdx.x & 63u) == 0) { bv[threadIdx.x >> 6] = wm; bi[threadIdx.x >> 6] = wi; }
+    __syncthreads();
+    if (threadIdx.x != 0) return;
+    for (int w = 1; w < 16; ++w)
+        if (bv[w] > v || (bv[w] == v && bi[w] < at)) { v = bv[w]; at = bi[w]; }
+    if (bv[0] > v || (bv[0] == v && bi[0] < at)) { at = bi[0]; }
+    out[blockIdx.x] = at == 0xFFFFFFFFu ? 0u : at;
+}
+
+}  // namespace nvmai

@@ -58,7 +58,7 @@ int launch_delta_chunked(nvmai_hip_ctx* ctx, const GdnDeltaParams& p, bool state
     if (DK != 128 || DV != 128) return 0;
     const uint32_t nchunks = (p.sh.rows + 15) / 16;
     const size_t count = (size_t)p.sh.batch * p.sh.v_heads * nchunks;
-    if (!ctx || nchunks > 65535 || p.sh.batch > 65535 || (p.sh.rows + 1) / 2 > 65535 || !aligned16(p.conv_out) || p.conv_stride % 8 ||
+    if (!act16(ctx) || nchunks > 65535 || p.sh.batch > 65535 || (p.sh.rows + 1) / 2 > 65535 || !aligned16(p.conv_out) || p.conv_stride % 8 ||
         (!state_bf16 && !aligned16(p.state)) || (reinterpret_cast<uintptr_t>(p.state) & 7u))
         return 0;
     // BF16 activations: the chain on the 16-bit matrix instructions from operands prepared per chunk
@@ -125,7 +125,7 @@ int launch_delta_shape(nvmai_hip_ctx* ctx, const GdnDeltaParams& p, bool state_b
 extern "C" int nvmai_hip_gdn_conv_norm(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_gdn_config* config,
                                        const void* qkv_raw, uint32_t qkv_stride, void* tail, const uint16_t* conv_weight,
                                        void* conv_out, uint32_t conv_out_stride, uint32_t rows, uint32_t batch) {
-    if (!ctx || !qkv_raw || !tail || !conv_weight || !conv_out) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !qkv_raw || !tail || !conv_weight || !conv_out) return NVMAI_ERR_INVALID_ARG;
     int rc = check_gdn(config, rows, batch);
     if (rc) return rc;
     const uint32_t C = 2 * config->num_k_heads * config->key_head_dim + config->num_v_heads * config->value_head_dim;
@@ -173,7 +173,7 @@ extern "C" int nvmai_hip_gdn_delta_gated_norm(nvmai_hip_ctx* ctx, nvmai_stream s
                                               const uint16_t* dt_bias, void* state, int state_is_bf16, const void* z,
                                               uint32_t z_stride, const uint16_t* norm_weight, void* out,
                                               uint32_t out_stride, uint32_t rows, uint32_t batch) {
-    if (!ctx || !conv_out || !a_proj || !b_proj || !a_log || !dt_bias || !state || !z || !norm_weight || !out)
+    if (!act16(ctx) || !conv_out || !a_proj || !b_proj || !a_log || !dt_bias || !state || !z || !norm_weight || !out)
         return NVMAI_ERR_INVALID_ARG;
     int rc = check_gdn(config, rows, batch);
     if (rc) return rc;
@@ -226,7 +226,7 @@ extern "C" int nvmai_hip_gdn_decode_step(nvmai_hip_ctx* ctx, nvmai_stream stream
                                          const uint16_t* dt_bias, void* state, int state_is_bf16, const void* z,
                                          uint32_t z_stride, const uint16_t* norm_weight, void* out, uint32_t out_stride,
                                          uint32_t batch) {
-    if (!ctx || !qkv_raw || !tail || !conv_weight || !a_proj || !b_proj || !a_log || !dt_bias || !state || !z ||
+    if (!act16(ctx) || !qkv_raw || !tail || !conv_weight || !a_proj || !b_proj || !a_log || !dt_bias || !state || !z ||
         !norm_weight || !out)
         return NVMAI_ERR_INVALID_ARG;
     int rc = check_gdn(config, 1, batch);
@@ -261,7 +261,7 @@ extern "C" int nvmai_hip_gdn_decode_step(nvmai_hip_ctx* ctx, nvmai_stream stream
 extern "C" int nvmai_hip_affine_gemv_fused(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_gemv_part* parts,
                                            uint32_t n_parts, uint32_t bits, const void* x, uint32_t x_stride,
                                            uint32_t n_tokens, uint32_t n) {
-    if (!ctx || !parts || n_parts == 0 || !x) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !parts || n_parts == 0 || !x) return NVMAI_ERR_INVALID_ARG;
     if (bits != 4 && bits != 8) return NVMAI_ERR_UNSUPPORTED;
     if (n == 0 || n % NVMAI_GROUP) return NVMAI_ERR_INVALID_ARG;
     const uint64_t row_bytes = (uint64_t)n * bits / 8, meta_bytes = (uint64_t)(n / NVMAI_GROUP) * 2;

@@ -16,7 +16,7 @@ bool gemv_mfma_ok(const uint8_t* w, const uint16_t* s, const uint16_t* b, uint32
 int gemv_mfma(nvmai_hip_ctx* ctx, hipStream_t s, const uint8_t* w, const uint16_t* scales, const uint16_t* biases,
               uint32_t bits, const void* x, uint32_t x_stride, uint32_t n_tokens, uint32_t m, uint32_t n, void* y,
               float* y_f32, uint32_t y_stride) {
-    if (!ctx || !gemv_mfma_ok(w, scales, biases, bits, x, x_stride, n_tokens, m, n, y, y_f32, y_stride))
+    if (!act16(ctx) || !gemv_mfma_ok(w, scales, biases, bits, x, x_stride, n_tokens, m, n, y, y_f32, y_stride))
         return NVMAI_ERR_INVALID_ARG;
     GemvMfmaParams p{w, scales, biases, (const uint16_t*)x, x_stride, n_tokens, m, n, (uint16_t*)y, y_f32, y_stride};
     // rows per block: 64 for a large matrix, 32 or 16 where that would leave compute units without a block

@@ -1,0 +1,94 @@
+// Entry point of gated linear attention.
+#include "ctx.hpp"
+#include "gla_kernels.hpp"
+
+using namespace nvmai;
+
+namespace {
+
+template <int ACT>
+int gla_recurrent(const GlaParams& p, uint32_t batch, hipStream_t s) {
+    const uint32_t groups = 512u / p.dv, per = (p.dk + groups - 1) / groups;
+    const size_t lds = ((size_t)3 * p.dk + (size_t)groups * p.dv + 8 + p.rank) * 4;
+    if (lds > 64 * 1024) return NVMAI_ERR_UNSUPPORTED;
+    const dim3 grid(p.heads, batch);
+    if (per <= 8) gla_recurrent_kernel<ACT, 8><<<grid, 512, lds, s>>>(p);
+    else if (per <= 32) gla_recurrent_kernel<ACT, 32><<<grid, 512, lds, s>>>(p);
+    else gla_recurrent_kernel<ACT, 0><<<grid, 512, lds, s>>>(p);
+    return launch_status();
+}
+
+template <int ACT, int KT>
+void gla_spans(const GlaParams& p, uint32_t subs, uint32_t spans, hipStream_t s) {
+    const dim3 grid(spans, p.heads);
+    const uint32_t threads = p.dv * 4u;              // a wave per sixteen value columns
+    gla_span_kernel<ACT, KT, false><<<grid, threads, 0, s>>>(p);
+    gla_span_decay_kernel<<<dim3((p.heads * p.dk + 255) / 256, spans), 256, 0, s>>>(p, subs);
+    gla_scan_kernel<<<dim3((p.dk * p.dv / 4 + 255) / 256, p.heads), 256, 0, s>>>(p, spans);
+    gla_span_kernel<ACT, KT, true><<<grid, threads, 0, s>>>(p);
+}
+
+template <int ACT>
+int gla_chunked(const GlaParams& p, hipStream_t s) {
+    const uint32_t subs = (p.rows + GLA_SUB - 1) / GLA_SUB, spans = (subs + GLA_SPAN - 1) / GLA_SPAN;
+    const size_t lds = ((size_t)48 * (p.dk + 4) + (size_t)16 * p.rank) * 4;
+    static bool raised = false;
+    if (!raised) {
+        NVMAI_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void*>(gla_prep_kernel<ACT>), hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024));
+        raised = true;
+    }
+    if (lds > 128 * 1024) return NVMAI_ERR_UNSUPPORTED;
+    gla_prep_kernel<ACT><<<dim3(subs, p.heads), 256, lds, s>>>(p);
+    const uint32_t kt = (p.dk + 15) / 16;
+    if (kt <= 2) gla_spans<ACT, 2>(p, subs, spans, s);
+    else if (kt <= 4) gla_spans<ACT, 4>(p, subs, spans, s);
+    else if (kt <= 8) gla_spans<ACT, 8>(p, subs, spans, s);
+    else gla_spans<ACT, 16>(p, subs, spans, s);
+    return launch_status();
+}
+
+}  // namespace
+
+extern "C" int nvmai_hip_gla(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_gla_config* config, const void* q, const void* k,
+                             const void* v, const void* g, const void* a1, uint32_t proj_stride, const uint16_t* a2,
+                             const uint16_t* a2_bias, const uint16_t* norm_weight, float* state, const uint32_t* slots,
+                             uint32_t slot, void* out, uint32_t out_stride, uint32_t rows, uint32_t batch, int form) {
+    if (!ctx || !config || !q || !k || !v || !g || !a1 || !a2 || !a2_bias || !norm_weight || !state || !out) return NVMAI_ERR_INVALID_ARG;
+    if (ctx->act != NVMAI_ACT_BF16 && ctx->act != NVMAI_ACT_FP32) return NVMAI_ERR_UNSUPPORTED;
+    const nvmai_gla_config& c = *config;
+    if (c.heads == 0 || c.key_dim == 0 || c.value_dim == 0 || c.rank == 0 || c.value_count == 0 || c.value_count > c.value_dim) return NVMAI_ERR_INVALID_ARG;
+    if (c.key_dim % 16 || c.value_dim % 16 || c.rank % 8) return NVMAI_ERR_INVALID_ARG;
+    if (c.value_dim > 512) return NVMAI_ERR_UNSUPPORTED;
+    if (!(c.tau > 0.0f)) return NVMAI_ERR_INVALID_ARG;
+    if (proj_stride < c.heads * c.key_dim || proj_stride < c.heads * c.value_dim || proj_stride < c.rank || out_stride < c.heads * c.value_dim)
+        return NVMAI_ERR_INVALID_ARG;
+    if (!aligned16(a2) || !aligned16(state)) return NVMAI_ERR_ALIGNMENT;
+    if (form < NVMAI_FORM_AUTO || form > NVMAI_GLA_CHUNKED) return NVMAI_ERR_INVALID_ARG;
+    if (rows == 0 || batch == 0) return NVMAI_OK;
+    if (batch > 65535) return NVMAI_ERR_UNSUPPORTED;
+    GlaParams p{};
+    p.q = q; p.k = k; p.v = v; p.g = g; p.a1 = a1; p.a2 = a2; p.a2_bias = a2_bias; p.norm_weight = norm_weight;
+    p.state = state; p.slots = slots; p.slot0 = slot; p.out = out; p.proj_stride = proj_stride; p.out_stride = out_stride;
+    p.heads = c.heads; p.dk = c.key_dim; p.dv = c.value_dim; p.dv_count = c.value_count; p.rank = c.rank; p.rows = rows;
+    p.inv_tau = 1.0f / c.tau; p.q_scale = c.q_scale; p.eps = c.eps;
+    hipStream_t s = (hipStream_t)stream;
+    const bool can_chunk = batch == 1 && !slots && c.key_dim <= GLA_MAX_DIM && c.value_dim <= GLA_MAX_DIM && c.rank <= 512 &&
+                           (rows + GLA_SUB - 1) / GLA_SUB <= 0x7FFFFFFFu;
+    if (form == NVMAI_GLA_CHUNKED && !can_chunk) return NVMAI_ERR_UNSUPPORTED;
+    // below two spans' worth of rows the launches of the chunked form cost more than the rows
+    const bool chunk = form == NVMAI_GLA_CHUNKED || (form == NVMAI_FORM_AUTO && can_chunk && rows >= 32);
+    if (!chunk) return ctx->act == NVMAI_ACT_BF16 ? gla_recurrent<ACT_BF16>(p, batch, s) : gla_recurrent<ACT_FP32>(p, batch, s);
+    const size_t subs = (rows + GLA_SUB - 1) / GLA_SUB, spans = (subs + GLA_SPAN - 1) / GLA_SPAN;
+    if (spans > 65535) return NVMAI_ERR_UNSUPPORTED;
+    const size_t n_qd = subs * c.heads * 16 * c.key_dim, n_edge = subs * c.heads * c.key_dim, n_att = subs * c.heads * 256;
+    const size_t n_spans = spans * c.heads * c.key_dim * c.value_dim, n_dec = spans * c.heads * c.key_dim;
+    const int rc = ws_begin(ctx, stream, 2 * ws_round(n_qd * 4) + ws_round(n_edge * 4) + ws_round(n_att * 4) + ws_round(n_spans * 4) + ws_round(n_dec * 4));
+    if (rc) return rc;
+    p.qd = ws_take<float>(ctx, n_qd);
+    p.kd = ws_take<float>(ctx, n_qd);
+    p.edge = ws_take<float>(ctx, n_edge);
+    p.att = ws_take<float>(ctx, n_att);
+    p.spans = ws_take<float>(ctx, n_spans);
+    p.span_decay = ws_take<float>(ctx, n_dec);
+    return ctx->act == NVMAI_ACT_BF16 ? gla_chunked<ACT_BF16>(p, s) : gla_chunked<ACT_FP32>(p, s);
+}

@@ -1,0 +1,188 @@
+// Entry points of latent attention.
+#include "ctx.hpp"
+#include "dense_internal.hpp"
+#include "latent_kernels.hpp"
+
+using namespace nvmai;
+
+namespace {
+
+int check_config(const nvmai_hip_ctx* ctx, const nvmai_latent_config* c, const nvmai_latent_cache* cache) {
+    if (!ctx || !c || !cache || !cache->base) return NVMAI_ERR_INVALID_ARG;
+    if (ctx->act != NVMAI_ACT_BF16 && ctx->act != NVMAI_ACT_FP32) return NVMAI_ERR_UNSUPPORTED;
+    if (c->heads == 0 || c->nope_dim == 0 || c->value_dim == 0 || c->rank == 0) return NVMAI_ERR_INVALID_ARG;
+    if (c->nope_dim % 16 || c->rope_dim % 16 || c->value_dim % 16 || c->rank % 64) return NVMAI_ERR_INVALID_ARG;
+    if (c->rotary_dims > c->rope_dim || c->rotary_dims % 2 || (c->rotary_dims && !c->inv_freq)) return NVMAI_ERR_INVALID_ARG;
+    if (c->rank_count == 0 || c->rank_count > c->rank) return NVMAI_ERR_INVALID_ARG;
+    if (cache->row_stride < c->rank + c->rope_dim || cache->row_stride % 32 || cache->capacity < 64) return NVMAI_ERR_INVALID_ARG;
+    if (!aligned16(cache->base) || cache->slot_stride % 8 || cache->slot_stride < (uint64_t)cache->capacity * cache->row_stride) return NVMAI_ERR_ALIGNMENT;
+    return NVMAI_OK;
+}
+
+LatentRows rows_of(const nvmai_row_map* m) { return LatentRows{m->slots, m->positions, m->slot, m->position}; }
+LatentCache cache_of(const nvmai_latent_cache* c) { return LatentCache{c->base, c->slot_stride, c->row_stride, c->capacity}; }
+
+int raise_lds(const void* kernel, size_t bytes) {
+    if (bytes > 160 * 1024) return NVMAI_ERR_UNSUPPORTED;
+    if (bytes > 64 * 1024) NVMAI_HIP_TRY(hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes));
+    return NVMAI_OK;
+}
+
+template <int NT>
+int launch_partial(const LatentAttnParams& p, hipStream_t s) {
+    const size_t lds = (size_t)p.rank * 80;
+    const int rc = raise_lds(reinterpret_cast<const void*>(latent_partial_mfma_kernel<NT>), lds);
+    if (rc) return rc;
+    latent_partial_mfma_kernel<NT><<<dim3(p.splits, (p.heads + 15) / 16, p.n_rows), 256, lds, s>>>(p);
+    return NVMAI_OK;
+}
+
+template <int ACT>
+int absorbed(const LatentAttnParams& p, hipStream_t s) {
+    const size_t lds_a = ((size_t)p.nope + 4 * (size_t)p.rank) * 4;
+    int rc = raise_lds(reinterpret_cast<const void*>(latent_absorb_kernel<ACT>), lds_a);
+    if (rc) return rc;
+    latent_absorb_kernel<ACT><<<dim3(p.heads, p.n_rows), 256, lds_a, s>>>(p);
+    const uint32_t rest = p.cache.row_stride - p.rank;
+    if (ACT == ACT_BF16 && p.rank <= 1024 && rest <= 128) {
+        rc = p.rank <= 128 ? launch_partial<2>(p, s) : p.rank <= 256 ? launch_partial<4>(p, s) : p.rank <= 512 ? launch_partial<8>(p, s) : launch_partial<16>(p, s);
+    } else {
+        const size_t lds = ((size_t)p.cache.row_stride + p.rank + 256 + 8) * 4;
+        rc = raise_lds(reinterpret_cast<const void*>(latent_partial_plain_kernel<ACT>), lds);
+        if (!rc) latent_partial_plain_kernel<ACT><<<dim3(p.splits, p.heads, p.n_rows), 256, lds, s>>>(p);
+    }
+    if (rc) return rc;
+    const size_t lds_c = ((size_t)p.rank + p.splits) * 4;
+    rc = raise_lds(reinterpret_cast<const void*>(latent_combine_kernel<ACT>), lds_c);
+    if (rc) return rc;
+    const uint32_t slices = p.n_rows * p.heads >= 128 ? 1 : p.vdim >= 64 ? 4 : 1;
+    latent_combine_kernel<ACT><<<dim3(p.heads, p.n_rows, slices), 256, lds_c, s>>>(p);
+    return launch_status();
+}
+
+template <int DQ, int DV>
+void launch_flash(const LatentAttnParams& p, hipStream_t s) {
+    latent_flash_kernel<DQ, DV><<<dim3((p.n_rows + 127) / 128, p.heads), 256, 0, s>>>(p);
+}
+template <int DQ>
+void launch_flash_v(const LatentAttnParams& p, hipStream_t s) {
+    if (p.vdim <= 64) launch_flash<DQ, 64>(p, s);
+    else if (p.vdim <= 128) launch_flash<DQ, 128>(p, s);
+    else launch_flash<DQ, 256>(p, s);
+}
+
+}  // namespace
+
+extern "C" int nvmai_hip_latent_epilogue(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_latent_config* config, const void* proj,
+                                         uint32_t proj_stride, uint32_t q_at, uint32_t q_count, const uint16_t* q_norm,
+                                         uint32_t kv_at, uint32_t rope_at, const uint16_t* kv_norm, void* cq, uint32_t cq_stride,
+                                         const nvmai_latent_cache* cache, const nvmai_row_map* map, uint32_t rows) {
+    const int rc = check_config(ctx, config, cache);
+    if (rc) return rc;
+    const nvmai_latent_config& c = *config;
+    if (!proj || !q_norm || !kv_norm || !cq || !map || q_count == 0 || cq_stride < q_count) return NVMAI_ERR_INVALID_ARG;
+    if (proj_stride < q_at + q_count || proj_stride < kv_at + c.rank_count || proj_stride < rope_at + c.rope_dim) return NVMAI_ERR_INVALID_ARG;
+    if (!map->positions && rows > cache->capacity) return NVMAI_ERR_INVALID_ARG;       // two rows of one call in one place
+    if (rows == 0) return NVMAI_OK;
+    LatentEpilogueParams p{};
+    p.proj = proj; p.q_norm = q_norm; p.kv_norm = kv_norm; p.inv_freq = c.inv_freq; p.cq = cq; p.rows = rows_of(map); p.cache = cache_of(cache);
+    p.proj_stride = proj_stride; p.q_at = q_at; p.kv_at = kv_at; p.rot_at = rope_at; p.cq_stride = cq_stride; p.q_count = q_count;
+    p.rank_count = c.rank_count; p.rank = c.rank; p.rot_dim = c.rope_dim; p.rot_dims = c.rotary_dims; p.eps = c.eps;
+    hipStream_t s = (hipStream_t)stream;
+    if (ctx->act == NVMAI_ACT_BF16) latent_epilogue_kernel<ACT_BF16><<<rows, 256, 0, s>>>(p);
+    else latent_epilogue_kernel<ACT_FP32><<<rows, 256, 0, s>>>(p);
+    return launch_status();
+}
+
+extern "C" int nvmai_hip_latent_attention(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_latent_config* config, void* q,
+                                          uint32_t q_stride, const void* gate, uint32_t gate_stride, const uint16_t* uk,
+                                          const uint16_t* uv, const nvmai_latent_cache* cache, const nvmai_row_map* map, void* out,
+                                          uint32_t out_stride, uint32_t rows, int form) {
+    int rc = check_config(ctx, config, cache);
+    if (rc) return rc;
+    const nvmai_latent_config& c = *config;
+    if (!q || !uk || !uv || !map || !out) return NVMAI_ERR_INVALID_ARG;
+    if (q_stride < c.heads * (c.nope_dim + c.rope_dim) || out_stride < c.heads * c.value_dim || (gate && gate_stride < c.heads)) return NVMAI_ERR_INVALID_ARG;
+    if (!aligned16(q) || q_stride % 8 || !aligned16(out) || out_stride % 4 || !aligned16(uk) || !aligned16(uv)) return NVMAI_ERR_ALIGNMENT;
+    if (form < NVMAI_FORM_AUTO || form > NVMAI_LATENT_EXPANDED) return NVMAI_ERR_INVALID_ARG;
+    if ((map->slots == nullptr) != (map->positions == nullptr)) return NVMAI_ERR_INVALID_ARG;
+    if (rows == 0) return NVMAI_OK;
+    if (rows > 65535) return NVMAI_ERR_UNSUPPORTED;
+    const bool known = map->positions == nullptr;
+    // every key a row may look at has to be in the ring while the call runs
+    const uint32_t last = known ? map->position + rows : 0;
+    if (known) {
+        const uint64_t span = c.window ? (uint64_t)c.window + rows - 1 : (uint64_t)last;
+        if ((span < last ? span : last) > cache->capacity) return NVMAI_ERR_INVALID_ARG;
+    }
+    LatentAttnParams p{};
+    p.q = q; p.gate = gate; p.uk = uk; p.uv = uv; p.inv_freq = c.inv_freq; p.rows = rows_of(map); p.cache = cache_of(cache); p.out = out;
+    p.q_stride = q_stride; p.gate_stride = gate_stride; p.out_stride = out_stride; p.n_rows = rows; p.heads = c.heads; p.nope = c.nope_dim;
+    p.rot = c.rope_dim; p.vdim = c.value_dim; p.rank = c.rank; p.rot_dims = c.rotary_dims; p.window = c.window;
+    p.scale_log2 = c.scale * LA_LOG2E;
+    hipStream_t s = (hipStream_t)stream;
+    const bool f32 = ctx->act == NVMAI_ACT_FP32;
+    const size_t esz = f32 ? 4 : 2;
+    if (form == NVMAI_LATENT_EXPANDED && !known) return NVMAI_ERR_UNSUPPORTED;
+    const bool expand = form == NVMAI_LATENT_EXPANDED || (form == NVMAI_FORM_AUTO && known && rows >= 32);
+    if (!expand) {
+        uint32_t keys = known ? last : cache->capacity;
+        if (c.window && c.window < keys) keys = c.window;
+        // about four blocks per compute unit, at least 64 keys each
+        const uint32_t groups = f32 ? c.heads : (c.heads + 15) / 16;
+        const uint32_t want = 4u * (uint32_t)ctx->compute_units / (rows * groups) + 1u;
+        uint32_t per = ((keys + want - 1) / want + 31) / 32 * 32;
+        if (per < 64) per = 64;
+        p.split_keys = per;
+        p.splits = (keys + per - 1) / per;
+        const size_t cells = (size_t)rows * c.heads * p.splits, n_qa = (size_t)rows * c.heads * cache->row_stride;
+        rc = ws_begin(ctx, stream, ws_round(n_qa * esz) + ws_round(cells * c.rank * 4) + 2 * ws_round(cells * 4));
+        if (rc) return rc;
+        p.qa = ws_take<uint8_t>(ctx, n_qa * esz);
+        p.part_o = ws_take<float>(ctx, cells * c.rank);
+        p.part_m = ws_take<float>(ctx, cells);
+        p.part_l = ws_take<float>(ctx, cells);
+        return f32 ? absorbed<ACT_FP32>(p, s) : absorbed<ACT_BF16>(p, s);
+    }
+    p.key0 = c.window && map->position + 1 > c.window ? map->position + 1 - c.window : 0;
+    p.nk = last - p.key0;
+    p.nk_pad = (p.nk + 63) / 64 * 64;
+    const uint32_t dq = c.nope_dim + c.rope_dim;
+    const bool flash = !f32 && dq <= 256 && c.value_dim <= 256;
+    const size_t n_lat = (size_t)p.nk_pad * cache->row_stride, n_kn = (size_t)p.nk_pad * c.heads * c.nope_dim, n_v = (size_t)p.nk_pad * c.heads * c.value_dim;
+    rc = ws_begin(ctx, stream, ws_round(n_lat * esz) + ws_round(n_kn * esz) + ws_round(n_v * esz));
+    if (rc) return rc;
+    p.lat = ws_take<uint8_t>(ctx, n_lat * esz);
+    p.kn = ws_take<uint8_t>(ctx, n_kn * esz);
+    p.v = ws_take<uint8_t>(ctx, n_v * esz);
+    const uint32_t nh = c.heads * c.nope_dim, vh = c.heads * c.value_dim;
+    const DenseLinearParams lk{uk, p.lat, p.kn, nullptr, c.rank, cache->row_stride, nh, p.nk_pad, nh, c.rank, NVMAI_LINEAR_NONE};
+    const DenseLinearParams lv = flash ? DenseLinearParams{static_cast<const uint16_t*>(p.lat), uv, p.v, nullptr, cache->row_stride, c.rank, p.nk_pad, vh, p.nk_pad, c.rank, NVMAI_LINEAR_NONE}
+                                       : DenseLinearParams{uv, p.lat, p.v, nullptr, c.rank, cache->row_stride, vh, p.nk_pad, vh, c.rank, NVMAI_LINEAR_NONE};
+    if ((rc = dense_linear_check(ctx, lk)) || (rc = dense_linear_check(ctx, lv))) return rc;
+    const size_t lds_rot = (size_t)c.rotary_dims * 4;
+    if (f32) {
+        latent_gather_kernel<ACT_FP32><<<p.nk_pad, 256, 0, s>>>(p);
+        if (c.rotary_dims) latent_rotate_q_kernel<ACT_FP32><<<rows, 256, lds_rot, s>>>(p);
+    } else {
+        latent_gather_kernel<ACT_BF16><<<p.nk_pad, 256, 0, s>>>(p);
+        if (c.rotary_dims) latent_rotate_q_kernel<ACT_BF16><<<rows, 256, lds_rot, s>>>(p);
+    }
+    if ((rc = dense_linear(ctx, s, lk)) || (rc = dense_linear(ctx, s, lv))) return rc;
+    if (!flash) {
+        const size_t lds = ((size_t)dq + c.value_dim + 256 + 8) * 4;
+        if (f32) {
+            if ((rc = raise_lds(reinterpret_cast<const void*>(latent_expanded_plain_kernel<ACT_FP32>), lds))) return rc;
+            latent_expanded_plain_kernel<ACT_FP32><<<dim3(c.heads, rows), 256, lds, s>>>(p);
+        } else {
+            if ((rc = raise_lds(reinterpret_cast<const void*>(latent_expanded_plain_kernel<ACT_BF16>), lds))) return rc;
+            latent_expanded_plain_kernel<ACT_BF16><<<dim3(c.heads, rows), 256, lds, s>>>(p);
+        }
+        return launch_status();
+    }
+    if (dq <= 64) launch_flash_v<64>(p, s);
+    else if (dq <= 128) launch_flash_v<128>(p, s);
+    else if (dq <= 192) launch_flash_v<192>(p, s);
+    else launch_flash_v<256>(p, s);
+    return launch_status();
+}

@@ -1,0 +1,657 @@
+// Latent attention: keys and values are linear images of one cached latent per position, plus one rotated key part
+// that all heads share.  gfx950, wave64.
+//
+//   score(h, i, j) = scale * (q_n(h, i) . W_uk(h) c_j + q_r(h, i) . k_r(j)),   window: 0 <= i - j < window
+//   out(h, i)      = sigmoid(gate(h, i)) * W_uv(h) sum_j softmax_j(score) c_j
+//
+// A cache row holds [c | rotated key part | zeros], row stride `row_stride`.  Two forms of the same sum:
+//   * absorbed, for decoding and short portions: q_n is taken through W_uk(h)^T once, every head then reads the
+//     latents themselves (each cache row is fetched once per sixteen heads), W_uv(h) is applied to the sum;
+//   * expanded, for prompts: keys and values of the range are formed by two matrix products, then flash attention.
+#pragma once
+
+#include "common.hpp"
+
+namespace nvmai {
+
+typedef __bf16 la_b8 __attribute__((ext_vector_type(8)));
+typedef float la_f4 __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ la_f4 la_mfma(const uint4& a, const uint4& b, la_f4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(la_b8, a), __builtin_bit_cast(la_b8, b), c, 0, 0, 0);
+}
+
+constexpr float LA_LOG2E = 1.4426950408889634f;
+constexpr float LA_NONE = -1e30f;        // maximum of no scores
+
+// Where a row's token sits: by arrays (a decode batch) or consecutive from (slot, position) (a prompt's portion).
+struct LatentRows {
+    const uint32_t *slots, *positions;
+    uint32_t slot, position;
+    __device__ __forceinline__ uint32_t slot_of(uint32_t r) const { return slots ? slots[r] : slot; }
+    __device__ __forceinline__ uint32_t position_of(uint32_t r) const { return positions ? positions[r] : position + r; }
+};
+
+struct LatentCache {
+    void* base;
+    uint64_t slot_stride;    // elements
+    uint32_t row_stride, capacity;
+};
+
+// (cos, sin) of position * inv_freq with the angle reduced in double: exact to fp32 at any position.
+__device__ __forceinline__ void la_rotation(uint32_t position, double inv_freq, float& c, float& s) {
+    double a = (double)position * inv_freq;
+    a -= 6.283185307179586476925 * rint(a * 0.15915494309189533577);
+    sincosf((float)a, &s, &c);
+}
+
+__device__ __forceinline__ float la_block_sum(float v, float* lds) {
+    v = wave_sum_bcast(v);
+    if ((threadIdx.x & 63u) == 0) lds[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return (lds[0] + lds[1]) + (lds[2] + lds[3]);
+}
+
+__device__ __forceinline__ float la_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+
+// ---- after the down projections: both latents normed, the key part rotated, the cache row written ---------
+struct LatentEpilogueParams {
+    const void* proj;                    // [rows, proj_stride]: [W_dq h | W_dkv h: latent, rotated part]
+    const uint16_t *q_norm, *kv_norm;
+    const double* inv_freq;              // [rot_dims / 2]
+    void* cq;                            // [rows, cq_stride]
+    LatentRows rows;
+    LatentCache cache;
+    uint32_t proj_stride, q_at, kv_at, rot_at, cq_stride, q_count, rank_count, rank, rot_dim, rot_dims;
+    float eps;
+};
+
+template <int ACT>
+__global__ __launch_bounds__(256) void latent_epilogue_kernel(LatentEpilogueParams p) {
+    __shared__ float lds[8];
+    const uint32_t row = blockIdx.x, tid = threadIdx.x;
+    const act_t<ACT>* proj = static_cast<const act_t<ACT>*>(p.proj) + (size_t)row * p.proj_stride;
+    const uint32_t position = p.rows.position_of(row);
+    act_t<ACT>* out = static_cast<act_t<ACT>*>(p.cache.base) + (size_t)p.rows.slot_of(row) * p.cache.slot_stride +
+                      (size_t)(position % p.cache.capacity) * p.cache.row_stride;
+    float qs = 0.0f, ks = 0.0f;
+    for (uint32_t j = tid; j < p.q_count; j += 256u) { const float v = act_to_f32<ACT>(proj[p.q_at + j]); qs = fmaf(v, v, qs); }
+    for (uint32_t j = tid; j < p.rank_count; j += 256u) { const float v = act_to_f32<ACT>(proj[p.kv_at + j]); ks = fmaf(v, v, ks); }
+    const float qi = 1.0f / sqrtf(la_block_sum(qs, lds) / (float)p.q_count + p.eps);
+    const float ki = 1.0f / sqrtf(la_block_sum(ks, lds + 4) / (float)p.rank_count + p.eps);
+    act_t<ACT>* cq = static_cast<act_t<ACT>*>(p.cq) + (size_t)row * p.cq_stride;
+    for (uint32_t j = tid; j < p.q_count; j += 256u) cq[j] = f32_to_act<ACT>(act_to_f32<ACT>(proj[p.q_at + j]) * qi * bf16_to_f32(p.q_norm[j]));
+    for (uint32_t j = tid; j < p.rank_count; j += 256u) out[j] = f32_to_act<ACT>(act_to_f32<ACT>(proj[p.kv_at + j]) * ki * bf16_to_f32(p.kv_norm[j]));
+    const uint32_t half = p.rot_dims / 2u;
+    for (uint32_t j = tid; j < p.rot_dim; j += 256u) {
+        if (j < half) {
+            float c, s;
+            la_rotation(position, p.inv_freq[j], c, s);
+            const float u = act_to_f32<ACT>(proj[p.rot_at + j]), v = act_to_f32<ACT>(proj[p.rot_at + half + j]);
+            out[p.rank + j] = f32_to_act<ACT>(u * c - v * s);
+            out[p.rank + half + j] = f32_to_act<ACT>(v * c + u * s);
+        } else if (j >= p.rot_dims) {
+            out[p.rank + j] = proj[p.rot_at + j];
+        }
+    }
+}
+
+struct LatentAttnParams {
+    const void* q;                       // [rows, q_stride]: head by head [nope | rot], not yet rotated
+    const void* gate;                    // [rows, gate_stride]: one logit per head, nullptr = no gate
+    const uint16_t *uk, *uv;             // [heads * nope, rank], [heads * vdim, rank] BF16
+    const double* inv_freq;
+    LatentRows rows;
+    LatentCache cache;
+    void* out;                           // [rows, out_stride]: head by head [vdim]
+    uint32_t q_stride, gate_stride, out_stride, n_rows, heads, nope, rot, vdim, rank, rot_dims, window;
+    float scale_log2;                    // scale * log2(e)
+    // absorbed form
+    void* qa;                            // [rows, heads, row_stride]
+    float *part_o, *part_m, *part_l;     // [rows, heads, splits, rank], [rows, heads, splits] x 2
+    uint32_t splits, split_keys;
+    // expanded form
+    void *lat, *kn, *v;                  // [nk_pad, row_stride], [nk_pad, heads * nope], V (or V^T [heads * vdim, nk_pad])
+    uint32_t nk, nk_pad, key0;           // keys of the call, the position of the first
+};
+
+__device__ __forceinline__ uint32_t la_first_key(uint32_t position, uint32_t window) {
+    return window != 0u && position + 1u > window ? position + 1u - window : 0u;
+}
+
+// ---- absorbed: q_n -> W_uk(h)^T q_n, q_r rotated ----------------------------------------------------
+// A block per (head, row): the waves split the rows of W_uk(h), a lane owns eight latent dims per 512.
+template <int ACT>
+__global__ __launch_bounds__(256) void latent_absorb_kernel(LatentAttnParams p) {
+    extern __shared__ __attribute__((aligned(16))) float la_lds[];
+    const uint32_t head = blockIdx.x, row = blockIdx.y, tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6;
+    float* qs = la_lds;                  // [nope]
+    float* part = qs + p.nope;           // [4][rank]
+    const act_t<ACT>* q = static_cast<const act_t<ACT>*>(p.q) + (size_t)row * p.q_stride + head * (p.nope + p.rot);
+    for (uint32_t d = tid; d < p.nope; d += 256u) qs[d] = act_to_f32<ACT>(q[d]);
+    act_t<ACT>* out = static_cast<act_t<ACT>*>(p.qa) + ((size_t)row * p.heads + head) * p.cache.row_stride;
+    const uint32_t position = p.rows.position_of(row), half = p.rot_dims / 2u;
+    for (uint32_t j = tid; j < p.cache.row_stride - p.rank; j += 256u) {
+        if (j < half) {
+            float c, s;
+            la_rotation(position, p.inv_freq[j], c, s);
+            const float u = act_to_f32<ACT>(q[p.nope + j]), v = act_to_f32<ACT>(q[p.nope + half + j]);
+            out[p.rank + j] = f32_to_act<ACT>(u * c - v * s);
+            out[p.rank + half + j] = f32_to_act<ACT>(v * c + u * s);
+        } else if (j >= p.rot_dims) {
+            out[p.rank + j] = j < p.rot ? q[p.nope + j] : f32_to_act<ACT>(0.0f);
+        }
+    }
+    __syncthreads();
+    for (uint32_t c0 = 0; c0 < p.rank; c0 += 512u) {
+        const uint32_t r = c0 + lane * 8u;
+        if (r < p.rank) {
+            float acc[8] = {};
+            const uint16_t* uk = p.uk + (size_t)head * p.nope * p.rank + r;
+#pragma unroll 8
+            for (uint32_t d = wave; d < p.nope; d += 4u) {
+                const uint4 w = *reinterpret_cast<const uint4*>(uk + (size_t)d * p.rank);
+                float f[8];
+                act2_to_f32<ACT_BF16>(w.x, f[0], f[1]);
+                act2_to_f32<ACT_BF16>(w.y, f[2], f[3]);
+                act2_to_f32<ACT_BF16>(w.z, f[4], f[5]);
+                act2_to_f32<ACT_BF16>(w.w, f[6], f[7]);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) acc[e] = fmaf(f[e], qs[d], acc[e]);
+            }
+#pragma unroll
+            for (int e = 0; e < 8; ++e) part[wave * p.rank + r + e] = acc[e];
+        }
+    }
+    __syncthreads();
+    for (uint32_t r = tid; r < p.rank; r += 256u)
+        out[r] = f32_to_act<ACT>((part[r] + part[p.rank + r]) + (part[2u * p.rank + r] + part[3u * p.rank + r]));
+}
+
+// ---- absorbed: scores and sums over one split of the window, sixteen heads per block --------------------
+// Per 32 keys: S^T[key, head] = K Q^T with the waves splitting the row's elements (cache rows are the A operand as
+// they lie in memory), the partial scores summed through LDS, the softmax in registers, and
+// O^T[latent, head] += C^T P^T with the waves splitting the latent.  C^T comes from LDS: a thread transposes four
+// keys x eight latents on the way in.  The score registers of a lane are the B operand of the second product when
+// its eight keys are read as 4 g .. 4 g + 3 and 16 + 4 g .. 16 + 4 g + 3, so the columns of C^T lie in that order.
+// P enters as two BF16 halves (hi + lo): fp32 weights.
+template <int NT>
+__global__ __launch_bounds__(256) void latent_partial_mfma_kernel(LatentAttnParams p) {
+    constexpr int NQ = (2 * NT + 7) / 4;             // 32-element steps of a row per wave: rank <= 64 NT, rest <= 128
+    constexpr int NV = (NT + 3) / 4;                 // transposed units per thread
+    extern __shared__ __attribute__((aligned(16))) float la_lds[];
+    uint16_t* ct = reinterpret_cast<uint16_t*>(la_lds);      // [rank][40]: 32 keys, rows 16 bytes off a power of two
+    __shared__ __attribute__((aligned(16))) float sc[4][16][36];
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, i = lane & 15u, g = lane >> 4;
+    const uint32_t split = blockIdx.x, h0 = blockIdx.y * 16u, row = blockIdx.z;
+    const uint32_t position = p.rows.position_of(row), first = la_first_key(position, p.window);
+    const uint32_t lo = first + split * p.split_keys, hi = min(position + 1u, lo + p.split_keys);
+    const uint32_t head = min(h0 + i, p.heads - 1u);
+    const size_t cell = ((size_t)row * p.heads + head) * p.splits + split;
+    if (lo >= hi) {                                  // uniform
+        if (tid < 16u && h0 + tid < p.heads) { p.part_m[cell] = LA_NONE; p.part_l[cell] = 0.0f; }
+        return;
+    }
+    const uint32_t rs = p.cache.row_stride, steps = rs / 32u, tiles = p.rank / 16u;
+    const uint16_t* cache = static_cast<const uint16_t*>(p.cache.base) + (size_t)p.rows.slot_of(row) * p.cache.slot_stride;
+    const uint16_t* q = static_cast<const uint16_t*>(p.qa) + ((size_t)row * p.heads + head) * rs;
+    uint4 qf[NQ];
+#pragma unroll
+    for (int n = 0; n < NQ; ++n) qf[n] = *reinterpret_cast<const uint4*>(q + min(wave + 4u * n, steps - 1u) * 32u + 8u * g);
+    la_f4 acc[NT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n) acc[n] = la_f4{0.0f, 0.0f, 0.0f, 0.0f};
+    float m = LA_NONE, l = 0.0f;
+    const uint32_t units = p.rank;                   // 8 groups of four keys x rank / 8 pieces
+    for (uint32_t k0 = lo; k0 < hi; k0 += 32u) {
+        const uint32_t ring0 = k0 % p.cache.capacity, most = hi - 1u - k0;
+        auto row_of = [&](uint32_t key) {            // keys past the split repeat its last one
+            uint32_t r = ring0 + min(key, most);
+            r -= r >= p.cache.capacity ? p.cache.capacity : 0u;
+            return cache + (size_t)r * rs;
+        };
+        uint4 vv[NV][4];
+#pragma unroll
+        for (int n = 0; n < NV; ++n) {
+            const uint32_t u = min(tid + 256u * n, units - 1u), kg = u & 7u, piece = u >> 3;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) vv[n][e] = *reinterpret_cast<const uint4*>(row_of(4u * kg + e) + piece * 8u);
+        }
+        const uint16_t *ka = row_of(i) + 8u * g, *kb = row_of(16u + i) + 8u * g;
+        la_f4 s0 = la_f4{0.0f, 0.0f, 0.0f, 0.0f}, s1 = s0;
+        uint4 fa[NQ], fb[NQ];
+#pragma unroll
+        for (int n = 0; n < NQ; ++n) {
+            const uint32_t at = min(wave + 4u * n, steps - 1u) * 32u;
+            fa[n] = *reinterpret_cast<const uint4*>(ka + at);
+            fb[n] = *reinterpret_cast<const uint4*>(kb + at);
+        }
+#pragma unroll
+        for (int n = 0; n < NQ; ++n)
+            if (wave + 4u * n < steps) {             // uniform
+                s0 = la_mfma(fa[n], qf[n], s0);
+                s1 = la_mfma(fb[n], qf[n], s1);
+            }
+        *reinterpret_cast<la_f4*>(&sc[wave][i][4u * g]) = s0;
+        *reinterpret_cast<la_f4*>(&sc[wave][i][16u + 4u * g]) = s1;
+#pragma unroll
+        for (int n = 0; n < NV; ++n) {
+            const uint32_t u = tid + 256u * n, kg = u & 7u, piece = u >> 3;
+            if (u < units) {
+                const uint32_t at = kg < 4u ? 8u * kg : 8u * (kg - 4u) + 4u;
+                const uint32_t a[4][4] = {{vv[n][0].x, vv[n][0].y, vv[n][0].z, vv[n][0].w}, {vv[n][1].x, vv[n][1].y, vv[n][1].z, vv[n][1].w},
+                                          {vv[n][2].x, vv[n][2].y, vv[n][2].z, vv[n][2].w}, {vv[n][3].x, vv[n][3].y, vv[n][3].z, vv[n][3].w}};
+#pragma unroll
+                for (int e = 0; e < 8; ++e) {
+                    const uint32_t sel = (e & 1) ? 0x07060302u : 0x05040100u;     // high or low halves of two dwords
+                    uint2 w;
+                    w.x = __builtin_amdgcn_perm(a[1][e >> 1], a[0][e >> 1], sel);
+                    w.y = __builtin_amdgcn_perm(a[3][e >> 1], a[2][e >> 1], sel);
+                    *reinterpret_cast<uint2*>(&ct[(piece * 8u + e) * 40u + at]) = w;
+                }
+            }
+        }
+        __syncthreads();
+        float s[8];
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+            la_f4 v = *reinterpret_cast<const la_f4*>(&sc[0][i][16 * h + 4u * g]);
+#pragma unroll
+            for (int w = 1; w < 4; ++w) v += *reinterpret_cast<const la_f4*>(&sc[w][i][16 * h + 4u * g]);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) s[4 * h + j] = k0 + 16u * h + 4u * g + j < hi ? v[j] * p.scale_log2 : LA_NONE;
+        }
+        float tm = s[0];
+#pragma unroll
+        for (int j = 1; j < 8; ++j) tm = fmaxf(tm, s[j]);
+        tm = fmaxf(tm, shfl_xor_f(tm, 16));
+        tm = fmaxf(tm, shfl_xor_f(tm, 32));
+        const float mn = fmaxf(m, tm), alpha = __builtin_amdgcn_exp2f(m - mn);
+        m = mn;
+        float ts = 0.0f;
+        uint16_t ph[8], pl[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+            const float e = s[j] > LA_NONE ? __builtin_amdgcn_exp2f(s[j] - mn) : 0.0f;
+            ts += e;
+            ph[j] = f32_to_bf16(e);
+            pl[j] = f32_to_bf16(e - bf16_to_f32(ph[j]));
+        }
+        ts += shfl_xor_f(ts, 16);
+        ts += shfl_xor_f(ts, 32);
+        l = fmaf(l, alpha, ts);
+        uint4 bh, bl;
+        bh.x = ph[0] | ((uint32_t)ph[1] << 16); bh.y = ph[2] | ((uint32_t)ph[3] << 16);
+        bh.z = ph[4] | ((uint32_t)ph[5] << 16); bh.w = ph[6] | ((uint32_t)ph[7] << 16);
+        bl.x = pl[0] | ((uint32_t)pl[1] << 16); bl.y = pl[2] | ((uint32_t)pl[3] << 16);
+        bl.z = pl[4] | ((uint32_t)pl[5] << 16); bl.w = pl[6] | ((uint32_t)pl[7] << 16);
+#pragma unroll
+        for (int n = 0; n < NT; ++n) {
+            const uint32_t tile = wave + 4u * n;
+            if (tile < tiles) {                      // uniform
+                const uint4 a = *reinterpret_cast<const uint4*>(&ct[(16u * tile + i) * 40u + 8u * g]);
+                acc[n] *= alpha;
+                acc[n] = la_mfma(a, bh, acc[n]);
+                acc[n] = la_mfma(a, bl, acc[n]);
+            }
+        }
+        __syncthreads();
+    }
+    if (h0 + i >= p.heads) return;
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+        const uint32_t tile = wave + 4u * n;
+        if (tile < tiles) *reinterpret_cast<la_f4*>(p.part_o + cell * p.rank + 16u * tile + 4u * g) = acc[n];
+    }
+    if (wave == 0 && g == 0) { p.part_m[cell] = m; p.part_l[cell] = l; }
+}
+
+// One query row against keys [lo, hi) in blocks of 256, a thread per key, any sizes: the plain form behind both
+// kernels below.  dot(key) is the score without scale, value(key, j) one value element; acc (LDS, [vd]) receives
+// sum p v, and every thread the maximum and the sum.
+template <typename Dot, typename Value>
+__device__ __forceinline__ void la_plain_rows(uint32_t lo, uint32_t hi, uint32_t vd, float scale_log2, float* acc, float* ps,
+                                              float* red, float& m, float& l, Dot dot, Value value) {
+    const uint32_t tid = threadIdx.x;
+    m = LA_NONE;
+    l = 0.0f;
+    for (uint32_t j = tid; j < vd; j += 256u) acc[j] = 0.0f;
+    for (uint32_t k0 = lo; k0 < hi; k0 += 256u) {
+        const uint32_t key = k0 + tid;
+        const float s = key < hi ? dot(key) * scale_log2 : LA_NONE;
+        const float wm = wave_max_f32(s);
+        __syncthreads();                             // the previous block's ps and red have been read
+        if ((tid & 63u) == 0) red[tid >> 6] = wm;
+        __syncthreads();
+        const float mn = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), m), alpha = __builtin_amdgcn_exp2f(m - mn);
+        m = mn;
+        const float e = key < hi ? __builtin_amdgcn_exp2f(s - mn) : 0.0f;
+        ps[tid] = e;
+        const float ws = wave_sum_bcast(e);
+        if ((tid & 63u) == 0) red[4 + (tid >> 6)] = ws;
+        __syncthreads();
+        l = fmaf(l, alpha, (red[4] + red[5]) + (red[6] + red[7]));
+        const uint32_t n = min(256u, hi - k0);
+        for (uint32_t j = tid; j < vd; j += 256u) {
+            float a = acc[j] * alpha;
+            for (uint32_t k = 0; k < n; ++k) a = fmaf(ps[k], value(k0 + k, j), a);
+            acc[j] = a;
+        }
+    }
+    __syncthreads();
+}
+
+template <int ACT>
+__global__ __launch_bounds__(256) void latent_partial_plain_kernel(LatentAttnParams p) {
+    extern __shared__ __attribute__((aligned(16))) float la_lds[];
+    const uint32_t tid = threadIdx.x, split = blockIdx.x, head = blockIdx.y, row = blockIdx.z, rs = p.cache.row_stride;
+    float *qs = la_lds, *acc = qs + rs, *ps = acc + p.rank, *red = ps + 256;
+    const uint32_t position = p.rows.position_of(row), first = la_first_key(position, p.window);
+    const uint32_t lo = first + split * p.split_keys, hi = min(position + 1u, lo + p.split_keys);
+    const size_t cell = ((size_t)row * p.heads + head) * p.splits + split;
+    if (lo >= hi) {
+        if (tid == 0) { p.part_m[cell] = LA_NONE; p.part_l[cell] = 0.0f; }
+        return;
+    }
+    const act_t<ACT>* q = static_cast<const act_t<ACT>*>(p.qa) + ((size_t)row * p.heads + head) * rs;
+    for (uint32_t j = tid; j < rs; j += 256u) qs[j] = act_to_f32<ACT>(q[j]);
+    __syncthreads();
+    const act_t<ACT>* cache = static_cast<const act_t<ACT>*>(p.cache.base) + (size_t)p.rows.slot_of(row) * p.cache.slot_stride;
+    float m, l;
+    la_plain_rows(lo, hi, p.rank, p.scale_log2, acc, ps, red, m, l,
+        [&](uint32_t key) {
+            const act_t<ACT>* k = cache + (size_t)(key % p.cache.capacity) * rs;
+            float s = 0.0f;
+            for (uint32_t j = 0; j < p.rank + p.rot; ++j) s = fmaf(act_to_f32<ACT>(k[j]), qs[j], s);
+            return s;
+        },
+        [&](uint32_t key, uint32_t j) { return act_to_f32<ACT>(cache[(size_t)(key % p.cache.capacity) * rs + j]); });
+    for (uint32_t j = tid; j < p.rank; j += 256u) p.part_o[cell * p.rank + j] = acc[j];
+    if (tid == 0) { p.part_m[cell] = m; p.part_l[cell] = l; }
+}
+
+// ---- absorbed: splits combined, W_uv(h), the output gate ------------------------------------------------
+// Grid (heads, rows, slices of the value rows).
+template <int ACT>
+__global__ __launch_bounds__(256) void latent_combine_kernel(LatentAttnParams p) {
+    extern __shared__ __attribute__((aligned(16))) float la_lds[];
+    const uint32_t head = blockIdx.x, row = blockIdx.y, tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6;
+    float* o = la_lds;                   // [rank]
+    float* wt = o + p.rank;              // [splits]
+    const size_t cell = ((size_t)row * p.heads + head) * p.splits;
+    const float gate = p.gate ? la_sigmoid(act_to_f32<ACT>(static_cast<const act_t<ACT>*>(p.gate)[(size_t)row * p.gate_stride + head])) : 1.0f;
+    float m = LA_NONE;
+    for (uint32_t s = lane; s < p.splits; s += 64u) m = fmaxf(m, p.part_m[cell + s]);
+    m = wave_max_f32(m);
+    float l = 0.0f;
+    for (uint32_t s = lane; s < p.splits; s += 64u) {
+        const float ls = p.part_l[cell + s];
+        const float w = ls > 0.0f ? __builtin_amdgcn_exp2f(p.part_m[cell + s] - m) : 0.0f;
+        l = fmaf(ls, w, l);
+        if (wave == 0) wt[s] = w;
+    }
+    l = wave_sum_bcast(l);
+    const float inv = 1.0f / l;
+    __syncthreads();
+    // splits past the last key of this row wrote no sums and weigh nothing: the live ones are a prefix
+    const uint32_t first = la_first_key(p.rows.position_of(row), p.window);
+    const uint32_t live = min(p.splits, (p.rows.position_of(row) + 1u - first + p.split_keys - 1u) / p.split_keys);
+    for (uint32_t r = tid * 4u; r < p.rank; r += 1024u) {
+        la_f4 a = la_f4{0.0f, 0.0f, 0.0f, 0.0f};
+        const float* po = p.part_o + cell * p.rank + r;
+#pragma unroll 8
+        for (uint32_t s = 0; s < live; ++s) a += *reinterpret_cast<const la_f4*>(po + (size_t)s * p.rank) * wt[s];
+        *reinterpret_cast<la_f4*>(o + r) = a * inv;
+    }
+    __syncthreads();
+    const uint32_t per = (p.vdim + gridDim.z - 1u) / gridDim.z, j1 = min(p.vdim, (blockIdx.z + 1u) * per);
+#pragma unroll 4
+    for (uint32_t j = blockIdx.z * per + wave; j < j1; j += 4u) {
+        const uint16_t* uv = p.uv + (size_t)(head * p.vdim + j) * p.rank;
+        float a = 0.0f;
+        for (uint32_t r = lane * 8u; r < p.rank; r += 512u) {
+            const uint4 w = *reinterpret_cast<const uint4*>(uv + r);
+            float f[8];
+            act2_to_f32<ACT_BF16>(w.x, f[0], f[1]);
+            act2_to_f32<ACT_BF16>(w.y, f[2], f[3]);
+            act2_to_f32<ACT_BF16>(w.z, f[4], f[5]);
+            act2_to_f32<ACT_BF16>(w.w, f[6], f[7]);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) a = fmaf(f[e], o[r + e], a);
+        }
+        a = wave_sum_bcast(a);
+        if (lane == 0) static_cast<act_t<ACT>*>(p.out)[(size_t)row * p.out_stride + head * p.vdim + j] = f32_to_act<ACT>(a * gate);
+    }
+}
+
+// ---- expanded: the range's cache rows gathered from the ring, queries rotated in place --------------------
+template <int ACT>
+__global__ __launch_bounds__(256) void latent_gather_kernel(LatentAttnParams p) {
+    constexpr uint32_t PER = 16u / sizeof(act_t<ACT>);
+    const uint32_t key = blockIdx.x, pieces = p.cache.row_stride / PER;
+    const act_t<ACT>* src = static_cast<const act_t<ACT>*>(p.cache.base) + (size_t)p.rows.slot * p.cache.slot_stride +
+                            (size_t)((p.key0 + min(key, p.nk - 1u)) % p.cache.capacity) * p.cache.row_stride;
+    act_t<ACT>* dst = static_cast<act_t<ACT>*>(p.lat) + (size_t)key * p.cache.row_stride;
+    for (uint32_t j = threadIdx.x; j < pieces; j += 256u) {
+        const uint4 v = reinterpret_cast<const uint4*>(src)[j];
+        reinterpret_cast<uint4*>(dst)[j] = key < p.nk ? v : make_uint4(0u, 0u, 0u, 0u);
+    }
+}
+
+template <int ACT>
+__global__ __launch_bounds__(256) void latent_rotate_q_kernel(LatentAttnParams p) {
+    const uint32_t row = blockIdx.x, half = p.rot_dims / 2u, position = p.rows.position + row;
+    extern __shared__ __attribute__((aligned(16))) float la_lds[];      // [half] cos, [half] sin
+    for (uint32_t j = threadIdx.x; j < half; j += 256u) la_rotation(position, p.inv_freq[j], la_lds[j], la_lds[half + j]);
+    __syncthreads();
+    act_t<ACT>* q = static_cast<act_t<ACT>*>(const_cast<void*>(p.q)) + (size_t)row * p.q_stride;
+    for (uint32_t e = threadIdx.x; e < p.heads * half; e += 256u) {
+        const uint32_t head = e / half, j = e % half;
+        act_t<ACT>* r = q + head * (p.nope + p.rot) + p.nope + j;
+        const float u = act_to_f32<ACT>(r[0]), v = act_to_f32<ACT>(r[half]), c = la_lds[j], s = la_lds[half + j];
+        r[0] = f32_to_act<ACT>(u * c - v * s);
+        r[half] = f32_to_act<ACT>(v * c + u * s);
+    }
+}
+
+template <int ACT>
+__global__ __launch_bounds__(256) void latent_expanded_plain_kernel(LatentAttnParams p) {
+    extern __shared__ __attribute__((aligned(16))) float la_lds[];
+    const uint32_t tid = threadIdx.x, head = blockIdx.x, row = blockIdx.y, dq = p.nope + p.rot;
+    float *qs = la_lds, *acc = qs + dq, *ps = acc + p.vdim, *red = ps + 256;
+    const act_t<ACT>* q = static_cast<const act_t<ACT>*>(p.q) + (size_t)row * p.q_stride + head * dq;
+    for (uint32_t j = tid; j < dq; j += 256u) qs[j] = act_to_f32<ACT>(q[j]);
+    __syncthreads();
+    const uint32_t position = p.rows.position + row, lo = la_first_key(position, p.window) - p.key0, hi = position + 1u - p.key0;
+    const act_t<ACT>*kn = static_cast<const act_t<ACT>*>(p.kn), *lat = static_cast<const act_t<ACT>*>(p.lat), *v = static_cast<const act_t<ACT>*>(p.v);
+    float m, l;
+    la_plain_rows(lo, hi, p.vdim, p.scale_log2, acc, ps, red, m, l,
+        [&](uint32_t key) {
+            const act_t<ACT>* a = kn + (size_t)key * p.heads * p.nope + head * p.nope;
+            const act_t<ACT>* b = lat + (size_t)key * p.cache.row_stride + p.rank;
+            float s = 0.0f;
+            for (uint32_t j = 0; j < p.nope; ++j) s = fmaf(act_to_f32<ACT>(a[j]), qs[j], s);
+            for (uint32_t j = 0; j < p.rot; ++j) s = fmaf(act_to_f32<ACT>(b[j]), qs[p.nope + j], s);
+            return s;
+        },
+        [&](uint32_t key, uint32_t j) { return act_to_f32<ACT>(v[(size_t)key * p.heads * p.vdim + head * p.vdim + j]); });
+    const float gate = p.gate ? la_sigmoid(act_to_f32<ACT>(static_cast<const act_t<ACT>*>(p.gate)[(size_t)row * p.gate_stride + head])) : 1.0f;
+    for (uint32_t j = tid; j < p.vdim; j += 256u)
+        static_cast<act_t<ACT>*>(p.out)[(size_t)row * p.out_stride + head * p.vdim + j] = f32_to_act<ACT>(acc[j] / l * gate);
+}
+
+// ---- expanded: flash attention over a window, BF16 -------------------------------------------------------
+// 128 queries of one head per block, 32 per wave; keys and V^T in tiles of 64 keys through LDS, the next tile's
+// loads in flight under the current tile's products.  S^T[key, query] = K Q^T and O^T[value, query] += V^T P^T: the
+// score registers are the B operand of the second product (see above for the order of the keys in V^T's columns).
+// DQ: query/key dims, DV: value dims, both padded with zeros in LDS.
+template <int DQ, int DV>
+__global__ __launch_bounds__(256) void latent_flash_kernel(LatentAttnParams p) {
+    constexpr int KS = DQ / 32, KU = DQ / 32, VU = DV / 32, NV = DV / 16;
+    constexpr uint32_t KLD = DQ + 8, VLD = 72;
+    __shared__ __attribute__((aligned(16))) uint16_t kt[64 * KLD];
+    __shared__ __attribute__((aligned(16))) uint16_t vt[DV * VLD];
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, i = lane & 15u, g = lane >> 4;
+    const uint32_t head = blockIdx.y, qb = gridDim.x - 1u - blockIdx.x;      // the blocks with the most keys first
+    const uint32_t q0 = qb * 128u, dq = p.nope + p.rot;
+    const uint16_t* q = static_cast<const uint16_t*>(p.q) + head * dq;
+    uint4 qf[2][KS];
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+        const uint32_t t = min(q0 + wave * 32u + 16u * b + i, p.n_rows - 1u);
+#pragma unroll
+        for (int s = 0; s < KS; ++s) {
+            const uint32_t d = 32u * s + 8u * g;
+            const uint4 v = *reinterpret_cast<const uint4*>(q + (size_t)t * p.q_stride + min(d, dq - 8u));
+            qf[b][s] = d < dq ? v : make_uint4(0u, 0u, 0u, 0u);
+        }
+    }
+    la_f4 acc[2][NV];
+    float m[2] = {LA_NONE, LA_NONE}, l[2] = {0.0f, 0.0f};
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int n = 0; n < NV; ++n) acc[b][n] = la_f4{0.0f, 0.0f, 0.0f, 0.0f};
+    // keys are numbered from key0
+    const uint32_t last_t = min(q0 + 127u, p.n_rows - 1u);
+    const uint32_t k_lo = (la_first_key(p.rows.position + q0, p.window) - p.key0) & ~63u;
+    const uint32_t k_hi = p.rows.position + last_t + 1u - p.key0;
+    const uint16_t *kn = static_cast<const uint16_t*>(p.kn) + head * p.nope, *kr = static_cast<const uint16_t*>(p.lat) + p.rank;
+    const uint16_t* v = static_cast<const uint16_t*>(p.v) + (size_t)head * p.vdim * p.nk_pad;
+    const uint32_t kn_stride = p.heads * p.nope;
+    uint4 kreg[KU], vreg[VU];
+    auto fetch = [&](uint32_t k0) {
+#pragma unroll
+        for (int n = 0; n < KU; ++n) {
+            const uint32_t u = tid + 256u * n, key = k0 + u / (DQ / 8u), d = (u % (DQ / 8u)) * 8u;
+            const uint32_t dc = min(d, dq - 8u);
+            const uint16_t* src = dc < p.nope ? kn + (size_t)key * kn_stride + dc : kr + (size_t)key * p.cache.row_stride + (dc - p.nope);
+            const uint4 w = *reinterpret_cast<const uint4*>(src);
+            kreg[n] = d < dq ? w : make_uint4(0u, 0u, 0u, 0u);
+        }
+#pragma unroll
+        for (int n = 0; n < VU; ++n) {
+            const uint32_t u = tid + 256u * n, d = u >> 3, piece = u & 7u;
+            const uint4 w = *reinterpret_cast<const uint4*>(v + (size_t)min(d, p.vdim - 1u) * p.nk_pad + k0 + piece * 8u);
+            vreg[n] = d < p.vdim ? w : make_uint4(0u, 0u, 0u, 0u);
+        }
+    };
+    fetch(k_lo);
+    // this wave's own range of keys
+    const uint32_t wt0 = q0 + wave * 32u, wt1 = min(wt0 + 31u, p.n_rows - 1u);
+    const bool wave_live = wt0 < p.n_rows;
+    const uint32_t w_lo = la_first_key(p.rows.position + wt0, p.window) - p.key0, w_hi = p.rows.position + wt1 + 1u - p.key0;
+    // a tile needs no mask when every query of the wave sees all of it
+    const uint32_t full_lo = la_first_key(p.rows.position + wt1, p.window) - p.key0, full_hi = p.rows.position + wt0 + 1u - p.key0;
+    for (uint32_t k0 = k_lo; k0 < k_hi; k0 += 64u) {
+        __syncthreads();
+#pragma unroll
+        for (int n = 0; n < KU; ++n) {
+            const uint32_t u = tid + 256u * n;
+            *reinterpret_cast<uint4*>(&kt[(u / (DQ / 8u)) * KLD + (u % (DQ / 8u)) * 8u]) = kreg[n];
+        }
+#pragma unroll
+        for (int n = 0; n < VU; ++n) {
+            const uint32_t u = tid + 256u * n, d = u >> 3, piece = u & 7u;      // keys 8 piece .. 8 piece + 7
+            const uint32_t kg = (2u * piece) & 7u, at = (piece >> 2) * 32u + (kg < 4u ? 8u * kg : 8u * (kg - 4u) + 4u);
+            *reinterpret_cast<uint2*>(&vt[d * VLD + at]) = make_uint2(vreg[n].x, vreg[n].y);
+            *reinterpret_cast<uint2*>(&vt[d * VLD + at + 8u]) = make_uint2(vreg[n].z, vreg[n].w);
+        }
+        __syncthreads();
+        if (k0 + 64u < k_hi) fetch(k0 + 64u);
+        if (!wave_live || k0 >= w_hi || k0 + 64u <= w_lo) continue;             // wave-uniform
+        la_f4 s[2][4];
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+            for (int t = 0; t < 4; ++t) s[b][t] = la_f4{0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+        for (int st = 0; st < KS; ++st)
+#pragma unroll
+            for (int t = 0; t < 4; ++t) {
+                const uint4 a = *reinterpret_cast<const uint4*>(&kt[(16 * t + i) * KLD + 32 * st + 8u * g]);
+#pragma unroll
+                for (int b = 0; b < 2; ++b) s[b][t] = la_mfma(a, qf[b][st], s[b][t]);
+            }
+        const bool masked = k0 < full_lo || k0 + 64u > full_hi;
+        uint4 pf[2][2];
+#pragma unroll
+        for (int b = 0; b < 2; ++b) {
+            if (masked) {
+                const uint32_t pos = p.rows.position + min(wt0 + 16u * b + i, p.n_rows - 1u);
+                const uint32_t lo = la_first_key(pos, p.window) - p.key0, hi = pos + 1u - p.key0;
+#pragma unroll
+                for (int t = 0; t < 4; ++t)
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) {
+                        const uint32_t key = k0 + 16u * t + 4u * g + j;
+                        s[b][t][j] = key >= lo && key < hi ? s[b][t][j] * p.scale_log2 : LA_NONE;
+                    }
+            } else {
+#pragma unroll
+                for (int t = 0; t < 4; ++t) s[b][t] *= p.scale_log2;
+            }
+            float tm = s[b][0][0];
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) tm = fmaxf(tm, s[b][t][j]);
+            tm = fmaxf(tm, shfl_xor_f(tm, 16));
+            tm = fmaxf(tm, shfl_xor_f(tm, 32));
+            if (__any(tm > m[b])) {
+                const float mn = fmaxf(m[b], tm), alpha = __builtin_amdgcn_exp2f(m[b] - mn);
+                m[b] = mn;
+                l[b] *= alpha;
+#pragma unroll
+                for (int n = 0; n < NV; ++n) acc[b][n] *= alpha;
+            }
+            uint32_t w[8];
+#pragma unroll
+            for (int t = 0; t < 4; ++t) {
+                float e[4];
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    e[j] = __builtin_amdgcn_exp2f(s[b][t][j] - m[b]);
+                    if (masked && s[b][t][j] <= LA_NONE) e[j] = 0.0f;           // a query without a key so far: m is LA_NONE too
+                    l[b] += e[j];
+                }
+                w[2 * t] = f32_to_bf16(e[0]) | ((uint32_t)f32_to_bf16(e[1]) << 16);
+                w[2 * t + 1] = f32_to_bf16(e[2]) | ((uint32_t)f32_to_bf16(e[3]) << 16);
+            }
+            pf[b][0] = make_uint4(w[0], w[1], w[2], w[3]);
+            pf[b][1] = make_uint4(w[4], w[5], w[6], w[7]);
+        }
+#pragma unroll
+        for (int h = 0; h < 2; ++h)
+#pragma unroll
+            for (int n = 0; n < NV; ++n) {
+                const uint4 a = *reinterpret_cast<const uint4*>(&vt[(16 * n + i) * VLD + 32 * h + 8u * g]);
+#pragma unroll
+                for (int b = 0; b < 2; ++b) acc[b][n] = la_mfma(a, pf[b][h], acc[b][n]);
+            }
+    }
+    if (!wave_live) return;
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+        float sum = l[b];
+        sum += shfl_xor_f(sum, 16);
+        sum += shfl_xor_f(sum, 32);
+        const uint32_t t = wt0 + 16u * b + i;
+        if (t >= p.n_rows) continue;
+        const float gate = p.gate ? la_sigmoid(bf16_to_f32(static_cast<const uint16_t*>(p.gate)[(size_t)t * p.gate_stride + head])) : 1.0f;
+        const float f = gate / sum;
+        uint16_t* out = static_cast<uint16_t*>(p.out) + (size_t)t * p.out_stride + head * p.vdim;
+#pragma unroll
+        for (int n = 0; n < NV; ++n) {
+            const uint32_t d = 16u * n + 4u * g;
+            if (d < p.vdim) {
+                uint2 w;
+                w.x = f32_to_bf16(acc[b][n][0] * f) | ((uint32_t)f32_to_bf16(acc[b][n][1] * f) << 16);
+                w.y = f32_to_bf16(acc[b][n][2] * f) | ((uint32_t)f32_to_bf16(acc[b][n][3] * f) << 16);
+                *reinterpret_cast<uint2*>(out + d) = w;
+            }
+        }
+    }
+}
+
+}  // namespace nvmai

@@ -1,145 +1,12 @@
-// Entry points of the decode-side MoE path: context, quantizer, affine GEMV,
+// Entry points of the decode-side MoE path: quantizer, affine GEMV,
 // router top-k, routed phase 1 / phase 2, shared expert, fused decode layer.
-#include <atomic>
 #include <cstdio>
 #include <cstdlib>
-#include <new>
 
 #include "ctx.hpp"
 #include "moe_kernels.hpp"
 
 using namespace nvmai;
-
-namespace {
-
-// Scratch of the allocation-free decode entry point: one array per device, in the library's image,
-// so that a caller which may not allocate (HIP graph capture, a serving loop, a harness that
-// forbids hipMalloc) still has the step's intermediate buffers.  Host code never uses the
-// array's name as an address: the device address comes from hipGetSymbolAddress, once per device.
-constexpr size_t STATIC_SCRATCH_BYTES = (size_t)4 << 20;
-static __device__ __align__(256) __attribute__((used)) uint8_t scratch[STATIC_SCRATCH_BYTES];
-constexpr int STATIC_SCRATCH_MAX_DEVICES = 64;
-// Device address of `scratch` on each device, nullptr = not asked yet.  Contexts may be created from several
-// threads: the slots are atomics (every thread that fills one stores the same address, so no lock is needed).
-std::atomic<uint8_t*> g_static_scratch[STATIC_SCRATCH_MAX_DEVICES];
-
-// The device address of this device's copy of the array (the device must be current).
-int static_scratch_ptr(int device, uint8_t** out) {
-    if (device < 0 || device >= STATIC_SCRATCH_MAX_DEVICES) return NVMAI_ERR_INVALID_ARG;
-    uint8_t* known = g_static_scratch[device].load(std::memory_order_acquire);
-    if (!known) {
-        void* ptr = nullptr;
-        if (hipGetSymbolAddress(&ptr, HIP_SYMBOL(scratch)) != hipSuccess || !ptr) {
-            (void)hipGetLastError();
-            return NVMAI_ERR_HIP;
-        }
-        known = static_cast<uint8_t*>(ptr);
-        g_static_scratch[device].store(known, std::memory_order_release);
-    }
-    *out = known;
-    return NVMAI_OK;
-}
-
-}  // namespace
-
-// ---------------------------------------------------------------------------
-// context
-// ---------------------------------------------------------------------------
-extern "C" int nvmai_hip_ctx_create(int device, int act_dtype, nvmai_hip_ctx** out) {
-    if (!out || (act_dtype != NVMAI_ACT_BF16 && act_dtype != NVMAI_ACT_FP16)) return NVMAI_ERR_INVALID_ARG;
-    int count = 0;
-    if (hipGetDeviceCount(&count) != hipSuccess || count <= 0) return NVMAI_ERR_NO_DEVICE;
-    if (device < 0 || device >= count) return NVMAI_ERR_INVALID_ARG;
-    NVMAI_HIP_TRY(hipSetDevice(device));
-    nvmai_hip_ctx* ctx = new (std::nothrow) nvmai_hip_ctx();
-    if (!ctx) return NVMAI_ERR_HIP;
-    ctx->device = device;
-    ctx->compute_units = 256;
-    {
-        int cus = 0;
-        if (hipDeviceGetAttribute(&cus, hipDeviceAttributeMultiprocessorCount, device) == hipSuccess && cus > 0)
-            ctx->compute_units = cus;
-    }
-    ctx->act = act_dtype;
-    ctx->ws = nullptr;
-    ctx->ws_cap = 0;
-    ctx->ws_used = 0;
-    ctx->prof_on = false;
-    ctx->tickets = nullptr;
-    if (hipMalloc(reinterpret_cast<void**>(&ctx->tickets), TICKET_WORDS * 4) != hipSuccess ||
-        hipMemset(ctx->tickets, 0, TICKET_WORDS * 4) != hipSuccess) {
-        delete ctx;
-        return NVMAI_ERR_HIP;
-    }
-    // device address of this device's static scratch array (nullptr if the lookup fails: only the
-    // allocation-free entry point needs it, and it then reports the failure)
-    ctx->static_scratch = nullptr;
-    (void)static_scratch_ptr(device, &ctx->static_scratch);
-    *out = ctx;
-    return NVMAI_OK;
-}
-
-extern "C" void nvmai_hip_ctx_destroy(nvmai_hip_ctx* ctx) {
-    if (!ctx) return;
-    if (ctx->ws) (void)hipFree(ctx->ws);
-    for (void* block : ctx->ws_retired) (void)hipFree(block);
-    if (ctx->tickets) (void)hipFree(ctx->tickets);
-    for (auto& sp : ctx->prof_spans) { (void)hipEventDestroy(sp.start); (void)hipEventDestroy(sp.stop); }
-    for (auto& e : ctx->prof_free) (void)hipEventDestroy(e);
-    delete ctx;
-}
-
-extern "C" int nvmai_hip_ctx_reserve(nvmai_hip_ctx* ctx, size_t bytes) {
-    if (!ctx) return NVMAI_ERR_INVALID_ARG;
-    NVMAI_HIP_TRY(hipSetDevice(ctx->device));
-    return ws_begin(ctx, nullptr, bytes);
-}
-
-extern "C" size_t nvmai_hip_ctx_workspace_bytes(const nvmai_hip_ctx* ctx) { return ctx ? ctx->ws_cap : 0; }
-
-extern "C" int nvmai_hip_profile_enable(nvmai_hip_ctx* ctx, int on) {
-    if (!ctx) return NVMAI_ERR_INVALID_ARG;
-    if (on) {
-        for (auto& sp : ctx->prof_spans) {
-            NVMAI_HIP_TRY(hipEventSynchronize(sp.stop));
-            ctx->prof_free.push_back(sp.start);
-            ctx->prof_free.push_back(sp.stop);
-        }
-        ctx->prof_spans.clear();
-    }
-    ctx->prof_on = on != 0;
-    return NVMAI_OK;
-}
-
-extern "C" int nvmai_hip_profile_read(nvmai_hip_ctx* ctx, int tag, double* total_ms, uint32_t* launches) {
-    if (!ctx || !total_ms || !launches) return NVMAI_ERR_INVALID_ARG;
-    double total = 0.0;
-    uint32_t n = 0;
-    for (auto& sp : ctx->prof_spans) {
-        if (sp.tag != tag) continue;
-        NVMAI_HIP_TRY(hipEventSynchronize(sp.stop));
-        float ms = 0.0f;
-        NVMAI_HIP_TRY(hipEventElapsedTime(&ms, sp.start, sp.stop));
-        total += ms;
-        ++n;
-    }
-    *total_ms = total;
-    *launches = n;
-    return NVMAI_OK;
-}
-
-extern "C" const char* nvmai_hip_status_string(int status) {
-    switch (status) {
-        case NVMAI_OK: return "ok";
-        case NVMAI_ERR_INVALID_ARG: return "invalid argument";
-        case NVMAI_ERR_UNSUPPORTED: return "unsupported configuration";
-        case NVMAI_ERR_ALIGNMENT: return "pointer or stride not 16-byte aligned";
-        case NVMAI_ERR_SCRATCH: return "scratch too small";
-        case NVMAI_ERR_HIP: return "HIP runtime error";
-        case NVMAI_ERR_NO_DEVICE: return "no HIP device";
-        default: return "unknown status";
-    }
-}
 
 extern "C" int nvmai_expert_offsets_for(uint32_t d, uint32_t f, uint32_t bits,
                                         nvmai_expert_offsets* out, uint64_t* stride_bytes) {
@@ -510,7 +377,7 @@ void launch_down_combine(int act, uint32_t bits, const DownCombineParams& p, hip
 extern "C" int nvmai_hip_quantize_affine(nvmai_hip_ctx* ctx, nvmai_stream stream, const void* w,
                                          int w_is_bf16, uint32_t rows, uint32_t n, uint32_t bits,
                                          uint8_t* packed, uint16_t* scales, uint16_t* biases) {
-    if (!ctx || !w || !packed || !scales || !biases) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !w || !packed || !scales || !biases) return NVMAI_ERR_INVALID_ARG;
     if (bits != 4 && bits != 8) return NVMAI_ERR_UNSUPPORTED;
     if (n == 0 || n % NVMAI_GROUP) return NVMAI_ERR_INVALID_ARG;
     if (rows == 0) return NVMAI_OK;
@@ -524,7 +391,7 @@ extern "C" int nvmai_hip_dequantize_affine(nvmai_hip_ctx* ctx, nvmai_stream stre
                                            const uint8_t* packed, const uint16_t* scales,
                                            const uint16_t* biases, uint64_t count, uint32_t bits,
                                            uint8_t* codes_out, void* values_out) {
-    if (!ctx || !packed) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !packed) return NVMAI_ERR_INVALID_ARG;
     if (bits != 4 && bits != 8) return NVMAI_ERR_UNSUPPORTED;
     if (values_out && (!scales || !biases)) return NVMAI_ERR_INVALID_ARG;
     if (count % NVMAI_GROUP) return NVMAI_ERR_INVALID_ARG;
@@ -547,7 +414,7 @@ int affine_gemv_any(nvmai_hip_ctx* ctx, nvmai_stream stream, const uint8_t* weig
                     const uint16_t* scales, const uint16_t* biases, uint32_t bits, const void* x,
                     bool x_is_f32, uint32_t x_stride, uint32_t n_tokens, uint32_t m, uint32_t n, void* y,
                     float* y_f32, uint32_t y_stride) {
-    if (!ctx || !weights || !scales || !biases || !x || (!y && !y_f32)) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !weights || !scales || !biases || !x || (!y && !y_f32)) return NVMAI_ERR_INVALID_ARG;
     if (bits != 4 && bits != 8) return NVMAI_ERR_UNSUPPORTED;
     if (n == 0 || n % NVMAI_GROUP || x_stride < n || y_stride < m) return NVMAI_ERR_INVALID_ARG;
     if (!aligned16(weights) || !aligned16(x) || (x_stride % 8)) return NVMAI_ERR_ALIGNMENT;
@@ -601,7 +468,7 @@ extern "C" int nvmai_hip_affine_gemv(nvmai_hip_ctx* ctx, nvmai_stream stream, co
                                      uint32_t m, uint32_t n, void* y, float* y_f32,
                                      uint32_t y_stride) {
     if (bits == 16) {                     // dense BF16 rows: the BF16 LM head
-        if (!ctx || !weights || !x || (!y && !y_f32)) return NVMAI_ERR_INVALID_ARG;
+        if (!act16(ctx) || !weights || !x || (!y && !y_f32)) return NVMAI_ERR_INVALID_ARG;
         return nvmai::dense_bf16_gemv(ctx, (hipStream_t)stream, reinterpret_cast<const uint16_t*>(weights), x, x_stride,
                                       n_tokens, m, n, y, y_f32, y_stride);
     }
@@ -662,7 +529,7 @@ extern "C" int nvmai_hip_affine_gemv_prenorm(nvmai_hip_ctx* ctx, nvmai_stream st
                                              void* hidden_out, uint32_t hidden_out_stride, void* normed_scratch,
                                              uint32_t normed_stride, uint32_t n_tokens, uint32_t m, uint32_t n, void* y,
                                              uint32_t y_stride) {
-    if (!ctx || !weights || !scales || !biases || !hidden || !norm_weight || !hidden_out || !y) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !weights || !scales || !biases || !hidden || !norm_weight || !hidden_out || !y) return NVMAI_ERR_INVALID_ARG;
     if (bits != 4 && bits != 8) return NVMAI_ERR_UNSUPPORTED;
     if (n == 0 || n % NVMAI_GROUP || hidden_stride < n || hidden_out_stride < n || (delta && delta_stride < n) || y_stride < m)
         return NVMAI_ERR_INVALID_ARG;
@@ -751,7 +618,7 @@ extern "C" int nvmai_hip_moe_router_topk(nvmai_hip_ctx* ctx, nvmai_stream stream
                                          const uint16_t* eff_scale, const uint16_t* per_expert_scale,
                                          uint32_t num_experts, uint32_t d, uint32_t top_k,
                                          uint32_t* out_idx, uint16_t* out_w, float* logits_out) {
-    if (!ctx || !hidden || !out_idx || !out_w) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !hidden || !out_idx || !out_w) return NVMAI_ERR_INVALID_ARG;
     int rc = check_rows_desc(router, d, false);
     if (rc) return rc;
     if (num_experts == 0 || num_experts > 64 * TOPK_MAX_PER_LANE) return NVMAI_ERR_INVALID_ARG;
@@ -782,7 +649,7 @@ namespace {
 
 int slots_prologue(nvmai_hip_ctx* ctx, const void* const* blobs, const nvmai_expert_offsets* off,
                    uint32_t bits, uint32_t d, uint32_t f, uint32_t top_k, RowsParams& p) {
-    if (!ctx || !blobs) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !blobs) return NVMAI_ERR_INVALID_ARG;
     int rc = check_shape(d, f, bits);
     if (rc) return rc;
     rc = check_offsets(off);
@@ -902,7 +769,7 @@ extern "C" int nvmai_hip_shared_expert(nvmai_hip_ctx* ctx, nvmai_stream stream, 
                                        const nvmai_rows* shared_gate, const void* x,
                                        uint32_t x_stride, uint32_t n_tokens, void* y,
                                        uint32_t y_stride, uint32_t d, uint32_t f) {
-    if (!ctx || !blob || !x || !y) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !blob || !x || !y) return NVMAI_ERR_INVALID_ARG;
     int rc = check_shape(d, f, bits);
     if (rc) return rc;
     rc = check_offsets(off);
@@ -1063,7 +930,7 @@ int decode_layer_impl(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_moe_l
                       uint32_t x_stride, uint32_t n_tokens, void* y, uint32_t y_stride, uint32_t* out_idx,
                       uint16_t* out_w, uint32_t* stats, uint8_t* fixed_ws, size_t fixed_cap,
                       const PreNorm* pre = nullptr, PostNorm* post = nullptr) {
-    if (!ctx || !L || !x || !y) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !L || !x || !y) return NVMAI_ERR_INVALID_ARG;
     int rc = check_shape(L->d, L->f, L->bits);
     if (rc) return rc;
     rc = check_offsets(&L->offsets);
@@ -1210,7 +1077,7 @@ extern "C" int nvmai_hip_moe_decode_layer_prenorm(nvmai_hip_ctx* ctx, nvmai_stre
                                                   uint32_t normed_stride, uint32_t n_tokens, void* y,
                                                   uint32_t y_stride, uint32_t* out_idx, uint16_t* out_w,
                                                   uint32_t* stats) {
-    if (!ctx || !L || !hidden || !norm_weight || !hidden_out || !normed || !y) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !L || !hidden || !norm_weight || !hidden_out || !normed || !y) return NVMAI_ERR_INVALID_ARG;
     const uint32_t D = L->d;
     if (hidden_stride < D || hidden_out_stride < D || normed_stride < D || (delta && delta_stride < D))
         return NVMAI_ERR_INVALID_ARG;
@@ -1252,7 +1119,7 @@ extern "C" int nvmai_hip_moe_decode_layer_norms(nvmai_hip_ctx* ctx, nvmai_stream
                                                 uint32_t* out_idx, uint16_t* out_w, uint32_t* stats,
                                                 const uint16_t* next_norm_weight, void* next_normed,
                                                 uint32_t next_normed_stride) {
-    if (!ctx || !L || !hidden || !norm_weight || !hidden_out || !normed || !y || !next_norm_weight || !next_normed)
+    if (!act16(ctx) || !L || !hidden || !norm_weight || !hidden_out || !normed || !y || !next_norm_weight || !next_normed)
         return NVMAI_ERR_INVALID_ARG;
     const uint32_t D = L->d;
     if (hidden_stride < D || hidden_out_stride < D || normed_stride < D || next_normed_stride < D || (delta && delta_stride < D))
@@ -1287,7 +1154,7 @@ extern "C" int nvmai_hip_moe_decode_layer_noalloc(nvmai_hip_ctx* ctx, nvmai_stre
                                                   const nvmai_moe_layer* L, const void* x, uint32_t x_stride,
                                                   uint32_t n_tokens, void* y, uint32_t y_stride,
                                                   uint32_t* out_idx, uint16_t* out_w, uint32_t* stats) {
-    if (!ctx) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx)) return NVMAI_ERR_INVALID_ARG;
     if (!ctx->static_scratch) return NVMAI_ERR_HIP;     // the symbol lookup failed at context creation
     // every device holds its own copy of the array at its own address: the address this context keeps is
     // only good while its device is the current one

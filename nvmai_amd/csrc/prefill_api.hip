@@ -23,7 +23,7 @@ extern "C" int nvmai_prefill_grouping_check(int64_t n_pairs, int64_t query_count
 extern "C" int nvmai_hip_prefill_make_pairs(nvmai_hip_ctx* ctx, nvmai_stream stream, const uint32_t* idx,
                                             const uint16_t* w, uint32_t tokens, uint32_t top_k,
                                             nvmai_prefill_pair* pairs) {
-    if (!ctx || !idx || !w || !pairs || top_k == 0) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !idx || !w || !pairs || top_k == 0) return NVMAI_ERR_INVALID_ARG;
     const uint64_t n = (uint64_t)tokens * top_k;
     if (n >= (1u << 28)) return NVMAI_ERR_INVALID_ARG;
     if (n == 0) return NVMAI_OK;
@@ -77,7 +77,7 @@ extern "C" int nvmai_hip_prefill_group_pairs(nvmai_hip_ctx* ctx, nvmai_stream st
                                              uint32_t query_count, uint32_t top_k, uint32_t num_experts,
                                              uint32_t tile_expert_count, const uint64_t* sort_keys,
                                              uint64_t n_sort_keys, const nvmai_prefill_grouping* out) {
-    if (!ctx || (n_pairs && !pairs)) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || (n_pairs && !pairs)) return NVMAI_ERR_INVALID_ARG;
     int rc = check_grouping(out, n_pairs);
     if (rc) return rc;
     if (nvmai_prefill_grouping_check((int64_t)n_pairs, query_count, top_k, num_experts, tile_expert_count,
@@ -113,7 +113,7 @@ extern "C" int nvmai_hip_prefill_group_routes(nvmai_hip_ctx* ctx, nvmai_stream s
                                               const uint64_t* sort_keys, uint64_t n_sort_keys,
                                               const nvmai_prefill_grouping* out) {
     const uint64_t n_pairs = (uint64_t)query_count * top_k;
-    if (!ctx || (n_pairs && (!idx || !w))) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || (n_pairs && (!idx || !w))) return NVMAI_ERR_INVALID_ARG;
     int rc = check_grouping(out, n_pairs);
     if (rc) return rc;
     if (nvmai_prefill_grouping_check((int64_t)n_pairs, query_count, top_k, num_experts, tile_expert_count,
@@ -230,7 +230,7 @@ extern "C" int nvmai_hip_prefill_grouped_moe(nvmai_hip_ctx* ctx, nvmai_stream st
                                              const void* hidden, uint32_t hidden_stride, uint32_t query_count,
                                              uint32_t top_k, const nvmai_prefill_grouping* grouping,
                                              void* act_scratch, void* route_partials) {
-    if (!ctx || !experts_base || !off || !hidden || !act_scratch || !route_partials) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !experts_base || !off || !hidden || !act_scratch || !route_partials) return NVMAI_ERR_INVALID_ARG;
     int rc = check_grouping(grouping, (uint64_t)query_count * top_k);
     if (rc) return rc;
     if (bits != 4 && bits != 8) return NVMAI_ERR_UNSUPPORTED;
@@ -298,7 +298,7 @@ extern "C" int nvmai_hip_prefill_grouped_moe_streamed(nvmai_hip_ctx* ctx, nvmai_
                                                       uint64_t n_sorted_pairs, void* act_scratch, void* route_partials,
                                                       uint32_t* err) {
     static_assert(sizeof(nvmai_prefill_streamed_params) == 128, "PrefillGroupedRoutedMoEStreamedParams is 128 bytes");
-    if (!ctx || !params || !expert_blobs || !hidden || !sorted_pairs || !act_scratch || !route_partials)
+    if (!act16(ctx) || !params || !expert_blobs || !hidden || !sorted_pairs || !act_scratch || !route_partials)
         return NVMAI_ERR_INVALID_ARG;
     if (bits != 4 && bits != 8) return NVMAI_ERR_UNSUPPORTED;
     const uint32_t d = params->d, f = params->routed_intermediate, top_k = params->top_k;
@@ -385,7 +385,7 @@ extern "C" int nvmai_hip_affine_qmm(nvmai_hip_ctx* ctx, nvmai_stream stream, con
                                     const uint16_t* scales, const uint16_t* biases, uint32_t bits,
                                     const void* x, uint32_t x_stride, void* y, uint32_t y_stride, uint32_t m,
                                     uint32_t n, uint32_t k) {
-    if (!ctx || !weights || !scales || !biases || !x || !y) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !weights || !scales || !biases || !x || !y) return NVMAI_ERR_INVALID_ARG;
     if (bits != 4 && bits != 8) return NVMAI_ERR_UNSUPPORTED;
     if (n == 0 || k == 0 || k % NVMAI_GROUP || x_stride < k || y_stride < n) return NVMAI_ERR_INVALID_ARG;
     if (!aligned16(weights) || !aligned16(x) || x_stride % 8 || !aligned16(y) ||
@@ -418,7 +418,7 @@ extern "C" int nvmai_hip_prefill_moe_reduce_token_major(nvmai_hip_ctx* ctx, nvma
                                                         const void* route_partials, const uint16_t* route_weights,
                                                         void* h2, uint32_t h2_stride, uint32_t query_count,
                                                         uint32_t top_k, uint32_t d) {
-    if (!ctx || !route_partials || !route_weights || !h2) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !route_partials || !route_weights || !h2) return NVMAI_ERR_INVALID_ARG;
     if (query_count == 0 || top_k == 0 || d == 0 || d % 2 || h2_stride < d || h2_stride % 2) return NVMAI_ERR_INVALID_ARG;
     hipStream_t s = (hipStream_t)stream;
     ProfScope prof(ctx, NVMAI_PROF_PREFILL_COMBINE, s);

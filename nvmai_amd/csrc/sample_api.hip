@@ -32,7 +32,10 @@ extern "C" int nvmai_hip_softmax_tiled(nvmai_hip_ctx* ctx, nvmai_stream stream, 
     float* tsum = ws_take<float>(ctx, (size_t)rows * tiles);
     ProfScope ps(ctx, NVMAI_PROF_SOFTMAX, s);
     dim3 grid(tiles, rows);
-    if (ctx->act == ACT_BF16) {
+    if (ctx->act == ACT_FP32) {
+        softmax_stage1_kernel<ACT_FP32><<<grid, 256, 0, s>>>(logits, v, logits_stride, softcap, tmax, tsum, tiles);
+        softmax_normalize_kernel<ACT_FP32><<<grid, 256, 0, s>>>(logits, v, logits_stride, softcap, tmax, tsum, tiles, probs, probs_stride);
+    } else if (ctx->act == ACT_BF16) {
         softmax_stage1_kernel<ACT_BF16><<<grid, 256, 0, s>>>(logits, v, logits_stride, softcap, tmax, tsum, tiles);
         softmax_normalize_kernel<ACT_BF16><<<grid, 256, 0, s>>>(logits, v, logits_stride, softcap, tmax, tsum, tiles, probs, probs_stride);
     } else {
@@ -97,7 +100,7 @@ extern "C" int nvmai_hip_sample(nvmai_hip_ctx* ctx, nvmai_stream stream, const u
 extern "C" int nvmai_hip_repetition_penalty(nvmai_hip_ctx* ctx, nvmai_stream stream, void* logits, uint32_t v,
                                             const int32_t* history_ids, uint32_t n_ids, float penalty,
                                             float logit_softcap) {
-    if (!ctx || !logits || v == 0 || (n_ids && !history_ids)) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !logits || v == 0 || (n_ids && !history_ids)) return NVMAI_ERR_INVALID_ARG;
     if (!(penalty > 0.0f)) return NVMAI_ERR_INVALID_ARG;
     if (n_ids == 0 || penalty == 1.0f) return NVMAI_OK;          // Sampler.swift:181
     hipStream_t s = (hipStream_t)stream;

@@ -54,9 +54,16 @@ __device__ __forceinline__ void block_softmax_merge(float& m, float& d, float* l
 constexpr int SOFTMAX_PER_THREAD = SOFTMAX_TILE / 256;
 
 template <int ACT>
-__device__ __forceinline__ bool softmax_load(const uint16_t* z, uint32_t base, uint32_t v, float softcap, float* x) {
+__device__ __forceinline__ bool softmax_load(const act_t<ACT>* z, uint32_t base, uint32_t v, float softcap, float* x) {
     const bool vec = (reinterpret_cast<uintptr_t>(z + base) & 15u) == 0 && base + SOFTMAX_TILE <= v;
-    if (vec) {
+    if (vec && ACT == ACT_FP32) {
+#pragma unroll
+        for (int h = 0; h < 4; ++h) {          // the same entries per thread: two 16-byte loads per half
+            const float4 q = *reinterpret_cast<const float4*>(z + base + (h / 2) * (SOFTMAX_TILE / 2) + 8 * threadIdx.x + 4 * (h % 2));
+            x[4 * h] = softcap_value(q.x, softcap); x[4 * h + 1] = softcap_value(q.y, softcap);
+            x[4 * h + 2] = softcap_value(q.z, softcap); x[4 * h + 3] = softcap_value(q.w, softcap);
+        }
+    } else if (vec) {
 #pragma unroll
         for (int h = 0; h < 2; ++h) {
             const uint4 q = *reinterpret_cast<const uint4*>(z + base + h * (SOFTMAX_TILE / 2) + 8 * threadIdx.x);
@@ -86,7 +93,7 @@ __global__ __launch_bounds__(256) void softmax_stage1_kernel(const void* logits,
                                                             uint32_t tiles) {
     __shared__ float lds[8];
     const uint32_t tile = blockIdx.x, row = blockIdx.y;
-    const uint16_t* z = (const uint16_t*)logits + (size_t)row * row_stride;
+    const act_t<ACT>* z = (const act_t<ACT>*)logits + (size_t)row * row_stride;
     float x[SOFTMAX_PER_THREAD];
     softmax_load<ACT>(z, tile * SOFTMAX_TILE, v, softcap, x);
     float m = -INFINITY, d = 0.0f;
@@ -109,7 +116,7 @@ __global__ __launch_bounds__(256) void softmax_normalize_kernel(const void* logi
                                                                uint16_t* probs, uint32_t probs_stride) {
     __shared__ float lds[8];
     const uint32_t row = blockIdx.y;
-    const uint16_t* z = (const uint16_t*)logits + (size_t)row * row_stride;
+    const act_t<ACT>* z = (const act_t<ACT>*)logits + (size_t)row * row_stride;
     const uint32_t base = blockIdx.x * SOFTMAX_TILE;
     float x[SOFTMAX_PER_THREAD];
     const bool vec = softmax_load<ACT>(z, base, v, softcap, x);   // in flight while the partials merge

@@ -20,7 +20,7 @@ constexpr uint32_t RMS_DIRECT_ROWS = 256;
 extern "C" int nvmai_hip_rmsnorm(nvmai_hip_ctx* ctx, nvmai_stream stream, const void* x, uint32_t x_stride,
                                  const uint16_t* weight, void* out, uint32_t out_stride, uint32_t rows,
                                  uint32_t d, float eps) {
-    if (!ctx || !x || !out || d == 0 || x_stride < d || out_stride < d) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !x || !out || d == 0 || x_stride < d || out_stride < d) return NVMAI_ERR_INVALID_ARG;
     if (rows == 0) return NVMAI_OK;
     hipStream_t s = (hipStream_t)stream;
     const dim3 grid((rows + 3) / 4);
@@ -43,7 +43,7 @@ extern "C" int nvmai_hip_residual_add_rmsnorm(nvmai_hip_ctx* ctx, nvmai_stream s
                                               uint32_t hidden_stride, const void* delta, uint32_t delta_stride,
                                               const uint16_t* weight, void* out, uint32_t out_stride, uint32_t rows,
                                               uint32_t d, float eps) {
-    if (!ctx || !hidden || !delta || !out || d == 0 || hidden_stride < d || delta_stride < d || out_stride < d)
+    if (!act16(ctx) || !hidden || !delta || !out || d == 0 || hidden_stride < d || delta_stride < d || out_stride < d)
         return NVMAI_ERR_INVALID_ARG;
     if (rows == 0) return NVMAI_OK;
     hipStream_t s = (hipStream_t)stream;
@@ -70,7 +70,7 @@ int qkv_epilogue_impl(nvmai_hip_ctx* ctx, nvmai_stream stream, const void* proj,
                       uint32_t head_dim, uint32_t rotary_dim, int v_norm, const uint32_t* positions, uint32_t position,
                       float theta, float eps, const nvmai_kv_view* k_cache, const nvmai_kv_view* v_cache) {
     const bool cached = k_cache || v_cache;
-    if (!ctx || !proj || !q_out || (q_packed && !gate_out)) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !proj || !q_out || (q_packed && !gate_out)) return NVMAI_ERR_INVALID_ARG;
     if (cached ? (!k_cache || !v_cache) : (!k_out || !v_out)) return NVMAI_ERR_INVALID_ARG;
     if ((k_out == nullptr) != (v_out == nullptr)) return NVMAI_ERR_INVALID_ARG;
     if (head_dim == 0 || head_dim > 512 || num_q_heads == 0 || num_kv_heads == 0) return NVMAI_ERR_INVALID_ARG;   // kFusedMaxHeadDim
@@ -181,7 +181,7 @@ namespace {
 
 template <int OP>
 int run_elementwise(nvmai_hip_ctx* ctx, nvmai_stream stream, const void* a, const void* b, void* out, uint32_t count) {
-    if (!ctx || !a || !b || !out) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !a || !b || !out) return NVMAI_ERR_INVALID_ARG;
     if (count == 0) return NVMAI_OK;
     hipStream_t s = (hipStream_t)stream;
     if (count >= 4096 && count % 8 == 0 && aligned16(a) && aligned16(out) && (OP == EW_SIGMOID_SCALAR || aligned16(b))) {
@@ -224,7 +224,7 @@ extern "C" int nvmai_hip_residual_add(nvmai_hip_ctx* ctx, nvmai_stream stream, v
 
 extern "C" int nvmai_hip_split_q_gate(nvmai_hip_ctx* ctx, nvmai_stream stream, const void* packed, void* q,
                                       void* gate, uint32_t heads, uint32_t dim) {
-    if (!ctx || !packed || !q || !gate) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !packed || !q || !gate) return NVMAI_ERR_INVALID_ARG;
     if ((uint64_t)heads * dim > 0x7FFFFFFFull) return NVMAI_ERR_INVALID_ARG;
     if (heads * dim == 0) return NVMAI_OK;
     split_join_rows_kernel<false><<<(heads * dim + 255) / 256, 256, 0, (hipStream_t)stream>>>(
@@ -234,7 +234,7 @@ extern "C" int nvmai_hip_split_q_gate(nvmai_hip_ctx* ctx, nvmai_stream stream, c
 
 extern "C" int nvmai_hip_concat_rows(nvmai_hip_ctx* ctx, nvmai_stream stream, const void* lhs, const void* rhs,
                                      void* out, uint32_t rows, uint32_t dim) {
-    if (!ctx || !lhs || !rhs || !out) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !lhs || !rhs || !out) return NVMAI_ERR_INVALID_ARG;
     if ((uint64_t)rows * dim > 0x7FFFFFFFull) return NVMAI_ERR_INVALID_ARG;
     if (rows * dim == 0) return NVMAI_OK;
     split_join_rows_kernel<true><<<(rows * dim + 255) / 256, 256, 0, (hipStream_t)stream>>>(
@@ -246,7 +246,7 @@ extern "C" int nvmai_hip_embed_lookup(nvmai_hip_ctx* ctx, nvmai_stream stream, c
                                       const uint16_t* scales, const uint16_t* biases, uint32_t bits,
                                       const uint32_t* token_ids, uint32_t token_id, uint32_t n_tokens, void* out,
                                       uint32_t out_stride, uint32_t d, uint32_t vocab, float out_scale) {
-    if (!ctx || !table || !scales || !biases || !out) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !table || !scales || !biases || !out) return NVMAI_ERR_INVALID_ARG;
     if (bits != 4 && bits != 8) return NVMAI_ERR_UNSUPPORTED;
     if (d == 0 || d % NVMAI_GROUP || out_stride < d) return NVMAI_ERR_INVALID_ARG;
     if (n_tokens == 0) return NVMAI_OK;
@@ -276,7 +276,7 @@ extern "C" int nvmai_hip_lm_head_greedy(nvmai_hip_ctx* ctx, nvmai_stream stream,
                                         const uint8_t* weights, const uint16_t* scales, const uint16_t* biases,
                                         uint32_t bits, uint32_t* out_tokens, uint32_t d, uint32_t vocab,
                                         float rms_eps) {
-    if (!ctx || !hidden || !weights || !scales || !biases || !out_tokens) return NVMAI_ERR_INVALID_ARG;
+    if (!act16(ctx) || !hidden || !weights || !scales || !biases || !out_tokens) return NVMAI_ERR_INVALID_ARG;
     if (bits != 4 && bits != 8) return NVMAI_ERR_UNSUPPORTED;
     if (d == 0 || d % NVMAI_GROUP || hidden_stride < d || vocab == 0) return NVMAI_ERR_INVALID_ARG;   // LMHeadChainInt4.swift:76-77
     const uint32_t chunks = d * bits / 128;        // d is a multiple of 64: whole 16-byte chunks

@@ -265,12 +265,89 @@ def _from_gturbo(cls, ctx, model, gdn=None, kv_bits=8, gdn_state_bf16=True):
 HybridWeights.from_gturbo = classmethod(_from_gturbo)
 
 
-class HybridDecoder:
+class StepDecoder:
+    """What every model's step driver shares: the token and logit buffers, a prompt fed a chunk at a time, the sampler
+    at the end of a step, and the calls the session layer (generate.py) makes.  A model supplies
+    _prefill_chunk_rows (a portion of one sequence through every layer, from the state it has), forward_hidden (one
+    token of each sequence) and head_rows (logits of final-normed rows)."""
+    max_chunk = None            # most tokens of one pass over a prompt, None: no limit
+
+    def __init__(self, ctx, cfg, weights, batch, max_context):
+        self.ctx, self.cfg, self.w, self.batch, self.max_context = ctx, cfg, weights, batch, max_context
+        dev = ctx.device
+        self.logits = torch.zeros((batch, cfg.vocab), dtype=ctx.dtype, device=dev)
+        self.probs = torch.zeros((batch, cfg.vocab), dtype=torch.float16, device=dev)
+        self.tokens = torch.zeros(batch, dtype=torch.int32, device=dev)
+        self.next_tokens = torch.zeros(batch, dtype=torch.int32, device=dev)
+        self.positions = torch.zeros(batch, dtype=torch.int32, device=dev)
+        self.softmax = ops.LogitSoftcapSoftmaxTiled(ctx, cfg.vocab)
+
+    # -- prompts: the tokens of ONE sequence, a chunk at a time, through every layer ------------------------
+    def prefill_rows(self, tokens, sequence=0, start_position=0, want=None, chunk_tokens=2048):
+        """tokens: int32 device tensor [n] of sequence `sequence`, the first of them at start_position; continues
+        from the state that earlier calls left.  Returns the final-normed rows at the places `want` (indices into
+        tokens, in any order; None: the last one) as one tensor (None for an empty `want`)."""
+        n = tokens.numel()
+        if n == 0:
+            raise ValueError("prefill needs at least one token")
+        if start_position + n > self.max_context:
+            raise ValueError("prefill of %d tokens from %d exceeds the cache (%d rows)" % (n, start_position, self.max_context))
+        want = [n - 1] if want is None else list(want)
+        if any(not 0 <= p < n for p in want):
+            raise ValueError("a wanted place lies outside the portion")
+        if self.max_chunk is not None:
+            chunk_tokens = min(chunk_tokens, self.max_chunk)
+        out = {}
+        for c0 in range(0, n, chunk_tokens):
+            c1 = min(n, c0 + chunk_tokens)
+            rows = self._prefill_chunk_rows(tokens[c0:c1].contiguous(), sequence, start_position + c0)
+            for p in want:
+                if c0 <= p < c1:
+                    # the driver may reuse the rows' buffer for the next chunk
+                    out[p] = rows[p - c0:p - c0 + 1] if c1 == n else rows[p - c0:p - c0 + 1].clone()
+        if not want:
+            return None
+        return out[want[0]] if len(want) == 1 else torch.cat([out[p] for p in want])
+
+    def prefill_chunked(self, tokens, sequence=0, start_position=0, chunk_tokens=2048):
+        """The same; returns the final-normed row of the last token, [1, hidden] (the input of head())."""
+        return self.prefill_rows(tokens, sequence, start_position, None, chunk_tokens)
+
+    # -- what a session calls --------------------------------------------------------------------------
+    def decode_rows(self, sequences, positions, tokens):
+        """One more token of each of `sequences` (lists of equal length): final-normed rows in that order.  This form
+        makes one pass when every sequence takes part at one position, else a pass per sequence."""
+        if len(sequences) == self.batch and len(set(positions)) == 1 and list(sequences) == list(range(self.batch)):
+            self.tokens.copy_(torch.tensor(tokens, dtype=torch.int32))
+            return self.forward_hidden(positions[0])
+        one = lambda t: torch.tensor([t], dtype=torch.int32, device=self.ctx.device)
+        rows = [self._prefill_chunk_rows(one(t), b, p).clone() for b, p, t in zip(sequences, positions, tokens)]
+        return torch.cat(rows)
+
+    # -- the end of a step -----------------------------------------------------------------------------
+    def sample(self, seeds, temperature=0.6, top_k=20, top_p=0.95):
+        """Softcap + softmax and the tiled top-k sampler (Sampler.sample's production path): tokens in
+        self.next_tokens."""
+        self.softmax.encode(self.logits, self.probs, softcap=self.cfg.logit_softcap)
+        check(lib.nvmai_hip_sample_topk64(self.ctx.handle, ops._stream(), ops._ptr(self.probs), self.probs.stride(0),
+                                          self.batch, self.cfg.vocab, temperature, top_p,
+                                          (C.c_uint64 * self.batch)(*seeds), top_k, ops._ptr(self.next_tokens), None),
+              "sample_topk64")
+        return self.next_tokens
+
+    def step(self, position, seeds, temperature=0.6, top_k=20, top_p=0.95):
+        """tokens (self.tokens) at `position` -> next tokens (self.next_tokens)."""
+        self.forward_hidden(position)
+        self.head()
+        return self.sample(seeds, temperature, top_k, top_p)
+
+
+class HybridDecoder(StepDecoder):
     """One decode step for `batch` sequences: buffers, recurrent states and KV caches are allocated
     once; step() only enqueues kernels."""
 
     def __init__(self, ctx, cfg, weights, batch=1, max_context=32768):
-        self.ctx, self.cfg, self.w, self.batch, self.max_context = ctx, cfg, weights, batch, max_context
+        super().__init__(ctx, cfg, weights, batch, max_context)
         dev, dt = ctx.device, ctx.dtype
         D = cfg.hidden
         buf = lambda *shape: torch.zeros(shape, dtype=dt, device=dev)
@@ -287,11 +364,6 @@ class HybridDecoder:
         self.q, self.gate, self.attn_out = buf(batch, cfg.num_heads, cfg.head_dim), buf(batch, cfg.num_heads, cfg.head_dim), \
             buf(batch, cfg.num_heads, cfg.head_dim)
         self.k_stage, self.v_stage = buf(batch, cfg.kv_dim), buf(batch, cfg.kv_dim)
-        self.logits = buf(batch, cfg.vocab)
-        self.probs = torch.zeros((batch, cfg.vocab), dtype=torch.float16, device=dev)
-        self.tokens = torch.zeros(batch, dtype=torch.int32, device=dev)
-        self.next_tokens = torch.zeros(batch, dtype=torch.int32, device=dev)
-        self.positions = torch.zeros(batch, dtype=torch.int32, device=dev)
         self.gdn_states, self.kv = {}, {}
         for L in range(cfg.layers):
             if cfg.is_linear(L):
@@ -302,7 +374,6 @@ class HybridDecoder:
         self.moe = ops.MoE(ctx, cfg.expert_bits)
         self.attn = ops.Attention(ctx)
         self.quant = ops.KVCacheQuantizer(ctx)
-        self.softmax = ops.LogitSoftcapSoftmaxTiled(ctx, cfg.vocab)
         self.sampler = ops.SampleTopK64(ctx, cfg.vocab) if cfg.vocab <= 262144 else None
         self.ew = ops.Elementwise(ctx)
 
@@ -447,21 +518,7 @@ class HybridDecoder:
     # quantized cache, the tiled router, the permutation by expert and the grouped GEMM, the shared expert
     # in dense mode -- and they leave the sequence's KV rows, conv tails and recurrent states exactly
     # where step() expects them, so decoding continues at start_position + len(tokens).
-    def prefill_chunked(self, tokens, sequence=0, start_position=0, chunk_tokens=2048):
-        """tokens: int32 device tensor [n] of sequence `sequence`, the first of them at start_position.
-        Returns the final-normed row of the last token, [1, hidden] (the input of head())."""
-        n = tokens.numel()
-        if n == 0:
-            raise ValueError("prefill_chunked needs at least one token")
-        if start_position + n > self.max_context:
-            raise ValueError("prefill of %d tokens from %d exceeds the cache (%d rows)" % (n, start_position, self.max_context))
-        last = None
-        for c0 in range(0, n, chunk_tokens):
-            last = self._execute_prefill_chunk(tokens[c0:min(n, c0 + chunk_tokens)].contiguous(), sequence,
-                                               start_position + c0)
-        return last
-
-    def _execute_prefill_chunk(self, tokens, b, start):
+    def _prefill_chunk_rows(self, tokens, b, start):
         cfg, ctx = self.cfg, self.ctx
         T = tokens.numel()
         e_p, e_s, e_b = self.w.embed
@@ -481,7 +538,7 @@ class HybridDecoder:
             y = self._routed_moe_prefill(w, routed_x, T)
             nxt = self.w.layers[L + 1]["in_norm"] if L + 1 < cfg.layers else self.w.final_norm
             normed = ops.residual_add_rmsnorm(ctx, hidden, y, nxt, eps=cfg.rms_eps)
-        return normed[T - 1:T]
+        return normed
 
     def _linear_attention_prefill(self, L, w, normed, b, T):
         cfg = self.cfg
@@ -560,18 +617,14 @@ class HybridDecoder:
         ops.affine_gemv(self.ctx, p_, s_, b_, cfg.head_bits, self.normed, cfg.vocab, cfg.hidden, y=self.logits)
         return self.logits
 
-    def sample(self, seeds, temperature=0.6, top_k=20, top_p=0.95):
-        """Softcap + softmax and the tiled top-k sampler (Sampler.sample's production path): tokens in
-        self.next_tokens."""
-        self.softmax.encode(self.logits, self.probs, softcap=self.cfg.logit_softcap)
-        check(lib.nvmai_hip_sample_topk64(self.ctx.handle, ops._stream(), ops._ptr(self.probs), self.probs.stride(0),
-                                          self.batch, self.cfg.vocab, temperature, top_p,
-                                          (C.c_uint64 * self.batch)(*seeds), top_k, ops._ptr(self.next_tokens), None),
-              "sample_topk64")
-        return self.next_tokens
+    def reset(self, sequence):
+        """Forget what the sequence left: recurrent states start from zero (KV rows are overwritten as they are used)."""
+        for tail, state in self.gdn_states.values():
+            tail[sequence].zero_()
+            state[sequence].zero_()
 
-    def step(self, position, seeds, temperature=0.6, top_k=20, top_p=0.95):
-        """tokens (self.tokens) at `position` -> next tokens (self.next_tokens)."""
-        self.forward_hidden(position)
-        self.head()
-        return self.sample(seeds, temperature, top_k, top_p)
+    def head_rows(self, normed):
+        """Logits of any number of final-normed rows: (activations [n, vocab], None)."""
+        cfg = self.cfg
+        p_, s_, b_ = self.w.lm_head
+        return ops.affine_gemv(self.ctx, p_, s_, b_, cfg.head_bits, normed, cfg.vocab, cfg.hidden), None

@@ -7,13 +7,14 @@ import ctypes as C
 import torch
 
 from . import _lib
-from ._lib import ExpertOffsets, GdnConfig, GemvPart, GenerationConfig as _CGenerationConfig, KvView, MoeLayer, PrefillGrouping, Rows, check, lib
+from ._lib import (ExpertOffsets, GdnConfig, GemvPart, GenerationConfig as _CGenerationConfig, GlaConfig, KvView,
+                   LatentCacheView, LatentConfig, MoeLayer, PrefillGrouping, RowMap, Rows, check, lib)
 
-ACT_BF16, ACT_FP16 = 0, 1
+ACT_BF16, ACT_FP16, ACT_FP32 = 0, 1, 2
 (PROF_ROUTER, PROF_SELECT, PROF_GROUP, PROF_PHASE1, PROF_PHASE2, PROF_COMBINE, PROF_KV_QUANT,
  PROF_ATTN_PARTIAL, PROF_ATTN_COMBINE, PROF_SOFTMAX, PROF_SAMPLE, PROF_PREFILL_GROUP,
  PROF_PREFILL_GEMM1, PROF_PREFILL_GEMM2, PROF_PREFILL_COMBINE) = range(15)
-_ACT_TORCH = {ACT_BF16: torch.bfloat16, ACT_FP16: torch.float16}
+_ACT_TORCH = {ACT_BF16: torch.bfloat16, ACT_FP16: torch.float16, ACT_FP32: torch.float32}
 
 
 def _ptr(t):
@@ -1080,4 +1081,116 @@ class Elementwise:
         out = torch.empty((rows, 2 * dim), dtype=lhs.dtype, device=lhs.device)
         check(lib.nvmai_hip_concat_rows(self.ctx.handle, _stream(), _ptr(lhs), _ptr(rhs), _ptr(out), rows, dim),
               "concat_rows")
+        return out
+
+
+# ---------------------------------------------------------------------------------------------
+# dense models: BF16 weights, BF16 or 32-bit activations, a 32-bit residual stream
+FORM_AUTO = 0
+GLA_RECURRENT, GLA_CHUNKED = 1, 2
+LATENT_ABSORBED, LATENT_EXPANDED = 1, 2
+LINEAR_NONE, LINEAR_GELU_ERF = 0, 1
+
+
+def dense_linear(ctx, weight, x, y=None, y_f32=None, n=None, activation=LINEAR_NONE):
+    """y[t] = act(W x[t]): weight [n, k] BF16 (k a multiple of 64), x [tokens, >= k] activations; y (activations) and /
+    or y_f32 are buffers [tokens, >= n] with one row stride."""
+    rows, k = weight.shape
+    out = y if y is not None else y_f32
+    assert y is None or y_f32 is None or y.stride(0) == y_f32.stride(0)
+    check(lib.nvmai_hip_dense_linear(ctx.handle, _stream(), _ptr(weight), weight.stride(0), _ptr(x), x.stride(0), x.shape[0],
+                                     rows if n is None else n, k, _ptr(y), _ptr(y_f32), out.stride(0), activation),
+          "dense_linear")
+    return out
+
+
+def norm_residual(ctx, x, d, delta=None, post=None, mult=1.0, next_norm=None, out=None, eps=1e-6):
+    """x += mult * LN(delta) (post = (weight, bias), None: delta as it is), then out = LN(x) with next_norm =
+    (weight, bias): the end of a sublayer and the start of the next over the 32-bit residual x [tokens, >= d]."""
+    pw, pb = post if post is not None else (None, None)
+    nw, nb = next_norm if next_norm is not None else (None, None)
+    check(lib.nvmai_hip_norm_residual(ctx.handle, _stream(), _ptr(x), x.stride(0), _ptr(delta),
+                                      0 if delta is None else delta.stride(0), _ptr(pw), _ptr(pb), mult, _ptr(nw), _ptr(nb),
+                                      _ptr(out), 0 if out is None else out.stride(0), x.shape[0], d, eps), "norm_residual")
+    return out
+
+
+def embed_rows(ctx, table, token_ids, d, vocab, out):
+    """Rows of a BF16 table as 32-bit residual rows."""
+    check(lib.nvmai_hip_embed_rows(ctx.handle, _stream(), _ptr(table), table.stride(0), _ptr(token_ids), token_ids.numel(),
+                                   _ptr(out), out.stride(0), d, vocab), "embed_rows")
+    return out
+
+
+def argmax_rows(ctx, logits, out=None):
+    """Greedy token of each row of 32-bit logits, ties to the lower id."""
+    if out is None:
+        out = torch.empty(logits.shape[0], dtype=torch.int32, device=logits.device)
+    check(lib.nvmai_hip_argmax_rows(ctx.handle, _stream(), _ptr(logits), logits.stride(0), logits.shape[0], logits.shape[1],
+                                    _ptr(out)), "argmax_rows")
+    return out
+
+
+def row_map(slot=0, position=0, slots=None, positions=None):
+    """Rows position, position + 1, ... of one slot, or (int32 device arrays) one slot and position per row."""
+    m = RowMap(None if slots is None else slots.data_ptr(), None if positions is None else positions.data_ptr(), slot, position)
+    m._keep = (slots, positions)
+    return m
+
+
+class GLA:
+    """Gated linear attention with a decay per key channel (nvmai_hip_gla).  key_dim and value_dim are multiples of 16,
+    value_count (of value_dim) and key_count (of key_dim) the real sizes behind them."""
+
+    def __init__(self, ctx, heads, key_dim, value_dim, rank, tau, eps, key_count=None, value_count=None):
+        self.ctx, self.heads, self.key_dim, self.value_dim = ctx, heads, key_dim, value_dim
+        self.cfg = GlaConfig(heads, key_dim, value_dim, value_dim if value_count is None else value_count, rank, tau,
+                             (key_dim if key_count is None else key_count) ** -0.5, eps)
+
+    def new_state(self, slots):
+        return torch.zeros((slots, self.heads, self.key_dim, self.value_dim), dtype=torch.float32, device=self.ctx.device)
+
+    def encode(self, q, k, v, g, a1, a2, a2_bias, norm_weight, state, out, rows, batch=1, slot=0, slots=None, form=FORM_AUTO):
+        """q, k, v, g, a1: column ranges of one projected matrix [batch * rows, ...]."""
+        stride = q.stride(0)
+        assert all(t.stride(0) == stride for t in (k, v, g, a1))
+        check(lib.nvmai_hip_gla(self.ctx.handle, _stream(), C.byref(self.cfg), _ptr(q), _ptr(k), _ptr(v), _ptr(g), _ptr(a1),
+                                stride, _ptr(a2), _ptr(a2_bias), _ptr(norm_weight), _ptr(state), _ptr(slots), slot, _ptr(out),
+                                out.stride(0), rows, batch, form), "gla")
+        return out
+
+
+class LatentCache:
+    """One layer's cached latents: per slot a ring of `capacity` rows [latent | rotated key part | zeros] of
+    activations; position p lies at row p % capacity.  The counterpart of KVCache for latent attention."""
+
+    def __init__(self, ctx, slots, capacity, rank, rope_dim):
+        self.capacity = max(64, capacity)
+        self.row_stride = (rank + rope_dim + 31) // 32 * 32
+        self.rows = torch.zeros((slots, self.capacity, self.row_stride), dtype=ctx.dtype, device=ctx.device)
+        self.view = LatentCacheView(self.rows.data_ptr(), self.rows.stride(0), self.row_stride, self.capacity)
+
+
+class LatentAttention:
+    """Latent attention (nvmai_hip_latent_epilogue, nvmai_hip_latent_attention).  nope_dim, rope_dim and value_dim are
+    multiples of 16 and rank of 64; rank_count is the real latent size.  window 0: every earlier position."""
+
+    def __init__(self, ctx, heads, nope_dim, rope_dim, value_dim, rank, rank_count, scale, window, rotary_dims, rope_base, eps):
+        self.ctx, self.heads, self.nope_dim, self.rope_dim, self.value_dim, self.rank = ctx, heads, nope_dim, rope_dim, value_dim, rank
+        # frequencies in double: the angle position * frequency is reduced in double by the kernels
+        i = torch.arange(rotary_dims // 2, dtype=torch.float64)
+        self.inv_freq = (float(rope_base) ** (-2.0 * i / max(1, rotary_dims))).to(ctx.device)
+        self.cfg = LatentConfig(heads, nope_dim, rope_dim, value_dim, rank, rank_count, rotary_dims, window, scale, eps,
+                                self.inv_freq.data_ptr() if rotary_dims else None)
+
+    def encode_epilogue(self, proj, q_at, q_count, q_norm, kv_at, rope_at, kv_norm, cq, cache, rows_at):
+        check(lib.nvmai_hip_latent_epilogue(self.ctx.handle, _stream(), C.byref(self.cfg), _ptr(proj), proj.stride(0), q_at, q_count,
+                                            _ptr(q_norm), kv_at, rope_at, _ptr(kv_norm), _ptr(cq), cq.stride(0),
+                                            C.byref(cache.view), C.byref(rows_at), proj.shape[0]), "latent_epilogue")
+        return cq
+
+    def encode(self, q, gate, uk, uv, cache, rows_at, out, form=FORM_AUTO):
+        check(lib.nvmai_hip_latent_attention(self.ctx.handle, _stream(), C.byref(self.cfg), _ptr(q), q.stride(0), _ptr(gate),
+                                             0 if gate is None else gate.stride(0), _ptr(uk), _ptr(uv), C.byref(cache.view),
+                                             C.byref(rows_at), _ptr(out), out.stride(0), q.shape[0], form), "latent_attention")
         return out
