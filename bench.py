@@ -26,6 +26,13 @@ RAMP_STEPS = 200       # untimed steps ahead of the --warmup steps of the decode
                        # milliseconds of work to reach its clock, and --steps 20 of this workload are under 3 ms
 
 
+# width, layers, heads, (GLA dim, vdim), (latent dim, rot_dim, vdim, kv_rank, q_rank, window), ff, vocab; layers alternate
+# GLA (no feed-forward) and windowed latent attention (dense feed-forward)
+PAKIRAX_SIZES = {"1k": (1024, 24, 8, (128, 128), (128, 64, 128, 256, 768, 2048), 4096, 65536),
+                 "2k": (2048, 40, 16, (128, 128), (128, 64, 128, 512, 1536, 4096), 8192, 248320),
+                 "4k": (4096, 32, 32, (128, 128), (128, 64, 128, 512, 1536, 4096), 16384, 131072)}
+
+
 def parse():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -38,7 +45,7 @@ def parse():
     ap.add_argument("--sweep", action="store_true", help="also print batch/bits sweep lines to stderr")
     ap.add_argument("--no-extra", action="store_true", help="skip the `extra` object (the other cells of the metric) "
                     "that the default invocation appends")
-    ap.add_argument("--workload", default="decode", choices=["decode", "prefill", "attention", "prefill_attention", "sampler", "greedy", "step", "prefill_step", "copy", "read"],
+    ap.add_argument("--workload", default="decode", choices=["decode", "prefill", "attention", "prefill_attention", "sampler", "greedy", "step", "prefill_step", "pakirax_step", "pakirax_prefill", "copy", "read"],
                     help="decode = configs[1] (the headline line); prefill = configs[2] grouped GEMM; "
                          "attention = configs[3] quantized-KV decode attention; prefill_attention = causal attention of --tokens queries "
                          "at the end of a --context cache; sampler = the end of configs[4]: "
@@ -46,7 +53,10 @@ def parse():
                          "(RMSNorm + logits in a fixed order + argmax) over the same head; step = configs[4], the full 40-layer decode "
                          "step (tok/s at --batch 1..16, KV at --context); prefill_step = --tokens prompt tokens of one sequence through the "
                          "same 40 layers with the prefill kernels, in chunks of --chunk; copy = a plain 1 GiB device copy, "
-                         "the known-size kernel the FETCH_SIZE / WRITE_SIZE counters are calibrated on")
+                         "the known-size kernel the FETCH_SIZE / WRITE_SIZE counters are calibrated on; "
+                         "pakirax_step / pakirax_prefill = a decode step (--batch sequences at --context) / a --tokens prompt of the Pakirax "
+                         "model at --size, random weights")
+    ap.add_argument("--size", default="2k", choices=sorted(PAKIRAX_SIZES), help="pakirax_*: width of the model")
     ap.add_argument("--context", type=int, default=None, help="attention: tokens in the KV cache (default 32768; "
                     "prefill_attention: the chunk itself)")
     ap.add_argument("--tokens", type=int, default=4096, help="prefill: tokens per step")
@@ -760,6 +770,108 @@ def run_prefill_step(nv, ctx, torch, a):
     }
 
 
+def pakirax_model(nv, torch, a, batch, max_context, max_chunk):
+    from nvmai_amd.pakirax import PakiraxConfig, PakiraxDecoder, PakiraxWeights
+    width, layers, heads, (gk, gv), (dim, rot, vdim, kv_rank, q_rank, window), ff, vocab = PAKIRAX_SIZES[a.size]
+    g = {"type": "gla", "mixer": {"heads": heads, "dim": gk, "vdim": gv, "tau": 16.0}, "mlp": None}
+    at = {"type": "latent_attention", "mlp": {"kind": "dense", "ff": ff},
+          "mixer": {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": vdim, "kv_rank": kv_rank, "q_rank": q_rank,
+                    "scale": (dim + rot) ** -0.5, "mask": {"size": window}, "rot": {"base": 10000.0, "dims": rot}}}
+    cfg = PakiraxConfig({"architecture": "Pakirax", "vocab": vocab, "width": width, "residual_mult": 0.3, "norm": {"eps": 1e-6},
+                         "layers": [g, at] * (layers // 2)})
+    ctx = nv.Context(0, nv.ACT_BF16)
+    return ctx, cfg, PakiraxDecoder(ctx, cfg, PakiraxWeights.random(ctx, cfg, seed=2024), batch, max_context, max_chunk)
+
+
+def run_pakirax_step(nv, torch, a):
+    """One decode step of the Pakirax model at `--size` (random weights; half the layers gated linear attention with a
+    32-bit state, half latent attention over a window): embedding to greedy token for `--batch` sequences, each at the end
+    of a full window, captured once into a HIP graph and replayed."""
+    B, context = min(a.batch, 16), a.context
+    ctx, cfg, dec = pakirax_model(nv, torch, a, B, context + 1, 2048)
+    gen = torch.Generator(device="cuda").manual_seed(5)
+    for c in dec.caches.values():
+        c.rows.normal_(0.0, 1.0, generator=gen)
+    for s in dec.states.values():
+        s.normal_(0.0, 0.1, generator=gen)
+    dec.tokens.copy_(torch.randint(0, cfg.vocab, (B,), generator=gen, device="cuda", dtype=torch.int32))
+    dec.positions.fill_(context - 1)
+
+    def step():
+        dec.forward_hidden(None)
+        dec.head()
+        dec.greedy()
+    step()                                                  # warm-up: sizes the workspace
+    torch.cuda.synchronize()
+    stream, graph = torch.cuda.Stream(), torch.cuda.CUDAGraph()
+    with torch.cuda.stream(stream):
+        with torch.cuda.graph(graph, stream=stream):
+            step()
+    torch.cuda.synchronize()
+    for _ in range(max(1, a.warmup)):
+        graph.replay()
+    torch.cuda.synchronize()
+    t0 = time.perf_counter()
+    for _ in range(a.steps):
+        graph.replay()
+    torch.cuda.synchronize()
+    dt = (time.perf_counter() - t0) / a.steps
+    bpt = cfg.bytes_per_token(B, context)
+    gbps = bpt * B / dt / 1e9
+    assert bool(((dec.next_tokens >= 0) & (dec.next_tokens < cfg.vocab)).all()) and bool(torch.isfinite(dec.logits_f32).all())
+    return {
+        "metric": METRIC, "value": round(B / dt, 1), "unit": "tok/s", "n_gpus": 1, "steps": a.steps, "warmup": a.warmup,
+        "ms_per_step": round(dt * 1e3, 4), "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+        "dtype": "bf16 weights and activations, f32 accumulate, residual, norms, attention weights and recurrent state", "data": "synthetic",
+        "config": {"workload": "decode step of the Pakirax model, size %s: %d layers, width %d, vocab %d, window %d, greedy; batch %d at "
+                               "context %d, one HIP graph per step" % (a.size, len(cfg.layers), cfg.width, cfg.vocab,
+                                                                     cfg.layers[1][0].window, B, context),
+                   "batch": B, "context": context, "bytes_per_token_MB": round(bpt / 1e6, 1),
+                   "roofline_tok_per_s_at_8TBps": round(HBM_PEAK_GBPS * 1e9 / bpt, 1)},
+        "roofline": {"kernel": "whole step (all kernels of one graph replay)", "bound": "hbm", "achieved": round(gbps, 2),
+                     "peak": HBM_PEAK_GBPS, "unit": "GB/s", "frac": round(gbps / HBM_PEAK_GBPS, 4), "traffic": None,
+                     "traffic_source": None, "bytes_per_launch": round(bpt * B), "avg_launch_us": round(dt * 1e6, 2)},
+        "cpu_baseline": None,
+    }
+
+
+def run_pakirax_prefill(nv, torch, a):
+    """A prompt of `--tokens` tokens of one sequence through the Pakirax model at `--size` (random weights) in chunks of
+    `--chunk`, launched eagerly through the C ABI; the logits of the last token are not computed."""
+    T, chunk = a.tokens, a.chunk
+    ctx, cfg, dec = pakirax_model(nv, torch, a, 1, T, chunk)
+    gen = torch.Generator(device="cuda").manual_seed(9)
+    tokens = torch.randint(0, cfg.vocab, (T,), generator=gen, device="cuda", dtype=torch.int32)
+
+    def once():
+        dec.reset(0)
+        return dec.prefill_chunked(tokens, 0, 0, chunk)
+    for _ in range(max(1, a.warmup)):
+        last = once()
+    torch.cuda.synchronize()
+    assert bool(torch.isfinite(last.float()).all())
+    steps = max(1, a.steps)
+    t0 = time.perf_counter()
+    for _ in range(steps):
+        once()
+    torch.cuda.synchronize()
+    dt = (time.perf_counter() - t0) / steps
+    flops = cfg.prefill_flops(T) - 2.0 * cfg.vocab * cfg.width
+    tf = flops / dt / 1e12
+    return {
+        "metric": METRIC, "value": round(T / dt, 1), "unit": "tok/s", "n_gpus": 1, "steps": steps, "warmup": a.warmup,
+        "ms_per_step": round(dt * 1e3, 3), "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+        "dtype": "bf16 weights and activations, f32 accumulate, residual, norms, attention weights and recurrent state", "data": "synthetic",
+        "config": {"workload": "prompt of %d tokens through the Pakirax model, size %s (%d layers, width %d, window %d) in chunks of %d"
+                               % (T, a.size, len(cfg.layers), cfg.width, cfg.layers[1][0].window, chunk),
+                   "tokens": T, "chunk": chunk, "model_gflop_per_token": round(flops / T / 1e9, 2)},
+        "roofline": {"kernel": "whole prompt (all kernels)", "bound": "mfma", "achieved": round(tf, 2), "peak": MFMA_BF16_PEAK_TFLOPS,
+                     "unit": "TFLOP/s", "frac": round(tf / MFMA_BF16_PEAK_TFLOPS, 4), "traffic": None, "traffic_source": None,
+                     "flops_per_launch": flops, "avg_launch_us": round(dt * 1e6, 1)},
+        "cpu_baseline": None,
+    }
+
+
 def run_copy(torch, a):
     """A plain copy kernel of known size: 1 GiB read + 1 GiB written per launch."""
     n = 1 << 30
@@ -825,6 +937,8 @@ def main():
                 run_greedy(nv, ctx, torch, a) if a.workload == "greedy" else
                 run_step(nv, ctx, torch, a) if a.workload == "step" else
                 run_prefill_step(nv, ctx, torch, a) if a.workload == "prefill_step" else
+                run_pakirax_step(nv, torch, a) if a.workload == "pakirax_step" else
+                run_pakirax_prefill(nv, torch, a) if a.workload == "pakirax_prefill" else
                 run_read(nv, ctx, torch, a) if a.workload == "read" else run_copy(torch, a))
         print(json.dumps(line), flush=True)
         return

@@ -791,7 +791,7 @@ typedef struct {
  * with one row stride; a2 [heads * key_dim, rank] and a2_bias BF16; norm_weight BF16 [value_dim]; state
  * [slots, heads, key_dim, value_dim] floats, updated in place.  `batch` sequences of `rows` rows each: sequence b
  * uses slot slots[b] (device array), or slot + b when slots is NULL.  key_dim, value_dim multiples of 16, rank of 8,
- * value_dim <= 512.  The chunked form (one sequence, NULL slots, key_dim and value_dim <= 256) takes workspace. */
+ * none above 512.  The chunked form (one sequence, NULL slots, key_dim and value_dim <= 256) takes workspace. */
 typedef struct {
     uint32_t heads, key_dim, value_dim, value_count, rank;
     float tau, q_scale, eps;
@@ -818,7 +818,9 @@ typedef struct {
 } nvmai_latent_cache;
 
 /* From the down projections proj[t] = [.. c_q at q_at .. c_kv at kv_at .. rope part at rope_at ..]:
- * cq[t] = rmsnorm(c_q) * q_norm, and the token's cache row = [rmsnorm(c_kv) * kv_norm | rotated rope part]. */
+ * cq[t] = rmsnorm(c_q) * q_norm, and the token's cache row = [rmsnorm(c_kv) * kv_norm | rotated rope part].
+ * q_at, kv_at and the strides are multiples of 8; the columns up to the next multiple of 8 after q_count and
+ * rank_count are zero, and the norm weights are readable there. */
 int nvmai_hip_latent_epilogue(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_latent_config* config, const void* proj,
                               uint32_t proj_stride, uint32_t q_at, uint32_t q_count, const uint16_t* q_norm, uint32_t kv_at,
                               uint32_t rope_at, const uint16_t* kv_norm, void* cq, uint32_t cq_stride,

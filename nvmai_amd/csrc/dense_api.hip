@@ -22,9 +22,9 @@ int dense_linear_check(const nvmai_hip_ctx* ctx, const DenseLinearParams& p) {
 
 template <int NT>
 static void launch_gemv(const DenseLinearParams& p, hipStream_t s) {
-    // rows per wave: enough blocks for the device first, then more loads in flight per wave
-    if (p.n >= 8192) dense_gemv_kernel<NT, 4><<<(p.n + 15) / 16, 256, 0, s>>>(p);
-    else if (p.n >= 3072) dense_gemv_kernel<NT, 2><<<(p.n + 7) / 8, 256, 0, s>>>(p);
+    // rows per wave: one (short blocks, many of them) until the inputs' own loads weigh more than that
+    if (p.n >= 65536) dense_gemv_kernel<NT, 4><<<(p.n + 15) / 16, 256, 0, s>>>(p);
+    else if (NT > 2 && p.n >= 8192) dense_gemv_kernel<NT, 2><<<(p.n + 7) / 8, 256, 0, s>>>(p);
     else dense_gemv_kernel<NT, 1><<<(p.n + 3) / 4, 256, 0, s>>>(p);
 }
 
@@ -46,10 +46,21 @@ int dense_linear(nvmai_hip_ctx* ctx, hipStream_t s, const DenseLinearParams& p) 
         return launch_status();
     }
     if (p.rows <= 64) {
-        const uint32_t blocks = (p.n + 15) / 16;
-        if (p.rows <= 16) dense_skinny_kernel<1><<<blocks, 256, 0, s>>>(p);
-        else if (p.rows <= 32) dense_skinny_kernel<2><<<blocks, 256, 0, s>>>(p);
-        else dense_skinny_kernel<4><<<blocks, 256, 0, s>>>(p);
+        // row tiles per block: as many as leave every compute unit several blocks; waves: about four steps of k each
+        const int nr = p.n >= 32768 ? 4 : p.n >= 8192 ? 2 : 1;
+        const uint32_t blocks = (p.n + 16 * nr - 1) / (16 * nr);
+#define NVMAI_SKINNY(TT)                                                              \
+    do {                                                                              \
+        if (nr == 4) dense_skinny_kernel<TT, 4, 4><<<blocks, 256, 0, s>>>(p);         \
+        else if (nr == 2) dense_skinny_kernel<TT, 2, 4><<<blocks, 256, 0, s>>>(p);    \
+        else if (p.k <= 1024) dense_skinny_kernel<TT, 1, 4><<<blocks, 256, 0, s>>>(p); \
+        else if (p.k <= 2048) dense_skinny_kernel<TT, 1, 8><<<blocks, 512, 0, s>>>(p); \
+        else dense_skinny_kernel<TT, 1, 16><<<blocks, 1024, 0, s>>>(p);               \
+    } while (0)
+        if (p.rows <= 16) NVMAI_SKINNY(1);
+        else if (p.rows <= 32) NVMAI_SKINNY(2);
+        else NVMAI_SKINNY(4);
+#undef NVMAI_SKINNY
         return launch_status();
     }
     // the largest tile that still gives every compute unit one
@@ -73,6 +84,37 @@ extern "C" int nvmai_hip_dense_linear(nvmai_hip_ctx* ctx, nvmai_stream stream, c
     return dense_linear(ctx, (hipStream_t)stream, p);
 }
 
+namespace {
+
+template <int ACT, bool DELTA, bool POST, bool NEXT>
+void norm_residual_sized(const NormResidualParams& p, uint32_t rows, hipStream_t s) {
+    const bool vec = p.d % 4 == 0 && p.x_stride % 4 == 0 && aligned16(p.x) && (!DELTA || (p.delta_stride % 4 == 0 && aligned16(p.delta))) &&
+                     (!NEXT || (p.out_stride % 4 == 0 && aligned16(p.out))) && aligned16(p.post_w) && aligned16(p.post_b) &&
+                     aligned16(p.next_w) && aligned16(p.next_b);
+    const uint32_t vpt = (p.d + 1023) / 1024;
+    if (!vec) {
+        if (vpt <= 2) norm_residual_kernel<ACT, 2, DELTA, POST, NEXT, false><<<rows, 256, 0, s>>>(p);
+        else norm_residual_kernel<ACT, 16, DELTA, POST, NEXT, false><<<rows, 256, 0, s>>>(p);
+    } else if (vpt <= 1) norm_residual_kernel<ACT, 1, DELTA, POST, NEXT, true><<<rows, 256, 0, s>>>(p);
+    else if (vpt <= 2) norm_residual_kernel<ACT, 2, DELTA, POST, NEXT, true><<<rows, 256, 0, s>>>(p);
+    else if (vpt <= 4) norm_residual_kernel<ACT, 4, DELTA, POST, NEXT, true><<<rows, 256, 0, s>>>(p);
+    else if (vpt <= 8) norm_residual_kernel<ACT, 8, DELTA, POST, NEXT, true><<<rows, 256, 0, s>>>(p);
+    else norm_residual_kernel<ACT, 16, DELTA, POST, NEXT, true><<<rows, 256, 0, s>>>(p);
+}
+
+template <int ACT>
+int norm_residual(const NormResidualParams& p, uint32_t rows, hipStream_t s) {
+    const bool delta = p.delta, post = p.post_w, next = p.next_w;
+    if (delta && post && next) norm_residual_sized<ACT, true, true, true>(p, rows, s);
+    else if (delta && post) norm_residual_sized<ACT, true, true, false>(p, rows, s);
+    else if (delta && next) norm_residual_sized<ACT, true, false, true>(p, rows, s);
+    else if (delta) norm_residual_sized<ACT, true, false, false>(p, rows, s);
+    else if (next) norm_residual_sized<ACT, false, false, true>(p, rows, s);
+    return launch_status();
+}
+
+}  // namespace
+
 extern "C" int nvmai_hip_norm_residual(nvmai_hip_ctx* ctx, nvmai_stream stream, float* x, uint32_t x_stride, const float* delta,
                                        uint32_t delta_stride, const uint16_t* post_weight, const uint16_t* post_bias, float mult,
                                        const uint16_t* next_weight, const uint16_t* next_bias, void* out, uint32_t out_stride,
@@ -82,22 +124,10 @@ extern "C" int nvmai_hip_norm_residual(nvmai_hip_ctx* ctx, nvmai_stream stream, 
     if (ctx->act != NVMAI_ACT_BF16 && ctx->act != NVMAI_ACT_FP32) return NVMAI_ERR_UNSUPPORTED;
     if (d > 16384) return NVMAI_ERR_UNSUPPORTED;
     if (rows == 0) return NVMAI_OK;
+    if ((post_weight == nullptr) != (post_bias == nullptr) || (post_weight && !delta) || (next_weight == nullptr) != (next_bias == nullptr))
+        return NVMAI_ERR_INVALID_ARG;
     const NormResidualParams p{x, delta, post_weight, post_bias, next_weight, next_bias, out, x_stride, delta_stride, out_stride, d, mult, eps};
-    hipStream_t s = (hipStream_t)stream;
-    const uint32_t vpt = (d + 255) / 256;
-#define NVMAI_NR(ACT)                                                                            \
-    do {                                                                                         \
-        if (vpt <= 1) norm_residual_kernel<ACT, 1><<<rows, 256, 0, s>>>(p);                      \
-        else if (vpt <= 2) norm_residual_kernel<ACT, 2><<<rows, 256, 0, s>>>(p);                 \
-        else if (vpt <= 4) norm_residual_kernel<ACT, 4><<<rows, 256, 0, s>>>(p);                 \
-        else if (vpt <= 8) norm_residual_kernel<ACT, 8><<<rows, 256, 0, s>>>(p);                 \
-        else if (vpt <= 16) norm_residual_kernel<ACT, 16><<<rows, 256, 0, s>>>(p);               \
-        else if (vpt <= 32) norm_residual_kernel<ACT, 32><<<rows, 256, 0, s>>>(p);               \
-        else norm_residual_kernel<ACT, 64><<<rows, 256, 0, s>>>(p);                              \
-    } while (0)
-    if (ctx->act == NVMAI_ACT_BF16) NVMAI_NR(ACT_BF16); else NVMAI_NR(ACT_FP32);
-#undef NVMAI_NR
-    return launch_status();
+    return ctx->act == NVMAI_ACT_BF16 ? norm_residual<ACT_BF16>(p, rows, (hipStream_t)stream) : norm_residual<ACT_FP32>(p, rows, (hipStream_t)stream);
 }
 
 extern "C" int nvmai_hip_embed_rows(nvmai_hip_ctx* ctx, nvmai_stream stream, const uint16_t* table, uint32_t table_stride,
@@ -114,6 +144,13 @@ extern "C" int nvmai_hip_argmax_rows(nvmai_hip_ctx* ctx, nvmai_stream stream, co
                                      uint32_t n, uint32_t* out_index) {
     if (!ctx || !x || !out_index || n == 0 || x_stride < n) return NVMAI_ERR_INVALID_ARG;
     if (rows == 0) return NVMAI_OK;
-    argmax_rows_kernel<<<rows, 1024, 0, (hipStream_t)stream>>>(x, x_stride, n, out_index);
+    if (rows > 65535) return NVMAI_ERR_UNSUPPORTED;
+    const int rc = ws_begin(ctx, stream, ws_round((size_t)rows * ARGMAX_BLOCKS * 8));
+    if (rc) return rc;
+    uint64_t* part = ws_take<uint64_t>(ctx, (size_t)rows * ARGMAX_BLOCKS);
+    uint32_t blocks = (n + 1023) / 1024;
+    if (blocks > ARGMAX_BLOCKS) blocks = ARGMAX_BLOCKS;
+    argmax_stage1_kernel<<<dim3(blocks, rows), 256, 0, (hipStream_t)stream>>>(x, x_stride, n, part);
+    argmax_stage2_kernel<<<rows, 256, 0, (hipStream_t)stream>>>(part, blocks, out_index);
     return launch_status();
 }

@@ -104,52 +104,66 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(DenseLinearParams p) {
         }
 }
 
-// ---- 5 .. 64 input rows: 16 weight rows per block, the waves split k, MFMA, sums through LDS ---------
+// ---- 5 .. 64 input rows: 16 NR weight rows per block, the waves split k, MFMA, sums through LDS ---------
 // Weight rows are the A operand as they lie in memory: lane (i = lane % 16, g = lane / 16) loads the 32 bytes
 // W[r0 + i, k + 16 g .. + 16), four lanes cover 128 contiguous bytes of a row; the inputs are the B operand in
-// the same order of k.
-template <int TT>
-__global__ __launch_bounds__(256) void dense_skinny_kernel(DenseLinearParams p) {
-    __shared__ __attribute__((aligned(16))) float part[3][64][TT * 4];
+// the same order of k, read from L2 once per NR row tiles.
+template <int TT, int NR, int NW>
+__global__ __launch_bounds__(64 * NW) void dense_skinny_kernel(DenseLinearParams p) {
+    __shared__ __attribute__((aligned(16))) float part[NW - 1][64][TT * NR * 4];
     const uint32_t lane = threadIdx.x & 63u, wave = threadIdx.x >> 6, i = lane & 15u, g = lane >> 4;
-    const uint32_t r0 = blockIdx.x * 16u;
-    const uint16_t* wp = p.w + (size_t)min(r0 + i, p.n - 1u) * p.w_stride + g * 16u;
+    const uint32_t r0 = blockIdx.x * (16u * NR);
+    const uint16_t* wp[NR];
+#pragma unroll
+    for (int r = 0; r < NR; ++r) wp[r] = p.w + (size_t)min(r0 + 16u * r + i, p.n - 1u) * p.w_stride + g * 16u;
     const uint16_t* x = static_cast<const uint16_t*>(p.x);
     const uint16_t* xp[TT];
 #pragma unroll
     for (int t = 0; t < TT; ++t) xp[t] = x + (size_t)min(16u * t + i, p.rows - 1u) * p.x_stride + g * 16u;
-    dn_f4 acc[TT];
+    dn_f4 acc[NR][TT];
 #pragma unroll
-    for (int t = 0; t < TT; ++t) acc[t] = dn_f4{0.0f, 0.0f, 0.0f, 0.0f};
+    for (int r = 0; r < NR; ++r)
+#pragma unroll
+        for (int t = 0; t < TT; ++t) acc[r][t] = dn_f4{0.0f, 0.0f, 0.0f, 0.0f};
     const uint32_t steps = p.k / 64u;
 #pragma unroll 4
-    for (uint32_t st = wave; st < steps; st += 4u) {
-        const uint4 a0 = *reinterpret_cast<const uint4*>(wp + st * 64u), a1 = *reinterpret_cast<const uint4*>(wp + st * 64u + 8u);
-        uint4 b0[TT], b1[TT];
+    for (uint32_t st = wave; st < steps; st += NW) {
+        uint4 a0[NR], a1[NR], b0[TT], b1[TT];
+#pragma unroll
+        for (int r = 0; r < NR; ++r) {
+            a0[r] = *reinterpret_cast<const uint4*>(wp[r] + st * 64u);
+            a1[r] = *reinterpret_cast<const uint4*>(wp[r] + st * 64u + 8u);
+        }
 #pragma unroll
         for (int t = 0; t < TT; ++t) {
             b0[t] = *reinterpret_cast<const uint4*>(xp[t] + st * 64u);
             b1[t] = *reinterpret_cast<const uint4*>(xp[t] + st * 64u + 8u);
         }
 #pragma unroll
-        for (int t = 0; t < TT; ++t) {
-            acc[t] = dn_mfma(a0, b0[t], acc[t]);
-            acc[t] = dn_mfma(a1, b1[t], acc[t]);
-        }
+        for (int r = 0; r < NR; ++r)
+#pragma unroll
+            for (int t = 0; t < TT; ++t) {
+                acc[r][t] = dn_mfma(a0[r], b0[t], acc[r][t]);
+                acc[r][t] = dn_mfma(a1[r], b1[t], acc[r][t]);
+            }
     }
     if (wave != 0) {
 #pragma unroll
-        for (int t = 0; t < TT; ++t) *reinterpret_cast<dn_f4*>(&part[wave - 1][lane][4 * t]) = acc[t];
+        for (int r = 0; r < NR; ++r)
+#pragma unroll
+            for (int t = 0; t < TT; ++t) *reinterpret_cast<dn_f4*>(&part[wave - 1][lane][4 * (r * TT + t)]) = acc[r][t];
     }
     __syncthreads();
     if (wave != 0) return;
 #pragma unroll
-    for (int t = 0; t < TT; ++t) {
+    for (int r = 0; r < NR; ++r)
 #pragma unroll
-        for (int w = 0; w < 3; ++w) acc[t] += *reinterpret_cast<const dn_f4*>(&part[w][lane][4 * t]);
-        // acc[t][j] = y[token 16 t + i, row r0 + 4 g + j]
-        if (16u * t + i < p.rows) dense_store4_bf16(p, 16u * t + i, r0 + 4u * g, acc[t]);
-    }
+        for (int t = 0; t < TT; ++t) {
+#pragma unroll
+            for (int w = 0; w < NW - 1; ++w) acc[r][t] += *reinterpret_cast<const dn_f4*>(&part[w][lane][4 * (r * TT + t)]);
+            // acc[r][t][j] = y[token 16 t + i, row r0 + 16 r + 4 g + j]
+            if (16u * t + i < p.rows) dense_store4_bf16(p, 16u * t + i, r0 + 16u * r + 4u * g, acc[r][t]);
+        }
 }
 
 // ---- many input rows: tiles of BN weight rows x BM tokens, k in steps of 64 through double-buffered LDS --------
@@ -283,71 +297,117 @@ __device__ __forceinline__ float block_sum256(float v, float* lds) {
     return (lds[0] + lds[1]) + (lds[2] + lds[3]);
 }
 
-// (v - mean) / sqrt(mean((v - mean)^2) + eps) over the d elements tid, tid + 256, ... held in v; dead slots are zero.
+// (v - mean) / sqrt(mean((v - mean)^2) + eps) over the row's d elements, dead slots zero before and after.
+// Thread t holds the elements 4 (t + 256 j) .. + 3.
 template <int VPT>
-__device__ __forceinline__ void block_layernorm(float (&v)[VPT], uint32_t d, float eps, float* lds) {
+__device__ __forceinline__ void block_layernorm(float (&v)[VPT][4], uint32_t d, float eps, float* lds) {
     float s = 0.0f;
 #pragma unroll
-    for (int j = 0; j < VPT; ++j) s += v[j];
+    for (int j = 0; j < VPT; ++j) s += (v[j][0] + v[j][1]) + (v[j][2] + v[j][3]);
     const float mean = block_sum256(s, lds) / (float)d;
     float q = 0.0f;
 #pragma unroll
-    for (int j = 0; j < VPT; ++j) {
-        const bool live = threadIdx.x + 256u * j < d;
-        v[j] = live ? v[j] - mean : 0.0f;
-        q = fmaf(v[j], v[j], q);
-    }
+    for (int j = 0; j < VPT; ++j)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            v[j][e] = 4u * (threadIdx.x + 256u * j) + e < d ? v[j][e] - mean : 0.0f;
+            q = fmaf(v[j][e], v[j][e], q);
+        }
     const float inv = 1.0f / sqrtf(block_sum256(q, lds + 4) / (float)d + eps);
 #pragma unroll
-    for (int j = 0; j < VPT; ++j) v[j] *= inv;
+    for (int j = 0; j < VPT; ++j)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[j][e] *= inv;
 }
 
 struct NormResidualParams {
     float* x;                        // [rows, x_stride] residual stream
-    const float* delta;              // sublayer output, nullptr = none
-    const uint16_t *post_w, *post_b; // norm of delta, nullptr = delta is added as it is
-    const uint16_t *next_w, *next_b; // norm that opens the next sublayer, nullptr = no output
+    const float* delta;              // sublayer output
+    const uint16_t *post_w, *post_b; // norm of delta
+    const uint16_t *next_w, *next_b; // norm that opens the next sublayer
     void* out;
     uint32_t x_stride, delta_stride, out_stride, d;
     float mult, eps;
 };
 
-// x += mult * LN(delta); out = LN(x): one block per row, the row in registers.
-template <int ACT, int VPT>
+__device__ __forceinline__ void norm_bf4(const uint16_t* p, float* v) {
+    const uint2 q = *reinterpret_cast<const uint2*>(p);
+    act2_to_f32<ACT_BF16>(q.x, v[0], v[1]);
+    act2_to_f32<ACT_BF16>(q.y, v[2], v[3]);
+}
+
+// x += mult * LN(delta) (POST; DELTA: x += mult * delta); out = LN(x) (NEXT): one block per row, the row in registers.
+// Every operand is requested before the first sum.  VEC: four elements per load (d and the strides are multiples
+// of 4); dead slots reread the row's last elements.
+template <int ACT, int VPT, bool DELTA, bool POST, bool NEXT, bool VEC>
 __global__ __launch_bounds__(256) void norm_residual_kernel(NormResidualParams p) {
     __shared__ float lds[16];
     const uint32_t row = blockIdx.x, tid = threadIdx.x;
     float* x = p.x + (size_t)row * p.x_stride;
-    float xv[VPT], dv[VPT], pw[VPT], pb[VPT], nw[VPT], nb[VPT];
+    const float* delta = p.delta + (size_t)row * p.delta_stride;
+    float xv[VPT][4], dv[VPT][4], pw[VPT][4], pb[VPT][4], nw[VPT][4], nb[VPT][4];
 #pragma unroll
-    for (int j = 0; j < VPT; ++j) {          // every operand requested up front, dead slots reread the last element
-        const uint32_t at = min(tid + 256u * j, p.d - 1u);
-        xv[j] = x[at];
-        dv[j] = p.delta ? p.delta[(size_t)row * p.delta_stride + at] : 0.0f;
-        pw[j] = p.post_w ? bf16_to_f32(p.post_w[at]) : 1.0f;
-        pb[j] = p.post_b ? bf16_to_f32(p.post_b[at]) : 0.0f;
-        nw[j] = p.next_w ? bf16_to_f32(p.next_w[at]) : 1.0f;
-        nb[j] = p.next_b ? bf16_to_f32(p.next_b[at]) : 0.0f;
+    for (int j = 0; j < VPT; ++j) {
+        const uint32_t at = 4u * (tid + 256u * j);
+        if (VEC) {
+            const uint32_t c = min(at, p.d - 4u);
+            *reinterpret_cast<dn_f4*>(xv[j]) = *reinterpret_cast<const dn_f4*>(x + c);
+            if (DELTA) *reinterpret_cast<dn_f4*>(dv[j]) = *reinterpret_cast<const dn_f4*>(delta + c);
+            if (POST) { norm_bf4(p.post_w + c, pw[j]); norm_bf4(p.post_b + c, pb[j]); }
+            if (NEXT) { norm_bf4(p.next_w + c, nw[j]); norm_bf4(p.next_b + c, nb[j]); }
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const uint32_t c = min(at + e, p.d - 1u);
+                xv[j][e] = x[c];
+                if (DELTA) dv[j][e] = delta[c];
+                if (POST) { pw[j][e] = bf16_to_f32(p.post_w[c]); pb[j][e] = bf16_to_f32(p.post_b[c]); }
+                if (NEXT) { nw[j][e] = bf16_to_f32(p.next_w[c]); nb[j][e] = bf16_to_f32(p.next_b[c]); }
+            }
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+            if (at + e >= p.d) { xv[j][e] = 0.0f; if (DELTA) dv[j][e] = 0.0f; }
     }
-#pragma unroll
-    for (int j = 0; j < VPT; ++j)
-        if (tid + 256u * j >= p.d) { xv[j] = 0.0f; dv[j] = 0.0f; }
-    if (p.delta) {
-        if (p.post_w) block_layernorm<VPT>(dv, p.d, p.eps, lds);
+    if (DELTA) {
+        if (POST) block_layernorm<VPT>(dv, p.d, p.eps, lds);
 #pragma unroll
         for (int j = 0; j < VPT; ++j) {
-            const bool live = tid + 256u * j < p.d;
-            const float add = p.post_w ? fmaf(dv[j], pw[j], pb[j]) : dv[j];
-            xv[j] = live ? fmaf(p.mult, add, xv[j]) : 0.0f;
-            if (live) x[tid + 256u * j] = xv[j];
+            const uint32_t at = 4u * (tid + 256u * j);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const float add = POST ? fmaf(dv[j][e], pw[j][e], pb[j][e]) : dv[j][e];
+                xv[j][e] = at + e < p.d ? fmaf(p.mult, add, xv[j][e]) : 0.0f;
+            }
+            if (VEC) {
+                if (at < p.d) *reinterpret_cast<dn_f4*>(x + at) = *reinterpret_cast<dn_f4*>(xv[j]);
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (at + e < p.d) x[at + e] = xv[j][e];
+            }
         }
     }
-    if (!p.next_w) return;
+    if (!NEXT) return;
     block_layernorm<VPT>(xv, p.d, p.eps, lds + 8);
     act_t<ACT>* out = static_cast<act_t<ACT>*>(p.out) + (size_t)row * p.out_stride;
 #pragma unroll
-    for (int j = 0; j < VPT; ++j)
-        if (tid + 256u * j < p.d) out[tid + 256u * j] = f32_to_act<ACT>(fmaf(xv[j], nw[j], nb[j]));
+    for (int j = 0; j < VPT; ++j) {
+        const uint32_t at = 4u * (tid + 256u * j);
+        act_t<ACT> o[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] = f32_to_act<ACT>(fmaf(xv[j][e], nw[j][e], nb[j][e]));
+        if (VEC) {
+            if (at < p.d) {
+                if constexpr (ACT == ACT_FP32) *reinterpret_cast<dn_f4*>(out + at) = dn_f4{o[0], o[1], o[2], o[3]};
+                else *reinterpret_cast<uint2*>(out + at) = make_uint2(o[0] | ((uint32_t)o[1] << 16), o[2] | ((uint32_t)o[3] << 16));
+            }
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (at + e < p.d) out[at + e] = o[e];
+        }
+    }
 }
 
 // Rows of a BF16 table as 32-bit residual rows; an id past the table gives zeros.
@@ -359,26 +419,47 @@ __global__ __launch_bounds__(256) void embed_rows_kernel(const uint16_t* table, 
     out[(size_t)row * out_stride + j] = id < vocab ? bf16_to_f32(table[(size_t)id * table_stride + j]) : 0.0f;
 }
 
-// Index of the largest finite value of each row, ties to the lower index, 0 when none is finite.
-__global__ __launch_bounds__(1024) void argmax_rows_kernel(const float* x, uint32_t x_stride, uint32_t n, uint32_t* out) {
-    __shared__ float bv[16];
-    __shared__ uint32_t bi[16];
-    const float* row = x + (size_t)blockIdx.x * x_stride;
-    float v = -INFINITY;
-    uint32_t at = 0xFFFFFFFFu;
-    for (uint32_t j = threadIdx.x; j < n; j += 1024u) {
-        const float c = row[j];
-        if (c > v && c < INFINITY) { v = c; at = j; }
+// Index of the largest finite value of each row, ties to the lower index, 0 when none is finite.  A candidate is one
+// 64-bit key: the value in the upper half (mapped so that unsigned order is the order of the floats), the complement
+// of the index in the lower; 0 = none.
+constexpr uint32_t ARGMAX_BLOCKS = 64;
+
+__device__ __forceinline__ uint64_t argmax_key(float v, uint32_t index) {
+    const uint32_t b = __float_as_uint(v);
+    if ((b & 0x7F800000u) == 0x7F800000u) return 0ull;         // infinite or not a number
+    const uint32_t o = b == 0x80000000u ? 0x80000000u : (b & 0x80000000u) ? ~b : b | 0x80000000u;    // -0 ranks as 0
+    return ((uint64_t)o << 32) | (uint32_t)~index;
+}
+
+__device__ __forceinline__ uint64_t argmax_block(uint64_t best, uint64_t* lds) {
+#pragma unroll
+    for (int off = 32; off >= 1; off >>= 1) {
+        const uint64_t o = ((uint64_t)shfl_xor_u((uint32_t)(best >> 32), off) << 32) | shfl_xor_u((uint32_t)best, off);
+        best = o > best ? o : best;
     }
-    const float wm = wave_max_f32(v);
-    const uint32_t wi = wave_min_u32(v == wm ? at : 0xFFFFFFFFu);
-    if ((threadIdx.x & 63u) == 0) { bv[threadIdx.x >> 6] = wm; bi[threadIdx.x >> 6] = wi; }
+    if ((threadIdx.x & 63u) == 0) lds[threadIdx.x >> 6] = best;
     __syncthreads();
-    if (threadIdx.x != 0) return;
-    for (int w = 1; w < 16; ++w)
-        if (bv[w] > v || (bv[w] == v && bi[w] < at)) { v = bv[w]; at = bi[w]; }
-    if (bv[0] > v || (bv[0] == v && bi[0] < at)) { at = bi[0]; }
-    out[blockIdx.x] = at == 0xFFFFFFFFu ? 0u : at;
+    for (int w = 0; w < 4; ++w) best = lds[w] > best ? lds[w] : best;
+    return best;
+}
+
+__global__ __launch_bounds__(256) void argmax_stage1_kernel(const float* x, uint32_t x_stride, uint32_t n, uint64_t* part) {
+    __shared__ uint64_t lds[4];
+    const float* row = x + (size_t)blockIdx.y * x_stride;
+    uint64_t best = 0;
+#pragma unroll 4
+    for (uint32_t j = blockIdx.x * 256u + threadIdx.x; j < n; j += 256u * gridDim.x) {
+        const uint64_t k = argmax_key(row[j], j);
+        best = k > best ? k : best;
+    }
+    best = argmax_block(best, lds);
+    if (threadIdx.x == 0) part[blockIdx.y * ARGMAX_BLOCKS + blockIdx.x] = best;
+}
+
+__global__ __launch_bounds__(256) void argmax_stage2_kernel(const uint64_t* part, uint32_t blocks, uint32_t* out) {
+    __shared__ uint64_t lds[4];
+    const uint64_t best = argmax_block(threadIdx.x < blocks ? part[blockIdx.x * ARGMAX_BLOCKS + threadIdx.x] : 0ull, lds);
+    if (threadIdx.x == 0) out[blockIdx.x] = best == 0ull ? 0u : ~(uint32_t)best;
 }
 
 }  // namespace nvmai

@@ -6,16 +6,24 @@ using namespace nvmai;
 
 namespace {
 
+template <int ACT, int PER, uint32_t NTH>
+int gla_recurrent_sized(const GlaParams& p, uint32_t batch, hipStream_t s) {
+    const size_t groups = NTH / p.dv, chans = PER > 0 ? groups * PER : p.dk;
+    if (chans > NTH) return NVMAI_ERR_UNSUPPORTED;
+    const size_t lds = (3 * chans + 16 + groups * p.dv + p.rank) * 4;
+    if (lds > 64 * 1024) return NVMAI_ERR_UNSUPPORTED;
+    gla_recurrent_kernel<ACT, PER, NTH><<<dim3(p.heads, batch), NTH, lds, s>>>(p);
+    return launch_status();
+}
+
 template <int ACT>
 int gla_recurrent(const GlaParams& p, uint32_t batch, hipStream_t s) {
-    const uint32_t groups = 512u / p.dv, per = (p.dk + groups - 1) / groups;
-    const size_t lds = ((size_t)3 * p.dk + (size_t)groups * p.dv + 8 + p.rank) * 4;
-    if (lds > 64 * 1024) return NVMAI_ERR_UNSUPPORTED;
-    const dim3 grid(p.heads, batch);
-    if (per <= 8) gla_recurrent_kernel<ACT, 8><<<grid, 512, lds, s>>>(p);
-    else if (per <= 32) gla_recurrent_kernel<ACT, 32><<<grid, 512, lds, s>>>(p);
-    else gla_recurrent_kernel<ACT, 0><<<grid, 512, lds, s>>>(p);
-    return launch_status();
+    auto per = [&](uint32_t threads) { return (p.dk + threads / p.dv - 1) / (threads / p.dv); };
+    if (per(1024) <= 4) return gla_recurrent_sized<ACT, 4, 1024>(p, batch, s);
+    if (per(1024) <= 8) return gla_recurrent_sized<ACT, 8, 1024>(p, batch, s);
+    if (per(1024) <= 16) return gla_recurrent_sized<ACT, 16, 1024>(p, batch, s);
+    if (per(1024) <= 32) return gla_recurrent_sized<ACT, 32, 1024>(p, batch, s);
+    return gla_recurrent_sized<ACT, 0, 1024>(p, batch, s);
 }
 
 template <int ACT, int KT>
@@ -30,8 +38,8 @@ void gla_spans(const GlaParams& p, uint32_t subs, uint32_t spans, hipStream_t s)
 
 template <int ACT>
 int gla_chunked(const GlaParams& p, hipStream_t s) {
-    const uint32_t subs = (p.rows + GLA_SUB - 1) / GLA_SUB, spans = (subs + GLA_SPAN - 1) / GLA_SPAN;
-    const size_t lds = ((size_t)48 * (p.dk + 4) + (size_t)16 * p.rank) * 4;
+    const uint32_t subs = (p.rows + GLA_SUB - 1) / GLA_SUB, spans = (subs + p.span - 1) / p.span;
+    const size_t lds = ((size_t)48 * (p.dk + 4) + 2 * (size_t)p.dk + 1024 + (size_t)16 * p.rank) * 4;
     static bool raised = false;
     if (!raised) {
         NVMAI_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void*>(gla_prep_kernel<ACT>), hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024));
@@ -58,7 +66,7 @@ extern "C" int nvmai_hip_gla(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvma
     const nvmai_gla_config& c = *config;
     if (c.heads == 0 || c.key_dim == 0 || c.value_dim == 0 || c.rank == 0 || c.value_count == 0 || c.value_count > c.value_dim) return NVMAI_ERR_INVALID_ARG;
     if (c.key_dim % 16 || c.value_dim % 16 || c.rank % 8) return NVMAI_ERR_INVALID_ARG;
-    if (c.value_dim > 512) return NVMAI_ERR_UNSUPPORTED;
+    if (c.value_dim > 512 || c.key_dim > 512 || c.rank > 512) return NVMAI_ERR_UNSUPPORTED;
     if (!(c.tau > 0.0f)) return NVMAI_ERR_INVALID_ARG;
     if (proj_stride < c.heads * c.key_dim || proj_stride < c.heads * c.value_dim || proj_stride < c.rank || out_stride < c.heads * c.value_dim)
         return NVMAI_ERR_INVALID_ARG;
@@ -72,13 +80,15 @@ extern "C" int nvmai_hip_gla(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvma
     p.heads = c.heads; p.dk = c.key_dim; p.dv = c.value_dim; p.dv_count = c.value_count; p.rank = c.rank; p.rows = rows;
     p.inv_tau = 1.0f / c.tau; p.q_scale = c.q_scale; p.eps = c.eps;
     hipStream_t s = (hipStream_t)stream;
-    const bool can_chunk = batch == 1 && !slots && c.key_dim <= GLA_MAX_DIM && c.value_dim <= GLA_MAX_DIM && c.rank <= 512 &&
-                           (rows + GLA_SUB - 1) / GLA_SUB <= 0x7FFFFFFFu;
+    const bool can_chunk = batch == 1 && !slots && c.key_dim <= GLA_MAX_DIM && c.value_dim <= GLA_MAX_DIM;
     if (form == NVMAI_GLA_CHUNKED && !can_chunk) return NVMAI_ERR_UNSUPPORTED;
     // below two spans' worth of rows the launches of the chunked form cost more than the rows
     const bool chunk = form == NVMAI_GLA_CHUNKED || (form == NVMAI_FORM_AUTO && can_chunk && rows >= 32);
     if (!chunk) return ctx->act == NVMAI_ACT_BF16 ? gla_recurrent<ACT_BF16>(p, batch, s) : gla_recurrent<ACT_FP32>(p, batch, s);
-    const size_t subs = (rows + GLA_SUB - 1) / GLA_SUB, spans = (subs + GLA_SPAN - 1) / GLA_SPAN;
+    const size_t subs = (rows + GLA_SUB - 1) / GLA_SUB;
+    // long spans (fewer states through memory) as soon as they still make two blocks per compute unit
+    p.span = (subs / 8) * c.heads >= 2 * (size_t)ctx->compute_units ? 8 : 4;
+    const size_t spans = (subs + p.span - 1) / p.span;
     if (spans > 65535) return NVMAI_ERR_UNSUPPORTED;
     const size_t n_qd = subs * c.heads * 16 * c.key_dim, n_edge = subs * c.heads * c.key_dim, n_att = subs * c.heads * 256;
     const size_t n_spans = spans * c.heads * c.key_dim * c.value_dim, n_dec = spans * c.heads * c.key_dim;

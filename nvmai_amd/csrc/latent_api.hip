@@ -39,10 +39,10 @@ int launch_partial(const LatentAttnParams& p, hipStream_t s) {
 
 template <int ACT>
 int absorbed(const LatentAttnParams& p, hipStream_t s) {
-    const size_t lds_a = ((size_t)p.nope + 4 * (size_t)p.rank) * 4;
+    const size_t lds_a = (size_t)p.nope * 4;
     int rc = raise_lds(reinterpret_cast<const void*>(latent_absorb_kernel<ACT>), lds_a);
     if (rc) return rc;
-    latent_absorb_kernel<ACT><<<dim3(p.heads, p.n_rows), 256, lds_a, s>>>(p);
+    latent_absorb_kernel<ACT><<<dim3(p.heads, p.n_rows, (p.rank + 127) / 128 + 1), 256, lds_a, s>>>(p);
     const uint32_t rest = p.cache.row_stride - p.rank;
     if (ACT == ACT_BF16 && p.rank <= 1024 && rest <= 128) {
         rc = p.rank <= 128 ? launch_partial<2>(p, s) : p.rank <= 256 ? launch_partial<4>(p, s) : p.rank <= 512 ? launch_partial<8>(p, s) : launch_partial<16>(p, s);
@@ -52,23 +52,25 @@ int absorbed(const LatentAttnParams& p, hipStream_t s) {
         if (!rc) latent_partial_plain_kernel<ACT><<<dim3(p.splits, p.heads, p.n_rows), 256, lds, s>>>(p);
     }
     if (rc) return rc;
-    const size_t lds_c = ((size_t)p.rank + p.splits) * 4;
+    const size_t lds_c = (9 * (size_t)p.rank + p.splits) * 4;
     rc = raise_lds(reinterpret_cast<const void*>(latent_combine_kernel<ACT>), lds_c);
     if (rc) return rc;
-    const uint32_t slices = p.n_rows * p.heads >= 128 ? 1 : p.vdim >= 64 ? 4 : 1;
-    latent_combine_kernel<ACT><<<dim3(p.heads, p.n_rows, slices), 256, lds_c, s>>>(p);
+    latent_combine_kernel<ACT><<<dim3(p.heads, p.n_rows), 1024, lds_c, s>>>(p);
     return launch_status();
 }
 
-template <int DQ, int DV>
-void launch_flash(const LatentAttnParams& p, hipStream_t s) {
-    latent_flash_kernel<DQ, DV><<<dim3((p.n_rows + 127) / 128, p.heads), 256, 0, s>>>(p);
+template <int NP, int RP, int DV>
+int launch_flash(const LatentAttnParams& p, hipStream_t s) {
+    const size_t lds = 2 * ((size_t)64 * (NP + RP) * 2 + (size_t)DV * 128);
+    const int rc = raise_lds(reinterpret_cast<const void*>(latent_flash_kernel<NP, RP, DV>), lds);
+    if (rc) return rc;
+    latent_flash_kernel<NP, RP, DV><<<(p.n_rows + 127) / 128 * p.heads, 256, lds, s>>>(p);
+    return launch_status();
 }
-template <int DQ>
-void launch_flash_v(const LatentAttnParams& p, hipStream_t s) {
-    if (p.vdim <= 64) launch_flash<DQ, 64>(p, s);
-    else if (p.vdim <= 128) launch_flash<DQ, 128>(p, s);
-    else launch_flash<DQ, 256>(p, s);
+
+template <int NP, int RP>
+int launch_flash_v(const LatentAttnParams& p, hipStream_t s) {
+    return p.vdim <= 64 ? launch_flash<NP, RP, 64>(p, s) : launch_flash<NP, RP, 128>(p, s);
 }
 
 }  // namespace
@@ -81,6 +83,9 @@ extern "C" int nvmai_hip_latent_epilogue(nvmai_hip_ctx* ctx, nvmai_stream stream
     if (rc) return rc;
     const nvmai_latent_config& c = *config;
     if (!proj || !q_norm || !kv_norm || !cq || !map || q_count == 0 || cq_stride < q_count) return NVMAI_ERR_INVALID_ARG;
+    if (q_at % 8 || kv_at % 8 || proj_stride % 8 || cq_stride % 8 || !aligned16(proj) || !aligned16(cq) || !aligned16(q_norm) || !aligned16(kv_norm))
+        return NVMAI_ERR_ALIGNMENT;
+    if (cq_stride < (q_count + 7) / 8 * 8) return NVMAI_ERR_INVALID_ARG;
     if (proj_stride < q_at + q_count || proj_stride < kv_at + c.rank_count || proj_stride < rope_at + c.rope_dim) return NVMAI_ERR_INVALID_ARG;
     if (!map->positions && rows > cache->capacity) return NVMAI_ERR_INVALID_ARG;       // two rows of one call in one place
     if (rows == 0) return NVMAI_OK;
@@ -89,8 +94,17 @@ extern "C" int nvmai_hip_latent_epilogue(nvmai_hip_ctx* ctx, nvmai_stream stream
     p.proj_stride = proj_stride; p.q_at = q_at; p.kv_at = kv_at; p.rot_at = rope_at; p.cq_stride = cq_stride; p.q_count = q_count;
     p.rank_count = c.rank_count; p.rank = c.rank; p.rot_dim = c.rope_dim; p.rot_dims = c.rotary_dims; p.eps = c.eps;
     hipStream_t s = (hipStream_t)stream;
-    if (ctx->act == NVMAI_ACT_BF16) latent_epilogue_kernel<ACT_BF16><<<rows, 256, 0, s>>>(p);
-    else latent_epilogue_kernel<ACT_FP32><<<rows, 256, 0, s>>>(p);
+    const uint32_t pieces = (q_count + 7) / 8 + (c.rank_count + 7) / 8;
+#define NVMAI_LE(NP)                                                                              \
+    do {                                                                                          \
+        if (ctx->act == NVMAI_ACT_BF16) latent_epilogue_kernel<ACT_BF16, NP><<<rows, 256, 0, s>>>(p); \
+        else latent_epilogue_kernel<ACT_FP32, NP><<<rows, 256, 0, s>>>(p);                        \
+    } while (0)
+    if (pieces <= 256) NVMAI_LE(1);
+    else if (pieces <= 512) NVMAI_LE(2);
+    else if (pieces <= 2048) NVMAI_LE(8);
+    else return NVMAI_ERR_UNSUPPORTED;
+#undef NVMAI_LE
     return launch_status();
 }
 
@@ -128,11 +142,10 @@ extern "C" int nvmai_hip_latent_attention(nvmai_hip_ctx* ctx, nvmai_stream strea
     if (!expand) {
         uint32_t keys = known ? last : cache->capacity;
         if (c.window && c.window < keys) keys = c.window;
-        // about four blocks per compute unit, at least 64 keys each
+        // about two blocks per compute unit, at least 32 keys each
         const uint32_t groups = f32 ? c.heads : (c.heads + 15) / 16;
-        const uint32_t want = 4u * (uint32_t)ctx->compute_units / (rows * groups) + 1u;
-        uint32_t per = ((keys + want - 1) / want + 31) / 32 * 32;
-        if (per < 64) per = 64;
+        const uint32_t want = 2u * (uint32_t)ctx->compute_units / (rows * groups) + 1u;
+        const uint32_t per = ((keys + want - 1) / want + 31) / 32 * 32;
         p.split_keys = per;
         p.splits = (keys + per - 1) / per;
         const size_t cells = (size_t)rows * c.heads * p.splits, n_qa = (size_t)rows * c.heads * cache->row_stride;
@@ -148,17 +161,24 @@ extern "C" int nvmai_hip_latent_attention(nvmai_hip_ctx* ctx, nvmai_stream strea
     p.nk = last - p.key0;
     p.nk_pad = (p.nk + 63) / 64 * 64;
     const uint32_t dq = c.nope_dim + c.rope_dim;
-    const bool flash = !f32 && dq <= 256 && c.value_dim <= 256;
-    const size_t n_lat = (size_t)p.nk_pad * cache->row_stride, n_kn = (size_t)p.nk_pad * c.heads * c.nope_dim, n_v = (size_t)p.nk_pad * c.heads * c.value_dim;
+    bool flash = !f32 && c.nope_dim <= 256 && c.rope_dim <= 128 && c.value_dim <= 256;
+    // rows an odd number of 128-byte lines apart: a tile's rows then spread over the memory channels
+    auto odd_lines = [](uint32_t n) { return (n + 63) / 64 % 2 ? (n + 63) / 64 * 64 : ((n + 63) / 64 + 1) * 64; };
+    const uint32_t nh = c.heads * c.nope_dim, vh = c.heads * c.value_dim;
+    p.kn_stride = odd_lines(nh);
+    // 31-bit byte offsets inside its operands
+    const uint64_t widest = (uint64_t)p.nk_pad * (p.kn_stride > cache->row_stride ? p.kn_stride : cache->row_stride);
+    flash = flash && widest * 2 < 0x7FFFFFFFull && (uint64_t)vh * (p.nk_pad + 64) * 2 < 0x7FFFFFFFull;
+    p.v_stride = odd_lines(flash ? p.nk_pad : vh);
+    const size_t n_lat = (size_t)p.nk_pad * cache->row_stride, n_kn = (size_t)p.nk_pad * p.kn_stride, n_v = (size_t)(flash ? vh : p.nk_pad) * p.v_stride;
     rc = ws_begin(ctx, stream, ws_round(n_lat * esz) + ws_round(n_kn * esz) + ws_round(n_v * esz));
     if (rc) return rc;
     p.lat = ws_take<uint8_t>(ctx, n_lat * esz);
     p.kn = ws_take<uint8_t>(ctx, n_kn * esz);
     p.v = ws_take<uint8_t>(ctx, n_v * esz);
-    const uint32_t nh = c.heads * c.nope_dim, vh = c.heads * c.value_dim;
-    const DenseLinearParams lk{uk, p.lat, p.kn, nullptr, c.rank, cache->row_stride, nh, p.nk_pad, nh, c.rank, NVMAI_LINEAR_NONE};
-    const DenseLinearParams lv = flash ? DenseLinearParams{static_cast<const uint16_t*>(p.lat), uv, p.v, nullptr, cache->row_stride, c.rank, p.nk_pad, vh, p.nk_pad, c.rank, NVMAI_LINEAR_NONE}
-                                       : DenseLinearParams{uv, p.lat, p.v, nullptr, c.rank, cache->row_stride, vh, p.nk_pad, vh, c.rank, NVMAI_LINEAR_NONE};
+    const DenseLinearParams lk{uk, p.lat, p.kn, nullptr, c.rank, cache->row_stride, p.kn_stride, p.nk_pad, nh, c.rank, NVMAI_LINEAR_NONE};
+    const DenseLinearParams lv = flash ? DenseLinearParams{static_cast<const uint16_t*>(p.lat), uv, p.v, nullptr, cache->row_stride, c.rank, p.v_stride, vh, p.nk_pad, c.rank, NVMAI_LINEAR_NONE}
+                                       : DenseLinearParams{uv, p.lat, p.v, nullptr, c.rank, cache->row_stride, p.v_stride, p.nk_pad, vh, c.rank, NVMAI_LINEAR_NONE};
     if ((rc = dense_linear_check(ctx, lk)) || (rc = dense_linear_check(ctx, lv))) return rc;
     const size_t lds_rot = (size_t)c.rotary_dims * 4;
     if (f32) {
@@ -180,9 +200,7 @@ extern "C" int nvmai_hip_latent_attention(nvmai_hip_ctx* ctx, nvmai_stream strea
         }
         return launch_status();
     }
-    if (dq <= 64) launch_flash_v<64>(p, s);
-    else if (dq <= 128) launch_flash_v<128>(p, s);
-    else if (dq <= 192) launch_flash_v<192>(p, s);
-    else launch_flash_v<256>(p, s);
-    return launch_status();
+    if (c.nope_dim > 128 || c.rope_dim > 64 || c.value_dim > 128) return launch_flash<256, 128, 256>(p, s);
+    if (c.nope_dim <= 64) return c.rope_dim <= 32 ? launch_flash_v<64, 32>(p, s) : launch_flash_v<64, 64>(p, s);
+    return c.rope_dim <= 32 ? launch_flash_v<128, 32>(p, s) : launch_flash_v<128, 64>(p, s);
 }

@@ -21,6 +21,13 @@ __device__ __forceinline__ la_f4 la_mfma(const uint4& a, const uint4& b, la_f4 c
     return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(la_b8, a), __builtin_bit_cast(la_b8, b), c, 0, 0, 0);
 }
 
+// Two floats rounded to BF16 (nearest even) in one dword: one hardware conversion.
+typedef float la_f2 __attribute__((ext_vector_type(2)));
+typedef __bf16 la_b2 __attribute__((ext_vector_type(2)));
+__device__ __forceinline__ uint32_t la_pack2(float lo, float hi) {
+    return __builtin_bit_cast(uint32_t, __builtin_convertvector(la_f2{lo, hi}, la_b2));
+}
+
 constexpr float LA_LOG2E = 1.4426950408889634f;
 constexpr float LA_NONE = -1e30f;        // maximum of no scores
 
@@ -45,19 +52,12 @@ __device__ __forceinline__ void la_rotation(uint32_t position, double inv_freq, 
     sincosf((float)a, &s, &c);
 }
 
-__device__ __forceinline__ float la_block_sum(float v, float* lds) {
-    v = wave_sum_bcast(v);
-    if ((threadIdx.x & 63u) == 0) lds[threadIdx.x >> 6] = v;
-    __syncthreads();
-    return (lds[0] + lds[1]) + (lds[2] + lds[3]);
-}
-
 __device__ __forceinline__ float la_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 
 // ---- after the down projections: both latents normed, the key part rotated, the cache row written ---------
 struct LatentEpilogueParams {
     const void* proj;                    // [rows, proj_stride]: [W_dq h | W_dkv h: latent, rotated part]
-    const uint16_t *q_norm, *kv_norm;
+    const uint16_t *q_norm, *kv_norm;    // readable up to the counts rounded up to 8
     const double* inv_freq;              // [rot_dims / 2]
     void* cq;                            // [rows, cq_stride]
     LatentRows rows;
@@ -66,7 +66,40 @@ struct LatentEpilogueParams {
     float eps;
 };
 
+// Eight activations.
 template <int ACT>
+__device__ __forceinline__ void la_load8(const act_t<ACT>* p, float* v) {
+    if constexpr (ACT == ACT_FP32) {
+        const la_f4 a = reinterpret_cast<const la_f4*>(p)[0], b = reinterpret_cast<const la_f4*>(p)[1];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) { v[e] = a[e]; v[4 + e] = b[e]; }
+    } else {
+        const uint4 q = *reinterpret_cast<const uint4*>(p);
+        act2_to_f32<ACT>(q.x, v[0], v[1]);
+        act2_to_f32<ACT>(q.y, v[2], v[3]);
+        act2_to_f32<ACT>(q.z, v[4], v[5]);
+        act2_to_f32<ACT>(q.w, v[6], v[7]);
+    }
+}
+
+template <int ACT>
+__device__ __forceinline__ void la_store8(act_t<ACT>* p, const float* v) {
+    if constexpr (ACT == ACT_FP32) {
+        reinterpret_cast<la_f4*>(p)[0] = la_f4{v[0], v[1], v[2], v[3]};
+        reinterpret_cast<la_f4*>(p)[1] = la_f4{v[4], v[5], v[6], v[7]};
+    } else {
+        uint4 q;
+        q.x = f32_to_act<ACT>(v[0]) | ((uint32_t)f32_to_act<ACT>(v[1]) << 16);
+        q.y = f32_to_act<ACT>(v[2]) | ((uint32_t)f32_to_act<ACT>(v[3]) << 16);
+        q.z = f32_to_act<ACT>(v[4]) | ((uint32_t)f32_to_act<ACT>(v[5]) << 16);
+        q.w = f32_to_act<ACT>(v[6]) | ((uint32_t)f32_to_act<ACT>(v[7]) << 16);
+        *reinterpret_cast<uint4*>(p) = q;
+    }
+}
+
+// Both latents in pieces of eight elements, NP per thread, in registers between the sums and the stores; every load
+// (norm weights and rotation included) is issued before the first sum.  Elements past a latent's count are zero in proj.
+template <int ACT, int NP>
 __global__ __launch_bounds__(256) void latent_epilogue_kernel(LatentEpilogueParams p) {
     __shared__ float lds[8];
     const uint32_t row = blockIdx.x, tid = threadIdx.x;
@@ -74,25 +107,58 @@ __global__ __launch_bounds__(256) void latent_epilogue_kernel(LatentEpiloguePara
     const uint32_t position = p.rows.position_of(row);
     act_t<ACT>* out = static_cast<act_t<ACT>*>(p.cache.base) + (size_t)p.rows.slot_of(row) * p.cache.slot_stride +
                       (size_t)(position % p.cache.capacity) * p.cache.row_stride;
-    float qs = 0.0f, ks = 0.0f;
-    for (uint32_t j = tid; j < p.q_count; j += 256u) { const float v = act_to_f32<ACT>(proj[p.q_at + j]); qs = fmaf(v, v, qs); }
-    for (uint32_t j = tid; j < p.rank_count; j += 256u) { const float v = act_to_f32<ACT>(proj[p.kv_at + j]); ks = fmaf(v, v, ks); }
-    const float qi = 1.0f / sqrtf(la_block_sum(qs, lds) / (float)p.q_count + p.eps);
-    const float ki = 1.0f / sqrtf(la_block_sum(ks, lds + 4) / (float)p.rank_count + p.eps);
     act_t<ACT>* cq = static_cast<act_t<ACT>*>(p.cq) + (size_t)row * p.cq_stride;
-    for (uint32_t j = tid; j < p.q_count; j += 256u) cq[j] = f32_to_act<ACT>(act_to_f32<ACT>(proj[p.q_at + j]) * qi * bf16_to_f32(p.q_norm[j]));
-    for (uint32_t j = tid; j < p.rank_count; j += 256u) out[j] = f32_to_act<ACT>(act_to_f32<ACT>(proj[p.kv_at + j]) * ki * bf16_to_f32(p.kv_norm[j]));
+    const uint32_t qp = (p.q_count + 7u) / 8u, kp = (p.rank_count + 7u) / 8u, pieces = qp + kp;
+    float v[NP][8];
+    uint4 w[NP];
+#pragma unroll
+    for (int n = 0; n < NP; ++n) {
+        const uint32_t u = min(tid + 256u * n, pieces - 1u);
+        la_load8<ACT>(proj + (u < qp ? p.q_at + 8u * u : p.kv_at + 8u * (u - qp)), v[n]);
+        w[n] = *reinterpret_cast<const uint4*>(u < qp ? p.q_norm + 8u * u : p.kv_norm + 8u * (u - qp));
+    }
+    // the rope part, by the last threads (the first have the longest lists of pieces)
     const uint32_t half = p.rot_dims / 2u;
-    for (uint32_t j = tid; j < p.rot_dim; j += 256u) {
+    for (uint32_t j = 255u - tid; j < p.rot_dim; j += 256u) {
         if (j < half) {
             float c, s;
             la_rotation(position, p.inv_freq[j], c, s);
-            const float u = act_to_f32<ACT>(proj[p.rot_at + j]), v = act_to_f32<ACT>(proj[p.rot_at + half + j]);
-            out[p.rank + j] = f32_to_act<ACT>(u * c - v * s);
-            out[p.rank + half + j] = f32_to_act<ACT>(v * c + u * s);
+            const float a = act_to_f32<ACT>(proj[p.rot_at + j]), b = act_to_f32<ACT>(proj[p.rot_at + half + j]);
+            out[p.rank + j] = f32_to_act<ACT>(a * c - b * s);
+            out[p.rank + half + j] = f32_to_act<ACT>(b * c + a * s);
         } else if (j >= p.rot_dims) {
             out[p.rank + j] = proj[p.rot_at + j];
         }
+    }
+    float qs = 0.0f, ks = 0.0f;
+#pragma unroll
+    for (int n = 0; n < NP; ++n) {
+        const uint32_t u = tid + 256u * n;
+        float s = 0.0f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) s = fmaf(v[n][e], v[n][e], s);
+        qs += u < qp ? s : 0.0f;
+        ks += u >= qp && u < pieces ? s : 0.0f;
+    }
+    qs = wave_sum_bcast(qs);
+    ks = wave_sum_bcast(ks);
+    if ((tid & 63u) == 0) { lds[tid >> 6] = qs; lds[4 + (tid >> 6)] = ks; }
+    __syncthreads();
+    const float qi = 1.0f / sqrtf(((lds[0] + lds[1]) + (lds[2] + lds[3])) / (float)p.q_count + p.eps);
+    const float ki = 1.0f / sqrtf(((lds[4] + lds[5]) + (lds[6] + lds[7])) / (float)p.rank_count + p.eps);
+#pragma unroll
+    for (int n = 0; n < NP; ++n) {
+        const uint32_t u = tid + 256u * n;
+        if (u >= pieces) break;
+        const float inv = u < qp ? qi : ki;
+        float f[8];
+        act2_to_f32<ACT_BF16>(w[n].x, f[0], f[1]);
+        act2_to_f32<ACT_BF16>(w[n].y, f[2], f[3]);
+        act2_to_f32<ACT_BF16>(w[n].z, f[4], f[5]);
+        act2_to_f32<ACT_BF16>(w[n].w, f[6], f[7]);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) f[e] *= v[n][e] * inv;
+        la_store8<ACT>(u < qp ? cq + 8u * u : out + 8u * (u - qp), f);
     }
 }
 
@@ -111,8 +177,9 @@ struct LatentAttnParams {
     float *part_o, *part_m, *part_l;     // [rows, heads, splits, rank], [rows, heads, splits] x 2
     uint32_t splits, split_keys;
     // expanded form
-    void *lat, *kn, *v;                  // [nk_pad, row_stride], [nk_pad, heads * nope], V (or V^T [heads * vdim, nk_pad])
+    void *lat, *kn, *v;                  // [nk_pad, row_stride], [nk_pad, kn_stride], V (or V^T) rows of v_stride
     uint32_t nk, nk_pad, key0;           // keys of the call, the position of the first
+    uint32_t kn_stride, v_stride;
 };
 
 __device__ __forceinline__ uint32_t la_first_key(uint32_t position, uint32_t window) {
@@ -120,52 +187,64 @@ __device__ __forceinline__ uint32_t la_first_key(uint32_t position, uint32_t win
 }
 
 // ---- absorbed: q_n -> W_uk(h)^T q_n, q_r rotated ----------------------------------------------------
-// A block per (head, row): the waves split the rows of W_uk(h), a lane owns eight latent dims per 512.
+// A block per (head, row, 128 latent dims): sixteen lanes cover the latents in pieces of eight, sixteen groups of
+// lanes split the rows of W_uk(h).
 template <int ACT>
 __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentAttnParams p) {
     extern __shared__ __attribute__((aligned(16))) float la_lds[];
-    const uint32_t head = blockIdx.x, row = blockIdx.y, tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6;
+    __shared__ __attribute__((aligned(16))) float part[16][132];
+    const uint32_t head = blockIdx.x, row = blockIdx.y, tid = threadIdx.x, piece = tid & 15u, group = tid >> 4;
     float* qs = la_lds;                  // [nope]
-    float* part = qs + p.nope;           // [4][rank]
     const act_t<ACT>* q = static_cast<const act_t<ACT>*>(p.q) + (size_t)row * p.q_stride + head * (p.nope + p.rot);
-    for (uint32_t d = tid; d < p.nope; d += 256u) qs[d] = act_to_f32<ACT>(q[d]);
     act_t<ACT>* out = static_cast<act_t<ACT>*>(p.qa) + ((size_t)row * p.heads + head) * p.cache.row_stride;
-    const uint32_t position = p.rows.position_of(row), half = p.rot_dims / 2u;
-    for (uint32_t j = tid; j < p.cache.row_stride - p.rank; j += 256u) {
-        if (j < half) {
-            float c, s;
-            la_rotation(position, p.inv_freq[j], c, s);
-            const float u = act_to_f32<ACT>(q[p.nope + j]), v = act_to_f32<ACT>(q[p.nope + half + j]);
-            out[p.rank + j] = f32_to_act<ACT>(u * c - v * s);
-            out[p.rank + half + j] = f32_to_act<ACT>(v * c + u * s);
-        } else if (j >= p.rot_dims) {
-            out[p.rank + j] = j < p.rot ? q[p.nope + j] : f32_to_act<ACT>(0.0f);
-        }
-    }
-    __syncthreads();
-    for (uint32_t c0 = 0; c0 < p.rank; c0 += 512u) {
-        const uint32_t r = c0 + lane * 8u;
-        if (r < p.rank) {
-            float acc[8] = {};
-            const uint16_t* uk = p.uk + (size_t)head * p.nope * p.rank + r;
-#pragma unroll 8
-            for (uint32_t d = wave; d < p.nope; d += 4u) {
-                const uint4 w = *reinterpret_cast<const uint4*>(uk + (size_t)d * p.rank);
-                float f[8];
-                act2_to_f32<ACT_BF16>(w.x, f[0], f[1]);
-                act2_to_f32<ACT_BF16>(w.y, f[2], f[3]);
-                act2_to_f32<ACT_BF16>(w.z, f[4], f[5]);
-                act2_to_f32<ACT_BF16>(w.w, f[6], f[7]);
-#pragma unroll
-                for (int e = 0; e < 8; ++e) acc[e] = fmaf(f[e], qs[d], acc[e]);
+    if (blockIdx.z == gridDim.z - 1u) {              // the rotated part has a block of its own
+        const uint32_t position = p.rows.position_of(row), half = p.rot_dims / 2u;
+        for (uint32_t j = tid; j < p.cache.row_stride - p.rank; j += 256u) {
+            if (j < half) {
+                float c, s;
+                la_rotation(position, p.inv_freq[j], c, s);
+                const float u = act_to_f32<ACT>(q[p.nope + j]), v = act_to_f32<ACT>(q[p.nope + half + j]);
+                out[p.rank + j] = f32_to_act<ACT>(u * c - v * s);
+                out[p.rank + half + j] = f32_to_act<ACT>(v * c + u * s);
+            } else if (j >= p.rot_dims) {
+                out[p.rank + j] = j < p.rot ? q[p.nope + j] : f32_to_act<ACT>(0.0f);
             }
+        }
+        return;
+    }
+    const uint32_t r0 = blockIdx.z * 128u, r = min(r0 + piece * 8u, p.rank - 8u);
+    const uint16_t* uk = p.uk + (size_t)head * p.nope * p.rank + r;
+    float acc[8] = {};
+    for (uint32_t d0 = 0; d0 < p.nope; d0 += 128u) {
+        uint4 w[8];                                  // eight rows of W_uk in flight per lane
 #pragma unroll
-            for (int e = 0; e < 8; ++e) part[wave * p.rank + r + e] = acc[e];
+        for (int u = 0; u < 8; ++u) w[u] = *reinterpret_cast<const uint4*>(uk + (size_t)min(d0 + group + 16u * u, p.nope - 1u) * p.rank);
+        if (d0 == 0) {
+            for (uint32_t d = tid; d < p.nope; d += 256u) qs[d] = act_to_f32<ACT>(q[d]);
+            __syncthreads();
+        }
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            const uint32_t d = d0 + group + 16u * u;
+            const float x = d < p.nope ? qs[min(d, p.nope - 1u)] : 0.0f;
+            float f[8];
+            act2_to_f32<ACT_BF16>(w[u].x, f[0], f[1]);
+            act2_to_f32<ACT_BF16>(w[u].y, f[2], f[3]);
+            act2_to_f32<ACT_BF16>(w[u].z, f[4], f[5]);
+            act2_to_f32<ACT_BF16>(w[u].w, f[6], f[7]);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) acc[e] = fmaf(f[e], x, acc[e]);
         }
     }
+    *reinterpret_cast<la_f4*>(&part[group][piece * 8u]) = la_f4{acc[0], acc[1], acc[2], acc[3]};
+    *reinterpret_cast<la_f4*>(&part[group][piece * 8u + 4u]) = la_f4{acc[4], acc[5], acc[6], acc[7]};
     __syncthreads();
-    for (uint32_t r = tid; r < p.rank; r += 256u)
-        out[r] = f32_to_act<ACT>((part[r] + part[p.rank + r]) + (part[2u * p.rank + r] + part[3u * p.rank + r]));
+    if (tid < 128u && r0 + tid < p.rank) {
+        float a = 0.0f;
+#pragma unroll
+        for (int g = 0; g < 16; ++g) a += part[g][tid];
+        out[r0 + tid] = f32_to_act<ACT>(a);
+    }
 }
 
 // ---- absorbed: scores and sums over one split of the window, sixteen heads per block --------------------
@@ -371,15 +450,24 @@ __global__ __launch_bounds__(256) void latent_partial_plain_kernel(LatentAttnPar
 }
 
 // ---- absorbed: splits combined, W_uv(h), the output gate ------------------------------------------------
-// Grid (heads, rows, slices of the value rows).
+// A block of 1024 per (head, row): eight groups of threads share the splits, the waves then the value rows.
 template <int ACT>
-__global__ __launch_bounds__(256) void latent_combine_kernel(LatentAttnParams p) {
+__global__ __launch_bounds__(1024) void latent_combine_kernel(LatentAttnParams p) {
     extern __shared__ __attribute__((aligned(16))) float la_lds[];
     const uint32_t head = blockIdx.x, row = blockIdx.y, tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6;
     float* o = la_lds;                   // [rank]
-    float* wt = o + p.rank;              // [splits]
+    float* sums = o + p.rank;            // [8][rank]
+    float* wt = sums + 8u * p.rank;      // [splits]
     const size_t cell = ((size_t)row * p.heads + head) * p.splits;
     const float gate = p.gate ? la_sigmoid(act_to_f32<ACT>(static_cast<const act_t<ACT>*>(p.gate)[(size_t)row * p.gate_stride + head])) : 1.0f;
+    // splits past the last key of this row wrote no sums and weigh nothing: the live ones are a prefix
+    const uint32_t position = p.rows.position_of(row);
+    const uint32_t live = min(p.splits, (position + 1u - la_first_key(position, p.window) + p.split_keys - 1u) / p.split_keys);
+    const uint32_t group = tid >> 7, r0 = min((tid & 127u) * 4u, p.rank - 4u);
+    const float* po = p.part_o + cell * p.rank;
+    la_f4 ahead[8];                      // this group's first eight splits, requested before their weights are known
+#pragma unroll
+    for (int u = 0; u < 8; ++u) ahead[u] = *reinterpret_cast<const la_f4*>(po + (size_t)min(group + 8u * u, live - 1u) * p.rank + r0);
     float m = LA_NONE;
     for (uint32_t s = lane; s < p.splits; s += 64u) m = fmaxf(m, p.part_m[cell + s]);
     m = wave_max_f32(m);
@@ -393,34 +481,51 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(LatentAttnParams p)
     l = wave_sum_bcast(l);
     const float inv = 1.0f / l;
     __syncthreads();
-    // splits past the last key of this row wrote no sums and weigh nothing: the live ones are a prefix
-    const uint32_t first = la_first_key(p.rows.position_of(row), p.window);
-    const uint32_t live = min(p.splits, (p.rows.position_of(row) + 1u - first + p.split_keys - 1u) / p.split_keys);
-    for (uint32_t r = tid * 4u; r < p.rank; r += 1024u) {
+    for (uint32_t r = (tid & 127u) * 4u; r < p.rank; r += 512u) {
         la_f4 a = la_f4{0.0f, 0.0f, 0.0f, 0.0f};
-        const float* po = p.part_o + cell * p.rank + r;
+        uint32_t s = group;
+        if (r < 512u) {
+#pragma unroll
+            for (int u = 0; u < 8; ++u)
+                if (group + 8u * u < live) a += ahead[u] * wt[group + 8u * u];
+            s += 64u;
+        }
 #pragma unroll 8
-        for (uint32_t s = 0; s < live; ++s) a += *reinterpret_cast<const la_f4*>(po + (size_t)s * p.rank) * wt[s];
-        *reinterpret_cast<la_f4*>(o + r) = a * inv;
+        for (; s < live; s += 8u) a += *reinterpret_cast<const la_f4*>(po + (size_t)s * p.rank + r) * wt[s];
+        *reinterpret_cast<la_f4*>(sums + group * p.rank + r) = a;
     }
     __syncthreads();
-    const uint32_t per = (p.vdim + gridDim.z - 1u) / gridDim.z, j1 = min(p.vdim, (blockIdx.z + 1u) * per);
-#pragma unroll 4
-    for (uint32_t j = blockIdx.z * per + wave; j < j1; j += 4u) {
-        const uint16_t* uv = p.uv + (size_t)(head * p.vdim + j) * p.rank;
+    for (uint32_t r = tid; r < p.rank; r += 1024u) {
         float a = 0.0f;
-        for (uint32_t r = lane * 8u; r < p.rank; r += 512u) {
-            const uint4 w = *reinterpret_cast<const uint4*>(uv + r);
-            float f[8];
-            act2_to_f32<ACT_BF16>(w.x, f[0], f[1]);
-            act2_to_f32<ACT_BF16>(w.y, f[2], f[3]);
-            act2_to_f32<ACT_BF16>(w.z, f[4], f[5]);
-            act2_to_f32<ACT_BF16>(w.w, f[6], f[7]);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) a = fmaf(f[e], o[r + e], a);
+        for (int u = 0; u < 8; ++u) a += sums[u * p.rank + r];
+        o[r] = a * inv;
+    }
+    __syncthreads();
+    for (uint32_t j0 = wave * 4u; j0 < p.vdim; j0 += 64u) {      // four value rows of a wave in flight
+        float a[4] = {};
+        for (uint32_t r = lane * 8u; r < p.rank; r += 512u) {
+            uint4 w[4];
+#pragma unroll
+            for (int u = 0; u < 4; ++u) w[u] = *reinterpret_cast<const uint4*>(p.uv + (size_t)(head * p.vdim + min(j0 + u, p.vdim - 1u)) * p.rank + r);
+            const la_f4 o0 = *reinterpret_cast<const la_f4*>(o + r), o1 = *reinterpret_cast<const la_f4*>(o + r + 4u);
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                float f[8];
+                act2_to_f32<ACT_BF16>(w[u].x, f[0], f[1]);
+                act2_to_f32<ACT_BF16>(w[u].y, f[2], f[3]);
+                act2_to_f32<ACT_BF16>(w[u].z, f[4], f[5]);
+                act2_to_f32<ACT_BF16>(w[u].w, f[6], f[7]);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) a[u] = fmaf(f[4 + e], o1[e], fmaf(f[e], o0[e], a[u]));
+            }
         }
-        a = wave_sum_bcast(a);
-        if (lane == 0) static_cast<act_t<ACT>*>(p.out)[(size_t)row * p.out_stride + head * p.vdim + j] = f32_to_act<ACT>(a * gate);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            const float v = wave_sum_bcast(a[u]);
+            if (lane == (uint32_t)u && j0 + u < p.vdim)
+                static_cast<act_t<ACT>*>(p.out)[(size_t)row * p.out_stride + head * p.vdim + j0 + u] = f32_to_act<ACT>(v * gate);
+        }
     }
 }
 
@@ -467,43 +572,60 @@ __global__ __launch_bounds__(256) void latent_expanded_plain_kernel(LatentAttnPa
     float m, l;
     la_plain_rows(lo, hi, p.vdim, p.scale_log2, acc, ps, red, m, l,
         [&](uint32_t key) {
-            const act_t<ACT>* a = kn + (size_t)key * p.heads * p.nope + head * p.nope;
+            const act_t<ACT>* a = kn + (size_t)key * p.kn_stride + head * p.nope;
             const act_t<ACT>* b = lat + (size_t)key * p.cache.row_stride + p.rank;
             float s = 0.0f;
             for (uint32_t j = 0; j < p.nope; ++j) s = fmaf(act_to_f32<ACT>(a[j]), qs[j], s);
             for (uint32_t j = 0; j < p.rot; ++j) s = fmaf(act_to_f32<ACT>(b[j]), qs[p.nope + j], s);
             return s;
         },
-        [&](uint32_t key, uint32_t j) { return act_to_f32<ACT>(v[(size_t)key * p.heads * p.vdim + head * p.vdim + j]); });
+        [&](uint32_t key, uint32_t j) { return act_to_f32<ACT>(v[(size_t)key * p.v_stride + head * p.vdim + j]); });
     const float gate = p.gate ? la_sigmoid(act_to_f32<ACT>(static_cast<const act_t<ACT>*>(p.gate)[(size_t)row * p.gate_stride + head])) : 1.0f;
     for (uint32_t j = tid; j < p.vdim; j += 256u)
         static_cast<act_t<ACT>*>(p.out)[(size_t)row * p.out_stride + head * p.vdim + j] = f32_to_act<ACT>(acc[j] / l * gate);
 }
 
 // ---- expanded: flash attention over a window, BF16 -------------------------------------------------------
-// 128 queries of one head per block, 32 per wave; keys and V^T in tiles of 64 keys through LDS, the next tile's
-// loads in flight under the current tile's products.  S^T[key, query] = K Q^T and O^T[value, query] += V^T P^T: the
-// score registers are the B operand of the second product (see above for the order of the keys in V^T's columns).
-// DQ: query/key dims, DV: value dims, both padded with zeros in LDS.
-template <int DQ, int DV>
-__global__ __launch_bounds__(256) void latent_flash_kernel(LatentAttnParams p) {
-    constexpr int KS = DQ / 32, KU = DQ / 32, VU = DV / 32, NV = DV / 16;
-    constexpr uint32_t KLD = DQ + 8, VLD = 72;
-    __shared__ __attribute__((aligned(16))) uint16_t kt[64 * KLD];
-    __shared__ __attribute__((aligned(16))) uint16_t vt[DV * VLD];
-    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, i = lane & 15u, g = lane >> 4;
-    const uint32_t head = blockIdx.y, qb = gridDim.x - 1u - blockIdx.x;      // the blocks with the most keys first
+// 128 queries of one head per block, 32 per wave; K rows (in two regions, the head's own part and the shared rotated
+// part) and V^T rows in tiles of 64 keys, loaded straight into LDS, the next tile under the current tile's products.
+// S^T[key, query] = K Q^T and O^T[value, query] += V^T P^T.  Row m of score tile 2 h (2 h + 1) is key
+// 32 h + 8 (m / 4) + m % 4 (+ 4): a lane's registers of the two tiles are then the keys 8 g .. 8 g + 7, in order, and
+// stand as the B operand of the second product beside 16 contiguous bytes of V^T.
+// LDS pieces of 16 bytes are exchanged within a row (la_swizzle) so that the eight lanes that a read serves at once
+// fall into different banks.  NP, RP: the two parts of a key, DV: value dims, padded with zeros (a lane whose column
+// does not exist loads from past the end of the buffer, which reads as zero).
+template <int W>                         // row width in pieces
+__device__ __forceinline__ uint32_t la_swizzle(uint32_t key) {
+    return W >= 8 ? (key & 3u) | ((key >> 1) & 4u) : (key >> 3) & (W - 1u);
+}
+
+constexpr uint32_t LA_OUT_OF_BOUNDS = 0x80000000u;
+
+template <int NP, int RP, int DV>
+__global__ __launch_bounds__(256, NP + RP + DV <= 320 ? 2 : 1) void latent_flash_kernel(LatentAttnParams p) {
+    constexpr int KN = NP / 32, KR = RP / 32, NV = DV / 16;
+    constexpr int LN = NP / 32, LR = RP / 32, LV = DV / 32;      // 1 KB loads per wave and tile
+    constexpr uint32_t AT_R = 64u * NP * 2u, AT_V = AT_R + 64u * RP * 2u, STAGE = AT_V + DV * 128u;
+    extern __shared__ __attribute__((aligned(16))) float la_lds[];
+    uint8_t* lds = reinterpret_cast<uint8_t*>(la_lds);
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = __builtin_amdgcn_readfirstlane(tid >> 6), i = lane & 15u, g = lane >> 4;
+    // Blocks are dealt to the eight XCDs in turn: an XCD keeps to its own heads (their keys stay in its L2) where
+    // the heads divide.  Even rounds take the query blocks with the most keys first, odd ones last: a compute unit's
+    // two blocks then add up to the same work.
+    const uint32_t nqb = (p.n_rows + 127u) / 128u, id = blockIdx.x;
+    const uint32_t nth = p.heads % 8u == 0u ? id / 8u : id, round = nth / nqb, in_round = nth % nqb;
+    const uint32_t head = p.heads % 8u == 0u ? round * 8u + id % 8u : round, qb = round & 1u ? in_round : nqb - 1u - in_round;
     const uint32_t q0 = qb * 128u, dq = p.nope + p.rot;
     const uint16_t* q = static_cast<const uint16_t*>(p.q) + head * dq;
-    uint4 qf[2][KS];
+    uint4 qf[2][KN + KR];
 #pragma unroll
     for (int b = 0; b < 2; ++b) {
-        const uint32_t t = min(q0 + wave * 32u + 16u * b + i, p.n_rows - 1u);
+        const uint16_t* qr = q + (size_t)min(q0 + wave * 32u + 16u * b + i, p.n_rows - 1u) * p.q_stride;
 #pragma unroll
-        for (int s = 0; s < KS; ++s) {
-            const uint32_t d = 32u * s + 8u * g;
-            const uint4 v = *reinterpret_cast<const uint4*>(q + (size_t)t * p.q_stride + min(d, dq - 8u));
-            qf[b][s] = d < dq ? v : make_uint4(0u, 0u, 0u, 0u);
+        for (int s = 0; s < KN + KR; ++s) {
+            const uint32_t d = s < KN ? 32u * s + 8u * g : 32u * (s - KN) + 8u * g, n = s < KN ? p.nope : p.rot;
+            const uint4 v = *reinterpret_cast<const uint4*>(qr + (d < n ? (s < KN ? d : p.nope + d) : 0u));
+            qf[b][s] = d < n ? v : make_uint4(0u, 0u, 0u, 0u);
         }
     }
     la_f4 acc[2][NV];
@@ -516,67 +638,77 @@ __global__ __launch_bounds__(256) void latent_flash_kernel(LatentAttnParams p) {
     const uint32_t last_t = min(q0 + 127u, p.n_rows - 1u);
     const uint32_t k_lo = (la_first_key(p.rows.position + q0, p.window) - p.key0) & ~63u;
     const uint32_t k_hi = p.rows.position + last_t + 1u - p.key0;
-    const uint16_t *kn = static_cast<const uint16_t*>(p.kn) + head * p.nope, *kr = static_cast<const uint16_t*>(p.lat) + p.rank;
-    const uint16_t* v = static_cast<const uint16_t*>(p.v) + (size_t)head * p.vdim * p.nk_pad;
-    const uint32_t kn_stride = p.heads * p.nope;
-    uint4 kreg[KU], vreg[VU];
-    auto fetch = [&](uint32_t k0) {
+    const uint32_t kn_bytes = p.kn_stride * 2u, lat_bytes = p.cache.row_stride * 2u, v_bytes = p.v_stride * 2u;
+    [[maybe_unused]] const __amdgpu_buffer_rsrc_t nrs = __builtin_amdgcn_make_buffer_rsrc(p.kn, 0, (int)(p.nk_pad * kn_bytes), 0x00020000);
+    [[maybe_unused]] const __amdgpu_buffer_rsrc_t rrs = __builtin_amdgcn_make_buffer_rsrc(p.lat, 0, (int)(p.nk_pad * lat_bytes), 0x00020000);
+    [[maybe_unused]] const __amdgpu_buffer_rsrc_t vrs = __builtin_amdgcn_make_buffer_rsrc(p.v, 0, (int)(p.heads * p.vdim * v_bytes), 0x00020000);
+    uint32_t noff[LN], roff[LR], voff[LV];
 #pragma unroll
-        for (int n = 0; n < KU; ++n) {
-            const uint32_t u = tid + 256u * n, key = k0 + u / (DQ / 8u), d = (u % (DQ / 8u)) * 8u;
-            const uint32_t dc = min(d, dq - 8u);
-            const uint16_t* src = dc < p.nope ? kn + (size_t)key * kn_stride + dc : kr + (size_t)key * p.cache.row_stride + (dc - p.nope);
-            const uint4 w = *reinterpret_cast<const uint4*>(src);
-            kreg[n] = d < dq ? w : make_uint4(0u, 0u, 0u, 0u);
-        }
+    for (int j = 0; j < LN; ++j) {
+        const uint32_t u = (wave * LN + j) * 64u + lane, key = u / (NP / 8), d = ((u % (NP / 8)) ^ la_swizzle<NP / 8>(key)) * 8u;
+        noff[j] = d < p.nope ? key * kn_bytes + (head * p.nope + d) * 2u : LA_OUT_OF_BOUNDS;
+    }
 #pragma unroll
-        for (int n = 0; n < VU; ++n) {
-            const uint32_t u = tid + 256u * n, d = u >> 3, piece = u & 7u;
-            const uint4 w = *reinterpret_cast<const uint4*>(v + (size_t)min(d, p.vdim - 1u) * p.nk_pad + k0 + piece * 8u);
-            vreg[n] = d < p.vdim ? w : make_uint4(0u, 0u, 0u, 0u);
-        }
+    for (int j = 0; j < LR; ++j) {
+        const uint32_t u = (wave * LR + j) * 64u + lane, key = u / (RP / 8), d = ((u % (RP / 8)) ^ la_swizzle<RP / 8>(key)) * 8u;
+        roff[j] = d < p.rot ? key * lat_bytes + (p.rank + d) * 2u : LA_OUT_OF_BOUNDS;
+    }
+#pragma unroll
+    for (int j = 0; j < LV; ++j) {
+        const uint32_t u = (wave * LV + j) * 64u + lane, d = u >> 3, piece = (u & 7u) ^ (d & 7u);
+        voff[j] = d < p.vdim ? (head * p.vdim + d) * v_bytes + piece * 16u : LA_OUT_OF_BOUNDS;
+    }
+    auto issue = [&](uint32_t k0, uint8_t* dst) {
+#if defined(__HIP_DEVICE_COMPILE__)     // the host pass rejects the 16-byte form of the load
+#pragma unroll
+        for (int j = 0; j < LN; ++j)
+            __builtin_amdgcn_raw_ptr_buffer_load_lds(nrs, (__attribute__((address_space(3))) void*)(dst + (wave * LN + j) * 1024u), 16, noff[j], k0 * kn_bytes, 0, 0);
+#pragma unroll
+        for (int j = 0; j < LR; ++j)
+            __builtin_amdgcn_raw_ptr_buffer_load_lds(rrs, (__attribute__((address_space(3))) void*)(dst + AT_R + (wave * LR + j) * 1024u), 16, roff[j], k0 * lat_bytes, 0, 0);
+#pragma unroll
+        for (int j = 0; j < LV; ++j)
+            __builtin_amdgcn_raw_ptr_buffer_load_lds(vrs, (__attribute__((address_space(3))) void*)(dst + AT_V + (wave * LV + j) * 1024u), 16, voff[j], k0 * 2u, 0, 0);
+#endif
     };
-    fetch(k_lo);
-    // this wave's own range of keys
+    // this wave's own range of keys, and the part of it that every one of its queries sees
     const uint32_t wt0 = q0 + wave * 32u, wt1 = min(wt0 + 31u, p.n_rows - 1u);
     const bool wave_live = wt0 < p.n_rows;
     const uint32_t w_lo = la_first_key(p.rows.position + wt0, p.window) - p.key0, w_hi = p.rows.position + wt1 + 1u - p.key0;
-    // a tile needs no mask when every query of the wave sees all of it
     const uint32_t full_lo = la_first_key(p.rows.position + wt1, p.window) - p.key0, full_hi = p.rows.position + wt0 + 1u - p.key0;
-    for (uint32_t k0 = k_lo; k0 < k_hi; k0 += 64u) {
-        __syncthreads();
-#pragma unroll
-        for (int n = 0; n < KU; ++n) {
-            const uint32_t u = tid + 256u * n;
-            *reinterpret_cast<uint4*>(&kt[(u / (DQ / 8u)) * KLD + (u % (DQ / 8u)) * 8u]) = kreg[n];
-        }
-#pragma unroll
-        for (int n = 0; n < VU; ++n) {
-            const uint32_t u = tid + 256u * n, d = u >> 3, piece = u & 7u;      // keys 8 piece .. 8 piece + 7
-            const uint32_t kg = (2u * piece) & 7u, at = (piece >> 2) * 32u + (kg < 4u ? 8u * kg : 8u * (kg - 4u) + 4u);
-            *reinterpret_cast<uint2*>(&vt[d * VLD + at]) = make_uint2(vreg[n].x, vreg[n].y);
-            *reinterpret_cast<uint2*>(&vt[d * VLD + at + 8u]) = make_uint2(vreg[n].z, vreg[n].w);
-        }
-        __syncthreads();
-        if (k0 + 64u < k_hi) fetch(k0 + 64u);
+    const uint32_t krow = 8u * (i >> 2) + (i & 3u);              // key of this lane's row in an even score tile
+    issue(k_lo, lds);
+    uint32_t stage = 0;
+    for (uint32_t k0 = k_lo; k0 < k_hi; k0 += 64u, stage ^= 1u) {
+        __syncthreads();                             // this tile has landed; everyone is done with the other stage
+        if (k0 + 64u < k_hi) issue(k0 + 64u, lds + (stage ^ 1u) * STAGE);
         if (!wave_live || k0 >= w_hi || k0 + 64u <= w_lo) continue;             // wave-uniform
+        const uint8_t* cur = lds + stage * STAGE;
         la_f4 s[2][4];
 #pragma unroll
         for (int b = 0; b < 2; ++b)
 #pragma unroll
             for (int t = 0; t < 4; ++t) s[b][t] = la_f4{0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
-        for (int st = 0; st < KS; ++st)
+        for (int st = 0; st < KN + KR; ++st) {
+            uint4 a[4];
 #pragma unroll
             for (int t = 0; t < 4; ++t) {
-                const uint4 a = *reinterpret_cast<const uint4*>(&kt[(16 * t + i) * KLD + 32 * st + 8u * g]);
-#pragma unroll
-                for (int b = 0; b < 2; ++b) s[b][t] = la_mfma(a, qf[b][st], s[b][t]);
+                const uint32_t key = 32u * (t >> 1) + 4u * (t & 1) + krow;
+                a[t] = st < KN ? *reinterpret_cast<const uint4*>(cur + key * (NP * 2u) + ((4u * st + g) ^ la_swizzle<NP / 8>(key)) * 16u)
+                               : *reinterpret_cast<const uint4*>(cur + AT_R + key * (RP * 2u) + ((4u * (st - KN) + g) ^ la_swizzle<RP / 8>(key)) * 16u);
             }
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+#pragma unroll
+                for (int b = 0; b < 2; ++b) s[b][t] = la_mfma(a[t], qf[b][st], s[b][t]);
+        }
         const bool masked = k0 < full_lo || k0 + 64u > full_hi;
         uint4 pf[2][2];
 #pragma unroll
         for (int b = 0; b < 2; ++b) {
+#pragma unroll
+            for (int t = 0; t < 4; ++t) s[b][t] *= p.scale_log2;
             if (masked) {
                 const uint32_t pos = p.rows.position + min(wt0 + 16u * b + i, p.n_rows - 1u);
                 const uint32_t lo = la_first_key(pos, p.window) - p.key0, hi = pos + 1u - p.key0;
@@ -584,18 +716,13 @@ __global__ __launch_bounds__(256) void latent_flash_kernel(LatentAttnParams p) {
                 for (int t = 0; t < 4; ++t)
 #pragma unroll
                     for (int j = 0; j < 4; ++j) {
-                        const uint32_t key = k0 + 16u * t + 4u * g + j;
-                        s[b][t][j] = key >= lo && key < hi ? s[b][t][j] * p.scale_log2 : LA_NONE;
+                        const uint32_t key = k0 + 32u * (t >> 1) + 8u * g + 4u * (t & 1) + j;
+                        s[b][t][j] = key >= lo && key < hi ? s[b][t][j] : 2.0f * LA_NONE;
                     }
-            } else {
-#pragma unroll
-                for (int t = 0; t < 4; ++t) s[b][t] *= p.scale_log2;
             }
-            float tm = s[b][0][0];
+            float tm = fmaxf(fmaxf(s[b][0][0], s[b][0][1]), fmaxf(s[b][0][2], s[b][0][3]));
 #pragma unroll
-            for (int t = 0; t < 4; ++t)
-#pragma unroll
-                for (int j = 0; j < 4; ++j) tm = fmaxf(tm, s[b][t][j]);
+            for (int t = 1; t < 4; ++t) tm = fmaxf(fmaxf(fmaxf(s[b][t][0], s[b][t][1]), fmaxf(s[b][t][2], s[b][t][3])), tm);
             tm = fmaxf(tm, shfl_xor_f(tm, 16));
             tm = fmaxf(tm, shfl_xor_f(tm, 32));
             if (__any(tm > m[b])) {
@@ -605,18 +732,16 @@ __global__ __launch_bounds__(256) void latent_flash_kernel(LatentAttnParams p) {
 #pragma unroll
                 for (int n = 0; n < NV; ++n) acc[b][n] *= alpha;
             }
+            // a query without a key so far has m = LA_NONE, and exp2(2 LA_NONE - LA_NONE) = 0
             uint32_t w[8];
 #pragma unroll
             for (int t = 0; t < 4; ++t) {
                 float e[4];
 #pragma unroll
-                for (int j = 0; j < 4; ++j) {
-                    e[j] = __builtin_amdgcn_exp2f(s[b][t][j] - m[b]);
-                    if (masked && s[b][t][j] <= LA_NONE) e[j] = 0.0f;           // a query without a key so far: m is LA_NONE too
-                    l[b] += e[j];
-                }
-                w[2 * t] = f32_to_bf16(e[0]) | ((uint32_t)f32_to_bf16(e[1]) << 16);
-                w[2 * t + 1] = f32_to_bf16(e[2]) | ((uint32_t)f32_to_bf16(e[3]) << 16);
+                for (int j = 0; j < 4; ++j) e[j] = __builtin_amdgcn_exp2f(s[b][t][j] - m[b]);
+                l[b] += (e[0] + e[1]) + (e[2] + e[3]);
+                w[2 * t] = la_pack2(e[0], e[1]);
+                w[2 * t + 1] = la_pack2(e[2], e[3]);
             }
             pf[b][0] = make_uint4(w[0], w[1], w[2], w[3]);
             pf[b][1] = make_uint4(w[4], w[5], w[6], w[7]);
@@ -625,7 +750,7 @@ __global__ __launch_bounds__(256) void latent_flash_kernel(LatentAttnParams p) {
         for (int h = 0; h < 2; ++h)
 #pragma unroll
             for (int n = 0; n < NV; ++n) {
-                const uint4 a = *reinterpret_cast<const uint4*>(&vt[(16 * n + i) * VLD + 32 * h + 8u * g]);
+                const uint4 a = *reinterpret_cast<const uint4*>(cur + AT_V + (16u * n + i) * 128u + ((4u * h + g) ^ (i & 7u)) * 16u);
 #pragma unroll
                 for (int b = 0; b < 2; ++b) acc[b][n] = la_mfma(a, pf[b][h], acc[b][n]);
             }
@@ -644,12 +769,7 @@ __global__ __launch_bounds__(256) void latent_flash_kernel(LatentAttnParams p) {
 #pragma unroll
         for (int n = 0; n < NV; ++n) {
             const uint32_t d = 16u * n + 4u * g;
-            if (d < p.vdim) {
-                uint2 w;
-                w.x = f32_to_bf16(acc[b][n][0] * f) | ((uint32_t)f32_to_bf16(acc[b][n][1] * f) << 16);
-                w.y = f32_to_bf16(acc[b][n][2] * f) | ((uint32_t)f32_to_bf16(acc[b][n][3] * f) << 16);
-                *reinterpret_cast<uint2*>(out + d) = w;
-            }
+            if (d < p.vdim) *reinterpret_cast<uint2*>(out + d) = make_uint2(la_pack2(acc[b][n][0] * f, acc[b][n][1] * f), la_pack2(acc[b][n][2] * f, acc[b][n][3] * f));
         }
     }
 }

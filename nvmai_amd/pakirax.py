@@ -105,17 +105,32 @@ class PakiraxConfig:
                 out["l%d.mlp.up" % i], out["l%d.mlp.down" % i] = (ff, W), (W, ff)
         return out
 
-    def bytes_per_token(self, context, decay_rank=16, act_bytes=2):
-        """Algorithmic HBM bytes of one decode token of one sequence: every weight once, recurrent states read and
-        written, the cached rows the windows reach."""
-        import math
+    def matrix_elements(self, decay_rank=16):
+        """Elements of every matrix a token is multiplied by, the logits' included."""
         shapes = self.tensor_shapes(lambda i: decay_rank)
-        total = 2 * sum(math.prod(s) for s in shapes.values())
+        return sum(s[0] * s[1] for s in shapes.values() if len(s) == 2)
+
+    def bytes_per_token(self, batch=1, context=32768, act_bytes=2):
+        """Algorithmic HBM bytes of one decode step divided by the batch: every matrix once, recurrent states read and
+        written, the cached rows the windows reach."""
+        own = 0
         for m, _ in self.layers:
             if m.kind == "gla":
-                total += 2 * 4 * m.heads * m.dim * m.vdim
+                own += 2 * 4 * m.heads * m.dim * m.vdim
             else:
-                total += act_bytes * (min(context, m.window) if m.window else context) * (m.kv_rank + m.rot_dim)
+                own += act_bytes * (min(context, m.window) if m.window else context) * (m.kv_rank + m.rot_dim)
+        return 2 * self.matrix_elements() / batch + own
+
+    def prefill_flops(self, tokens):
+        """Useful flops of a prompt of `tokens`: 2 per matrix element and token (the logits of one token), the pairs
+        inside the windows, the recurrences' two products."""
+        total = 2.0 * tokens * (self.matrix_elements() - self.vocab * self.width) + 2.0 * self.vocab * self.width
+        for m, _ in self.layers:
+            if m.kind == "gla":
+                total += 4.0 * tokens * m.heads * m.dim * m.vdim
+            else:
+                w = min(m.window or tokens, tokens)
+                total += 2.0 * m.heads * (m.dim + m.rot_dim + m.vdim) * (w * (w + 1) / 2 + (tokens - w) * w)
         return total
 
 
@@ -189,7 +204,8 @@ class PakiraxWeights:
                 w["uq"] = cols(uq).contiguous()
                 w["uk"] = cols(_blocks(t(x + "uk"), 0, [(H, m.dim, m.dim_p)])).contiguous()
                 w["uv"] = cols(_blocks(t(x + "uv"), 0, [(H, m.vdim, m.vdim_p)])).contiguous()
-                w["q_norm"], w["kv_norm"] = t(x + "dq.norm").contiguous(), t(x + "dkv.norm").contiguous()
+                w["q_norm"] = _blocks(t(x + "dq.norm"), 0, [(1, m.q_rank, qp)]).contiguous()
+                w["kv_norm"] = _blocks(t(x + "dkv.norm"), 0, [(1, m.kv_rank, m.rank_p)]).contiguous()
             w["o"] = _blocks(t(x + "o"), 1, [(H, m.vdim, m.vdim_p)], _up(H * m.vdim_p, 64)).contiguous()
             if ff is not None:
                 w.update(norm2=norm(p + "norm2"), norm2b=norm(p + "norm2b"), up=cols(t(p + "mlp.up")).contiguous(),

@@ -240,7 +240,7 @@ class Latent:
         self.uv, self.uv64 = bf(rng, heads * vdim, rank, std=self.count ** -0.5)
         self.kvn, self.kvn64 = bf(rng, rank)
         self.qn, self.qn64 = bf(rng, qc)
-        self.proj, self.p64 = acts(ctx, down)
+        self.proj, self.p64 = acts(ctx, down, (down.shape[1] + 7) // 8 * 8)
         for i, j in spikes:                         # query i points at key j: W_uk c_j dominates its scores
             c = P.rms_norm(self.p64[j, qc:qc + self.count], self.kvn64[:self.count], self.eps)
             for h in range(heads):
