@@ -787,8 +787,8 @@ typedef struct {
 
 /* Gated linear attention with a decay per key channel: z = W_a2 a1 + b, alpha = sigmoid(z)^(1/tau),
  *   S_t = diag(alpha_t) S_(t-1) + k_t v_t^T,  o_t = S_t^T (q_scale q_t),  out = rmsnorm(o) * norm_weight * silu(g)
- * per head.  q, k [.., heads * key_dim], v, g [.., heads * value_dim], a1 [.., rank] are columns of projected rows
- * with one row stride; a2 [heads * key_dim, rank] and a2_bias BF16; norm_weight BF16 [value_dim]; state
+ * per head.  q, k [.., heads * key_dim], v, g [.., heads * value_dim], a1 [.., rank] are columns of projected rows,
+ * floats in either context, with one row stride; a2 [heads * key_dim, rank] and a2_bias BF16; norm_weight BF16 [value_dim]; state
  * [slots, heads, key_dim, value_dim] floats, updated in place.  `batch` sequences of `rows` rows each: sequence b
  * uses slot slots[b] (device array), or slot + b when slots is NULL.  key_dim, value_dim multiples of 16, rank of 8,
  * none above 512.  The chunked form (one sequence, NULL slots, key_dim and value_dim <= 256) takes workspace. */
@@ -796,8 +796,8 @@ typedef struct {
     uint32_t heads, key_dim, value_dim, value_count, rank;
     float tau, q_scale, eps;
 } nvmai_gla_config;
-int nvmai_hip_gla(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_gla_config* config, const void* q, const void* k,
-                  const void* v, const void* g, const void* a1, uint32_t proj_stride, const uint16_t* a2, const uint16_t* a2_bias,
+int nvmai_hip_gla(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_gla_config* config, const float* q, const float* k,
+                  const float* v, const float* g, const float* a1, uint32_t proj_stride, const uint16_t* a2, const uint16_t* a2_bias,
                   const uint16_t* norm_weight, float* state, const uint32_t* slots, uint32_t slot, void* out, uint32_t out_stride,
                   uint32_t rows, uint32_t batch, int form);
 
@@ -808,13 +808,15 @@ typedef struct {
     float scale, eps;
     const double* inv_freq;
 } nvmai_latent_config;
-/* Rows [latent: rank | rope part: rope_dim | zeros] of activations; position p of a slot lies at row p % capacity.
+/* Rows [latent: rank | rope part: rope_dim | zeros]; position p of a slot lies at row p % capacity.  type: the
+ * context's activation type, or NVMAI_ACT_BF16 in a 32-bit context (32-bit rows over a BF16 cache; absorbed form only).
  * Elements a model's counts leave out are zero and stay so (the caller clears the array once). */
 typedef struct {
     void* base;
     uint64_t slot_stride;      /* elements */
     uint32_t row_stride;       /* elements, a multiple of 32 */
     uint32_t capacity;         /* rows per slot, at least 64 */
+    int32_t type;              /* NVMAI_ACT_BF16 or NVMAI_ACT_FP32 */
 } nvmai_latent_cache;
 
 /* From the down projections proj[t] = [.. c_q at q_at .. c_kv at kv_at .. rope part at rope_at ..]:

@@ -92,7 +92,7 @@ class LatentConfig(C.Structure):
 
 class LatentCacheView(C.Structure):
     """nvmai_latent_cache"""
-    _fields_ = [("base", vp), ("slot_stride", u64), ("row_stride", u32), ("capacity", u32)]
+    _fields_ = [("base", vp), ("slot_stride", u64), ("row_stride", u32), ("capacity", u32), ("type", i32)]
 
 
 class PrefillStreamedParams(C.Structure):

@@ -20,29 +20,32 @@ int dense_linear_check(const nvmai_hip_ctx* ctx, const DenseLinearParams& p) {
     return NVMAI_OK;
 }
 
-template <int NT>
+template <int ACT, int NT>
 static void launch_gemv(const DenseLinearParams& p, hipStream_t s) {
     // rows per wave: one (short blocks, many of them) until the inputs' own loads weigh more than that
-    if (p.n >= 65536) dense_gemv_kernel<NT, 4><<<(p.n + 15) / 16, 256, 0, s>>>(p);
-    else if (NT > 2 && p.n >= 8192) dense_gemv_kernel<NT, 2><<<(p.n + 7) / 8, 256, 0, s>>>(p);
-    else dense_gemv_kernel<NT, 1><<<(p.n + 3) / 4, 256, 0, s>>>(p);
+    if (p.n >= 65536) dense_gemv_kernel<ACT, NT, 4><<<(p.n + 15) / 16, 256, 0, s>>>(p);
+    else if (NT * (ACT == ACT_FP32 ? 2 : 1) > 2 && p.n >= 8192) dense_gemv_kernel<ACT, NT, 2><<<(p.n + 7) / 8, 256, 0, s>>>(p);
+    else dense_gemv_kernel<ACT, NT, 1><<<(p.n + 3) / 4, 256, 0, s>>>(p);
+}
+
+template <int ACT>
+static int gemv(const DenseLinearParams& p, hipStream_t s) {
+    if (p.rows == 1) launch_gemv<ACT, 1>(p, s);
+    else if (p.rows == 2) launch_gemv<ACT, 2>(p, s);
+    else if (p.rows == 3) launch_gemv<ACT, 3>(p, s);
+    else launch_gemv<ACT, 4>(p, s);
+    return launch_status();
 }
 
 int dense_linear(nvmai_hip_ctx* ctx, hipStream_t s, const DenseLinearParams& p) {
     const int rc = dense_linear_check(ctx, p);
     if (rc) return rc;
     if (p.rows == 0) return NVMAI_OK;
+    if (p.rows <= 4) return ctx->act == NVMAI_ACT_FP32 ? gemv<ACT_FP32>(p, s) : gemv<ACT_BF16>(p, s);
     if (ctx->act == NVMAI_ACT_FP32) {
         const dim3 grid((p.n + 63) / 64, (p.rows + 63) / 64);
         if (grid.y > 65535) return NVMAI_ERR_UNSUPPORTED;
         dense_f32_kernel<<<grid, 256, 0, s>>>(p);
-        return launch_status();
-    }
-    if (p.rows <= 4) {
-        if (p.rows == 1) launch_gemv<1>(p, s);
-        else if (p.rows == 2) launch_gemv<2>(p, s);
-        else if (p.rows == 3) launch_gemv<3>(p, s);
-        else launch_gemv<4>(p, s);
         return launch_status();
     }
     if (p.rows <= 64) {

@@ -48,8 +48,9 @@ __device__ __forceinline__ void dense_store4_bf16(const DenseLinearParams& p, ui
 
 // ---- 1 .. 4 input rows: a wave owns RW weight rows, its lanes split k in 16-byte pieces -------------
 // Bound by the matrix's bytes.  The inputs are read from L1 / L2 beside the weights (no LDS, no barrier): every
-// load of a k step is independent of the others, so a wave has RW + NT 16-byte loads per lane in flight.
-template <int NT, int RW>
+// load of a k step is independent of the others, so a wave has RW + NT (32-bit inputs: RW + 2 NT) 16-byte loads per lane
+// in flight.
+template <int ACT, int NT, int RW>
 __global__ __launch_bounds__(256) void dense_gemv_kernel(DenseLinearParams p) {
     const uint32_t lane = threadIdx.x & 63u, wave = threadIdx.x >> 6;
     const uint32_t r0 = (blockIdx.x * 4u + wave) * RW;
@@ -57,42 +58,59 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(DenseLinearParams p) {
     const uint16_t* wp[RW];
 #pragma unroll
     for (int r = 0; r < RW; ++r) wp[r] = p.w + (size_t)min(r0 + r, p.n - 1u) * p.w_stride;
-    const uint16_t* x = static_cast<const uint16_t*>(p.x);
+    const act_t<ACT>* x = static_cast<const act_t<ACT>*>(p.x);
     float acc[NT][RW];
 #pragma unroll
     for (int t = 0; t < NT; ++t)
 #pragma unroll
         for (int r = 0; r < RW; ++r) acc[t][r] = 0.0f;
-#pragma unroll 4
-    for (uint32_t k0 = 0; k0 < p.k; k0 += 512u) {
-        const uint32_t k = k0 + lane * 8u;
-        const bool live = k < p.k;
-        const uint32_t at = live ? k : p.k - 8u;             // past the end: reload the last piece, multiply by zero
-        uint4 wv[RW], xv[NT];
+    constexpr int XP = ACT == ACT_FP32 ? 2 : 1;
+    constexpr int U = NT * XP + RW <= 3 ? 4 : 2;             // steps of 512 k whose loads are all issued before the first product
+    for (uint32_t k0 = 0; k0 < p.k; k0 += 512u * U) {
+        uint4 wv[U][RW], xv[U][NT][XP];
 #pragma unroll
-        for (int r = 0; r < RW; ++r) wv[r] = *reinterpret_cast<const uint4*>(wp[r] + at);
+        for (int s = 0; s < U; ++s) {
+            const uint32_t at = min(k0 + 512u * s + lane * 8u, p.k - 8u);        // past the end: the last piece, multiplied by zero
 #pragma unroll
-        for (int t = 0; t < NT; ++t) xv[t] = *reinterpret_cast<const uint4*>(x + (size_t)t * p.x_stride + at);
-        float wf[RW][8];
+            for (int r = 0; r < RW; ++r) wv[s][r] = *reinterpret_cast<const uint4*>(wp[r] + at);
 #pragma unroll
-        for (int r = 0; r < RW; ++r) {
-            act2_to_f32<ACT_BF16>(wv[r].x, wf[r][0], wf[r][1]);
-            act2_to_f32<ACT_BF16>(wv[r].y, wf[r][2], wf[r][3]);
-            act2_to_f32<ACT_BF16>(wv[r].z, wf[r][4], wf[r][5]);
-            act2_to_f32<ACT_BF16>(wv[r].w, wf[r][6], wf[r][7]);
+            for (int t = 0; t < NT; ++t)
+#pragma unroll
+                for (int u = 0; u < XP; ++u) xv[s][t][u] = reinterpret_cast<const uint4*>(x + (size_t)t * p.x_stride + at)[u];
         }
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-        for (int t = 0; t < NT; ++t) {
-            const uint4 q = live ? xv[t] : make_uint4(0u, 0u, 0u, 0u);
-            float xf[8];
-            act2_to_f32<ACT_BF16>(q.x, xf[0], xf[1]);
-            act2_to_f32<ACT_BF16>(q.y, xf[2], xf[3]);
-            act2_to_f32<ACT_BF16>(q.z, xf[4], xf[5]);
-            act2_to_f32<ACT_BF16>(q.w, xf[6], xf[7]);
+        for (int s = 0; s < U; ++s) {
+            const bool live = k0 + 512u * s + lane * 8u < p.k;
+            float wf[RW][8];
 #pragma unroll
-            for (int r = 0; r < RW; ++r)
+            for (int r = 0; r < RW; ++r) {
+                const uint4 q = live ? wv[s][r] : make_uint4(0u, 0u, 0u, 0u);
+                act2_to_f32<ACT_BF16>(q.x, wf[r][0], wf[r][1]);
+                act2_to_f32<ACT_BF16>(q.y, wf[r][2], wf[r][3]);
+                act2_to_f32<ACT_BF16>(q.z, wf[r][4], wf[r][5]);
+                act2_to_f32<ACT_BF16>(q.w, wf[r][6], wf[r][7]);
+            }
 #pragma unroll
-                for (int j = 0; j < 8; ++j) acc[t][r] = fmaf(wf[r][j], xf[j], acc[t][r]);
+            for (int t = 0; t < NT; ++t) {
+                float xf[8];
+                if constexpr (ACT == ACT_FP32) {
+#pragma unroll
+                    for (int u = 0; u < 2; ++u) {
+                        xf[4 * u] = __uint_as_float(xv[s][t][u].x); xf[4 * u + 1] = __uint_as_float(xv[s][t][u].y);
+                        xf[4 * u + 2] = __uint_as_float(xv[s][t][u].z); xf[4 * u + 3] = __uint_as_float(xv[s][t][u].w);
+                    }
+                } else {
+                    act2_to_f32<ACT_BF16>(xv[s][t][0].x, xf[0], xf[1]);
+                    act2_to_f32<ACT_BF16>(xv[s][t][0].y, xf[2], xf[3]);
+                    act2_to_f32<ACT_BF16>(xv[s][t][0].z, xf[4], xf[5]);
+                    act2_to_f32<ACT_BF16>(xv[s][t][0].w, xf[6], xf[7]);
+                }
+#pragma unroll
+                for (int r = 0; r < RW; ++r)
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) acc[t][r] = fmaf(wf[r][j], xf[j], acc[t][r]);
+            }
         }
     }
 #pragma unroll
@@ -100,7 +118,7 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(DenseLinearParams p) {
 #pragma unroll
         for (int r = 0; r < RW; ++r) {
             const float v = wave_sum_bcast(acc[t][r]);
-            if (lane == (uint32_t)(t * RW + r) && r0 + r < p.n && (uint32_t)t < p.rows) dense_store<ACT_BF16>(p, t, r0 + r, v);
+            if (lane == (uint32_t)(t * RW + r) && r0 + r < p.n && (uint32_t)t < p.rows) dense_store<ACT>(p, t, r0 + r, v);
         }
 }
 
@@ -246,7 +264,7 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(DenseLinearParams p, ui
     }
 }
 
-// ---- 32-bit activations: 64 x 64 tiles on the vector pipe, BF16 weights widened, fp32 FMA ------------
+// ---- 32-bit activations, more than four rows: 64 x 64 tiles on the vector pipe, BF16 weights widened, fp32 FMA ------------
 // Sums are two-level (a step of 16 k, then the running total), which keeps the rounding error of a long k small.
 __global__ __launch_bounds__(256) void dense_f32_kernel(DenseLinearParams p) {
     __shared__ float ws[16][65], xs[16][65];

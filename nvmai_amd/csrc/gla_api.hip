@@ -42,11 +42,11 @@ int gla_chunked(const GlaParams& p, hipStream_t s) {
     const size_t lds = ((size_t)48 * (p.dk + 4) + 2 * (size_t)p.dk + 1024 + (size_t)16 * p.rank) * 4;
     static bool raised = false;
     if (!raised) {
-        NVMAI_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void*>(gla_prep_kernel<ACT>), hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024));
+        NVMAI_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void*>(gla_prep_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024));
         raised = true;
     }
     if (lds > 128 * 1024) return NVMAI_ERR_UNSUPPORTED;
-    gla_prep_kernel<ACT><<<dim3(subs, p.heads), 256, lds, s>>>(p);
+    gla_prep_kernel<<<dim3(subs, p.heads), 256, lds, s>>>(p);
     const uint32_t kt = (p.dk + 15) / 16;
     if (kt <= 2) gla_spans<ACT, 2>(p, subs, spans, s);
     else if (kt <= 4) gla_spans<ACT, 4>(p, subs, spans, s);
@@ -57,8 +57,8 @@ int gla_chunked(const GlaParams& p, hipStream_t s) {
 
 }  // namespace
 
-extern "C" int nvmai_hip_gla(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_gla_config* config, const void* q, const void* k,
-                             const void* v, const void* g, const void* a1, uint32_t proj_stride, const uint16_t* a2,
+extern "C" int nvmai_hip_gla(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_gla_config* config, const float* q, const float* k,
+                             const float* v, const float* g, const float* a1, uint32_t proj_stride, const uint16_t* a2,
                              const uint16_t* a2_bias, const uint16_t* norm_weight, float* state, const uint32_t* slots,
                              uint32_t slot, void* out, uint32_t out_stride, uint32_t rows, uint32_t batch, int form) {
     if (!ctx || !config || !q || !k || !v || !g || !a1 || !a2 || !a2_bias || !norm_weight || !state || !out) return NVMAI_ERR_INVALID_ARG;

@@ -4,7 +4,8 @@
 //   S_t = diag(alpha_t) S_(t-1) + k_t v_t^T,   o_t = S_t^T (scale q_t)
 //   out_t = rmsnorm(o_t) * w * silu(g_t)                               (per head, over the value channels)
 //
-// Two forms of the same recurrence, both in fp32 throughout:
+// Two forms of the same recurrence, both in fp32 throughout, from projections kept in 32 bits (the norm of a first token's
+// output leaves little but the sign of q . k, which a rounding of q and k may turn):
 //   * row by row, a block per (head, sequence), the state in registers: decoding and short portions;
 //   * in chunks, for prompts.  With b_t = sum of log2 alpha from the start of a sub-chunk of 16 rows to t,
 //         o_t  = (q_t 2^b_t)^T S_0 + sum_{s<=t} A_ts v_s,    A_ts = sum_d q_td k_sd 2^(b_td - b_sd)
@@ -27,7 +28,7 @@ constexpr uint32_t GLA_SUB = 16;         // rows of a sub-chunk
 constexpr uint32_t GLA_MAX_DIM = 256;    // of the chunked form
 
 struct GlaParams {
-    const void *q, *k, *v, *g, *a1;      // activations, row stride proj_stride
+    const float *q, *k, *v, *g, *a1;     // projected rows in 32 bits, row stride proj_stride
     const uint16_t *a2, *a2_bias, *norm_weight;
     float* state;                        // [slots, heads, dk, dv]
     const uint32_t* slots;               // slot of a sequence, nullptr = slot0 + sequence
@@ -87,14 +88,12 @@ __global__ __launch_bounds__(NTH) void gla_recurrent_kernel(GlaParams p) {
     float* a1s = part + groups * dv;     // [rank]
     const uint32_t slot = p.slots ? p.slots[seq] : p.slot0 + seq;
     float* S = p.state + ((size_t)slot * p.heads + head) * dk * dv + j;
-    const act_t<ACT>*qp = static_cast<const act_t<ACT>*>(p.q) + head * dk, *kp = static_cast<const act_t<ACT>*>(p.k) + head * dk;
-    const act_t<ACT>*vp = static_cast<const act_t<ACT>*>(p.v) + head * dv, *gp = static_cast<const act_t<ACT>*>(p.g) + head * dv;
-    const act_t<ACT>* a1p = static_cast<const act_t<ACT>*>(p.a1);
+    const float *qp = p.q + head * dk, *kp = p.k + head * dk, *vp = p.v + head * dv, *gp = p.g + head * dv;
     const uint32_t dc = min(tid, dk - 1u), jc = min(tid, dv - 1u), rc = min(tid, p.rank - 1u), ch = head * dk + dc;
-    act_t<ACT> a1v, q0, k0, vj, gj;
+    float a1v, q0, k0, vj, gj;
     auto fetch = [&](uint32_t t) {
         const size_t at = ((size_t)seq * p.rows + t) * p.proj_stride;
-        a1v = a1p[at + rc];
+        a1v = p.a1[at + rc];
         q0 = qp[at + dc];
         k0 = kp[at + dc];
         vj = vp[at + j];
@@ -111,7 +110,7 @@ __global__ __launch_bounds__(NTH) void gla_recurrent_kernel(GlaParams p) {
     }
     for (uint32_t t = 0; t < p.rows; ++t) {
         const size_t row = (size_t)seq * p.rows + t;
-        if (tid < p.rank) a1s[tid] = act_to_f32<ACT>(a1v);
+        if (tid < p.rank) a1s[tid] = a1v;
         __syncthreads();
         float z = b0, w[8];
         gla_unpack8(w0, w);
@@ -134,11 +133,11 @@ __global__ __launch_bounds__(NTH) void gla_recurrent_kernel(GlaParams p) {
         }
         if (tid < chans) {
             const bool real = tid < dk;
-            qs[tid] = real ? act_to_f32<ACT>(q0) * p.q_scale : 0.0f;
-            ks[tid] = real ? act_to_f32<ACT>(k0) : 0.0f;
+            qs[tid] = real ? q0 * p.q_scale : 0.0f;
+            ks[tid] = real ? k0 : 0.0f;
             al[tid] = real ? __builtin_amdgcn_exp2f(gla_log2_decay(z, p.inv_tau)) : 0.0f;
         }
-        const float v = act_to_f32<ACT>(vj), gate = act_to_f32<ACT>(gj);
+        const float v = vj, gate = gj;
         fetch(min(t + 1u, p.rows - 1u));
         __syncthreads();
         float o = 0.0f;
@@ -195,7 +194,6 @@ __global__ __launch_bounds__(NTH) void gla_recurrent_kernel(GlaParams p) {
 // exponent of the difference otherwise.
 constexpr float GLA_SAFE = 60.0f;
 
-template <int ACT>
 __global__ __launch_bounds__(256) void gla_prep_kernel(GlaParams p) {
     extern __shared__ __attribute__((aligned(16))) float gla_lds[];
     const uint32_t tid = threadIdx.x, sub = blockIdx.x, head = blockIdx.y, dk = p.dk, ld = dk + 4u;
@@ -208,7 +206,7 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(GlaParams p) {
     const uint32_t t0 = sub * GLA_SUB, live = min(GLA_SUB, p.rows > t0 ? p.rows - t0 : 0u);
     for (uint32_t e = tid; e < 16u * p.rank; e += 256u) {
         const uint32_t t = e / p.rank, r = e % p.rank;
-        a1s[e] = t < live ? act_to_f32<ACT>(static_cast<const act_t<ACT>*>(p.a1)[(size_t)(t0 + t) * p.proj_stride + r]) : 0.0f;
+        a1s[e] = t < live ? p.a1[(size_t)(t0 + t) * p.proj_stride + r] : 0.0f;
     }
     const size_t cell = (size_t)sub * p.heads + head;
     __syncthreads();
@@ -220,8 +218,8 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(GlaParams p) {
 #pragma unroll
         for (int t = 0; t < 8; ++t) {
             const size_t at = (size_t)min(t0 + 8u * half + t, p.rows - 1u) * p.proj_stride + ch;
-            qv[t] = act_to_f32<ACT>(static_cast<const act_t<ACT>*>(p.q)[at]);
-            kv[t] = act_to_f32<ACT>(static_cast<const act_t<ACT>*>(p.k)[at]);
+            qv[t] = p.q[at];
+            kv[t] = p.k[at];
             z[t] = bias;
         }
         for (uint32_t r = 0; r < p.rank; r += 8u) {
@@ -336,14 +334,14 @@ __global__ __launch_bounds__(1024) void gla_span_kernel(GlaParams p) {
 #pragma unroll
         for (int ks = 0; ks < 4; ++ks) {
             const uint32_t t = t0 + 4u * ks + g;
-            const float v = act_to_f32<ACT>(static_cast<const act_t<ACT>*>(p.v)[(size_t)min(t, p.rows - 1u) * p.proj_stride + head * dv + col]);
+            const float v = p.v[(size_t)min(t, p.rows - 1u) * p.proj_stride + head * dv + col];
             vb[ks] = t < p.rows ? v : 0.0f;
         }
         float gate[4];
         if (OUT) {
 #pragma unroll
             for (int r = 0; r < 4; ++r)
-                gate[r] = act_to_f32<ACT>(static_cast<const act_t<ACT>*>(p.g)[(size_t)min(t0 + 4u * g + r, p.rows - 1u) * p.proj_stride + head * dv + col]);
+                gate[r] = p.g[(size_t)min(t0 + 4u * g + r, p.rows - 1u) * p.proj_stride + head * dv + col];
         }
         __syncthreads();
         if (OUT) {

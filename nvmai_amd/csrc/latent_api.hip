@@ -14,6 +14,7 @@ int check_config(const nvmai_hip_ctx* ctx, const nvmai_latent_config* c, const n
     if (c->nope_dim % 16 || c->rope_dim % 16 || c->value_dim % 16 || c->rank % 64) return NVMAI_ERR_INVALID_ARG;
     if (c->rotary_dims > c->rope_dim || c->rotary_dims % 2 || (c->rotary_dims && !c->inv_freq)) return NVMAI_ERR_INVALID_ARG;
     if (c->rank_count == 0 || c->rank_count > c->rank) return NVMAI_ERR_INVALID_ARG;
+    if (cache->type != ctx->act && !(ctx->act == NVMAI_ACT_FP32 && cache->type == NVMAI_ACT_BF16)) return NVMAI_ERR_UNSUPPORTED;
     if (cache->row_stride < c->rank + c->rope_dim || cache->row_stride % 32 || cache->capacity < 64) return NVMAI_ERR_INVALID_ARG;
     if (!aligned16(cache->base) || cache->slot_stride % 8 || cache->slot_stride < (uint64_t)cache->capacity * cache->row_stride) return NVMAI_ERR_ALIGNMENT;
     return NVMAI_OK;
@@ -37,19 +38,19 @@ int launch_partial(const LatentAttnParams& p, hipStream_t s) {
     return NVMAI_OK;
 }
 
-template <int ACT>
+template <int ACT, int CT>
 int absorbed(const LatentAttnParams& p, hipStream_t s) {
     const size_t lds_a = (size_t)p.nope * 4;
-    int rc = raise_lds(reinterpret_cast<const void*>(latent_absorb_kernel<ACT>), lds_a);
+    int rc = raise_lds(reinterpret_cast<const void*>(latent_absorb_kernel<ACT, CT>), lds_a);
     if (rc) return rc;
-    latent_absorb_kernel<ACT><<<dim3(p.heads, p.n_rows, (p.rank + 127) / 128 + 1), 256, lds_a, s>>>(p);
+    latent_absorb_kernel<ACT, CT><<<dim3(p.heads, p.n_rows, (p.rank + 127) / 128 + 1), 256, lds_a, s>>>(p);
     const uint32_t rest = p.cache.row_stride - p.rank;
-    if (ACT == ACT_BF16 && p.rank <= 1024 && rest <= 128) {
+    if (CT == ACT_BF16 && p.rank <= 1024 && rest <= 128) {
         rc = p.rank <= 128 ? launch_partial<2>(p, s) : p.rank <= 256 ? launch_partial<4>(p, s) : p.rank <= 512 ? launch_partial<8>(p, s) : launch_partial<16>(p, s);
     } else {
         const size_t lds = ((size_t)p.cache.row_stride + p.rank + 256 + 8) * 4;
-        rc = raise_lds(reinterpret_cast<const void*>(latent_partial_plain_kernel<ACT>), lds);
-        if (!rc) latent_partial_plain_kernel<ACT><<<dim3(p.splits, p.heads, p.n_rows), 256, lds, s>>>(p);
+        rc = raise_lds(reinterpret_cast<const void*>(latent_partial_plain_kernel<CT>), lds);
+        if (!rc) latent_partial_plain_kernel<CT><<<dim3(p.splits, p.heads, p.n_rows), 256, lds, s>>>(p);
     }
     if (rc) return rc;
     const size_t lds_c = (9 * (size_t)p.rank + p.splits) * 4;
@@ -97,8 +98,9 @@ extern "C" int nvmai_hip_latent_epilogue(nvmai_hip_ctx* ctx, nvmai_stream stream
     const uint32_t pieces = (q_count + 7) / 8 + (c.rank_count + 7) / 8;
 #define NVMAI_LE(NP)                                                                              \
     do {                                                                                          \
-        if (ctx->act == NVMAI_ACT_BF16) latent_epilogue_kernel<ACT_BF16, NP><<<rows, 256, 0, s>>>(p); \
-        else latent_epilogue_kernel<ACT_FP32, NP><<<rows, 256, 0, s>>>(p);                        \
+        if (ctx->act == NVMAI_ACT_BF16) latent_epilogue_kernel<ACT_BF16, ACT_BF16, NP><<<rows, 256, 0, s>>>(p); \
+        else if (cache->type == NVMAI_ACT_BF16) latent_epilogue_kernel<ACT_FP32, ACT_BF16, NP><<<rows, 256, 0, s>>>(p); \
+        else latent_epilogue_kernel<ACT_FP32, ACT_FP32, NP><<<rows, 256, 0, s>>>(p);              \
     } while (0)
     if (pieces <= 256) NVMAI_LE(1);
     else if (pieces <= 512) NVMAI_LE(2);
@@ -135,15 +137,15 @@ extern "C" int nvmai_hip_latent_attention(nvmai_hip_ctx* ctx, nvmai_stream strea
     p.rot = c.rope_dim; p.vdim = c.value_dim; p.rank = c.rank; p.rot_dims = c.rotary_dims; p.window = c.window;
     p.scale_log2 = c.scale * LA_LOG2E;
     hipStream_t s = (hipStream_t)stream;
-    const bool f32 = ctx->act == NVMAI_ACT_FP32;
-    const size_t esz = f32 ? 4 : 2;
-    if (form == NVMAI_LATENT_EXPANDED && !known) return NVMAI_ERR_UNSUPPORTED;
-    const bool expand = form == NVMAI_LATENT_EXPANDED || (form == NVMAI_FORM_AUTO && known && rows >= 32);
+    const bool f32 = ctx->act == NVMAI_ACT_FP32, cache32 = cache->type == NVMAI_ACT_FP32;
+    const size_t esz = cache32 ? 4 : 2;
+    if (form == NVMAI_LATENT_EXPANDED && (!known || f32 != cache32)) return NVMAI_ERR_UNSUPPORTED;
+    const bool expand = form == NVMAI_LATENT_EXPANDED || (form == NVMAI_FORM_AUTO && known && f32 == cache32 && rows >= 32);
     if (!expand) {
         uint32_t keys = known ? last : cache->capacity;
         if (c.window && c.window < keys) keys = c.window;
         // about two blocks per compute unit, at least 32 keys each
-        const uint32_t groups = f32 ? c.heads : (c.heads + 15) / 16;
+        const uint32_t groups = cache32 ? c.heads : (c.heads + 15) / 16;
         const uint32_t want = 2u * (uint32_t)ctx->compute_units / (rows * groups) + 1u;
         const uint32_t per = ((keys + want - 1) / want + 31) / 32 * 32;
         p.split_keys = per;
@@ -155,7 +157,8 @@ extern "C" int nvmai_hip_latent_attention(nvmai_hip_ctx* ctx, nvmai_stream strea
         p.part_o = ws_take<float>(ctx, cells * c.rank);
         p.part_m = ws_take<float>(ctx, cells);
         p.part_l = ws_take<float>(ctx, cells);
-        return f32 ? absorbed<ACT_FP32>(p, s) : absorbed<ACT_BF16>(p, s);
+        if (!f32) return absorbed<ACT_BF16, ACT_BF16>(p, s);
+        return cache32 ? absorbed<ACT_FP32, ACT_FP32>(p, s) : absorbed<ACT_FP32, ACT_BF16>(p, s);
     }
     p.key0 = c.window && map->position + 1 > c.window ? map->position + 1 - c.window : 0;
     p.nk = last - p.key0;

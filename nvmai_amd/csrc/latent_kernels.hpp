@@ -4,7 +4,8 @@
 //   score(h, i, j) = scale * (q_n(h, i) . W_uk(h) c_j + q_r(h, i) . k_r(j)),   window: 0 <= i - j < window
 //   out(h, i)      = sigmoid(gate(h, i)) * W_uv(h) sum_j softmax_j(score) c_j
 //
-// A cache row holds [c | rotated key part | zeros], row stride `row_stride`.  Two forms of the same sum:
+// A cache row holds [c | rotated key part | zeros], row stride `row_stride`, in the activation type or (CT) in BF16 beside
+// 32-bit activations.  Two forms of the same sum:
 //   * absorbed, for decoding and short portions: q_n is taken through W_uk(h)^T once, every head then reads the
 //     latents themselves (each cache row is fetched once per sixteen heads), W_uv(h) is applied to the sum;
 //   * expanded, for prompts: keys and values of the range are formed by two matrix products, then flash attention.
@@ -99,13 +100,13 @@ __device__ __forceinline__ void la_store8(act_t<ACT>* p, const float* v) {
 
 // Both latents in pieces of eight elements, NP per thread, in registers between the sums and the stores; every load
 // (norm weights and rotation included) is issued before the first sum.  Elements past a latent's count are zero in proj.
-template <int ACT, int NP>
+template <int ACT, int CT, int NP>
 __global__ __launch_bounds__(256) void latent_epilogue_kernel(LatentEpilogueParams p) {
     __shared__ float lds[8];
     const uint32_t row = blockIdx.x, tid = threadIdx.x;
     const act_t<ACT>* proj = static_cast<const act_t<ACT>*>(p.proj) + (size_t)row * p.proj_stride;
     const uint32_t position = p.rows.position_of(row);
-    act_t<ACT>* out = static_cast<act_t<ACT>*>(p.cache.base) + (size_t)p.rows.slot_of(row) * p.cache.slot_stride +
+    act_t<CT>* out = static_cast<act_t<CT>*>(p.cache.base) + (size_t)p.rows.slot_of(row) * p.cache.slot_stride +
                       (size_t)(position % p.cache.capacity) * p.cache.row_stride;
     act_t<ACT>* cq = static_cast<act_t<ACT>*>(p.cq) + (size_t)row * p.cq_stride;
     const uint32_t qp = (p.q_count + 7u) / 8u, kp = (p.rank_count + 7u) / 8u, pieces = qp + kp;
@@ -124,10 +125,10 @@ __global__ __launch_bounds__(256) void latent_epilogue_kernel(LatentEpiloguePara
             float c, s;
             la_rotation(position, p.inv_freq[j], c, s);
             const float a = act_to_f32<ACT>(proj[p.rot_at + j]), b = act_to_f32<ACT>(proj[p.rot_at + half + j]);
-            out[p.rank + j] = f32_to_act<ACT>(a * c - b * s);
-            out[p.rank + half + j] = f32_to_act<ACT>(b * c + a * s);
+            out[p.rank + j] = f32_to_act<CT>(a * c - b * s);
+            out[p.rank + half + j] = f32_to_act<CT>(b * c + a * s);
         } else if (j >= p.rot_dims) {
-            out[p.rank + j] = proj[p.rot_at + j];
+            out[p.rank + j] = f32_to_act<CT>(act_to_f32<ACT>(proj[p.rot_at + j]));
         }
     }
     float qs = 0.0f, ks = 0.0f;
@@ -158,7 +159,8 @@ __global__ __launch_bounds__(256) void latent_epilogue_kernel(LatentEpiloguePara
         act2_to_f32<ACT_BF16>(w[n].w, f[6], f[7]);
 #pragma unroll
         for (int e = 0; e < 8; ++e) f[e] *= v[n][e] * inv;
-        la_store8<ACT>(u < qp ? cq + 8u * u : out + 8u * (u - qp), f);
+        if (u < qp) la_store8<ACT>(cq + 8u * u, f);
+        else la_store8<CT>(out + 8u * (u - qp), f);
     }
 }
 
@@ -189,14 +191,14 @@ __device__ __forceinline__ uint32_t la_first_key(uint32_t position, uint32_t win
 // ---- absorbed: q_n -> W_uk(h)^T q_n, q_r rotated ----------------------------------------------------
 // A block per (head, row, 128 latent dims): sixteen lanes cover the latents in pieces of eight, sixteen groups of
 // lanes split the rows of W_uk(h).
-template <int ACT>
+template <int ACT, int CT>
 __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentAttnParams p) {
     extern __shared__ __attribute__((aligned(16))) float la_lds[];
     __shared__ __attribute__((aligned(16))) float part[16][132];
     const uint32_t head = blockIdx.x, row = blockIdx.y, tid = threadIdx.x, piece = tid & 15u, group = tid >> 4;
     float* qs = la_lds;                  // [nope]
     const act_t<ACT>* q = static_cast<const act_t<ACT>*>(p.q) + (size_t)row * p.q_stride + head * (p.nope + p.rot);
-    act_t<ACT>* out = static_cast<act_t<ACT>*>(p.qa) + ((size_t)row * p.heads + head) * p.cache.row_stride;
+    act_t<CT>* out = static_cast<act_t<CT>*>(p.qa) + ((size_t)row * p.heads + head) * p.cache.row_stride;
     if (blockIdx.z == gridDim.z - 1u) {              // the rotated part has a block of its own
         const uint32_t position = p.rows.position_of(row), half = p.rot_dims / 2u;
         for (uint32_t j = tid; j < p.cache.row_stride - p.rank; j += 256u) {
@@ -204,10 +206,10 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentAttnParams p) 
                 float c, s;
                 la_rotation(position, p.inv_freq[j], c, s);
                 const float u = act_to_f32<ACT>(q[p.nope + j]), v = act_to_f32<ACT>(q[p.nope + half + j]);
-                out[p.rank + j] = f32_to_act<ACT>(u * c - v * s);
-                out[p.rank + half + j] = f32_to_act<ACT>(v * c + u * s);
+                out[p.rank + j] = f32_to_act<CT>(u * c - v * s);
+                out[p.rank + half + j] = f32_to_act<CT>(v * c + u * s);
             } else if (j >= p.rot_dims) {
-                out[p.rank + j] = j < p.rot ? q[p.nope + j] : f32_to_act<ACT>(0.0f);
+                out[p.rank + j] = f32_to_act<CT>(j < p.rot ? act_to_f32<ACT>(q[p.nope + j]) : 0.0f);
             }
         }
         return;
@@ -243,7 +245,7 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentAttnParams p) 
         float a = 0.0f;
 #pragma unroll
         for (int g = 0; g < 16; ++g) a += part[g][tid];
-        out[r0 + tid] = f32_to_act<ACT>(a);
+        out[r0 + tid] = f32_to_act<CT>(a);
     }
 }
 

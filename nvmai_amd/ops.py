@@ -1151,9 +1151,9 @@ class GLA:
         return torch.zeros((slots, self.heads, self.key_dim, self.value_dim), dtype=torch.float32, device=self.ctx.device)
 
     def encode(self, q, k, v, g, a1, a2, a2_bias, norm_weight, state, out, rows, batch=1, slot=0, slots=None, form=FORM_AUTO):
-        """q, k, v, g, a1: column ranges of one projected matrix [batch * rows, ...]."""
+        """q, k, v, g, a1: column ranges of one projected 32-bit matrix [batch * rows, ...]."""
         stride = q.stride(0)
-        assert all(t.stride(0) == stride for t in (k, v, g, a1))
+        assert all(t.stride(0) == stride and t.dtype == torch.float32 for t in (q, k, v, g, a1))
         check(lib.nvmai_hip_gla(self.ctx.handle, _stream(), C.byref(self.cfg), _ptr(q), _ptr(k), _ptr(v), _ptr(g), _ptr(a1),
                                 stride, _ptr(a2), _ptr(a2_bias), _ptr(norm_weight), _ptr(state), _ptr(slots), slot, _ptr(out),
                                 out.stride(0), rows, batch, form), "gla")
@@ -1168,7 +1168,7 @@ class LatentCache:
         self.capacity = max(64, capacity)
         self.row_stride = (rank + rope_dim + 31) // 32 * 32
         self.rows = torch.zeros((slots, self.capacity, self.row_stride), dtype=ctx.dtype, device=ctx.device)
-        self.view = LatentCacheView(self.rows.data_ptr(), self.rows.stride(0), self.row_stride, self.capacity)
+        self.view = LatentCacheView(self.rows.data_ptr(), self.rows.stride(0), self.row_stride, self.capacity, ctx.act)
 
 
 class LatentAttention:

@@ -20,7 +20,7 @@ from .decoder import StepDecoder
 from .gturbo import ModelError
 from .safetensors_file import SafetensorsFile
 
-ARCHITECTURE = "Pakirax"
+FEW_ROWS = 2        # passes whose products read 32-bit inputs at the price of 16-bit ones (dense_linear: bound by the weights)
 
 
 def _up(n, m):
@@ -255,72 +255,88 @@ class PakiraxDecoder(StepDecoder):
         super().__init__(ctx, cfg, weights, batch, max_context)
         self.max_chunk = min(max_chunk, max_context)
         self.max_rows = max(self.max_chunk, batch)
-        self.mixers, self.states, self.caches = [], {}, {}
+        # Passes of a few rows are bound by the weights' bytes: their activations stay in 32 bits (a context of its own
+        # over the same weights, states and caches); longer ones run in the context's type.
+        self.few_ctx = ctx if ctx.act == ops.ACT_FP32 else ops.Context(ctx.device.index, ops.ACT_FP32)
+        self.mixers, self.states, self.caches = {}, {}, {}
         for i, (m, _) in enumerate(cfg.layers):
+            for c in {ctx, self.few_ctx}:
+                if m.kind == "gla":
+                    op = ops.GLA(c, m.heads, m.dim_p, m.vdim_p, weights.layers[i]["rank"], m.tau, cfg.eps, m.dim, m.vdim)
+                else:
+                    op = ops.LatentAttention(c, m.heads, m.dim_p, m.rot_p, m.vdim_p, m.rank_p, m.kv_rank, m.scale, m.window,
+                                             m.rot_dims, m.rot_base, cfg.eps)
+                self.mixers[i, c] = op
             if m.kind == "gla":
-                op = ops.GLA(ctx, m.heads, m.dim_p, m.vdim_p, weights.layers[i]["rank"], m.tau, cfg.eps, m.dim, m.vdim)
                 self.states[i] = op.new_state(batch)
             else:
-                op = ops.LatentAttention(ctx, m.heads, m.dim_p, m.rot_p, m.vdim_p, m.rank_p, m.kv_rank, m.scale, m.window,
-                                         m.rot_dims, m.rot_base, cfg.eps)
                 capacity = min(max_context, m.window + self.max_chunk - 1) if m.window else max_context
                 self.caches[i] = ops.LatentCache(ctx, batch, capacity, m.rank_p, m.rot_p)
-            self.mixers.append(op)
         self.slots = torch.arange(batch, dtype=torch.int32, device=ctx.device)
         self._buffers = {}
         self.residual_hook = None        # called with (layer index, residual rows) after every layer
         self.logits_f32 = torch.zeros((batch, cfg.vocab), dtype=torch.float32, device=ctx.device)
 
-    def _buf(self, name, rows, cols, dtype=None):
+    def _buf(self, name, rows, cols, dtype):
         """Scratch rows.  Columns past a producer's own stay zero: a buffer's name goes with one width."""
         key = (name, cols, dtype)
         if key not in self._buffers:
-            self._buffers[key] = torch.zeros((self.max_rows, cols), dtype=dtype or self.ctx.dtype, device=self.ctx.device)
+            # buffers of passes in another type than the context's never see more than FEW_ROWS rows
+            most = self.max_rows if dtype == self.ctx.dtype or name in ("residual", "delta", "gla_proj") else FEW_ROWS
+            self._buffers[key] = torch.zeros((most, cols), dtype=dtype, device=self.ctx.device)
         return self._buffers[key][:rows]
 
     # -- mixers: normed rows in, the sublayer's output as 32-bit rows ---------------------------------------
-    def _gla(self, i, h, rows_at, T, slots):
-        m, w, op = self.cfg.layers[i][0], self.w.layers[i], self.mixers[i]
-        proj = ops.dense_linear(self.ctx, w["in_proj"], h, y=self._buf("gla_proj", T, w["in_proj"].shape[0]))
+    def _gla(self, ctx, i, h, rows_at, T, slots):
+        m, w, op = self.cfg.layers[i][0], self.w.layers[i], self.mixers[i, ctx]
+        proj = ops.dense_linear(ctx, w["in_proj"], h, y_f32=self._buf("gla_proj", T, w["in_proj"].shape[0], torch.float32))
         part = lambda n: proj[:, w["at"][n]:]
-        out = self._buf("gla_out%d" % (m.heads * m.vdim_p), T, w["o"].shape[1])
+        out = self._buf("gla_out%d" % (m.heads * m.vdim_p), T, w["o"].shape[1], ctx.dtype)
         batch, rows = (1, T) if slots is None else (T, 1)
         op.encode(part("q"), part("k"), part("v"), part("g"), part("a1"), w["a2"], w["a2_bias"], w["norm"], self.states[i], out,
                   rows, batch, rows_at.slot, slots)
-        return ops.dense_linear(self.ctx, w["o"], out, y_f32=self._buf("delta", T, self.cfg.width_p, torch.float32))
+        return ops.dense_linear(ctx, w["o"], out, y_f32=self._buf("delta", T, self.cfg.width_p, torch.float32))
 
-    def _latent_attention(self, i, h, rows_at, T, slots):
-        m, w, op = self.cfg.layers[i][0], self.w.layers[i], self.mixers[i]
-        at = w["at"]
-        proj = ops.dense_linear(self.ctx, w["in_proj"], h, y=self._buf("latent_proj", T, w["in_proj"].shape[0]))
-        cq = self._buf("cq%d" % m.q_rank, T, w["uq"].shape[1])
+    def _latent_attention(self, ctx, i, h, rows_at, T, slots):
+        m, w, op = self.cfg.layers[i][0], self.w.layers[i], self.mixers[i, ctx]
+        at, dt = w["at"], ctx.dtype
+        proj = ops.dense_linear(ctx, w["in_proj"], h, y=self._buf("latent_proj", T, w["in_proj"].shape[0], dt))
+        cq = self._buf("cq%d" % m.q_rank, T, w["uq"].shape[1], dt)
         op.encode_epilogue(proj, at["q"], m.q_rank, w["q_norm"], at["kv"], at["rope"], w["kv_norm"], cq, self.caches[i], rows_at)
-        q = ops.dense_linear(self.ctx, w["uq"], cq, y=self._buf("latent_q", T, w["uq"].shape[0]))
-        out = self._buf("latent_out%d" % (m.heads * m.vdim_p), T, w["o"].shape[1])
+        q = ops.dense_linear(ctx, w["uq"], cq, y=self._buf("latent_q", T, w["uq"].shape[0], dt))
+        out = self._buf("latent_out%d" % (m.heads * m.vdim_p), T, w["o"].shape[1], dt)
         op.encode(q, proj[:, at["g"]:], w["uk"], w["uv"], self.caches[i], rows_at, out)
-        return ops.dense_linear(self.ctx, w["o"], out, y_f32=self._buf("delta", T, self.cfg.width_p, torch.float32))
+        return ops.dense_linear(ctx, w["o"], out, y_f32=self._buf("delta", T, self.cfg.width_p, torch.float32))
 
     # -- the layers -------------------------------------------------------------------------------------
     def _forward(self, tokens, rows_at, slots=None):
         """tokens (int32 device tensor) through every layer: final-normed rows [T, width padded]."""
-        cfg, ctx, T = self.cfg, self.ctx, tokens.numel()
+        cfg, T = self.cfg, tokens.numel()
+        ctx = self.few_ctx if T <= FEW_ROWS else self.ctx
         D, mult = cfg.width, cfg.residual_mult
         x = self._buf("residual", T, D, torch.float32)
-        h = self._buf("normed", T, cfg.width_p)
+        h, last = self._buf("normed", T, cfg.width_p, ctx.dtype), self._buf("normed", T, cfg.width_p, self.ctx.dtype)
         ops.embed_rows(ctx, self.w.embed, tokens, D, cfg.vocab, x)
-        ops.norm_residual(ctx, x, D, next_norm=self.w.layers[0]["norm1"] if self.w.layers else self.w.final_norm, out=h, eps=cfg.eps)
+
+        def close(delta, post, layer):           # the end of a sublayer and the norm of layer `layer` (the final one: the head's type)
+            if layer < len(cfg.layers):
+                ops.norm_residual(ctx, x, D, delta, post, mult, self.w.layers[layer]["norm1"], h, cfg.eps)
+            else:
+                ops.norm_residual(self.ctx, x, D, delta, post, mult, self.w.final_norm, last, cfg.eps)
+        close(None, None, 0)
         for i, (m, ff) in enumerate(cfg.layers):
             w = self.w.layers[i]
-            after = self.w.layers[i + 1]["norm1"] if i + 1 < len(cfg.layers) else self.w.final_norm
-            delta = (self._gla if m.kind == "gla" else self._latent_attention)(i, h, rows_at, T, slots)
-            ops.norm_residual(ctx, x, D, delta, w["norm1b"], mult, after if ff is None else w["norm2"], h, cfg.eps)
-            if ff is not None:
-                act = ops.dense_linear(ctx, w["up"], h, y=self._buf("ff%d" % ff, T, w["down"].shape[1]), activation=ops.LINEAR_GELU_ERF)
+            delta = (self._gla if m.kind == "gla" else self._latent_attention)(ctx, i, h, rows_at, T, slots)
+            if ff is None:
+                close(delta, w["norm1b"], i + 1)
+            else:
+                ops.norm_residual(ctx, x, D, delta, w["norm1b"], mult, w["norm2"], h, cfg.eps)
+                act = ops.dense_linear(ctx, w["up"], h, y=self._buf("ff%d" % ff, T, w["down"].shape[1], ctx.dtype), activation=ops.LINEAR_GELU_ERF)
                 delta = ops.dense_linear(ctx, w["down"], act, y_f32=self._buf("delta", T, cfg.width_p, torch.float32))
-                ops.norm_residual(ctx, x, D, delta, w["norm2b"], mult, after, h, cfg.eps)
+                close(delta, w["norm2b"], i + 1)
             if self.residual_hook is not None:
                 self.residual_hook(i, x)
-        return h
+        return last
 
     def _prefill_chunk_rows(self, tokens, b, start):
         return self._forward(tokens, ops.row_map(b, start))

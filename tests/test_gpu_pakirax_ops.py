@@ -138,7 +138,8 @@ def gla_case(ctx, rng, heads, dk, dv, rank, rows, tau, bias, count=None):
     part = lambda n, c: np.where(np.arange(n) % (n // heads) < c, rng.standard_normal((rows, n)), 0.0)
     q, k, v, g = part(heads * dk, kc), part(heads * dk, kc), part(heads * dv, vc), rng.standard_normal((rows, heads * dv))
     a1 = rng.standard_normal((rows, rank))
-    proj, p64 = acts(ctx, np.concatenate([q, k, v, g, a1], 1))
+    proj = torch.from_numpy(np.concatenate([q, k, v, g, a1], 1).astype(np.float32)).cuda()
+    p64 = proj.double().cpu().numpy()
     cuts = np.cumsum([0, heads * dk, heads * dk, heads * dv, heads * dv, rank])
     dev = [proj[:, a:] for a in cuts[:5]]
     f64 = [p64[:, a:b] for a, b in zip(cuts, cuts[1:])]
@@ -225,7 +226,7 @@ def test_gla_batch_of_slots_equals_each_alone(ctx):
 class Latent:
     """One layer's operands and its plain restatement; rows are fed in portions through the library's two calls."""
 
-    def __init__(self, ctx, rng, heads, nope, rot, vdim, rank, window, n, capacity=None, slots=1, count=None, rotary=None, spikes=()):
+    def __init__(self, ctx, rng, heads, nope, rot, vdim, rank, window, n, capacity=None, slots=1, count=None, rotary=None, spikes=(), cache_ctx=None):
         import nvmai_amd as nv
         self.nv, self.ctx, self.n, self.window = nv, ctx, n, window
         self.heads, self.nope, self.rot, self.vdim, self.rank = heads, nope, rot, vdim, rank
@@ -249,7 +250,7 @@ class Latent:
         self.q, self.q64 = acts(ctx, q)
         self.qc = qc
         self.op = nv.LatentAttention(ctx, heads, nope, rot, vdim, rank, self.count, self.scale, window, self.rotary, self.base, self.eps)
-        self.cache = nv.LatentCache(ctx, slots, capacity or n, rank, rot)
+        self.cache = nv.LatentCache(cache_ctx or ctx, slots, capacity or n, rank, rot)
 
     def run(self, portions, form, slot=0, base=0):
         """Feed `portions` (row counts) from position base; the gated outputs of every row."""
@@ -387,3 +388,18 @@ def test_latent_decode_batch_of_unequal_positions(ctx):
     y = torch.zeros((B, L.heads * L.vdim), dtype=ctx.dtype, device="cuda")
     L.op.encode(q, proj[:, L.qc + L.rank + L.rot:], L.uk, L.uv, L.cache, rows, y)
     close(y, L.plain(lengths), 2e-5 if is32(ctx) else 2e-2)
+
+
+def test_latent_attention_in_32_bit_over_a_bf16_cache():
+    """32-bit rows beside a BF16 cache: what passes of one or two rows use.  The cached rows and the query on its way to them are
+    BF16, everything else 32-bit; the expanded form is refused."""
+    import nvmai_amd as nv
+    full, half = nv.Context(0, nv.ACT_FP32), nv.Context(0, nv.ACT_BF16)
+    for window, portions in [(33, [1] * 90), (64, [4, 3, 2, 1] * 9), (0, [50, 40])]:
+        n = sum(portions)
+        L = Latent(full, np.random.default_rng(window), 5, 48, 32, 48, 128, window, n, cache_ctx=half)
+        close(L.run(portions, nv.FORM_AUTO), L.plain(range(n)), 1e-2)
+    with pytest.raises(nv.NvmaiError):
+        L.run([90], nv.LATENT_EXPANDED)
+    with pytest.raises(nv.NvmaiError):
+        Latent(half, np.random.default_rng(0), 5, 48, 32, 48, 128, 33, 4, cache_ctx=full).run([4], nv.FORM_AUTO)
