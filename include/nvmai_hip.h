@@ -750,7 +750,7 @@ uint64_t nvmai_sampler_seed_for(uint64_t seed, int64_t position);
  * are [n, k] BF16 rows with k a multiple of 64; a model whose sizes are not multiples of 64 (rows of a matrix
  * product) or 16 (head sizes) is padded with zero weights when it is loaded, and the counts below that are called
  * `..._count` say how many of the elements are real where a mean is taken over them. */
-enum { NVMAI_LINEAR_NONE = 0, NVMAI_LINEAR_GELU_ERF = 1 };
+enum { NVMAI_LINEAR_NONE = 0, NVMAI_LINEAR_GELU_ERF = 1, NVMAI_LINEAR_GELU_TANH = 2, NVMAI_LINEAR_SILU_PAIRS = 3 };
 enum { NVMAI_FORM_AUTO = 0, NVMAI_GLA_RECURRENT = 1, NVMAI_GLA_CHUNKED = 2, NVMAI_LATENT_ABSORBED = 1, NVMAI_LATENT_EXPANDED = 2 };
 
 /* y[t, :] = act(W x[t, :]) for any number of rows: a wave per weight row up to 4 rows, split-k matrix-core products
@@ -759,6 +759,20 @@ enum { NVMAI_FORM_AUTO = 0, NVMAI_GLA_RECURRENT = 1, NVMAI_GLA_CHUNKED = 2, NVMA
 int nvmai_hip_dense_linear(nvmai_hip_ctx* ctx, nvmai_stream stream, const uint16_t* w, uint32_t w_stride, const void* x,
                            uint32_t x_stride, uint32_t rows, uint32_t n, uint32_t k, void* y, float* y_f32, uint32_t y_stride,
                            int activation);
+
+/* The same with more between the sum and the store: y[t, r] = act(sum + bias[r]) * mul[mul_ids[t], r].  bias: [n] BF16 or
+ * NULL; mul: a BF16 table [mul_rows, mul_stride] or NULL, mul_ids its row for each input row (a device array; an id
+ * >= mul_rows multiplies by zero).  SILU_PAIRS (n even, no bias, no mul): y[t, j] = silu(row 2 j) * (row 2 j + 1), n / 2 outputs. */
+typedef struct {
+    int32_t activation;
+    const uint16_t* bias;
+    const uint16_t* mul;
+    const uint32_t* mul_ids;
+    uint32_t mul_stride, mul_rows;
+} nvmai_linear_epilogue;
+int nvmai_hip_dense_linear_ex(nvmai_hip_ctx* ctx, nvmai_stream stream, const uint16_t* w, uint32_t w_stride, const void* x,
+                              uint32_t x_stride, uint32_t rows, uint32_t n, uint32_t k, void* y, float* y_f32, uint32_t y_stride,
+                              const nvmai_linear_epilogue* epilogue);
 
 /* The end of one sublayer and the start of the next over the 32-bit residual:
  *   x   += mult * LN(delta) * post_weight + post_bias   (post_weight NULL: x += mult * delta; delta NULL: x as it is)
@@ -769,9 +783,20 @@ int nvmai_hip_norm_residual(nvmai_hip_ctx* ctx, nvmai_stream stream, float* x, u
                             const uint16_t* next_weight, const uint16_t* next_bias, void* out, uint32_t out_stride, uint32_t rows,
                             uint32_t d, float eps);
 
+/* The same with RMS norms, RMS(v) = v / sqrt(mean(v^2) + eps):
+ *   x   += RMS(delta) * (post_add + post_weight)     (delta NULL with post_weight NULL: x as it is)
+ *   out  = RMS(x) * (next_add + next_weight)         (next_weight NULL: out = x as activations; out NULL: not written)
+ * The adds are 0 for a plain weight, 1 for one stored around zero. */
+int nvmai_hip_rms_residual(nvmai_hip_ctx* ctx, nvmai_stream stream, float* x, uint32_t x_stride, const float* delta,
+                           uint32_t delta_stride, const uint16_t* post_weight, float post_add, const uint16_t* next_weight,
+                           float next_add, void* out, uint32_t out_stride, uint32_t rows, uint32_t d, float eps);
+
 /* out[t, :] = row token_ids[t] of a BF16 table, as floats; an id >= vocab gives zeros. */
 int nvmai_hip_embed_rows(nvmai_hip_ctx* ctx, nvmai_stream stream, const uint16_t* table, uint32_t table_stride,
                          const uint32_t* token_ids, uint32_t n_tokens, float* out, uint32_t out_stride, uint32_t d, uint32_t vocab);
+
+/* x = cap * tanh(x / cap) over rows of floats. */
+int nvmai_hip_softcap_rows(nvmai_hip_ctx* ctx, nvmai_stream stream, float* x, uint32_t x_stride, uint32_t rows, uint32_t n, float cap);
 
 /* Index of the largest finite value of each row, ties to the lower index, 0 when none is finite. */
 int nvmai_hip_argmax_rows(nvmai_hip_ctx* ctx, nvmai_stream stream, const float* x, uint32_t x_stride, uint32_t rows, uint32_t n,
@@ -784,6 +809,14 @@ typedef struct {
     const uint32_t* positions;
     uint32_t slot, position;
 } nvmai_row_map;
+
+/* out[t, :] = scale * (row token_ids[t] of a BF16 table) + the sinusoid of the row's position, as floats, and once more as
+ * activations in act (or NULL).  inv_freq: device array of (d + 1) / 2 doubles; entry 2 i is the sine and 2 i + 1 the
+ * cosine of position * inv_freq[i]; NULL: no sinusoid (map may be NULL then). */
+int nvmai_hip_embed_positions(nvmai_hip_ctx* ctx, nvmai_stream stream, const uint16_t* table, uint32_t table_stride,
+                              const uint32_t* token_ids, uint32_t n_tokens, float scale, const double* inv_freq,
+                              const nvmai_row_map* map, float* out, uint32_t out_stride, void* act, uint32_t act_stride, uint32_t d,
+                              uint32_t vocab);
 
 /* Gated linear attention with a decay per key channel: z = W_a2 a1 + b, alpha = sigmoid(z)^(1/tau),
  *   S_t = diag(alpha_t) S_(t-1) + k_t v_t^T,  o_t = S_t^T (q_scale q_t),  out = rmsnorm(o) * norm_weight * silu(g)
@@ -837,6 +870,80 @@ int nvmai_hip_latent_attention(nvmai_hip_ctx* ctx, nvmai_stream stream, const nv
                                uint32_t q_stride, const void* gate, uint32_t gate_stride, const uint16_t* uk, const uint16_t* uv,
                                const nvmai_latent_cache* cache, const nvmai_row_map* map, void* out, uint32_t out_stride,
                                uint32_t rows, int form);
+
+/* ---- windowed grouped-query attention over a cache of normed keys --------------------------------------- *
+ * One layer's keys and values, per slot: k [kv_heads, pinned + ring, key_dim], v [kv_heads, value_dim, pinned + ring]
+ * (values transposed).  Position p lies in ring row pinned + p % ring and, when p < pinned, in row p too, where it stays.
+ * pinned (may be 0) and ring are multiples of 64, key_dim of 32, value_dim of 16.  type: NVMAI_ACT_BF16 or NVMAI_ACT_FP32, the
+ * context's activation type or BF16 in a 32-bit context.  The caller clears the arrays once.  Several layers may look at
+ * one cache. */
+typedef struct {
+    void* k;
+    void* v;
+    uint32_t kv_heads, key_dim, value_dim, pinned, ring;
+    int32_t type;
+} nvmai_kv_ring;
+
+/* Position i sees j <= i with i - j < window (0: every j) or j < keep_first (<= pinned).
+ *   score = scale * q . k;  softcap > 0: score = softcap * tanh(score / softcap);  alibi: score -= 2^(-8 (head + 1) / heads) (i - j)
+ * key_count is the real head size behind key_dim: the mean of the norms. */
+typedef struct {
+    uint32_t heads, key_count, window, keep_first;
+    float scale, softcap, eps;
+    int32_t alibi;
+} nvmai_window_config;
+
+/* From projected rows of floats: q[t] = rmsnorm(q part) * q_norm per head, in the cache's type, [rows, heads * key_dim];
+ * with k_norm not NULL also the token's cache entries, rmsnorm(k part) * k_norm and the value part (k_norm NULL: the
+ * cache is another layer's and already holds them).  q_at, k_at, v_at: columns of proj; norm weights BF16 [key_dim]. */
+int nvmai_hip_window_epilogue(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_window_config* config, const float* proj,
+                              uint32_t proj_stride, uint32_t q_at, uint32_t k_at, uint32_t v_at, const uint16_t* q_norm,
+                              const uint16_t* k_norm, void* q, uint32_t q_stride, const nvmai_kv_ring* cache, const nvmai_row_map* map,
+                              uint32_t rows);
+
+/* out[t, head * value_dim ..] = out_scale * sigmoid(gate[t, head]) * sum_j softmax_j(score) v_j; gate: floats
+ * [rows, gate_stride], NULL = none.  The rows' own cache entries must have been written.  The ring has to hold what the
+ * rows look at: window + rows - 1 positions.  Rows by arrays: max_position bounds their positions (sizes the launch).
+ * form: AUTO, NVMAI_WINDOW_SPLIT (decoding), NVMAI_WINDOW_FLASH (prompts, 16-bit) or NVMAI_WINDOW_PLAIN (any sizes).  Takes workspace. */
+enum { NVMAI_WINDOW_SPLIT = 1, NVMAI_WINDOW_FLASH = 2, NVMAI_WINDOW_PLAIN = 3 };
+int nvmai_hip_window_attention(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_window_config* config, const void* q,
+                               uint32_t q_stride, const float* gate, uint32_t gate_stride, const nvmai_kv_ring* cache,
+                               const nvmai_row_map* map, uint32_t max_position, float out_scale, void* out, uint32_t out_stride,
+                               uint32_t rows, int form);
+
+/* ---- recurrences with one decay per head ---------------------------------------------------------------------- *
+ * Per head, with a state S [key_dim, value_dim] of floats:
+ *   S_t = g_t S_(t-1) + k_t u_t^T,  o_t = S_t^T q_t,  g_t = exp(-exp(a_log) softplus(a_t + dt_bias))
+ *   NVMAI_SCAN_DELTA: u_t = sigmoid(b_t) (v_t - g_t S_(t-1)^T k_t); q and k unit vectors per head, q times q_scale
+ *   NVMAI_SCAN_SSD:   u_t = softplus(a_t + dt_bias) v_t;  o_t += skip v_t
+ * q, k (key_heads of them; head h uses h / (heads / key_heads)) and v come from projected rows of floats through a causal
+ * filter of `taps` per channel, a bias (conv_bias, or NULL) and silu.  The channels lie together from column conv_at:
+ * [q: key_heads * key_dim | k: the same | v: heads * value_dim]; a_at, b_at: columns of one number per head.  history
+ * [slots, history_rows, channels] floats holds the filter's inputs, position p in row p % history_rows
+ * (>= taps + 31; positions before 0 read as zero, whatever it holds).  conv [channels, taps], a_log, dt_bias, skip: BF16.  state
+ * [slots, heads, key_dim, value_dim], updated in place.  out: floats [rows, heads * value_dim].
+ * Rows by arrays: one row each of distinct slots.  key_dim, value_dim: multiples of 16, at most 512 (the chunked form 256).
+ * form: AUTO, NVMAI_SCAN_RECURRENT, NVMAI_SCAN_CHUNKED (consecutive rows of one slot; takes workspace). */
+enum { NVMAI_SCAN_DELTA = 0, NVMAI_SCAN_SSD = 1 };
+enum { NVMAI_SCAN_RECURRENT = 1, NVMAI_SCAN_CHUNKED = 2 };
+typedef struct {
+    int32_t kind;
+    uint32_t heads, key_heads, key_dim, value_dim, taps, history_rows;
+    uint32_t conv_at, a_at, b_at;
+    float q_scale;
+} nvmai_scan_config;
+int nvmai_hip_scan(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_scan_config* config, const float* proj, uint32_t proj_stride,
+                   const uint16_t* conv, const uint16_t* conv_bias, const uint16_t* a_log, const uint16_t* dt_bias, const uint16_t* skip,
+                   float* history, float* state, const nvmai_row_map* map, float* out, uint32_t out_stride, uint32_t rows, int form);
+
+/* The gated norm behind a recurrence.  x, gate: floats, heads of value_dim columns of which value_count are real; the
+ * heads * value_count real ones in order make `parts` equal parts, each normed by its own root mean square:
+ *   gate_first: out = RMS(x * silu(gate)) * weight * out_scale, weight [heads * value_dim]
+ *   else        out = RMS(x) * weight * silu(gate) * out_scale, weight [value_dim], shared by the heads
+ * out: activations, columns laid out as x's; padding columns are not written. */
+int nvmai_hip_gated_norm(nvmai_hip_ctx* ctx, nvmai_stream stream, const float* x, uint32_t x_stride, const float* gate,
+                         uint32_t gate_stride, const uint16_t* weight, void* out, uint32_t out_stride, uint32_t rows, uint32_t heads,
+                         uint32_t value_dim, uint32_t value_count, uint32_t parts, int gate_first, float out_scale, float eps);
 
 #ifdef __cplusplus
 }

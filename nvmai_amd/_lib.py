@@ -2,7 +2,7 @@
 
 The library is the product; there is no fallback.  If it has not been built the
 import fails loudly.  A part library (build.PARTS: the entry points one family of models needs) serves where the
-whole one has not been built; an entry point it does not hold fails when it is called.
+whole one has not been built (NVMAI_HIP_PART names it where several have); an entry point it does not hold fails when it is called.
 """
 import ctypes as C
 import glob
@@ -21,10 +21,10 @@ class NvmaiLibraryMissing(ImportError):
 def load():
     if os.path.exists(LIB_PATH):
         return C.CDLL(LIB_PATH)
-    parts = sorted(glob.glob(LIB_PATH[:-3] + ".*.so"))
+    parts = sorted(glob.glob(LIB_PATH[:-3] + ".%s.so" % os.environ.get("NVMAI_HIP_PART", "*")))
     if not parts:
         raise NvmaiLibraryMissing(
-            "%s is missing: run `python -m nvmai_amd.build` (hipcc, gfx950) first" % LIB_PATH)
+            "%s is missing: run `python nvmai_amd/build.py` (hipcc, gfx950) first" % LIB_PATH)
     return C.CDLL(parts[0])
 
 
@@ -109,6 +109,28 @@ class PrefillGrouping(C.Structure):
     _fields_ = [(n, vp) for n in ("sorted_pairs", "expert_offsets", "expert_counts", "groups", "tiles", "info")]
 
 
+class LinearEpilogue(C.Structure):
+    """nvmai_linear_epilogue"""
+    _fields_ = [("activation", i32), ("bias", vp), ("mul", vp), ("mul_ids", vp), ("mul_stride", u32), ("mul_rows", u32)]
+
+
+class KvRingView(C.Structure):
+    """nvmai_kv_ring"""
+    _fields_ = [("k", vp), ("v", vp), ("kv_heads", u32), ("key_dim", u32), ("value_dim", u32), ("pinned", u32), ("ring", u32), ("type", i32)]
+
+
+class WindowConfig(C.Structure):
+    """nvmai_window_config"""
+    _fields_ = [("heads", u32), ("key_count", u32), ("window", u32), ("keep_first", u32), ("scale", C.c_float), ("softcap", C.c_float),
+                ("eps", C.c_float), ("alibi", i32)]
+
+
+class ScanConfig(C.Structure):
+    """nvmai_scan_config"""
+    _fields_ = [("kind", i32)] + [(n, u32) for n in ("heads", "key_heads", "key_dim", "value_dim", "taps", "history_rows", "conv_at", "a_at",
+                                                     "b_at")] + [("q_scale", C.c_float)]
+
+
 # name -> argtypes (every function returns int unless listed in _OTHER)
 SIGNATURES = {
     "nvmai_hip_ctx_create": [C.c_int, C.c_int, C.POINTER(vp)],
@@ -189,6 +211,16 @@ SIGNATURES = {
     "nvmai_hip_dense_linear": [vp, vp, vp, u32, vp, u32, u32, u32, u32, vp, vp, u32, C.c_int],
     "nvmai_hip_norm_residual": [vp, vp, vp, u32, vp, u32, vp, vp, C.c_float, vp, vp, vp, u32, u32, u32, C.c_float],
     "nvmai_hip_embed_rows": [vp, vp, vp, u32, vp, u32, vp, u32, u32, u32],
+    "nvmai_hip_dense_linear_ex": [vp, vp, vp, u32, vp, u32, u32, u32, u32, vp, vp, u32, C.POINTER(LinearEpilogue)],
+    "nvmai_hip_rms_residual": [vp, vp, vp, u32, vp, u32, vp, C.c_float, vp, C.c_float, vp, u32, u32, u32, C.c_float],
+    "nvmai_hip_embed_positions": [vp, vp, vp, u32, vp, u32, C.c_float, vp, C.POINTER(RowMap), vp, u32, vp, u32, u32, u32],
+    "nvmai_hip_softcap_rows": [vp, vp, vp, u32, u32, u32, C.c_float],
+    "nvmai_hip_window_epilogue": [vp, vp, C.POINTER(WindowConfig), vp, u32, u32, u32, u32, vp, vp, vp, u32, C.POINTER(KvRingView),
+                                  C.POINTER(RowMap), u32],
+    "nvmai_hip_window_attention": [vp, vp, C.POINTER(WindowConfig), vp, u32, vp, u32, C.POINTER(KvRingView), C.POINTER(RowMap), u32,
+                                   C.c_float, vp, u32, u32, C.c_int],
+    "nvmai_hip_scan": [vp, vp, C.POINTER(ScanConfig), vp, u32, vp, vp, vp, vp, vp, vp, vp, C.POINTER(RowMap), vp, u32, u32, C.c_int],
+    "nvmai_hip_gated_norm": [vp, vp, vp, u32, vp, u32, vp, vp, u32, u32, u32, u32, u32, u32, C.c_int, C.c_float, C.c_float],
     "nvmai_hip_argmax_rows": [vp, vp, vp, u32, u32, u32, vp],
     "nvmai_hip_gla": [vp, vp, C.POINTER(GlaConfig), vp, vp, vp, vp, vp, u32, vp, vp, vp, vp, vp, u32, vp, u32, u32, u32, C.c_int],
     "nvmai_hip_latent_epilogue": [vp, vp, C.POINTER(LatentConfig), vp, u32, u32, u32, vp, u32, u32, vp, vp, u32,

@@ -17,7 +17,8 @@ FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=o
 
 
 # Part libraries: the sources that one family of models needs, for a run that must not wait for the rest.
-PARTS = {"dense": ["ctx_api", "dense_api", "gla_api", "latent_api", "sample_api"]}
+PARTS = {"dense": ["ctx_api", "dense_api", "norm_api", "gla_api", "latent_api", "sample_api"],
+         "scan": ["ctx_api", "dense_api", "norm_api", "window_api", "scan_api", "sample_api"]}
 
 
 def part_path(part):
@@ -49,9 +50,11 @@ def build(verbose=False, jobs=8):
 
 def ensure(part, verbose=False, jobs=8):
     """The library if it is built, else the part library, built now if it is not there either."""
-    for path in (LIB, part_path(part)):
-        if os.path.exists(path):
-            return path
+    if os.path.exists(LIB):
+        return LIB
+    os.environ["NVMAI_HIP_PART"] = part              # which of several parts the package loads
+    if os.path.exists(part_path(part)):
+        return part_path(part)
     return _compile([os.path.join(CSRC, n + ".hip") for n in PARTS[part]], part_path(part), verbose, jobs)
 
 

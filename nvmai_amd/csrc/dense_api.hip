@@ -1,5 +1,5 @@
-// Entry points of the dense models: matrix products against BF16 weights, layer norms over the 32-bit residual,
-// embedding rows, argmax.
+// Entry points of the dense models: matrix products against BF16 weights, embedding rows, the cap of the
+// logits, argmax.
 #include "ctx.hpp"
 #include "dense_kernels.hpp"
 #include "dense_internal.hpp"
@@ -11,8 +11,12 @@ namespace nvmai {
 int dense_linear_check(const nvmai_hip_ctx* ctx, const DenseLinearParams& p) {
     if (!ctx || !p.w || !p.x || (!p.y && !p.y_f32)) return NVMAI_ERR_INVALID_ARG;
     if (ctx->act != NVMAI_ACT_BF16 && ctx->act != NVMAI_ACT_FP32) return NVMAI_ERR_UNSUPPORTED;
-    if (p.k == 0 || p.k % 64 || p.n == 0 || p.w_stride < p.k || p.x_stride < p.k || p.y_stride < p.n) return NVMAI_ERR_INVALID_ARG;
-    if (p.activation != NVMAI_LINEAR_NONE && p.activation != NVMAI_LINEAR_GELU_ERF) return NVMAI_ERR_UNSUPPORTED;
+    if (p.k == 0 || p.k % 64 || p.n == 0 || p.w_stride < p.k || p.x_stride < p.k) return NVMAI_ERR_INVALID_ARG;
+    if (p.activation < NVMAI_LINEAR_NONE || p.activation > NVMAI_LINEAR_SILU_PAIRS) return NVMAI_ERR_UNSUPPORTED;
+    const bool pairs = p.activation == NVMAI_LINEAR_SILU_PAIRS;
+    if (p.y_stride < (pairs ? p.n / 2 : p.n)) return NVMAI_ERR_INVALID_ARG;
+    if (pairs && (p.n % 2 || p.y_stride % 2 || p.bias || p.mul)) return NVMAI_ERR_INVALID_ARG;
+    if (p.mul && (!p.mul_ids || p.mul_stride < p.n)) return NVMAI_ERR_INVALID_ARG;
     if (!aligned16(p.w) || !aligned16(p.x) || p.w_stride % 8 || p.x_stride % 8) return NVMAI_ERR_ALIGNMENT;
     if ((p.y && !aligned16(p.y)) || (p.y_f32 && !aligned16(p.y_f32))) return NVMAI_ERR_ALIGNMENT;
     // 32-bit byte offsets inside an operand
@@ -24,7 +28,7 @@ template <int ACT, int NT>
 static void launch_gemv(const DenseLinearParams& p, hipStream_t s) {
     // rows per wave: one (short blocks, many of them) until the inputs' own loads weigh more than that
     if (p.n >= 65536) dense_gemv_kernel<ACT, NT, 4><<<(p.n + 15) / 16, 256, 0, s>>>(p);
-    else if (NT * (ACT == ACT_FP32 ? 2 : 1) > 2 && p.n >= 8192) dense_gemv_kernel<ACT, NT, 2><<<(p.n + 7) / 8, 256, 0, s>>>(p);
+    else if (p.activation == NVMAI_LINEAR_SILU_PAIRS || (NT * (ACT == ACT_FP32 ? 2 : 1) > 2 && p.n >= 8192)) dense_gemv_kernel<ACT, NT, 2><<<(p.n + 7) / 8, 256, 0, s>>>(p);
     else dense_gemv_kernel<ACT, NT, 1><<<(p.n + 3) / 4, 256, 0, s>>>(p);
 }
 
@@ -87,59 +91,44 @@ extern "C" int nvmai_hip_dense_linear(nvmai_hip_ctx* ctx, nvmai_stream stream, c
     return dense_linear(ctx, (hipStream_t)stream, p);
 }
 
-namespace {
-
-template <int ACT, bool DELTA, bool POST, bool NEXT>
-void norm_residual_sized(const NormResidualParams& p, uint32_t rows, hipStream_t s) {
-    const bool vec = p.d % 4 == 0 && p.x_stride % 4 == 0 && aligned16(p.x) && (!DELTA || (p.delta_stride % 4 == 0 && aligned16(p.delta))) &&
-                     (!NEXT || (p.out_stride % 4 == 0 && aligned16(p.out))) && aligned16(p.post_w) && aligned16(p.post_b) &&
-                     aligned16(p.next_w) && aligned16(p.next_b);
-    const uint32_t vpt = (p.d + 1023) / 1024;
-    if (!vec) {
-        if (vpt <= 2) norm_residual_kernel<ACT, 2, DELTA, POST, NEXT, false><<<rows, 256, 0, s>>>(p);
-        else norm_residual_kernel<ACT, 16, DELTA, POST, NEXT, false><<<rows, 256, 0, s>>>(p);
-    } else if (vpt <= 1) norm_residual_kernel<ACT, 1, DELTA, POST, NEXT, true><<<rows, 256, 0, s>>>(p);
-    else if (vpt <= 2) norm_residual_kernel<ACT, 2, DELTA, POST, NEXT, true><<<rows, 256, 0, s>>>(p);
-    else if (vpt <= 4) norm_residual_kernel<ACT, 4, DELTA, POST, NEXT, true><<<rows, 256, 0, s>>>(p);
-    else if (vpt <= 8) norm_residual_kernel<ACT, 8, DELTA, POST, NEXT, true><<<rows, 256, 0, s>>>(p);
-    else norm_residual_kernel<ACT, 16, DELTA, POST, NEXT, true><<<rows, 256, 0, s>>>(p);
-}
-
-template <int ACT>
-int norm_residual(const NormResidualParams& p, uint32_t rows, hipStream_t s) {
-    const bool delta = p.delta, post = p.post_w, next = p.next_w;
-    if (delta && post && next) norm_residual_sized<ACT, true, true, true>(p, rows, s);
-    else if (delta && post) norm_residual_sized<ACT, true, true, false>(p, rows, s);
-    else if (delta && next) norm_residual_sized<ACT, true, false, true>(p, rows, s);
-    else if (delta) norm_residual_sized<ACT, true, false, false>(p, rows, s);
-    else if (next) norm_residual_sized<ACT, false, false, true>(p, rows, s);
-    return launch_status();
-}
-
-}  // namespace
-
-extern "C" int nvmai_hip_norm_residual(nvmai_hip_ctx* ctx, nvmai_stream stream, float* x, uint32_t x_stride, const float* delta,
-                                       uint32_t delta_stride, const uint16_t* post_weight, const uint16_t* post_bias, float mult,
-                                       const uint16_t* next_weight, const uint16_t* next_bias, void* out, uint32_t out_stride,
-                                       uint32_t rows, uint32_t d, float eps) {
-    if (!ctx || !x || d == 0 || x_stride < d || (delta && delta_stride < d)) return NVMAI_ERR_INVALID_ARG;
-    if ((next_weight == nullptr) != (out == nullptr) || (out && out_stride < d)) return NVMAI_ERR_INVALID_ARG;
-    if (ctx->act != NVMAI_ACT_BF16 && ctx->act != NVMAI_ACT_FP32) return NVMAI_ERR_UNSUPPORTED;
-    if (d > 16384) return NVMAI_ERR_UNSUPPORTED;
-    if (rows == 0) return NVMAI_OK;
-    if ((post_weight == nullptr) != (post_bias == nullptr) || (post_weight && !delta) || (next_weight == nullptr) != (next_bias == nullptr))
-        return NVMAI_ERR_INVALID_ARG;
-    const NormResidualParams p{x, delta, post_weight, post_bias, next_weight, next_bias, out, x_stride, delta_stride, out_stride, d, mult, eps};
-    return ctx->act == NVMAI_ACT_BF16 ? norm_residual<ACT_BF16>(p, rows, (hipStream_t)stream) : norm_residual<ACT_FP32>(p, rows, (hipStream_t)stream);
+extern "C" int nvmai_hip_dense_linear_ex(nvmai_hip_ctx* ctx, nvmai_stream stream, const uint16_t* w, uint32_t w_stride, const void* x,
+                                         uint32_t x_stride, uint32_t rows, uint32_t n, uint32_t k, void* y, float* y_f32,
+                                         uint32_t y_stride, const nvmai_linear_epilogue* e) {
+    if (!e) return NVMAI_ERR_INVALID_ARG;
+    const DenseLinearParams p{w, x, y, y_f32, w_stride, x_stride, y_stride, rows, n, k, e->activation, e->bias, e->mul, e->mul_ids,
+                              e->mul_stride, e->mul_rows};
+    return dense_linear(ctx, (hipStream_t)stream, p);
 }
 
 extern "C" int nvmai_hip_embed_rows(nvmai_hip_ctx* ctx, nvmai_stream stream, const uint16_t* table, uint32_t table_stride,
                                     const uint32_t* token_ids, uint32_t n_tokens, float* out, uint32_t out_stride, uint32_t d,
                                     uint32_t vocab) {
+    return nvmai_hip_embed_positions(ctx, stream, table, table_stride, token_ids, n_tokens, 1.0f, nullptr, nullptr, out, out_stride, nullptr, 0, d, vocab);
+}
+
+extern "C" int nvmai_hip_embed_positions(nvmai_hip_ctx* ctx, nvmai_stream stream, const uint16_t* table, uint32_t table_stride,
+                                         const uint32_t* token_ids, uint32_t n_tokens, float scale, const double* inv_freq,
+                                         const nvmai_row_map* map, float* out, uint32_t out_stride, void* act, uint32_t act_stride,
+                                         uint32_t d, uint32_t vocab) {
     if (!ctx || !table || !token_ids || !out || d == 0 || table_stride < d || out_stride < d || vocab == 0) return NVMAI_ERR_INVALID_ARG;
+    if ((inv_freq && !map) || (act && act_stride < d)) return NVMAI_ERR_INVALID_ARG;
+    if (act && ctx->act != NVMAI_ACT_BF16 && ctx->act != NVMAI_ACT_FP32) return NVMAI_ERR_UNSUPPORTED;
     if (n_tokens == 0) return NVMAI_OK;
     if (n_tokens > 65535) return NVMAI_ERR_UNSUPPORTED;
-    embed_rows_kernel<<<dim3((d + 255) / 256, n_tokens), 256, 0, (hipStream_t)stream>>>(table, table_stride, token_ids, out, out_stride, d, vocab);
+    EmbedParams p{table, token_ids, out, act, inv_freq, SeqRows{}, table_stride, out_stride, act_stride, d, vocab, scale};
+    if (map) p.rows = SeqRows{map->slots, map->positions, map->slot, map->position};
+    const dim3 grid((d + 511) / 512, n_tokens);
+    if (ctx->act == NVMAI_ACT_FP32) embed_rows_kernel<ACT_FP32><<<grid, 256, 0, (hipStream_t)stream>>>(p);
+    else embed_rows_kernel<ACT_BF16><<<grid, 256, 0, (hipStream_t)stream>>>(p);
+    return launch_status();
+}
+
+extern "C" int nvmai_hip_softcap_rows(nvmai_hip_ctx* ctx, nvmai_stream stream, float* x, uint32_t x_stride, uint32_t rows, uint32_t n,
+                                      float cap) {
+    if (!ctx || !x || n == 0 || x_stride < n || !(cap > 0.0f)) return NVMAI_ERR_INVALID_ARG;
+    if (rows == 0) return NVMAI_OK;
+    if (rows > 65535) return NVMAI_ERR_UNSUPPORTED;
+    softcap_rows_kernel<<<dim3((n + 255) / 256, rows), 256, 0, (hipStream_t)stream>>>(x, x_stride, n, cap);
     return launch_status();
 }
 

@@ -12,6 +12,10 @@ struct DenseLinearParams {
     float* y_f32;           // floats, or nullptr
     uint32_t w_stride, x_stride, y_stride, rows, n, k;
     int activation;         // NVMAI_LINEAR_*
+    const uint16_t* bias;   // [n] BF16, or nullptr
+    const uint16_t* mul;    // BF16 table [mul_rows, mul_stride]: y[t, r] *= mul[mul_ids[t], r]; or nullptr
+    const uint32_t* mul_ids;
+    uint32_t mul_stride, mul_rows;
 };
 
 int dense_linear_check(const nvmai_hip_ctx* ctx, const DenseLinearParams& p);

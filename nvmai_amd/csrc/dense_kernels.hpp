@@ -1,10 +1,10 @@
 // Kernels of the dense models (BF16 weights; 16-bit BF16 or 32-bit activations; a 32-bit residual stream):
-// the matrix products, layer norm with bias, the norm-scale-add that closes a sublayer, embedding rows, argmax.
+// the matrix products, embedding rows, the cap of the logits, argmax.
 // gfx950, wave64.
 #pragma once
 
-#include "common.hpp"
 #include "dense_internal.hpp"
+#include "rows.hpp"
 
 namespace nvmai {
 
@@ -18,20 +18,50 @@ __device__ __forceinline__ dn_f4 dn_mfma(const uint4& a, const uint4& b, dn_f4 c
 // z/2 (1 + erf(z / sqrt 2))
 __device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
 
-__device__ __forceinline__ float dense_act(float v, int activation) { return activation == 1 ? gelu_erf(v) : v; }
+// z/2 (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))
+__device__ __forceinline__ float gelu_tanh(float z) { return 0.5f * z * (1.0f + tanhf(0.79788456080286536f * fmaf(0.044715f * z * z, z, z))); }
+
+// What stands between a sum and its store: bias, activation, the token's own multiplier (an id past the table: zero).
+__device__ __forceinline__ float dense_finish(const DenseLinearParams& p, uint32_t t, uint32_t r, float v) {
+    if (p.bias) v += bf16_to_f32(p.bias[r]);
+    v = p.activation == NVMAI_LINEAR_GELU_ERF ? gelu_erf(v) : p.activation == NVMAI_LINEAR_GELU_TANH ? gelu_tanh(v) : v;
+    if (p.mul) {
+        const uint32_t id = p.mul_ids[t];
+        v *= id < p.mul_rows ? bf16_to_f32(p.mul[(size_t)id * p.mul_stride + r]) : 0.0f;
+    }
+    return v;
+}
 
 template <int ACT>
-__device__ __forceinline__ void dense_store(const DenseLinearParams& p, uint32_t t, uint32_t r, float v) {
-    v = dense_act(v, p.activation);
+__device__ __forceinline__ void dense_put(const DenseLinearParams& p, uint32_t t, uint32_t r, float v) {
     if (p.y) static_cast<act_t<ACT>*>(p.y)[(size_t)t * p.y_stride + r] = f32_to_act<ACT>(v);
     if (p.y_f32) p.y_f32[(size_t)t * p.y_stride + r] = v;
 }
 
+template <int ACT>
+__device__ __forceinline__ void dense_store(const DenseLinearParams& p, uint32_t t, uint32_t r, float v) {
+    dense_put<ACT>(p, t, r, dense_finish(p, t, r, v));
+}
+
+// Rows 2 j and 2 j + 1 of the matrix make output j: silu(gate) * up.
+template <int ACT>
+__device__ __forceinline__ void dense_store_pair(const DenseLinearParams& p, uint32_t t, uint32_t j, float gate, float up) {
+    dense_put<ACT>(p, t, j, silu(gate) * up);
+}
+
 // Four neighbouring outputs of one token (r0 a multiple of 4).
 __device__ __forceinline__ void dense_store4_bf16(const DenseLinearParams& p, uint32_t t, uint32_t r0, dn_f4 v) {
-    if (r0 + 4u <= p.n && (p.y_stride & 3u) == 0) {
+    if (p.activation == NVMAI_LINEAR_SILU_PAIRS) {           // n and the row stride are even
+        const float a = silu(v[0]) * v[1], b = silu(v[2]) * v[3];
+        if (r0 + 4u <= p.n) {
+            if (p.y) *reinterpret_cast<uint32_t*>(static_cast<uint16_t*>(p.y) + (size_t)t * p.y_stride + r0 / 2u) = f32_to_bf16(a) | ((uint32_t)f32_to_bf16(b) << 16);
+            if (p.y_f32) *reinterpret_cast<float2*>(p.y_f32 + (size_t)t * p.y_stride + r0 / 2u) = float2{a, b};
+        } else if (r0 < p.n) {
+            dense_put<ACT_BF16>(p, t, r0 / 2u, a);
+        }
+    } else if (r0 + 4u <= p.n && (p.y_stride & 3u) == 0) {
 #pragma unroll
-        for (int j = 0; j < 4; ++j) v[j] = dense_act(v[j], p.activation);
+        for (int j = 0; j < 4; ++j) v[j] = dense_finish(p, t, r0 + j, v[j]);
         if (p.y) {
             uint2 q;
             q.x = f32_to_bf16(v[0]) | ((uint32_t)f32_to_bf16(v[1]) << 16);
@@ -111,6 +141,18 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(DenseLinearParams p) {
 #pragma unroll
                     for (int j = 0; j < 8; ++j) acc[t][r] = fmaf(wf[r][j], xf[j], acc[t][r]);
             }
+        }
+    }
+    if constexpr (RW > 1) {
+        if (p.activation == NVMAI_LINEAR_SILU_PAIRS) {
+#pragma unroll
+            for (int t = 0; t < NT; ++t)
+#pragma unroll
+                for (int r = 0; r < RW; r += 2) {
+                    const float gate = wave_sum_bcast(acc[t][r]), up = wave_sum_bcast(acc[t][r + 1]);
+                    if (lane == (uint32_t)(t * RW + r) && r0 + r < p.n && (uint32_t)t < p.rows) dense_store_pair<ACT>(p, t, (r0 + r) / 2u, gate, up);
+                }
+            return;
         }
     }
 #pragma unroll
@@ -302,139 +344,62 @@ __global__ __launch_bounds__(256) void dense_f32_kernel(DenseLinearParams p) {
 #pragma unroll
         for (int n = 0; n < 4; ++n) {
             const uint32_t t = m0 + ty + 16u * m, r = n0 + tx + 16u * n;
-            if (t < p.rows && r < p.n) dense_store<ACT_FP32>(p, t, r, acc[m][n]);
+            const float next = shfl_xor_f(acc[m][n], 1);         // the neighbouring weight row's sum
+            if (t >= p.rows || r >= p.n) continue;
+            if (p.activation != NVMAI_LINEAR_SILU_PAIRS) dense_store<ACT_FP32>(p, t, r, acc[m][n]);
+            else if ((r & 1u) == 0) dense_store_pair<ACT_FP32>(p, t, r / 2u, acc[m][n], next);
         }
 }
 
-// ---- norms over the 32-bit residual -----------------------------------------------------------------
-// Sum over the 256 threads of a block, every thread gets it.  `lds` holds four floats per call site.
-__device__ __forceinline__ float block_sum256(float v, float* lds) {
-    v = wave_sum_bcast(v);
-    if ((threadIdx.x & 63u) == 0) lds[threadIdx.x >> 6] = v;
-    __syncthreads();
-    return (lds[0] + lds[1]) + (lds[2] + lds[3]);
-}
-
-// (v - mean) / sqrt(mean((v - mean)^2) + eps) over the row's d elements, dead slots zero before and after.
-// Thread t holds the elements 4 (t + 256 j) .. + 3.
-template <int VPT>
-__device__ __forceinline__ void block_layernorm(float (&v)[VPT][4], uint32_t d, float eps, float* lds) {
-    float s = 0.0f;
-#pragma unroll
-    for (int j = 0; j < VPT; ++j) s += (v[j][0] + v[j][1]) + (v[j][2] + v[j][3]);
-    const float mean = block_sum256(s, lds) / (float)d;
-    float q = 0.0f;
-#pragma unroll
-    for (int j = 0; j < VPT; ++j)
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            v[j][e] = 4u * (threadIdx.x + 256u * j) + e < d ? v[j][e] - mean : 0.0f;
-            q = fmaf(v[j][e], v[j][e], q);
-        }
-    const float inv = 1.0f / sqrtf(block_sum256(q, lds + 4) / (float)d + eps);
-#pragma unroll
-    for (int j = 0; j < VPT; ++j)
-#pragma unroll
-        for (int e = 0; e < 4; ++e) v[j][e] *= inv;
-}
-
-struct NormResidualParams {
-    float* x;                        // [rows, x_stride] residual stream
-    const float* delta;              // sublayer output
-    const uint16_t *post_w, *post_b; // norm of delta
-    const uint16_t *next_w, *next_b; // norm that opens the next sublayer
-    void* out;
-    uint32_t x_stride, delta_stride, out_stride, d;
-    float mult, eps;
+// ---- the two ends of a model ----------------------------------------------------------------------
+// Rows of a BF16 table as 32-bit residual rows; an id past the table gives zeros.  scale: factor of the table's rows;
+// inv_freq (nullptr: none): plus the sinusoid of the row's position, entry 2 i its sine and 2 i + 1 its cosine at
+// inv_freq[i]; act (nullptr: none): the row once more as activations.
+struct EmbedParams {
+    const uint16_t* table;
+    const uint32_t* ids;
+    float* out;
+    void* act;
+    const double* inv_freq;
+    SeqRows rows;
+    uint32_t table_stride, out_stride, act_stride, d, vocab;
+    float scale;
 };
 
-__device__ __forceinline__ void norm_bf4(const uint16_t* p, float* v) {
-    const uint2 q = *reinterpret_cast<const uint2*>(p);
-    act2_to_f32<ACT_BF16>(q.x, v[0], v[1]);
-    act2_to_f32<ACT_BF16>(q.y, v[2], v[3]);
-}
-
-// x += mult * LN(delta) (POST; DELTA: x += mult * delta); out = LN(x) (NEXT): one block per row, the row in registers.
-// Every operand is requested before the first sum.  VEC: four elements per load (d and the strides are multiples
-// of 4); dead slots reread the row's last elements.
-template <int ACT, int VPT, bool DELTA, bool POST, bool NEXT, bool VEC>
-__global__ __launch_bounds__(256) void norm_residual_kernel(NormResidualParams p) {
-    __shared__ float lds[16];
-    const uint32_t row = blockIdx.x, tid = threadIdx.x;
-    float* x = p.x + (size_t)row * p.x_stride;
-    const float* delta = p.delta + (size_t)row * p.delta_stride;
-    float xv[VPT][4], dv[VPT][4], pw[VPT][4], pb[VPT][4], nw[VPT][4], nb[VPT][4];
-#pragma unroll
-    for (int j = 0; j < VPT; ++j) {
-        const uint32_t at = 4u * (tid + 256u * j);
-        if (VEC) {
-            const uint32_t c = min(at, p.d - 4u);
-            *reinterpret_cast<dn_f4*>(xv[j]) = *reinterpret_cast<const dn_f4*>(x + c);
-            if (DELTA) *reinterpret_cast<dn_f4*>(dv[j]) = *reinterpret_cast<const dn_f4*>(delta + c);
-            if (POST) { norm_bf4(p.post_w + c, pw[j]); norm_bf4(p.post_b + c, pb[j]); }
-            if (NEXT) { norm_bf4(p.next_w + c, nw[j]); norm_bf4(p.next_b + c, nb[j]); }
-        } else {
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const uint32_t c = min(at + e, p.d - 1u);
-                xv[j][e] = x[c];
-                if (DELTA) dv[j][e] = delta[c];
-                if (POST) { pw[j][e] = bf16_to_f32(p.post_w[c]); pb[j][e] = bf16_to_f32(p.post_b[c]); }
-                if (NEXT) { nw[j][e] = bf16_to_f32(p.next_w[c]); nb[j][e] = bf16_to_f32(p.next_b[c]); }
-            }
-        }
-#pragma unroll
-        for (int e = 0; e < 4; ++e)
-            if (at + e >= p.d) { xv[j][e] = 0.0f; if (DELTA) dv[j][e] = 0.0f; }
+template <int ACT>
+__global__ __launch_bounds__(256) void embed_rows_kernel(EmbedParams p) {
+    const uint32_t row = blockIdx.y, pair = blockIdx.x * 256u + threadIdx.x, j = 2u * pair;
+    if (j >= p.d) return;
+    const uint32_t id = p.ids[row];
+    const bool two = j + 1u < p.d;
+    const uint16_t* e = p.table + (size_t)id * p.table_stride + j;
+    float a = 0.0f, b = 0.0f;
+    if (id < p.vocab) {
+        a = bf16_to_f32(e[0]) * p.scale;
+        b = two ? bf16_to_f32(e[1]) * p.scale : 0.0f;
     }
-    if (DELTA) {
-        if (POST) block_layernorm<VPT>(dv, p.d, p.eps, lds);
-#pragma unroll
-        for (int j = 0; j < VPT; ++j) {
-            const uint32_t at = 4u * (tid + 256u * j);
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const float add = POST ? fmaf(dv[j][e], pw[j][e], pb[j][e]) : dv[j][e];
-                xv[j][e] = at + e < p.d ? fmaf(p.mult, add, xv[j][e]) : 0.0f;
-            }
-            if (VEC) {
-                if (at < p.d) *reinterpret_cast<dn_f4*>(x + at) = *reinterpret_cast<dn_f4*>(xv[j]);
-            } else {
-#pragma unroll
-                for (int e = 0; e < 4; ++e)
-                    if (at + e < p.d) x[at + e] = xv[j][e];
-            }
-        }
+    if (p.inv_freq) {
+        float c, s;
+        position_angle(p.rows.position_of(row), p.inv_freq[pair], c, s);
+        a += s;
+        b += c;
     }
-    if (!NEXT) return;
-    block_layernorm<VPT>(xv, p.d, p.eps, lds + 8);
-    act_t<ACT>* out = static_cast<act_t<ACT>*>(p.out) + (size_t)row * p.out_stride;
-#pragma unroll
-    for (int j = 0; j < VPT; ++j) {
-        const uint32_t at = 4u * (tid + 256u * j);
-        act_t<ACT> o[4];
-#pragma unroll
-        for (int e = 0; e < 4; ++e) o[e] = f32_to_act<ACT>(fmaf(xv[j][e], nw[j][e], nb[j][e]));
-        if (VEC) {
-            if (at < p.d) {
-                if constexpr (ACT == ACT_FP32) *reinterpret_cast<dn_f4*>(out + at) = dn_f4{o[0], o[1], o[2], o[3]};
-                else *reinterpret_cast<uint2*>(out + at) = make_uint2(o[0] | ((uint32_t)o[1] << 16), o[2] | ((uint32_t)o[3] << 16));
-            }
-        } else {
-#pragma unroll
-            for (int e = 0; e < 4; ++e)
-                if (at + e < p.d) out[at + e] = o[e];
-        }
+    float* out = p.out + (size_t)row * p.out_stride + j;
+    out[0] = a;
+    if (two) out[1] = b;
+    if (p.act) {
+        act_t<ACT>* h = static_cast<act_t<ACT>*>(p.act) + (size_t)row * p.act_stride + j;
+        h[0] = f32_to_act<ACT>(a);
+        if (two) h[1] = f32_to_act<ACT>(b);
     }
 }
 
-// Rows of a BF16 table as 32-bit residual rows; an id past the table gives zeros.
-__global__ __launch_bounds__(256) void embed_rows_kernel(const uint16_t* table, uint32_t table_stride, const uint32_t* ids,
-                                                        float* out, uint32_t out_stride, uint32_t d, uint32_t vocab) {
-    const uint32_t row = blockIdx.y, j = blockIdx.x * 256u + threadIdx.x;
-    if (j >= d) return;
-    const uint32_t id = ids[row];
-    out[(size_t)row * out_stride + j] = id < vocab ? bf16_to_f32(table[(size_t)id * table_stride + j]) : 0.0f;
+// x <- cap tanh(x / cap)
+__global__ __launch_bounds__(256) void softcap_rows_kernel(float* x, uint32_t x_stride, uint32_t n, float cap) {
+    const uint32_t j = blockIdx.x * 256u + threadIdx.x;
+    if (j >= n) return;
+    float* v = x + (size_t)blockIdx.y * x_stride + j;
+    *v = cap * tanhf(*v / cap);
 }
 
 // Index of the largest finite value of each row, ties to the lower index, 0 when none is finite.  A candidate is one

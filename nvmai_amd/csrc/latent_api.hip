@@ -20,7 +20,7 @@ int check_config(const nvmai_hip_ctx* ctx, const nvmai_latent_config* c, const n
     return NVMAI_OK;
 }
 
-LatentRows rows_of(const nvmai_row_map* m) { return LatentRows{m->slots, m->positions, m->slot, m->position}; }
+SeqRows rows_of(const nvmai_row_map* m) { return SeqRows{m->slots, m->positions, m->slot, m->position}; }
 LatentCache cache_of(const nvmai_latent_cache* c) { return LatentCache{c->base, c->slot_stride, c->row_stride, c->capacity}; }
 
 int raise_lds(const void* kernel, size_t bytes) {

@@ -11,7 +11,7 @@
 //   * expanded, for prompts: keys and values of the range are formed by two matrix products, then flash attention.
 #pragma once
 
-#include "common.hpp"
+#include "rows.hpp"
 
 namespace nvmai {
 
@@ -32,26 +32,11 @@ __device__ __forceinline__ uint32_t la_pack2(float lo, float hi) {
 constexpr float LA_LOG2E = 1.4426950408889634f;
 constexpr float LA_NONE = -1e30f;        // maximum of no scores
 
-// Where a row's token sits: by arrays (a decode batch) or consecutive from (slot, position) (a prompt's portion).
-struct LatentRows {
-    const uint32_t *slots, *positions;
-    uint32_t slot, position;
-    __device__ __forceinline__ uint32_t slot_of(uint32_t r) const { return slots ? slots[r] : slot; }
-    __device__ __forceinline__ uint32_t position_of(uint32_t r) const { return positions ? positions[r] : position + r; }
-};
-
 struct LatentCache {
     void* base;
     uint64_t slot_stride;    // elements
     uint32_t row_stride, capacity;
 };
-
-// (cos, sin) of position * inv_freq with the angle reduced in double: exact to fp32 at any position.
-__device__ __forceinline__ void la_rotation(uint32_t position, double inv_freq, float& c, float& s) {
-    double a = (double)position * inv_freq;
-    a -= 6.283185307179586476925 * rint(a * 0.15915494309189533577);
-    sincosf((float)a, &s, &c);
-}
 
 __device__ __forceinline__ float la_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 
@@ -61,7 +46,7 @@ struct LatentEpilogueParams {
     const uint16_t *q_norm, *kv_norm;    // readable up to the counts rounded up to 8
     const double* inv_freq;              // [rot_dims / 2]
     void* cq;                            // [rows, cq_stride]
-    LatentRows rows;
+    SeqRows rows;
     LatentCache cache;
     uint32_t proj_stride, q_at, kv_at, rot_at, cq_stride, q_count, rank_count, rank, rot_dim, rot_dims;
     float eps;
@@ -123,7 +108,7 @@ __global__ __launch_bounds__(256) void latent_epilogue_kernel(LatentEpiloguePara
     for (uint32_t j = 255u - tid; j < p.rot_dim; j += 256u) {
         if (j < half) {
             float c, s;
-            la_rotation(position, p.inv_freq[j], c, s);
+            position_angle(position, p.inv_freq[j], c, s);
             const float a = act_to_f32<ACT>(proj[p.rot_at + j]), b = act_to_f32<ACT>(proj[p.rot_at + half + j]);
             out[p.rank + j] = f32_to_act<CT>(a * c - b * s);
             out[p.rank + half + j] = f32_to_act<CT>(b * c + a * s);
@@ -169,7 +154,7 @@ struct LatentAttnParams {
     const void* gate;                    // [rows, gate_stride]: one logit per head, nullptr = no gate
     const uint16_t *uk, *uv;             // [heads * nope, rank], [heads * vdim, rank] BF16
     const double* inv_freq;
-    LatentRows rows;
+    SeqRows rows;
     LatentCache cache;
     void* out;                           // [rows, out_stride]: head by head [vdim]
     uint32_t q_stride, gate_stride, out_stride, n_rows, heads, nope, rot, vdim, rank, rot_dims, window;
@@ -183,10 +168,6 @@ struct LatentAttnParams {
     uint32_t nk, nk_pad, key0;           // keys of the call, the position of the first
     uint32_t kn_stride, v_stride;
 };
-
-__device__ __forceinline__ uint32_t la_first_key(uint32_t position, uint32_t window) {
-    return window != 0u && position + 1u > window ? position + 1u - window : 0u;
-}
 
 // ---- absorbed: q_n -> W_uk(h)^T q_n, q_r rotated ----------------------------------------------------
 // A block per (head, row, 128 latent dims): sixteen lanes cover the latents in pieces of eight, sixteen groups of
@@ -204,7 +185,7 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentAttnParams p) 
         for (uint32_t j = tid; j < p.cache.row_stride - p.rank; j += 256u) {
             if (j < half) {
                 float c, s;
-                la_rotation(position, p.inv_freq[j], c, s);
+                position_angle(position, p.inv_freq[j], c, s);
                 const float u = act_to_f32<ACT>(q[p.nope + j]), v = act_to_f32<ACT>(q[p.nope + half + j]);
                 out[p.rank + j] = f32_to_act<CT>(u * c - v * s);
                 out[p.rank + half + j] = f32_to_act<CT>(v * c + u * s);
@@ -265,7 +246,7 @@ __global__ __launch_bounds__(256) void latent_partial_mfma_kernel(LatentAttnPara
     __shared__ __attribute__((aligned(16))) float sc[4][16][36];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, i = lane & 15u, g = lane >> 4;
     const uint32_t split = blockIdx.x, h0 = blockIdx.y * 16u, row = blockIdx.z;
-    const uint32_t position = p.rows.position_of(row), first = la_first_key(position, p.window);
+    const uint32_t position = p.rows.position_of(row), first = first_key(position, p.window);
     const uint32_t lo = first + split * p.split_keys, hi = min(position + 1u, lo + p.split_keys);
     const uint32_t head = min(h0 + i, p.heads - 1u);
     const size_t cell = ((size_t)row * p.heads + head) * p.splits + split;
@@ -427,7 +408,7 @@ __global__ __launch_bounds__(256) void latent_partial_plain_kernel(LatentAttnPar
     extern __shared__ __attribute__((aligned(16))) float la_lds[];
     const uint32_t tid = threadIdx.x, split = blockIdx.x, head = blockIdx.y, row = blockIdx.z, rs = p.cache.row_stride;
     float *qs = la_lds, *acc = qs + rs, *ps = acc + p.rank, *red = ps + 256;
-    const uint32_t position = p.rows.position_of(row), first = la_first_key(position, p.window);
+    const uint32_t position = p.rows.position_of(row), first = first_key(position, p.window);
     const uint32_t lo = first + split * p.split_keys, hi = min(position + 1u, lo + p.split_keys);
     const size_t cell = ((size_t)row * p.heads + head) * p.splits + split;
     if (lo >= hi) {
@@ -464,7 +445,7 @@ __global__ __launch_bounds__(1024) void latent_combine_kernel(LatentAttnParams p
     const float gate = p.gate ? la_sigmoid(act_to_f32<ACT>(static_cast<const act_t<ACT>*>(p.gate)[(size_t)row * p.gate_stride + head])) : 1.0f;
     // splits past the last key of this row wrote no sums and weigh nothing: the live ones are a prefix
     const uint32_t position = p.rows.position_of(row);
-    const uint32_t live = min(p.splits, (position + 1u - la_first_key(position, p.window) + p.split_keys - 1u) / p.split_keys);
+    const uint32_t live = min(p.splits, (position + 1u - first_key(position, p.window) + p.split_keys - 1u) / p.split_keys);
     const uint32_t group = tid >> 7, r0 = min((tid & 127u) * 4u, p.rank - 4u);
     const float* po = p.part_o + cell * p.rank;
     la_f4 ahead[8];                      // this group's first eight splits, requested before their weights are known
@@ -549,7 +530,7 @@ template <int ACT>
 __global__ __launch_bounds__(256) void latent_rotate_q_kernel(LatentAttnParams p) {
     const uint32_t row = blockIdx.x, half = p.rot_dims / 2u, position = p.rows.position + row;
     extern __shared__ __attribute__((aligned(16))) float la_lds[];      // [half] cos, [half] sin
-    for (uint32_t j = threadIdx.x; j < half; j += 256u) la_rotation(position, p.inv_freq[j], la_lds[j], la_lds[half + j]);
+    for (uint32_t j = threadIdx.x; j < half; j += 256u) position_angle(position, p.inv_freq[j], la_lds[j], la_lds[half + j]);
     __syncthreads();
     act_t<ACT>* q = static_cast<act_t<ACT>*>(const_cast<void*>(p.q)) + (size_t)row * p.q_stride;
     for (uint32_t e = threadIdx.x; e < p.heads * half; e += 256u) {
@@ -569,7 +550,7 @@ __global__ __launch_bounds__(256) void latent_expanded_plain_kernel(LatentAttnPa
     const act_t<ACT>* q = static_cast<const act_t<ACT>*>(p.q) + (size_t)row * p.q_stride + head * dq;
     for (uint32_t j = tid; j < dq; j += 256u) qs[j] = act_to_f32<ACT>(q[j]);
     __syncthreads();
-    const uint32_t position = p.rows.position + row, lo = la_first_key(position, p.window) - p.key0, hi = position + 1u - p.key0;
+    const uint32_t position = p.rows.position + row, lo = first_key(position, p.window) - p.key0, hi = position + 1u - p.key0;
     const act_t<ACT>*kn = static_cast<const act_t<ACT>*>(p.kn), *lat = static_cast<const act_t<ACT>*>(p.lat), *v = static_cast<const act_t<ACT>*>(p.v);
     float m, l;
     la_plain_rows(lo, hi, p.vdim, p.scale_log2, acc, ps, red, m, l,
@@ -638,7 +619,7 @@ __global__ __launch_bounds__(256, NP + RP + DV <= 320 ? 2 : 1) void latent_flash
         for (int n = 0; n < NV; ++n) acc[b][n] = la_f4{0.0f, 0.0f, 0.0f, 0.0f};
     // keys are numbered from key0
     const uint32_t last_t = min(q0 + 127u, p.n_rows - 1u);
-    const uint32_t k_lo = (la_first_key(p.rows.position + q0, p.window) - p.key0) & ~63u;
+    const uint32_t k_lo = (first_key(p.rows.position + q0, p.window) - p.key0) & ~63u;
     const uint32_t k_hi = p.rows.position + last_t + 1u - p.key0;
     const uint32_t kn_bytes = p.kn_stride * 2u, lat_bytes = p.cache.row_stride * 2u, v_bytes = p.v_stride * 2u;
     [[maybe_unused]] const __amdgpu_buffer_rsrc_t nrs = __builtin_amdgcn_make_buffer_rsrc(p.kn, 0, (int)(p.nk_pad * kn_bytes), 0x00020000);
@@ -676,8 +657,8 @@ __global__ __launch_bounds__(256, NP + RP + DV <= 320 ? 2 : 1) void latent_flash
     // this wave's own range of keys, and the part of it that every one of its queries sees
     const uint32_t wt0 = q0 + wave * 32u, wt1 = min(wt0 + 31u, p.n_rows - 1u);
     const bool wave_live = wt0 < p.n_rows;
-    const uint32_t w_lo = la_first_key(p.rows.position + wt0, p.window) - p.key0, w_hi = p.rows.position + wt1 + 1u - p.key0;
-    const uint32_t full_lo = la_first_key(p.rows.position + wt1, p.window) - p.key0, full_hi = p.rows.position + wt0 + 1u - p.key0;
+    const uint32_t w_lo = first_key(p.rows.position + wt0, p.window) - p.key0, w_hi = p.rows.position + wt1 + 1u - p.key0;
+    const uint32_t full_lo = first_key(p.rows.position + wt1, p.window) - p.key0, full_hi = p.rows.position + wt0 + 1u - p.key0;
     const uint32_t krow = 8u * (i >> 2) + (i & 3u);              // key of this lane's row in an even score tile
     issue(k_lo, lds);
     uint32_t stage = 0;
@@ -713,7 +694,7 @@ __global__ __launch_bounds__(256, NP + RP + DV <= 320 ? 2 : 1) void latent_flash
             for (int t = 0; t < 4; ++t) s[b][t] *= p.scale_log2;
             if (masked) {
                 const uint32_t pos = p.rows.position + min(wt0 + 16u * b + i, p.n_rows - 1u);
-                const uint32_t lo = la_first_key(pos, p.window) - p.key0, hi = pos + 1u - p.key0;
+                const uint32_t lo = first_key(pos, p.window) - p.key0, hi = pos + 1u - p.key0;
 #pragma unroll
                 for (int t = 0; t < 4; ++t)
 #pragma unroll

@@ -324,6 +324,13 @@ class StepDecoder:
         rows = [self._prefill_chunk_rows(one(t), b, p).clone() for b, p, t in zip(sequences, positions, tokens)]
         return torch.cat(rows)
 
+    def logits_rows(self, normed):
+        """32-bit logits of final-normed rows, capped where the model caps them (head_rows and the samplers' inputs are
+        not: the samplers cap them on the way)."""
+        y, y32 = self.head_rows(normed)
+        y32 = y32 if y32 is not None else y.float()
+        return ops.softcap_rows(self.ctx, y32, self.cfg.logit_softcap) if self.cfg.logit_softcap > 0.0 else y32
+
     # -- the end of a step -----------------------------------------------------------------------------
     def sample(self, seeds, temperature=0.6, top_k=20, top_p=0.95):
         """Softcap + softmax and the tiled top-k sampler (Sampler.sample's production path): tokens in

@@ -62,8 +62,7 @@ class Session:
 
     def logits(self, rows):
         """32-bit logits of final-normed rows."""
-        y, y32 = self.decoder.head_rows(rows)
-        return y32 if y32 is not None else y.float()
+        return self.decoder.logits_rows(rows)
 
 
 class Generator:

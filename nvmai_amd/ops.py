@@ -7,8 +7,9 @@ import ctypes as C
 import torch
 
 from . import _lib
-from ._lib import (ExpertOffsets, GdnConfig, GemvPart, GenerationConfig as _CGenerationConfig, GlaConfig, KvView,
-                   LatentCacheView, LatentConfig, MoeLayer, PrefillGrouping, RowMap, Rows, check, lib)
+from ._lib import (ExpertOffsets, GdnConfig, GemvPart, GenerationConfig as _CGenerationConfig, GlaConfig, KvRingView, KvView,
+                   LatentCacheView, LatentConfig, LinearEpilogue, MoeLayer, PrefillGrouping, RowMap, Rows, ScanConfig, WindowConfig,
+                   check, lib)
 
 ACT_BF16, ACT_FP16, ACT_FP32 = 0, 1, 2
 (PROF_ROUTER, PROF_SELECT, PROF_GROUP, PROF_PHASE1, PROF_PHASE2, PROF_COMBINE, PROF_KV_QUANT,
@@ -1089,18 +1090,26 @@ class Elementwise:
 FORM_AUTO = 0
 GLA_RECURRENT, GLA_CHUNKED = 1, 2
 LATENT_ABSORBED, LATENT_EXPANDED = 1, 2
-LINEAR_NONE, LINEAR_GELU_ERF = 0, 1
+WINDOW_SPLIT, WINDOW_FLASH, WINDOW_PLAIN = 1, 2, 3
+SCAN_RECURRENT, SCAN_CHUNKED = 1, 2
+SCAN_DELTA, SCAN_SSD = 0, 1
+LINEAR_NONE, LINEAR_GELU_ERF, LINEAR_GELU_TANH, LINEAR_SILU_PAIRS = range(4)
 
 
-def dense_linear(ctx, weight, x, y=None, y_f32=None, n=None, activation=LINEAR_NONE):
-    """y[t] = act(W x[t]): weight [n, k] BF16 (k a multiple of 64), x [tokens, >= k] activations; y (activations) and /
-    or y_f32 are buffers [tokens, >= n] with one row stride."""
+def dense_linear(ctx, weight, x, y=None, y_f32=None, n=None, activation=LINEAR_NONE, bias=None, mul=None, mul_ids=None):
+    """y[t] = act(W x[t] + bias) * mul[mul_ids[t]]: weight [n, k] BF16 (k a multiple of 64), x [tokens, >= k] activations; y
+    (activations) and / or y_f32 are buffers [tokens, >= n] with one row stride.  bias: BF16 [n]; mul: BF16 columns [.., n]
+    of a table.  LINEAR_SILU_PAIRS: y[t, j] = silu(row 2 j) * (row 2 j + 1)."""
     rows, k = weight.shape
     out = y if y is not None else y_f32
     assert y is None or y_f32 is None or y.stride(0) == y_f32.stride(0)
-    check(lib.nvmai_hip_dense_linear(ctx.handle, _stream(), _ptr(weight), weight.stride(0), _ptr(x), x.stride(0), x.shape[0],
-                                     rows if n is None else n, k, _ptr(y), _ptr(y_f32), out.stride(0), activation),
-          "dense_linear")
+    args = (ctx.handle, _stream(), _ptr(weight), weight.stride(0), _ptr(x), x.stride(0), x.shape[0], rows if n is None else n, k, _ptr(y),
+            _ptr(y_f32), out.stride(0))
+    if bias is None and mul is None:
+        check(lib.nvmai_hip_dense_linear(*args, activation), "dense_linear")
+    else:
+        e = LinearEpilogue(activation, _ptr(bias), _ptr(mul), _ptr(mul_ids), 0 if mul is None else mul.stride(0), 0 if mul is None else mul.shape[0])
+        check(lib.nvmai_hip_dense_linear_ex(*args, C.byref(e)), "dense_linear_ex")
     return out
 
 
@@ -1115,11 +1124,41 @@ def norm_residual(ctx, x, d, delta=None, post=None, mult=1.0, next_norm=None, ou
     return out
 
 
+def rms_residual(ctx, x, d, delta=None, post=None, post_add=0.0, next_norm=None, next_add=0.0, out=None, eps=1e-6):
+    """x += RMS(delta) * (post_add + post), then out = RMS(x) * (next_add + next_norm), or x as activations where
+    next_norm is None."""
+    check(lib.nvmai_hip_rms_residual(ctx.handle, _stream(), _ptr(x), x.stride(0), _ptr(delta), 0 if delta is None else delta.stride(0),
+                                     _ptr(post), post_add, _ptr(next_norm), next_add, _ptr(out), 0 if out is None else out.stride(0),
+                                     x.shape[0], d, eps), "rms_residual")
+    return out
+
+
 def embed_rows(ctx, table, token_ids, d, vocab, out):
     """Rows of a BF16 table as 32-bit residual rows."""
     check(lib.nvmai_hip_embed_rows(ctx.handle, _stream(), _ptr(table), table.stride(0), _ptr(token_ids), token_ids.numel(),
                                    _ptr(out), out.stride(0), d, vocab), "embed_rows")
     return out
+
+
+def sinusoid_frequencies(width, device, base=10000.0):
+    """base^(-2i / width), in double: the kernels reduce position * frequency in double."""
+    i = torch.arange((width + 1) // 2, dtype=torch.float64)
+    return (float(base) ** (-2.0 * i / width)).to(device)
+
+
+def embed_positions(ctx, table, token_ids, d, vocab, scale, inv_freq, rows_at, out, act=None):
+    """Rows of a BF16 table times `scale`, plus the sinusoids of their positions (inv_freq None: none), as 32-bit residual
+    rows, and as activations in `act`."""
+    check(lib.nvmai_hip_embed_positions(ctx.handle, _stream(), _ptr(table), table.stride(0), _ptr(token_ids), token_ids.numel(), scale,
+                                        _ptr(inv_freq), C.byref(rows_at), _ptr(out), out.stride(0), _ptr(act),
+                                        0 if act is None else act.stride(0), d, vocab), "embed_positions")
+    return out
+
+
+def softcap_rows(ctx, x, cap):
+    """cap * tanh(x / cap) over 32-bit rows, in place."""
+    check(lib.nvmai_hip_softcap_rows(ctx.handle, _stream(), _ptr(x), x.stride(0), x.shape[0], x.shape[1], cap), "softcap_rows")
+    return x
 
 
 def argmax_rows(ctx, logits, out=None):
@@ -1131,10 +1170,11 @@ def argmax_rows(ctx, logits, out=None):
     return out
 
 
-def row_map(slot=0, position=0, slots=None, positions=None):
-    """Rows position, position + 1, ... of one slot, or (int32 device arrays) one slot and position per row."""
+def row_map(slot=0, position=0, slots=None, positions=None, most=None):
+    """Rows position, position + 1, ... of one slot, or (int32 device arrays) one slot and position per row, none of the
+    positions past `most`."""
     m = RowMap(None if slots is None else slots.data_ptr(), None if positions is None else positions.data_ptr(), slot, position)
-    m._keep = (slots, positions)
+    m._keep, m.most = (slots, positions), most
     return m
 
 
@@ -1194,3 +1234,67 @@ class LatentAttention:
                                              0 if gate is None else gate.stride(0), _ptr(uk), _ptr(uv), C.byref(cache.view),
                                              C.byref(rows_at), _ptr(out), out.stride(0), q.shape[0], form), "latent_attention")
         return out
+
+
+class KvRing:
+    """Normed keys and transposed values of one layer (nvmai_kv_ring): per slot a ring of `window` positions or more behind
+    `keep` pinned ones.  The counterpart of KVCache for windowed attention; several layers may share one."""
+
+    def __init__(self, ctx, slots, kv_heads, key_dim, value_dim, capacity, keep=0):
+        up64 = lambda n: (n + 63) // 64 * 64
+        self.pinned, self.ring = up64(keep), up64(max(1, capacity))
+        rows = self.pinned + self.ring
+        self.k = torch.zeros((slots, kv_heads, rows, key_dim), dtype=ctx.dtype, device=ctx.device)
+        self.v = torch.zeros((slots, kv_heads, value_dim, rows), dtype=ctx.dtype, device=ctx.device)
+        self.view = KvRingView(self.k.data_ptr(), self.v.data_ptr(), kv_heads, key_dim, value_dim, self.pinned, self.ring, ctx.act)
+
+
+class WindowAttention:
+    """Windowed grouped-query attention (nvmai_hip_window_epilogue, nvmai_hip_window_attention): per-head RMS norms of
+    queries and keys, a sliding window (0: every earlier position) beside the first `keep` positions, a cap of the scores
+    (0: none), linear distance biases."""
+
+    def __init__(self, ctx, heads, key_count, scale, window, eps, keep=0, softcap=0.0, alibi=False):
+        self.ctx, self.cfg = ctx, WindowConfig(heads, key_count, window, keep, scale, softcap, eps, int(alibi))
+
+    def encode_epilogue(self, proj, q_at, k_at, v_at, q_norm, k_norm, q, cache, rows_at):
+        """k_norm None: the cache is another layer's and holds the rows' keys and values already."""
+        check(lib.nvmai_hip_window_epilogue(self.ctx.handle, _stream(), C.byref(self.cfg), _ptr(proj), proj.stride(0), q_at, k_at, v_at,
+                                            _ptr(q_norm), _ptr(k_norm), _ptr(q), q.stride(0), C.byref(cache.view), C.byref(rows_at),
+                                            proj.shape[0]), "window_epilogue")
+        return q
+
+    def encode(self, q, cache, rows_at, out, gate=None, out_scale=1.0, form=FORM_AUTO):
+        check(lib.nvmai_hip_window_attention(self.ctx.handle, _stream(), C.byref(self.cfg), _ptr(q), q.stride(0), _ptr(gate),
+                                             0 if gate is None else gate.stride(0), C.byref(cache.view), C.byref(rows_at),
+                                             rows_at.most or 0, out_scale, _ptr(out), out.stride(0), q.shape[0], form), "window_attention")
+        return out
+
+
+class HeadScan:
+    """A recurrence with one decay per head behind a short causal filter (nvmai_hip_scan): the gated delta rule or the
+    state-space form.  Channels of the projected rows from conv_at: q | k | v."""
+    AHEAD = 32
+
+    def __init__(self, ctx, kind, heads, key_heads, key_dim, value_dim, taps, conv_at, a_at, b_at=0, q_scale=1.0):
+        self.ctx, self.channels = ctx, 2 * key_heads * key_dim + heads * value_dim
+        self.cfg = ScanConfig(kind, heads, key_heads, key_dim, value_dim, taps, taps - 1 + self.AHEAD, conv_at, a_at, b_at, q_scale)
+
+    def new_state(self, slots):
+        """(filter inputs by position, recurrent state) of every slot; a new sequence needs the second one zeroed."""
+        c, f32 = self.cfg, dict(dtype=torch.float32, device=self.ctx.device)
+        return torch.zeros((slots, c.history_rows, self.channels), **f32), torch.zeros((slots, c.heads, c.key_dim, c.value_dim), **f32)
+
+    def encode(self, proj, conv, conv_bias, a_log, dt_bias, skip, history, state, rows_at, out, form=FORM_AUTO):
+        check(lib.nvmai_hip_scan(self.ctx.handle, _stream(), C.byref(self.cfg), _ptr(proj), proj.stride(0), _ptr(conv), _ptr(conv_bias),
+                                 _ptr(a_log), _ptr(dt_bias), _ptr(skip), _ptr(history), _ptr(state), C.byref(rows_at), _ptr(out),
+                                 out.stride(0), proj.shape[0], form), "scan")
+        return out
+
+
+def gated_norm(ctx, x, gate, weight, out, heads, value_dim, value_count, parts, gate_first, eps, out_scale=1.0):
+    """RMS norm over `parts` equal parts of the heads' real columns, with a SiLU gate before (gate_first) or after it."""
+    check(lib.nvmai_hip_gated_norm(ctx.handle, _stream(), _ptr(x), x.stride(0), _ptr(gate), gate.stride(0), _ptr(weight), _ptr(out),
+                                   out.stride(0), x.shape[0], heads, value_dim, value_count, parts, int(gate_first), out_scale, eps),
+          "gated_norm")
+    return out

@@ -1,6 +1,6 @@
 """Pakirax: a decoder-only language model of gated-linear-attention and windowed latent-attention layers, with a norm
-before and after every sublayer.  Configuration, weights and step driver; the session, sampling and prompt loop are
-StepDecoder's and generate.py's.
+before and after every sublayer.  Configuration, weights and step driver; what its step driver shares with the other
+dense models is in dense_model.py.
 
 A layer is  x <- x + m norm1b(mixer(norm1 x))  and, when it has a feed-forward,  x <- x + m norm2b(ff(norm2 x));  the
 residual x is 32-bit, the norms are layer norms with weight and bias, the logits are the embedding table times the
@@ -10,36 +10,19 @@ Weights are laid out for one launch per projection group (q, k, v, gate and the 
 down projections and the output gate of a latent-attention layer are rows of one matrix each) and padded with zeros so
 that the kernels see multiples of 16 (heads) and 64 (the k of a product); real counts go with them where a norm needs
 them."""
-import json
-import os
-
 import torch
 
 from . import ops
-from .decoder import StepDecoder
+from .dense_model import DenseDecoder, bf16_reader, blocks_of, check_shapes, need, open_directory, pad_columns, up
 from .gturbo import ModelError
-from .safetensors_file import SafetensorsFile
-
-FEW_ROWS = 2        # passes whose products read 32-bit inputs at the price of 16-bit ones (dense_linear: bound by the weights)
-
-
-def _up(n, m):
-    return (n + m - 1) // m * m
-
-
-def _need(d, where, *names):
-    for n in names:
-        if n not in d:
-            raise ModelError("indexCorrupt", "config.json: %s has no %s" % (where, n))
-    return [d[n] for n in names]
 
 
 class GlaLayer:
     kind = "gla"
 
     def __init__(self, m, where):
-        self.heads, self.dim, self.vdim, self.tau = _need(m, where, "heads", "dim", "vdim", "tau")
-        self.dim_p, self.vdim_p = _up(self.dim, 16), _up(self.vdim, 16)
+        self.heads, self.dim, self.vdim, self.tau = need(m, where, "heads", "dim", "vdim", "tau")
+        self.dim_p, self.vdim_p = up(self.dim, 16), up(self.vdim, 16)
 
     def shapes(self, width, rank):
         kd, vd = self.heads * self.dim, self.heads * self.vdim
@@ -52,13 +35,13 @@ class LatentLayer:
 
     def __init__(self, m, where):
         (self.heads, self.dim, self.rot_dim, self.vdim, self.kv_rank, self.q_rank, self.scale) = \
-            _need(m, where, "heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank", "scale")
+            need(m, where, "heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank", "scale")
         rot, mask = m.get("rot"), m.get("mask")
         self.rot_base, self.rot_dims = (float(rot["base"]), int(rot["dims"])) if rot else (1.0, 0)
         self.window = int(mask["size"]) if mask else 0
         if self.rot_dims > self.rot_dim or self.rot_dims % 2 or (mask and self.window < 1):
             raise ModelError("indexCorrupt", "config.json: %s: rot or mask out of range" % where)
-        self.dim_p, self.rot_p, self.vdim_p, self.rank_p = _up(self.dim, 16), _up(self.rot_dim, 16), _up(self.vdim, 16), _up(self.kv_rank, 64)
+        self.dim_p, self.rot_p, self.vdim_p, self.rank_p = up(self.dim, 16), up(self.rot_dim, 16), up(self.vdim, 16), up(self.kv_rank, 64)
 
     def shapes(self, width, rank):
         H = self.heads
@@ -75,19 +58,19 @@ class PakiraxConfig:
 
     def __init__(self, config):
         self.vocab, self.width, self.residual_mult, norm, layers = \
-            _need(config, "the model", "vocab", "width", "residual_mult", "norm", "layers")
-        self.eps, = _need(norm, "norm", "eps")
+            need(config, "the model", "vocab", "width", "residual_mult", "norm", "layers")
+        self.eps, = need(norm, "norm", "eps")
         self.hidden = self.width
-        self.width_p = _up(self.width, 64)
+        self.width_p = up(self.width, 64)
         self.logit_softcap = 0.0
         self.layers = []
         for i, e in enumerate(layers):
-            kind, mixer = _need(e, "layer %d" % i, "type", "mixer")
+            kind, mixer = need(e, "layer %d" % i, "type", "mixer")
             if kind not in MIXERS:
                 raise ModelError("unsupportedArch", "layer %d: mixer %s" % (i, kind))
             ff = None
             if e.get("mlp") is not None:
-                mlp_kind, ff = _need(e["mlp"], "layer %d's mlp" % i, "kind", "ff")
+                mlp_kind, ff = need(e["mlp"], "layer %d's mlp" % i, "kind", "ff")
                 if mlp_kind != "dense":
                     raise ModelError("unsupportedArch", "layer %d: feed-forward %s" % (i, mlp_kind))
             self.layers.append((MIXERS[kind](mixer, "layer %d" % i), ff))
@@ -134,44 +117,14 @@ class PakiraxConfig:
         return total
 
 
-def _blocks(t, dim, blocks, total=None):
-    """Lay out `dim` of t anew: consecutive runs of `size` entries, each padded with zeros to `padded` (blocks =
-    [(count, size, padded)]), the whole to `total`."""
-    out_n = sum(c * p for c, _, p in blocks)
-    total = out_n if total is None else total
-    shape = list(t.shape)
-    shape[dim] = total
-    if total == t.shape[dim] and all(s == p for _, s, p in blocks):
-        return t
-    out = torch.zeros(shape, dtype=t.dtype, device=t.device)
-    src = dst = 0
-    for count, size, padded in blocks:
-        lead = t.narrow(dim, src, count * size).unflatten(dim, (count, size))
-        out.narrow(dim, dst, count * padded).unflatten(dim, (count, padded)).narrow(dim + 1, 0, size).copy_(lead)
-        src, dst = src + count * size, dst + count * padded
-    return out
-
-
 class PakiraxWeights:
     """Device tensors of a model, padded and grouped.  source(name) -> BF16 tensor; shape(name) -> its shape."""
 
     def __init__(self, ctx, cfg, source, shape):
         self.ctx, self.cfg = ctx, cfg
         rank = lambda i: shape("l%d.mix.a1" % i)[0] if cfg.layers[i][0].kind == "gla" else 0
-        expected = cfg.tensor_shapes(rank)
-        for name, want in expected.items():
-            got = tuple(shape(name))
-            if got != tuple(want):
-                raise ModelError("indexCorrupt", "%s has shape %s, the configuration says %s" % (name, got, tuple(want)))
-
-        def t(name):
-            v = source(name)
-            if v.dtype != torch.bfloat16:
-                raise ModelError("indexCorrupt", "%s must be BF16" % name)
-            return v.to(ctx.device)
-
-        Wp = cfg.width_p
-        cols = lambda w: _blocks(w, 1, [(1, w.shape[1], _up(w.shape[1], 64))])
+        check_shapes(cfg.tensor_shapes(rank), shape)
+        t, cols = bf16_reader(ctx, source), pad_columns
         norm = lambda n: (t(n).contiguous(), t(n + ".b").contiguous())
         self.embed = cols(t("embed")).contiguous()
         self.final_norm = norm("final.norm")
@@ -181,32 +134,32 @@ class PakiraxWeights:
             w = dict(norm1=norm(p + "norm1"), norm1b=norm(p + "norm1b"))
             H = m.heads
             if m.kind == "gla":
-                r, rp = rank(i), _up(rank(i), 16)
+                r, rp = rank(i), up(rank(i), 16)
                 kd, vd = H * m.dim_p, H * m.vdim_p
-                rows = [_blocks(t(x + n), 0, [(H, m.dim, m.dim_p)]) for n in ("q", "k")] + \
-                       [_blocks(t(x + n), 0, [(H, m.vdim, m.vdim_p)]) for n in ("v", "g")] + [_blocks(t(x + "a1"), 0, [(1, r, rp)])]
+                rows = [blocks_of(t(x + n), 0, [(H, m.dim, m.dim_p)]) for n in ("q", "k")] + \
+                       [blocks_of(t(x + n), 0, [(H, m.vdim, m.vdim_p)]) for n in ("v", "g")] + [blocks_of(t(x + "a1"), 0, [(1, r, rp)])]
                 w["in_proj"] = cols(torch.cat(rows)).contiguous()
                 w["at"] = dict(q=0, k=kd, v=2 * kd, g=2 * kd + vd, a1=2 * kd + 2 * vd)
-                w["a2"] = _blocks(_blocks(t(x + "a2"), 0, [(H, m.dim, m.dim_p)]), 1, [(1, r, rp)]).contiguous()
-                w["a2_bias"] = _blocks(t(x + "a2.b"), 0, [(H, m.dim, m.dim_p)]).contiguous()
-                w["norm"] = _blocks(t(x + "norm"), 0, [(1, m.vdim, m.vdim_p)]).contiguous()
+                w["a2"] = blocks_of(blocks_of(t(x + "a2"), 0, [(H, m.dim, m.dim_p)]), 1, [(1, r, rp)]).contiguous()
+                w["a2_bias"] = blocks_of(t(x + "a2.b"), 0, [(H, m.dim, m.dim_p)]).contiguous()
+                w["norm"] = blocks_of(t(x + "norm"), 0, [(1, m.vdim, m.vdim_p)]).contiguous()
                 w["rank"] = rp
             else:
-                qp, gp = _up(m.q_rank, 16), _up(H, 16)
-                rows = [_blocks(t(x + "dq"), 0, [(1, m.q_rank, qp)]),
-                        _blocks(t(x + "dkv"), 0, [(1, m.kv_rank, m.rank_p), (1, m.rot_dim, m.rot_p)]),
-                        _blocks(t(x + "g"), 0, [(1, H, gp)])]
+                qp, gp = up(m.q_rank, 16), up(H, 16)
+                rows = [blocks_of(t(x + "dq"), 0, [(1, m.q_rank, qp)]),
+                        blocks_of(t(x + "dkv"), 0, [(1, m.kv_rank, m.rank_p), (1, m.rot_dim, m.rot_p)]),
+                        blocks_of(t(x + "g"), 0, [(1, H, gp)])]
                 w["in_proj"] = cols(torch.cat(rows)).contiguous()
                 w["at"] = dict(q=0, kv=qp, rope=qp + m.rank_p, g=qp + m.rank_p + m.rot_p)
                 uq = t(x + "uq").unflatten(0, (H, m.dim + m.rot_dim))
-                uq = torch.cat([_blocks(uq[:, :m.dim], 1, [(1, m.dim, m.dim_p)]),
-                                _blocks(uq[:, m.dim:], 1, [(1, m.rot_dim, m.rot_p)])], 1).flatten(0, 1)
+                uq = torch.cat([blocks_of(uq[:, :m.dim], 1, [(1, m.dim, m.dim_p)]),
+                                blocks_of(uq[:, m.dim:], 1, [(1, m.rot_dim, m.rot_p)])], 1).flatten(0, 1)
                 w["uq"] = cols(uq).contiguous()
-                w["uk"] = cols(_blocks(t(x + "uk"), 0, [(H, m.dim, m.dim_p)])).contiguous()
-                w["uv"] = cols(_blocks(t(x + "uv"), 0, [(H, m.vdim, m.vdim_p)])).contiguous()
-                w["q_norm"] = _blocks(t(x + "dq.norm"), 0, [(1, m.q_rank, qp)]).contiguous()
-                w["kv_norm"] = _blocks(t(x + "dkv.norm"), 0, [(1, m.kv_rank, m.rank_p)]).contiguous()
-            w["o"] = _blocks(t(x + "o"), 1, [(H, m.vdim, m.vdim_p)], _up(H * m.vdim_p, 64)).contiguous()
+                w["uk"] = cols(blocks_of(t(x + "uk"), 0, [(H, m.dim, m.dim_p)])).contiguous()
+                w["uv"] = cols(blocks_of(t(x + "uv"), 0, [(H, m.vdim, m.vdim_p)])).contiguous()
+                w["q_norm"] = blocks_of(t(x + "dq.norm"), 0, [(1, m.q_rank, qp)]).contiguous()
+                w["kv_norm"] = blocks_of(t(x + "dkv.norm"), 0, [(1, m.kv_rank, m.rank_p)]).contiguous()
+            w["o"] = blocks_of(t(x + "o"), 1, [(H, m.vdim, m.vdim_p)], up(H * m.vdim_p, 64)).contiguous()
             if ff is not None:
                 w.update(norm2=norm(p + "norm2"), norm2b=norm(p + "norm2b"), up=cols(t(p + "mlp.up")).contiguous(),
                          down=cols(t(p + "mlp.down")).contiguous())
@@ -215,15 +168,8 @@ class PakiraxWeights:
     @classmethod
     def from_directory(cls, ctx, path):
         """(config, weights) of a folder with config.json and model.safetensors."""
-        with open(os.path.join(path, "config.json")) as f:
-            cfg = PakiraxConfig(json.load(f))
-        tensors = SafetensorsFile(os.path.join(path, "model.safetensors"))
-
-        def shape(name):
-            if name not in tensors:
-                raise ModelError("indexCorrupt", "model.safetensors has no tensor %s" % name)
-            return tensors.shape(name)
-        return cfg, cls(ctx, cfg, tensors.tensor, shape)
+        cfg, tensor, shape = open_directory(path, PakiraxConfig)
+        return cfg, cls(ctx, cfg, tensor, shape)
 
     @classmethod
     def random(cls, ctx, cfg, seed=1234, decay_rank=16):
@@ -246,21 +192,16 @@ class PakiraxWeights:
         return cls(ctx, cfg, source, lambda n: shapes[n])
 
 
-class PakiraxDecoder(StepDecoder):
-    """Prompt portions and decode steps of a Pakirax model for `batch` sequences (slots).  Recurrent states and latent
-    rings are allocated once; every call only enqueues kernels.  A ring holds the layer's window beside one portion of
+class PakiraxDecoder(DenseDecoder):
+    """Prompt portions and decode steps of a Pakirax model.  A ring holds the layer's window beside one portion of
     max_chunk tokens, so a layer's cache does not grow with the context."""
+    long_f32 = ("residual", "delta", "gla_proj")
 
     def __init__(self, ctx, cfg, weights, batch=1, max_context=32768, max_chunk=2048):
-        super().__init__(ctx, cfg, weights, batch, max_context)
-        self.max_chunk = min(max_chunk, max_context)
-        self.max_rows = max(self.max_chunk, batch)
-        # Passes of a few rows are bound by the weights' bytes: their activations stay in 32 bits (a context of its own
-        # over the same weights, states and caches); longer ones run in the context's type.
-        self.few_ctx = ctx if ctx.act == ops.ACT_FP32 else ops.Context(ctx.device.index, ops.ACT_FP32)
+        super().__init__(ctx, cfg, weights, batch, max_context, max_chunk)
         self.mixers, self.states, self.caches = {}, {}, {}
         for i, (m, _) in enumerate(cfg.layers):
-            for c in {ctx, self.few_ctx}:
+            for c in self.contexts:
                 if m.kind == "gla":
                     op = ops.GLA(c, m.heads, m.dim_p, m.vdim_p, weights.layers[i]["rank"], m.tau, cfg.eps, m.dim, m.vdim)
                 else:
@@ -272,19 +213,6 @@ class PakiraxDecoder(StepDecoder):
             else:
                 capacity = min(max_context, m.window + self.max_chunk - 1) if m.window else max_context
                 self.caches[i] = ops.LatentCache(ctx, batch, capacity, m.rank_p, m.rot_p)
-        self.slots = torch.arange(batch, dtype=torch.int32, device=ctx.device)
-        self._buffers = {}
-        self.residual_hook = None        # called with (layer index, residual rows) after every layer
-        self.logits_f32 = torch.zeros((batch, cfg.vocab), dtype=torch.float32, device=ctx.device)
-
-    def _buf(self, name, rows, cols, dtype):
-        """Scratch rows.  Columns past a producer's own stay zero: a buffer's name goes with one width."""
-        key = (name, cols, dtype)
-        if key not in self._buffers:
-            # buffers of passes in another type than the context's never see more than FEW_ROWS rows
-            most = self.max_rows if dtype == self.ctx.dtype or name in ("residual", "delta", "gla_proj") else FEW_ROWS
-            self._buffers[key] = torch.zeros((most, cols), dtype=dtype, device=self.ctx.device)
-        return self._buffers[key][:rows]
 
     # -- mixers: normed rows in, the sublayer's output as 32-bit rows ---------------------------------------
     def _gla(self, ctx, i, h, rows_at, T, slots):
@@ -312,7 +240,7 @@ class PakiraxDecoder(StepDecoder):
     def _forward(self, tokens, rows_at, slots=None):
         """tokens (int32 device tensor) through every layer: final-normed rows [T, width padded]."""
         cfg, T = self.cfg, tokens.numel()
-        ctx = self.few_ctx if T <= FEW_ROWS else self.ctx
+        ctx = self.pass_context(T)
         D, mult = cfg.width, cfg.residual_mult
         x = self._buf("residual", T, D, torch.float32)
         h, last = self._buf("normed", T, cfg.width_p, ctx.dtype), self._buf("normed", T, cfg.width_p, self.ctx.dtype)
@@ -338,46 +266,7 @@ class PakiraxDecoder(StepDecoder):
                 self.residual_hook(i, x)
         return last
 
-    def _prefill_chunk_rows(self, tokens, b, start):
-        return self._forward(tokens, ops.row_map(b, start))
-
-    def forward_hidden(self, position):
-        """One token (self.tokens) of every sequence at `position` (None: each at its own, self.positions)."""
-        if position is not None:
-            self.positions.fill_(position)
-        self.normed = self._forward(self.tokens, ops.row_map(slots=self.slots, positions=self.positions), self.slots)
-        return self.normed
-
-    def decode_rows(self, sequences, positions, tokens):
-        if max(positions) >= self.max_context:
-            raise ValueError("position %d exceeds the context (%d)" % (max(positions), self.max_context))
-        ids = torch.tensor([tokens, sequences, positions], dtype=torch.int32).to(self.ctx.device)
-        if len(sequences) == 1:
-            return self._forward(ids[0], ops.row_map(sequences[0], positions[0]))
-        return self._forward(ids[0], ops.row_map(slots=ids[1], positions=ids[2]), ids[1])
-
     def reset(self, sequence):
         """Forget what the sequence left: recurrent states start from zero (ring rows are overwritten as they are used)."""
         for state in self.states.values():
             state[sequence].zero_()
-
-    # -- logits -----------------------------------------------------------------------------------------
-    def head_rows(self, normed):
-        """(activations, 32-bit) logits of any number of final-normed rows."""
-        n = normed.shape[0]
-        y32 = torch.empty((n, self.cfg.vocab), dtype=torch.float32, device=self.ctx.device)
-        if self.ctx.act == ops.ACT_FP32:
-            ops.dense_linear(self.ctx, self.w.embed, normed, y_f32=y32)
-            return y32, y32
-        y = torch.empty((n, self.cfg.vocab), dtype=self.ctx.dtype, device=self.ctx.device)
-        ops.dense_linear(self.ctx, self.w.embed, normed, y=y, y_f32=y32)
-        return y, y32
-
-    def head(self):
-        """Logits of the rows forward_hidden left: activations in self.logits, 32-bit in self.logits_f32."""
-        ops.dense_linear(self.ctx, self.w.embed, self.normed, y=self.logits, y_f32=self.logits_f32)
-        return self.logits
-
-    def greedy(self):
-        """Greedy tokens of self.logits_f32 in self.next_tokens."""
-        return ops.argmax_rows(self.ctx, self.logits_f32, out=self.next_tokens)

@@ -18,6 +18,12 @@ def _open_pakirax(ctx, path, batch=1, max_context=32768, max_chunk=2048):
     return PakiraxDecoder(ctx, cfg, weights, batch, max_context, max_chunk)
 
 
+def _open_kemuzen(ctx, path, batch=1, max_context=32768, max_chunk=2048):
+    from .kemuzen import KemuzenDecoder, KemuzenWeights
+    cfg, weights = KemuzenWeights.from_directory(ctx, path)
+    return KemuzenDecoder(ctx, cfg, weights, batch, max_context, max_chunk)
+
+
 def _open_hybrid(ctx, path, batch=1, max_context=32768, max_chunk=None):
     from . import gturbo
     from .decoder import HybridDecoder, HybridWeights
@@ -26,6 +32,7 @@ def _open_hybrid(ctx, path, batch=1, max_context=32768, max_chunk=None):
 
 
 FAMILIES = {"Pakirax": Family("Pakirax", "dense", ("bfloat16", "float32"), _open_pakirax),
+            "Kemuzen": Family("Kemuzen", "scan", ("bfloat16", "float32"), _open_kemuzen),
             "hybrid-moe": Family("hybrid-moe", None, ("bfloat16", "float16"), _open_hybrid)}
 
 
