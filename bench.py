@@ -31,6 +31,12 @@ RAMP_STEPS = 200       # untimed steps ahead of the --warmup steps of the decode
 PAKIRAX_SIZES = {"1k": (1024, 24, 8, (128, 128), (128, 64, 128, 256, 768, 2048), 4096, 65536),
                  "2k": (2048, 40, 16, (128, 128), (128, 64, 128, 512, 1536, 4096), 8192, 248320),
                  "4k": (4096, 32, 32, (128, 128), (128, 64, 128, 512, 1536, 4096), 16384, 131072)}
+# width, layers, window heads, kv heads, delta heads, key heads of them, state-space heads, window, ff, vocab, side dim; heads of
+# 128 (state-space: 64 with a state of 128); layers in fours: attention, delta rule, attention and state space side by
+# side, attention on the first one's keys
+KEMUZEN_SIZES = {"1k": (1024, 24, 8, 2, 16, 8, 32, 2048, 2816, 65536, 128),
+                 "2k": (2048, 40, 16, 4, 32, 16, 64, 4096, 5632, 248320, 256),
+                 "4k": (4096, 32, 32, 8, 64, 32, 128, 4096, 11264, 131072, 256)}
 
 
 def parse():
@@ -45,7 +51,7 @@ def parse():
     ap.add_argument("--sweep", action="store_true", help="also print batch/bits sweep lines to stderr")
     ap.add_argument("--no-extra", action="store_true", help="skip the `extra` object (the other cells of the metric) "
                     "that the default invocation appends")
-    ap.add_argument("--workload", default="decode", choices=["decode", "prefill", "attention", "prefill_attention", "sampler", "greedy", "step", "prefill_step", "pakirax_step", "pakirax_prefill", "copy", "read"],
+    ap.add_argument("--workload", default="decode", choices=["decode", "prefill", "attention", "prefill_attention", "sampler", "greedy", "step", "prefill_step", "pakirax_step", "pakirax_prefill", "kemuzen_step", "kemuzen_prefill", "copy", "read"],
                     help="decode = configs[1] (the headline line); prefill = configs[2] grouped GEMM; "
                          "attention = configs[3] quantized-KV decode attention; prefill_attention = causal attention of --tokens queries "
                          "at the end of a --context cache; sampler = the end of configs[4]: "
@@ -55,8 +61,8 @@ def parse():
                          "same 40 layers with the prefill kernels, in chunks of --chunk; copy = a plain 1 GiB device copy, "
                          "the known-size kernel the FETCH_SIZE / WRITE_SIZE counters are calibrated on; "
                          "pakirax_step / pakirax_prefill = a decode step (--batch sequences at --context) / a --tokens prompt of the Pakirax "
-                         "model at --size, random weights")
-    ap.add_argument("--size", default="2k", choices=sorted(PAKIRAX_SIZES), help="pakirax_*: width of the model")
+                         "model at --size, random weights; kemuzen_step / kemuzen_prefill = the same of the Kemuzen model")
+    ap.add_argument("--size", default="2k", choices=sorted(PAKIRAX_SIZES), help="pakirax_*, kemuzen_*: width of the model")
     ap.add_argument("--context", type=int, default=None, help="attention: tokens in the KV cache (default 32768; "
                     "prefill_attention: the chunk itself)")
     ap.add_argument("--tokens", type=int, default=4096, help="prefill: tokens per step")
@@ -783,17 +789,41 @@ def pakirax_model(nv, torch, a, batch, max_context, max_chunk):
     return ctx, cfg, PakiraxDecoder(ctx, cfg, PakiraxWeights.random(ctx, cfg, seed=2024), batch, max_context, max_chunk)
 
 
-def run_pakirax_step(nv, torch, a):
-    """One decode step of the Pakirax model at `--size` (random weights; half the layers gated linear attention with a
-    32-bit state, half latent attention over a window): embedding to greedy token for `--batch` sequences, each at the end
-    of a full window, captured once into a HIP graph and replayed."""
+def kemuzen_model(nv, torch, a, batch, max_context, max_chunk):
+    from nvmai_amd.kemuzen import KemuzenConfig, KemuzenDecoder, KemuzenWeights
+    width, layers, heads, kv, dheads, dkeys, sheads, window, ff, vocab, side = KEMUZEN_SIZES[a.size]
+    mlp = {"kind": "dense", "ff": ff}
+    at = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 50.0, "mask": {"size": window, "keep_first": 4}}
+    left = {k: v for k, v in at.items() if k != "softcap"}
+    left["mask"] = {"size": window}
+    right = {"heads": sheads, "vdim": 64, "state": 128, "groups": 1, "conv": 4, "norm_groups": 1}
+    four = lambda i: [{"type": "attention", "mixer": at, "mlp": mlp},
+                      {"type": "delta", "mixer": {"heads": dheads, "kv_heads": dkeys, "dim": 128, "vdim": 128, "conv": 4}, "mlp": mlp},
+                      {"type": "parallel", "mixer": {"left": left, "right": right, "left_scale": 0.7, "right_scale": 0.7}, "mlp": mlp},
+                      {"type": "attention", "mixer": dict(at, kv_from=i), "mlp": mlp}]
+    cfg = KemuzenConfig({"architecture": "Kemuzen", "vocab": vocab, "width": width, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-6},
+                         "logit_softcap": 30.0, "token_side": {"dim": side}, "layers": sum((four(i) for i in range(0, layers, 4)), [])})
+    ctx = nv.Context(0, nv.ACT_BF16)
+    return ctx, cfg, KemuzenDecoder(ctx, cfg, KemuzenWeights.random(ctx, cfg, seed=2024), batch, max_context, max_chunk)
+
+
+DENSE_MODELS = {"pakirax": ("Pakirax", pakirax_model, lambda cfg: cfg.layers[1][0].window),
+                "kemuzen": ("Kemuzen", kemuzen_model, lambda cfg: cfg.layers[0][0].window)}
+
+
+def run_dense_step(nv, torch, a, which):
+    """One decode step of a dense model at `--size` (random weights): embedding to greedy token for `--batch` sequences, each at
+    the end of a full window, captured once into a HIP graph and replayed."""
     B, context = min(a.batch, 16), a.context
-    ctx, cfg, dec = pakirax_model(nv, torch, a, B, context + 1, 2048)
+    title, build, window_of = DENSE_MODELS[which]
+    ctx, cfg, dec = build(nv, torch, a, B, context + 1, 2048)
     gen = torch.Generator(device="cuda").manual_seed(5)
-    for c in dec.caches.values():
-        c.rows.normal_(0.0, 1.0, generator=gen)
+    for c in set(dec.caches.values()):
+        for t in ([c.rows] if which == "pakirax" else [c.k, c.v]):
+            t.normal_(0.0, 1.0, generator=gen)
     for s in dec.states.values():
-        s.normal_(0.0, 0.1, generator=gen)
+        for t in ([s] if which == "pakirax" else s):
+            t.normal_(0.0, 0.1, generator=gen)
     dec.tokens.copy_(torch.randint(0, cfg.vocab, (B,), generator=gen, device="cuda", dtype=torch.int32))
     dec.positions.fill_(context - 1)
 
@@ -823,9 +853,9 @@ def run_pakirax_step(nv, torch, a):
         "metric": METRIC, "value": round(B / dt, 1), "unit": "tok/s", "n_gpus": 1, "steps": a.steps, "warmup": a.warmup,
         "ms_per_step": round(dt * 1e3, 4), "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
         "dtype": "bf16 weights and activations, f32 accumulate, residual, norms, attention weights and recurrent state", "data": "synthetic",
-        "config": {"workload": "decode step of the Pakirax model, size %s: %d layers, width %d, vocab %d, window %d, greedy; batch %d at "
-                               "context %d, one HIP graph per step" % (a.size, len(cfg.layers), cfg.width, cfg.vocab,
-                                                                     cfg.layers[1][0].window, B, context),
+        "config": {"workload": "decode step of the %s model, size %s: %d layers, width %d, vocab %d, window %d, greedy; batch %d at "
+                               "context %d, one HIP graph per step" % (title, a.size, len(cfg.layers), cfg.width, cfg.vocab, window_of(cfg), B,
+                                                                     context),
                    "batch": B, "context": context, "bytes_per_token_MB": round(bpt / 1e6, 1),
                    "roofline_tok_per_s_at_8TBps": round(HBM_PEAK_GBPS * 1e9 / bpt, 1)},
         "roofline": {"kernel": "whole step (all kernels of one graph replay)", "bound": "hbm", "achieved": round(gbps, 2),
@@ -835,11 +865,12 @@ def run_pakirax_step(nv, torch, a):
     }
 
 
-def run_pakirax_prefill(nv, torch, a):
-    """A prompt of `--tokens` tokens of one sequence through the Pakirax model at `--size` (random weights) in chunks of
+def run_dense_prefill(nv, torch, a, which):
+    """A prompt of `--tokens` tokens of one sequence through a dense model at `--size` (random weights) in chunks of
     `--chunk`, launched eagerly through the C ABI; the logits of the last token are not computed."""
     T, chunk = a.tokens, a.chunk
-    ctx, cfg, dec = pakirax_model(nv, torch, a, 1, T, chunk)
+    title, build, window_of = DENSE_MODELS[which]
+    ctx, cfg, dec = build(nv, torch, a, 1, T, chunk)
     gen = torch.Generator(device="cuda").manual_seed(9)
     tokens = torch.randint(0, cfg.vocab, (T,), generator=gen, device="cuda", dtype=torch.int32)
 
@@ -862,8 +893,8 @@ def run_pakirax_prefill(nv, torch, a):
         "metric": METRIC, "value": round(T / dt, 1), "unit": "tok/s", "n_gpus": 1, "steps": steps, "warmup": a.warmup,
         "ms_per_step": round(dt * 1e3, 3), "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
         "dtype": "bf16 weights and activations, f32 accumulate, residual, norms, attention weights and recurrent state", "data": "synthetic",
-        "config": {"workload": "prompt of %d tokens through the Pakirax model, size %s (%d layers, width %d, window %d) in chunks of %d"
-                               % (T, a.size, len(cfg.layers), cfg.width, cfg.layers[1][0].window, chunk),
+        "config": {"workload": "prompt of %d tokens through the %s model, size %s (%d layers, width %d, window %d) in chunks of %d"
+                               % (T, title, a.size, len(cfg.layers), cfg.width, window_of(cfg), chunk),
                    "tokens": T, "chunk": chunk, "model_gflop_per_token": round(flops / T / 1e9, 2)},
         "roofline": {"kernel": "whole prompt (all kernels)", "bound": "mfma", "achieved": round(tf, 2), "peak": MFMA_BF16_PEAK_TFLOPS,
                      "unit": "TFLOP/s", "frac": round(tf / MFMA_BF16_PEAK_TFLOPS, 4), "traffic": None, "traffic_source": None,
@@ -937,8 +968,8 @@ def main():
                 run_greedy(nv, ctx, torch, a) if a.workload == "greedy" else
                 run_step(nv, ctx, torch, a) if a.workload == "step" else
                 run_prefill_step(nv, ctx, torch, a) if a.workload == "prefill_step" else
-                run_pakirax_step(nv, torch, a) if a.workload == "pakirax_step" else
-                run_pakirax_prefill(nv, torch, a) if a.workload == "pakirax_prefill" else
+                run_dense_step(nv, torch, a, a.workload[:-5]) if a.workload in ("pakirax_step", "kemuzen_step") else
+                run_dense_prefill(nv, torch, a, a.workload[:-8]) if a.workload in ("pakirax_prefill", "kemuzen_prefill") else
                 run_read(nv, ctx, torch, a) if a.workload == "read" else run_copy(torch, a))
         print(json.dumps(line), flush=True)
         return

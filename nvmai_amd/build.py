@@ -17,8 +17,8 @@ FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=o
 
 
 # Part libraries: the sources that one family of models needs, for a run that must not wait for the rest.
-PARTS = {"dense": ["ctx_api", "dense_api", "norm_api", "gla_api", "latent_api", "sample_api"],
-         "scan": ["ctx_api", "dense_api", "norm_api", "window_api", "scan_api", "sample_api"]}
+_DENSE = ["ctx_api", "dense_api", "dense_erf_api", "dense_bias_api", "dense_pairs_api", "dense_full_api", "norm_api", "sample_api"]
+PARTS = {"dense": _DENSE + ["gla_api", "latent_api"], "scan": _DENSE + ["window_api", "scan_api"]}
 
 
 def part_path(part):

@@ -2,7 +2,7 @@
 // logits, argmax.
 #include "ctx.hpp"
 #include "dense_kernels.hpp"
-#include "dense_internal.hpp"
+#include "ends_kernels.hpp"
 
 using namespace nvmai;
 
@@ -24,62 +24,14 @@ int dense_linear_check(const nvmai_hip_ctx* ctx, const DenseLinearParams& p) {
     return NVMAI_OK;
 }
 
-template <int ACT, int NT>
-static void launch_gemv(const DenseLinearParams& p, hipStream_t s) {
-    // rows per wave: one (short blocks, many of them) until the inputs' own loads weigh more than that
-    if (p.n >= 65536) dense_gemv_kernel<ACT, NT, 4><<<(p.n + 15) / 16, 256, 0, s>>>(p);
-    else if (p.activation == NVMAI_LINEAR_SILU_PAIRS || (NT * (ACT == ACT_FP32 ? 2 : 1) > 2 && p.n >= 8192)) dense_gemv_kernel<ACT, NT, 2><<<(p.n + 7) / 8, 256, 0, s>>>(p);
-    else dense_gemv_kernel<ACT, NT, 1><<<(p.n + 3) / 4, 256, 0, s>>>(p);
-}
-
-template <int ACT>
-static int gemv(const DenseLinearParams& p, hipStream_t s) {
-    if (p.rows == 1) launch_gemv<ACT, 1>(p, s);
-    else if (p.rows == 2) launch_gemv<ACT, 2>(p, s);
-    else if (p.rows == 3) launch_gemv<ACT, 3>(p, s);
-    else launch_gemv<ACT, 4>(p, s);
-    return launch_status();
-}
-
 int dense_linear(nvmai_hip_ctx* ctx, hipStream_t s, const DenseLinearParams& p) {
     const int rc = dense_linear_check(ctx, p);
     if (rc) return rc;
     if (p.rows == 0) return NVMAI_OK;
-    if (p.rows <= 4) return ctx->act == NVMAI_ACT_FP32 ? gemv<ACT_FP32>(p, s) : gemv<ACT_BF16>(p, s);
-    if (ctx->act == NVMAI_ACT_FP32) {
-        const dim3 grid((p.n + 63) / 64, (p.rows + 63) / 64);
-        if (grid.y > 65535) return NVMAI_ERR_UNSUPPORTED;
-        dense_f32_kernel<<<grid, 256, 0, s>>>(p);
-        return launch_status();
-    }
-    if (p.rows <= 64) {
-        // row tiles per block: as many as leave every compute unit several blocks; waves: about four steps of k each
-        const int nr = p.n >= 32768 ? 4 : p.n >= 8192 ? 2 : 1;
-        const uint32_t blocks = (p.n + 16 * nr - 1) / (16 * nr);
-#define NVMAI_SKINNY(TT)                                                              \
-    do {                                                                              \
-        if (nr == 4) dense_skinny_kernel<TT, 4, 4><<<blocks, 256, 0, s>>>(p);         \
-        else if (nr == 2) dense_skinny_kernel<TT, 2, 4><<<blocks, 256, 0, s>>>(p);    \
-        else if (p.k <= 1024) dense_skinny_kernel<TT, 1, 4><<<blocks, 256, 0, s>>>(p); \
-        else if (p.k <= 2048) dense_skinny_kernel<TT, 1, 8><<<blocks, 512, 0, s>>>(p); \
-        else dense_skinny_kernel<TT, 1, 16><<<blocks, 1024, 0, s>>>(p);               \
-    } while (0)
-        if (p.rows <= 16) NVMAI_SKINNY(1);
-        else if (p.rows <= 32) NVMAI_SKINNY(2);
-        else NVMAI_SKINNY(4);
-#undef NVMAI_SKINNY
-        return launch_status();
-    }
-    // the largest tile that still gives every compute unit one
-    const uint32_t cus = (uint32_t)ctx->compute_units;
-    auto tiles = [](uint32_t v, uint32_t b) { return (v + b - 1) / b; };
-    if (tiles(p.n, 128) * tiles(p.rows, 128) >= cus)
-        dense_gemm_kernel<128, 128><<<tiles(p.n, 128) * tiles(p.rows, 128), 256, 0, s>>>(p, tiles(p.n, 128), tiles(p.rows, 128));
-    else if (tiles(p.n, 64) * tiles(p.rows, 128) >= cus)
-        dense_gemm_kernel<64, 128><<<tiles(p.n, 64) * tiles(p.rows, 128), 256, 0, s>>>(p, tiles(p.n, 64), tiles(p.rows, 128));
-    else
-        dense_gemm_kernel<64, 64><<<tiles(p.n, 64) * tiles(p.rows, 64), 256, 0, s>>>(p, tiles(p.n, 64), tiles(p.rows, 64));
-    return launch_status();
+    if (p.activation == NVMAI_LINEAR_SILU_PAIRS) return dense_launch_pairs(ctx, s, p);
+    if (p.mul || p.activation == NVMAI_LINEAR_GELU_TANH || (p.bias && p.activation != NVMAI_LINEAR_NONE)) return dense_launch_full(ctx, s, p);
+    if (p.bias) return dense_launch_bias(ctx, s, p);
+    return p.activation == NVMAI_LINEAR_GELU_ERF ? dense_launch_erf(ctx, s, p) : dense_launch<DE_PLAIN>(ctx, s, p);
 }
 
 }  // namespace nvmai

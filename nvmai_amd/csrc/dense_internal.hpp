@@ -19,6 +19,11 @@ struct DenseLinearParams {
 };
 
 int dense_linear_check(const nvmai_hip_ctx* ctx, const DenseLinearParams& p);
+// The launches behind it by what stands between sum and store (dense_*_api.hip, built side by side).
+int dense_launch_erf(nvmai_hip_ctx* ctx, hipStream_t s, const DenseLinearParams& p);
+int dense_launch_bias(nvmai_hip_ctx* ctx, hipStream_t s, const DenseLinearParams& p);
+int dense_launch_pairs(nvmai_hip_ctx* ctx, hipStream_t s, const DenseLinearParams& p);
+int dense_launch_full(nvmai_hip_ctx* ctx, hipStream_t s, const DenseLinearParams& p);
 int dense_linear(nvmai_hip_ctx* ctx, hipStream_t s, const DenseLinearParams& p);
 
 }  // namespace nvmai

@@ -1,10 +1,9 @@
 // Kernels of the dense models (BF16 weights; 16-bit BF16 or 32-bit activations; a 32-bit residual stream):
-// the matrix products, embedding rows, the cap of the logits, argmax.
-// gfx950, wave64.
+// the matrix products.  gfx950, wave64.
 #pragma once
 
 #include "dense_internal.hpp"
-#include "rows.hpp"
+#include "common.hpp"
 
 namespace nvmai {
 
@@ -21,11 +20,19 @@ __device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.0f + e
 // z/2 (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))
 __device__ __forceinline__ float gelu_tanh(float z) { return 0.5f * z * (1.0f + tanhf(0.79788456080286536f * fmaf(0.044715f * z * z, z, z))); }
 
-// What stands between a sum and its store: bias, activation, the token's own multiplier (an id past the table: zero).
+// What stands between a sum and its store, fixed when a kernel is built: a tile's store is unrolled many times, and code
+// that a call does not need costs instruction fetches in all of them.  PLAIN: the activation NONE; ERF: GELU_ERF; BIAS: a
+// bias; PAIRS: SILU_PAIRS; FULL: bias, any activation, the token's own multiplier.
+enum DenseEpilogue : int { DE_PLAIN, DE_ERF, DE_BIAS, DE_PAIRS, DE_FULL };
+
+template <int EPI>
 __device__ __forceinline__ float dense_finish(const DenseLinearParams& p, uint32_t t, uint32_t r, float v) {
+    if (EPI == DE_ERF) return gelu_erf(v);
+    if (EPI == DE_BIAS) return v + bf16_to_f32(p.bias[r]);
+    if (EPI != DE_FULL) return v;
     if (p.bias) v += bf16_to_f32(p.bias[r]);
     v = p.activation == NVMAI_LINEAR_GELU_ERF ? gelu_erf(v) : p.activation == NVMAI_LINEAR_GELU_TANH ? gelu_tanh(v) : v;
-    if (p.mul) {
+    if (p.mul) {                                     // an id past the table: zero
         const uint32_t id = p.mul_ids[t];
         v *= id < p.mul_rows ? bf16_to_f32(p.mul[(size_t)id * p.mul_stride + r]) : 0.0f;
     }
@@ -38,21 +45,20 @@ __device__ __forceinline__ void dense_put(const DenseLinearParams& p, uint32_t t
     if (p.y_f32) p.y_f32[(size_t)t * p.y_stride + r] = v;
 }
 
-template <int ACT>
+template <int EPI, int ACT>
 __device__ __forceinline__ void dense_store(const DenseLinearParams& p, uint32_t t, uint32_t r, float v) {
-    dense_put<ACT>(p, t, r, dense_finish(p, t, r, v));
+    dense_put<ACT>(p, t, r, dense_finish<EPI>(p, t, r, v));
 }
 
 // Rows 2 j and 2 j + 1 of the matrix make output j: silu(gate) * up.
 template <int ACT>
-__device__ __forceinline__ void dense_store_pair(const DenseLinearParams& p, uint32_t t, uint32_t j, float gate, float up) {
-    dense_put<ACT>(p, t, j, silu(gate) * up);
-}
+__device__ __forceinline__ float dense_pair(float gate, float up) { return (ACT == ACT_FP32 ? silu(gate) : silu_fast(gate)) * up; }
 
 // Four neighbouring outputs of one token (r0 a multiple of 4).
+template <int EPI>
 __device__ __forceinline__ void dense_store4_bf16(const DenseLinearParams& p, uint32_t t, uint32_t r0, dn_f4 v) {
-    if (p.activation == NVMAI_LINEAR_SILU_PAIRS) {           // n and the row stride are even
-        const float a = silu(v[0]) * v[1], b = silu(v[2]) * v[3];
+    if (EPI == DE_PAIRS) {                           // n and the row stride are even
+        const float a = dense_pair<ACT_BF16>(v[0], v[1]), b = dense_pair<ACT_BF16>(v[2], v[3]);
         if (r0 + 4u <= p.n) {
             if (p.y) *reinterpret_cast<uint32_t*>(static_cast<uint16_t*>(p.y) + (size_t)t * p.y_stride + r0 / 2u) = f32_to_bf16(a) | ((uint32_t)f32_to_bf16(b) << 16);
             if (p.y_f32) *reinterpret_cast<float2*>(p.y_f32 + (size_t)t * p.y_stride + r0 / 2u) = float2{a, b};
@@ -61,7 +67,7 @@ __device__ __forceinline__ void dense_store4_bf16(const DenseLinearParams& p, ui
         }
     } else if (r0 + 4u <= p.n && (p.y_stride & 3u) == 0) {
 #pragma unroll
-        for (int j = 0; j < 4; ++j) v[j] = dense_finish(p, t, r0 + j, v[j]);
+        for (int j = 0; j < 4; ++j) v[j] = dense_finish<EPI>(p, t, r0 + j, v[j]);
         if (p.y) {
             uint2 q;
             q.x = f32_to_bf16(v[0]) | ((uint32_t)f32_to_bf16(v[1]) << 16);
@@ -72,7 +78,7 @@ __device__ __forceinline__ void dense_store4_bf16(const DenseLinearParams& p, ui
     } else {
 #pragma unroll
         for (int j = 0; j < 4; ++j)
-            if (r0 + j < p.n) dense_store<ACT_BF16>(p, t, r0 + j, v[j]);
+            if (r0 + j < p.n) dense_store<EPI, ACT_BF16>(p, t, r0 + j, v[j]);
     }
 }
 
@@ -80,7 +86,7 @@ __device__ __forceinline__ void dense_store4_bf16(const DenseLinearParams& p, ui
 // Bound by the matrix's bytes.  The inputs are read from L1 / L2 beside the weights (no LDS, no barrier): every
 // load of a k step is independent of the others, so a wave has RW + NT (32-bit inputs: RW + 2 NT) 16-byte loads per lane
 // in flight.
-template <int ACT, int NT, int RW>
+template <int EPI, int ACT, int NT, int RW>
 __global__ __launch_bounds__(256) void dense_gemv_kernel(DenseLinearParams p) {
     const uint32_t lane = threadIdx.x & 63u, wave = threadIdx.x >> 6;
     const uint32_t r0 = (blockIdx.x * 4u + wave) * RW;
@@ -143,32 +149,25 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(DenseLinearParams p) {
             }
         }
     }
-    if constexpr (RW > 1) {
-        if (p.activation == NVMAI_LINEAR_SILU_PAIRS) {
 #pragma unroll
-            for (int t = 0; t < NT; ++t)
+    for (int t = 0; t < NT; ++t) {
+        float v[RW];
 #pragma unroll
-                for (int r = 0; r < RW; r += 2) {
-                    const float gate = wave_sum_bcast(acc[t][r]), up = wave_sum_bcast(acc[t][r + 1]);
-                    if (lane == (uint32_t)(t * RW + r) && r0 + r < p.n && (uint32_t)t < p.rows) dense_store_pair<ACT>(p, t, (r0 + r) / 2u, gate, up);
-                }
-            return;
+        for (int r = 0; r < RW; ++r) v[r] = wave_sum_bcast(acc[t][r]);
+#pragma unroll
+        for (int r = 0; r < RW; r += EPI == DE_PAIRS ? 2 : 1) {
+            if (lane != (uint32_t)(t * RW + r) || r0 + r >= p.n || (uint32_t)t >= p.rows) continue;
+            if constexpr (EPI == DE_PAIRS) dense_put<ACT>(p, t, (r0 + r) / 2u, dense_pair<ACT>(v[r], v[r + 1]));
+            else dense_store<EPI, ACT>(p, t, r0 + r, v[r]);
         }
     }
-#pragma unroll
-    for (int t = 0; t < NT; ++t)
-#pragma unroll
-        for (int r = 0; r < RW; ++r) {
-            const float v = wave_sum_bcast(acc[t][r]);
-            if (lane == (uint32_t)(t * RW + r) && r0 + r < p.n && (uint32_t)t < p.rows) dense_store<ACT>(p, t, r0 + r, v);
-        }
 }
 
 // ---- 5 .. 64 input rows: 16 NR weight rows per block, the waves split k, MFMA, sums through LDS ---------
 // Weight rows are the A operand as they lie in memory: lane (i = lane % 16, g = lane / 16) loads the 32 bytes
 // W[r0 + i, k + 16 g .. + 16), four lanes cover 128 contiguous bytes of a row; the inputs are the B operand in
 // the same order of k, read from L2 once per NR row tiles.
-template <int TT, int NR, int NW>
+template <int EPI, int TT, int NR, int NW>
 __global__ __launch_bounds__(64 * NW) void dense_skinny_kernel(DenseLinearParams p) {
     __shared__ __attribute__((aligned(16))) float part[NW - 1][64][TT * NR * 4];
     const uint32_t lane = threadIdx.x & 63u, wave = threadIdx.x >> 6, i = lane & 15u, g = lane >> 4;
@@ -222,7 +221,7 @@ __global__ __launch_bounds__(64 * NW) void dense_skinny_kernel(DenseLinearParams
 #pragma unroll
             for (int w = 0; w < NW - 1; ++w) acc[r][t] += *reinterpret_cast<const dn_f4*>(&part[w][lane][4 * (r * TT + t)]);
             // acc[r][t][j] = y[token 16 t + i, row r0 + 16 r + 4 g + j]
-            if (16u * t + i < p.rows) dense_store4_bf16(p, 16u * t + i, r0 + 16u * r + 4u * g, acc[r][t]);
+            if (16u * t + i < p.rows) dense_store4_bf16<EPI>(p, 16u * t + i, r0 + 16u * r + 4u * g, acc[r][t]);
         }
 }
 
@@ -230,7 +229,7 @@ __global__ __launch_bounds__(64 * NW) void dense_skinny_kernel(DenseLinearParams
 // Four waves, each a quarter of the tile (BN / 2 x BM / 2) in 16 x 16 x 32 products.  A tile's rows are 128 bytes
 // of LDS; the eight 16-byte pieces of row r lie in the order piece ^ (r % 8), so that the sixteen rows of an
 // operand read fall into different banks.  Loads go straight from memory into LDS.
-template <int BN, int BM>
+template <int EPI, int BN, int BM>
 __global__ __launch_bounds__(256) void dense_gemm_kernel(DenseLinearParams p, uint32_t tiles_n, uint32_t tiles_m) {
     constexpr int LA = BN / 32, LB = BM / 32;                // 1 KB pieces per wave
     constexpr int TN = BN / 32, TM = BM / 32;                // 16 x 16 tiles per wave
@@ -301,13 +300,14 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(DenseLinearParams p, ui
 #pragma unroll
         for (int a = 0; a < TN; ++a) {
             const uint32_t r = n0 + wn + 16 * a + 4u * g;
-            if (r < p.n) dense_store4_bf16(p, t, r, acc[a][b]);
+            if (r < p.n) dense_store4_bf16<EPI>(p, t, r, acc[a][b]);
         }
     }
 }
 
 // ---- 32-bit activations, more than four rows: 64 x 64 tiles on the vector pipe, BF16 weights widened, fp32 FMA ------------
 // Sums are two-level (a step of 16 k, then the running total), which keeps the rounding error of a long k small.
+template <int EPI>
 __global__ __launch_bounds__(256) void dense_f32_kernel(DenseLinearParams p) {
     __shared__ float ws[16][65], xs[16][65];
     const uint32_t tid = threadIdx.x, tx = tid & 15u, ty = tid >> 4;
@@ -344,105 +344,68 @@ __global__ __launch_bounds__(256) void dense_f32_kernel(DenseLinearParams p) {
 #pragma unroll
         for (int n = 0; n < 4; ++n) {
             const uint32_t t = m0 + ty + 16u * m, r = n0 + tx + 16u * n;
-            const float next = shfl_xor_f(acc[m][n], 1);         // the neighbouring weight row's sum
+            const float next = EPI == DE_PAIRS ? shfl_xor_f(acc[m][n], 1) : 0.0f;        // the neighbouring weight row's sum
             if (t >= p.rows || r >= p.n) continue;
-            if (p.activation != NVMAI_LINEAR_SILU_PAIRS) dense_store<ACT_FP32>(p, t, r, acc[m][n]);
-            else if ((r & 1u) == 0) dense_store_pair<ACT_FP32>(p, t, r / 2u, acc[m][n], next);
+            if (EPI != DE_PAIRS) dense_store<EPI, ACT_FP32>(p, t, r, acc[m][n]);
+            else if ((r & 1u) == 0) dense_put<ACT_FP32>(p, t, r / 2u, dense_pair<ACT_FP32>(acc[m][n], next));
         }
 }
 
-// ---- the two ends of a model ----------------------------------------------------------------------
-// Rows of a BF16 table as 32-bit residual rows; an id past the table gives zeros.  scale: factor of the table's rows;
-// inv_freq (nullptr: none): plus the sinusoid of the row's position, entry 2 i its sine and 2 i + 1 its cosine at
-// inv_freq[i]; act (nullptr: none): the row once more as activations.
-struct EmbedParams {
-    const uint16_t* table;
-    const uint32_t* ids;
-    float* out;
-    void* act;
-    const double* inv_freq;
-    SeqRows rows;
-    uint32_t table_stride, out_stride, act_stride, d, vocab;
-    float scale;
-};
-
-template <int ACT>
-__global__ __launch_bounds__(256) void embed_rows_kernel(EmbedParams p) {
-    const uint32_t row = blockIdx.y, pair = blockIdx.x * 256u + threadIdx.x, j = 2u * pair;
-    if (j >= p.d) return;
-    const uint32_t id = p.ids[row];
-    const bool two = j + 1u < p.d;
-    const uint16_t* e = p.table + (size_t)id * p.table_stride + j;
-    float a = 0.0f, b = 0.0f;
-    if (id < p.vocab) {
-        a = bf16_to_f32(e[0]) * p.scale;
-        b = two ? bf16_to_f32(e[1]) * p.scale : 0.0f;
-    }
-    if (p.inv_freq) {
-        float c, s;
-        position_angle(p.rows.position_of(row), p.inv_freq[pair], c, s);
-        a += s;
-        b += c;
-    }
-    float* out = p.out + (size_t)row * p.out_stride + j;
-    out[0] = a;
-    if (two) out[1] = b;
-    if (p.act) {
-        act_t<ACT>* h = static_cast<act_t<ACT>*>(p.act) + (size_t)row * p.act_stride + j;
-        h[0] = f32_to_act<ACT>(a);
-        if (two) h[1] = f32_to_act<ACT>(b);
-    }
+// ---- launches ---------------------------------------------------------------------------------------------
+template <int EPI, int ACT, int NT>
+void launch_gemv(const DenseLinearParams& p, hipStream_t s) {
+    // rows per wave: one (short blocks, many of them) until the inputs' own loads weigh more than that
+    if (p.n >= 65536) dense_gemv_kernel<EPI, ACT, NT, 4><<<(p.n + 15) / 16, 256, 0, s>>>(p);
+    else if (EPI == DE_PAIRS || (NT * (ACT == ACT_FP32 ? 2 : 1) > 2 && p.n >= 8192)) dense_gemv_kernel<EPI, ACT, NT, 2><<<(p.n + 7) / 8, 256, 0, s>>>(p);
+    else if constexpr (EPI != DE_PAIRS) dense_gemv_kernel<EPI, ACT, NT, 1><<<(p.n + 3) / 4, 256, 0, s>>>(p);
 }
 
-// x <- cap tanh(x / cap)
-__global__ __launch_bounds__(256) void softcap_rows_kernel(float* x, uint32_t x_stride, uint32_t n, float cap) {
-    const uint32_t j = blockIdx.x * 256u + threadIdx.x;
-    if (j >= n) return;
-    float* v = x + (size_t)blockIdx.y * x_stride + j;
-    *v = cap * tanhf(*v / cap);
+template <int EPI, int ACT>
+int gemv(const DenseLinearParams& p, hipStream_t s) {
+    if (p.rows == 1) launch_gemv<EPI, ACT, 1>(p, s);
+    else if (p.rows == 2) launch_gemv<EPI, ACT, 2>(p, s);
+    else if (p.rows == 3) launch_gemv<EPI, ACT, 3>(p, s);
+    else launch_gemv<EPI, ACT, 4>(p, s);
+    return launch_status();
 }
 
-// Index of the largest finite value of each row, ties to the lower index, 0 when none is finite.  A candidate is one
-// 64-bit key: the value in the upper half (mapped so that unsigned order is the order of the floats), the complement
-// of the index in the lower; 0 = none.
-constexpr uint32_t ARGMAX_BLOCKS = 64;
-
-__device__ __forceinline__ uint64_t argmax_key(float v, uint32_t index) {
-    const uint32_t b = __float_as_uint(v);
-    if ((b & 0x7F800000u) == 0x7F800000u) return 0ull;         // infinite or not a number
-    const uint32_t o = b == 0x80000000u ? 0x80000000u : (b & 0x80000000u) ? ~b : b | 0x80000000u;    // -0 ranks as 0
-    return ((uint64_t)o << 32) | (uint32_t)~index;
-}
-
-__device__ __forceinline__ uint64_t argmax_block(uint64_t best, uint64_t* lds) {
-#pragma unroll
-    for (int off = 32; off >= 1; off >>= 1) {
-        const uint64_t o = ((uint64_t)shfl_xor_u((uint32_t)(best >> 32), off) << 32) | shfl_xor_u((uint32_t)best, off);
-        best = o > best ? o : best;
+template <int EPI>
+int dense_launch(nvmai_hip_ctx* ctx, hipStream_t s, const DenseLinearParams& p) {
+    if (p.rows <= 4) return ctx->act == NVMAI_ACT_FP32 ? gemv<EPI, ACT_FP32>(p, s) : gemv<EPI, ACT_BF16>(p, s);
+    if (ctx->act == NVMAI_ACT_FP32) {
+        const dim3 grid((p.n + 63) / 64, (p.rows + 63) / 64);
+        if (grid.y > 65535) return NVMAI_ERR_UNSUPPORTED;
+        dense_f32_kernel<EPI><<<grid, 256, 0, s>>>(p);
+        return launch_status();
     }
-    if ((threadIdx.x & 63u) == 0) lds[threadIdx.x >> 6] = best;
-    __syncthreads();
-    for (int w = 0; w < 4; ++w) best = lds[w] > best ? lds[w] : best;
-    return best;
-}
-
-__global__ __launch_bounds__(256) void argmax_stage1_kernel(const float* x, uint32_t x_stride, uint32_t n, uint64_t* part) {
-    __shared__ uint64_t lds[4];
-    const float* row = x + (size_t)blockIdx.y * x_stride;
-    uint64_t best = 0;
-#pragma unroll 4
-    for (uint32_t j = blockIdx.x * 256u + threadIdx.x; j < n; j += 256u * gridDim.x) {
-        const uint64_t k = argmax_key(row[j], j);
-        best = k > best ? k : best;
+    if (p.rows <= 64) {
+        // row tiles per block: as many as leave every compute unit several blocks; waves: about four steps of k each
+        const int nr = p.n >= 32768 ? 4 : p.n >= 8192 ? 2 : 1;
+        const uint32_t blocks = (p.n + 16 * nr - 1) / (16 * nr);
+#define NVMAI_SKINNY(TT)                                                              \
+    do {                                                                              \
+        if (nr == 4) dense_skinny_kernel<EPI, TT, 4, 4><<<blocks, 256, 0, s>>>(p);         \
+        else if (nr == 2) dense_skinny_kernel<EPI, TT, 2, 4><<<blocks, 256, 0, s>>>(p);    \
+        else if (p.k <= 1024) dense_skinny_kernel<EPI, TT, 1, 4><<<blocks, 256, 0, s>>>(p); \
+        else if (p.k <= 2048) dense_skinny_kernel<EPI, TT, 1, 8><<<blocks, 512, 0, s>>>(p); \
+        else dense_skinny_kernel<EPI, TT, 1, 16><<<blocks, 1024, 0, s>>>(p);               \
+    } while (0)
+        if (p.rows <= 16) NVMAI_SKINNY(1);
+        else if (p.rows <= 32) NVMAI_SKINNY(2);
+        else NVMAI_SKINNY(4);
+#undef NVMAI_SKINNY
+        return launch_status();
     }
-    best = argmax_block(best, lds);
-    if (threadIdx.x == 0) part[blockIdx.y * ARGMAX_BLOCKS + blockIdx.x] = best;
-}
-
-__global__ __launch_bounds__(256) void argmax_stage2_kernel(const uint64_t* part, uint32_t blocks, uint32_t* out) {
-    __shared__ uint64_t lds[4];
-    const uint64_t best = argmax_block(threadIdx.x < blocks ? part[blockIdx.x * ARGMAX_BLOCKS + threadIdx.x] : 0ull, lds);
-    if (threadIdx.x == 0) out[blockIdx.x] = best == 0ull ? 0u : ~(uint32_t)best;
+    // the largest tile that still gives every compute unit one
+    const uint32_t cus = (uint32_t)ctx->compute_units;
+    auto tiles = [](uint32_t v, uint32_t b) { return (v + b - 1) / b; };
+    if (tiles(p.n, 128) * tiles(p.rows, 128) >= cus)
+        dense_gemm_kernel<EPI, 128, 128><<<tiles(p.n, 128) * tiles(p.rows, 128), 256, 0, s>>>(p, tiles(p.n, 128), tiles(p.rows, 128));
+    else if (tiles(p.n, 64) * tiles(p.rows, 128) >= cus)
+        dense_gemm_kernel<EPI, 64, 128><<<tiles(p.n, 64) * tiles(p.rows, 128), 256, 0, s>>>(p, tiles(p.n, 64), tiles(p.rows, 128));
+    else
+        dense_gemm_kernel<EPI, 64, 64><<<tiles(p.n, 64) * tiles(p.rows, 64), 256, 0, s>>>(p, tiles(p.n, 64), tiles(p.rows, 64));
+    return launch_status();
 }
 
 }  // namespace nvmai

@@ -6,26 +6,35 @@ using namespace nvmai;
 
 namespace {
 
-template <bool DELTA>
-int recurrent(ScanParams p, bool by_arrays, hipStream_t s) {
-    const uint32_t per = (p.dk + 15) / 16, rows = p.n_rows;
-    // consecutive rows: SCAN_AHEAD of them per launch, so that a launch overwrites no history it reads
-    const uint32_t step = by_arrays ? rows : SCAN_AHEAD;
-    for (uint32_t t0 = 0; t0 < rows; t0 += step) {
-        const uint32_t n = rows - t0 < step ? rows - t0 : step;
-        const dim3 grid(p.heads, p.dv / 16, by_arrays ? rows : 1);
-        const uint32_t seq_rows = by_arrays ? 1 : n;
-        p.n_rows = n;
-        if (per <= 2) scan_recurrent_kernel<DELTA, 2><<<grid, 256, 0, s>>>(p, seq_rows);
-        else if (per <= 4) scan_recurrent_kernel<DELTA, 4><<<grid, 256, 0, s>>>(p, seq_rows);
-        else if (per <= 8) scan_recurrent_kernel<DELTA, 8><<<grid, 256, 0, s>>>(p, seq_rows);
-        else if (per <= 16) scan_recurrent_kernel<DELTA, 16><<<grid, 256, 0, s>>>(p, seq_rows);
-        else scan_recurrent_kernel<DELTA, 32><<<grid, 256, 0, s>>>(p, seq_rows);
-        p.proj += (size_t)n * p.proj_stride;
-        p.out += (size_t)n * p.out_stride;
-        p.rows.position += n;
-    }
+template <bool DELTA, int CP>
+int recurrent_launch(const ScanParams& p, uint32_t sequences, uint32_t seq_rows, hipStream_t s) {
+    const uint32_t per = (p.dk + 15) / 16;
+    const dim3 grid(p.heads, p.dv / (16 * CP), sequences);
+    if (per <= 2) scan_recurrent_kernel<DELTA, 2, CP><<<grid, 256, 0, s>>>(p, seq_rows);
+    else if (per <= 4) scan_recurrent_kernel<DELTA, 4, CP><<<grid, 256, 0, s>>>(p, seq_rows);
+    else if (per <= 8) scan_recurrent_kernel<DELTA, 8, CP><<<grid, 256, 0, s>>>(p, seq_rows);
+    else if (CP == 1 && per <= 16) scan_recurrent_kernel<DELTA, 16, 1><<<grid, 256, 0, s>>>(p, seq_rows);
+    else if (CP == 1) scan_recurrent_kernel<DELTA, 32, 1><<<grid, 256, 0, s>>>(p, seq_rows);
     return launch_status();
+}
+
+template <bool DELTA>
+int recurrent(ScanParams p, bool by_arrays, uint32_t compute_units, hipStream_t s) {
+    // four columns per thread when blocks of sixteen columns would come in several rounds
+    const bool wide = by_arrays && p.dv % 64 == 0 && p.dk <= 128 && aligned16(p.state) && (uint64_t)p.heads * (p.dv / 16) * p.n_rows > 4ull * compute_units;
+    if (wide) return recurrent_launch<DELTA, 4>(p, p.n_rows, 1, s);
+    if (by_arrays) return recurrent_launch<DELTA, 1>(p, p.n_rows, 1, s);
+    // consecutive rows: SCAN_AHEAD of them per launch, so that a launch overwrites no history it reads
+    const uint32_t rows = p.n_rows;
+    for (uint32_t t0 = 0; t0 < rows; t0 += SCAN_AHEAD) {
+        p.n_rows = rows - t0 < SCAN_AHEAD ? rows - t0 : SCAN_AHEAD;
+        const int rc = recurrent_launch<DELTA, 1>(p, 1, p.n_rows, s);
+        if (rc) return rc;
+        p.proj += (size_t)p.n_rows * p.proj_stride;
+        p.out += (size_t)p.n_rows * p.out_stride;
+        p.rows.position += p.n_rows;
+    }
+    return NVMAI_OK;
 }
 
 template <bool DELTA, int TAPS>
@@ -45,19 +54,27 @@ int chunked(const ScanParams& p, uint32_t chunks, hipStream_t s) {
     if (p.taps == 4) filter<DELTA, 4>(p, s);
     else filter<DELTA, 0>(p, s);
     if (p.taps > 1) scan_history_kernel<<<dim3((p.channels + 255) / 256, p.taps - 1), 256, 0, s>>>(p);
-    scan_prep_kernel<DELTA><<<dim3(chunks, p.heads), 256, lds, s>>>(p);
+    // heads of one block: the state-space form shares q k^T among the heads of a group
+    const uint32_t ratio = p.heads / p.key_heads, per = DELTA ? 1 : ratio < 8 ? ratio : 8;
+    scan_prep_kernel<DELTA><<<dim3(chunks, p.key_heads * ((ratio + per - 1) / per)), 256, lds, s>>>(p, per);
     const dim3 grid(p.heads, p.dv / 16);
-    if (p.dk <= 64) scan_chain_kernel<DELTA, 4><<<grid, 512, 0, s>>>(p, chunks);
-    else if (p.dk <= 128) scan_chain_kernel<DELTA, 8><<<grid, 512, 0, s>>>(p, chunks);
-    else scan_chain_kernel<DELTA, 16><<<grid, 512, 0, s>>>(p, chunks);
+    if (p.dk <= 64) scan_chain_kernel<DELTA, 4, 2><<<grid, 512, 0, s>>>(p, chunks);
+    else if (p.dk <= 128) scan_chain_kernel<DELTA, 8, 2><<<grid, 512, 0, s>>>(p, chunks);
+    else scan_chain_kernel<DELTA, 16, 1><<<grid, 512, 0, s>>>(p, chunks);
     return launch_status();
 }
 
 template <int ACT, bool FIRST>
 int gated_norm(const GatedNormParams& p, hipStream_t s) {
     const uint32_t n = p.heads * p.dv_count / p.parts;
-    if (n <= 512) gated_norm_kernel<ACT, FIRST, 64><<<dim3(p.rows, (p.parts + 3) / 4), 256, 0, s>>>(p);
-    else gated_norm_kernel<ACT, FIRST, 256><<<dim3(p.rows, p.parts), 256, 0, s>>>(p);
+    const bool vec = p.dv == p.dv_count && n % 4 == 0 && p.x_stride % 4 == 0 && p.gate_stride % 4 == 0 && p.out_stride % 4 == 0 && aligned16(p.x) &&
+                     aligned16(p.gate) && aligned16(p.out);
+    if (vec && n <= 128) gated_norm_kernel<ACT, FIRST, 32, 1, true><<<dim3(p.rows, (p.parts + 7) / 8), 256, 0, s>>>(p);
+    else if (vec && n <= 512) gated_norm_kernel<ACT, FIRST, 64, 2, true><<<dim3(p.rows, (p.parts + 3) / 4), 256, 0, s>>>(p);
+    else if (vec && n <= 4096) gated_norm_kernel<ACT, FIRST, 256, 4, true><<<dim3(p.rows, p.parts), 256, 0, s>>>(p);
+    else if (vec && n <= 16384) gated_norm_kernel<ACT, FIRST, 1024, 4, true><<<dim3(p.rows, p.parts), 1024, 0, s>>>(p);
+    else if (n <= 512) gated_norm_kernel<ACT, FIRST, 64, 8, false><<<dim3(p.rows, (p.parts + 3) / 4), 256, 0, s>>>(p);
+    else gated_norm_kernel<ACT, FIRST, 256, 8, false><<<dim3(p.rows, p.parts), 256, 0, s>>>(p);
     return launch_status();
 }
 
@@ -90,7 +107,7 @@ extern "C" int nvmai_hip_scan(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvm
     const bool can_chunk = !by_arrays && c.key_dim <= 256 && c.value_dim <= 256 && c.taps <= 65536;
     if (form == NVMAI_SCAN_CHUNKED && !can_chunk) return NVMAI_ERR_UNSUPPORTED;
     if (form != NVMAI_SCAN_CHUNKED && !(form == NVMAI_FORM_AUTO && can_chunk && rows >= SCAN_AHEAD))
-        return delta ? recurrent<true>(p, by_arrays, s) : recurrent<false>(p, by_arrays, s);
+        return delta ? recurrent<true>(p, by_arrays, (uint32_t)ctx->compute_units, s) : recurrent<false>(p, by_arrays, (uint32_t)ctx->compute_units, s);
     const size_t cells = (size_t)chunks * c.heads, n_mixed = (size_t)rows * channels, n_kt = delta ? cells * 64 * c.key_dim : 0, n_u0 = delta ? cells * 64 * c.value_dim : 0;
     const int rc = ws_begin(ctx, stream, ws_round(n_mixed * 4) + ws_round(cells * 4096 * 4) + ws_round(cells * 192 * 4) + ws_round(n_kt * 4) + ws_round(n_u0 * 4));
     if (rc) return rc;

@@ -62,22 +62,28 @@ __device__ __forceinline__ float scan_filter(const ScanParams& p, uint32_t slot,
 }
 
 // ---- recurrent form --------------------------------------------------------------------------------------
-// Block (head, sixteen columns, sequence): thread (column j = tid % 16, group c = tid / 16) owns the state rows
-// c PER .. c PER + PER - 1 of its column.  Only the block that owns a channel (its value columns; the q and k of a key
-// head: the first block of its first head) writes the channel's history, in rows that no block of the launch reads.
-template <bool DELTA, int PER>
+// Block (head, 16 CP columns, sequence): thread (j = tid % 16, group c = tid / 16) owns the state rows c PER .. c PER + PER - 1
+// of the columns CP j .. CP j + CP - 1.  CP 1 makes many small blocks (one sequence), CP 4 fewer whose filter serves more
+// columns.  Only the block that owns a channel (its value columns; the q and k of a key head: the first block of its
+// first head) writes the channel's history, in rows that no block of the launch reads.
+template <bool DELTA, int PER, int CP>
 __global__ __launch_bounds__(256) void scan_recurrent_kernel(ScanParams p, uint32_t seq_rows) {
-    __shared__ __attribute__((aligned(16))) float qs[16 * PER], ks[16 * PER];
-    __shared__ float vs[16], red[3][4], part[2][4][16];
+    constexpr uint32_t COLS = 16u * CP;
+    __shared__ __attribute__((aligned(16))) float qs[16 * PER], ks[16 * PER], vs[COLS], part[2][4][COLS];
+    __shared__ float red[3][4];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, j = tid & 15u, c = tid >> 4;
-    const uint32_t head = blockIdx.x, c0 = blockIdx.y * 16u, seq = blockIdx.z, dk = p.dk;
+    const uint32_t head = blockIdx.x, c0 = blockIdx.y * COLS, seq = blockIdx.z, dk = p.dk;
     const uint32_t ratio = p.heads / p.key_heads, key_head = head / ratio;
     const uint32_t base = seq * seq_rows, slot = p.rows.slot_of(base), first = p.rows.position_of(base);
     const uint32_t q_ch = key_head * dk, k_ch = (p.key_heads + key_head) * dk, v_ch = 2u * p.key_heads * dk + head * p.dv + c0;
-    float* S = p.state + (((size_t)slot * p.heads + head) * dk) * p.dv + c0 + j;
-    float st[PER];
+    float* S = p.state + (((size_t)slot * p.heads + head) * dk) * p.dv + c0 + CP * j;
+    float st[PER][CP];
 #pragma unroll
-    for (int e = 0; e < PER; ++e) st[e] = S[(size_t)min(c * PER + e, dk - 1u) * p.dv];
+    for (int e = 0; e < PER; ++e) {
+        const float* at = S + (size_t)min(c * PER + e, dk - 1u) * p.dv;
+        if constexpr (CP == 4) *reinterpret_cast<sc_f4*>(st[e]) = *reinterpret_cast<const sc_f4*>(at);
+        else st[e][0] = at[0];
+    }
     const float rate = expf(bf16_to_f32(p.a_log[head])), dt_bias = bf16_to_f32(p.dt_bias[head]), skip = DELTA ? 0.0f : bf16_to_f32(p.skip[head]);
     const bool keys_owner = head % ratio == 0u && c0 == 0u;
     for (uint32_t t = 0; t < seq_rows; ++t) {
@@ -102,44 +108,69 @@ __global__ __launch_bounds__(256) void scan_recurrent_kernel(ScanParams p, uint3
             kk = fmaf(k, k, kk);
             qk = fmaf(q, k, qk);
         }
-        if (tid >= 240u) {                           // the last sixteen threads have the fewest q and k channels
-            vs[j] = scan_filter(p, slot, base, first, t, v_ch + j);
-            past[v_ch + j] = row[p.conv_at + v_ch + j];
+        if (tid >= 256u - COLS) {                    // the last threads have the fewest q and k channels
+            const uint32_t d = tid - (256u - COLS);
+            vs[d] = scan_filter(p, slot, base, first, t, v_ch + d);
+            past[v_ch + d] = row[p.conv_at + v_ch + d];
         }
         qq = wave_sum_bcast(qq);
         kk = wave_sum_bcast(kk);
         qk = wave_sum_bcast(qk);
         if (lane == 0) { red[0][wave] = qq; red[1][wave] = kk; red[2][wave] = qk; }
         __syncthreads();
-        float sq = 0.0f, sk = 0.0f;                  // S^T q, S^T k over this thread's rows
+        float sq[CP] = {}, sk[CP] = {};              // S^T q, S^T k over this thread's rows
 #pragma unroll
         for (int e = 0; e < PER; ++e) {
-            sq = fmaf(st[e], qs[c * PER + e], sq);
-            if (DELTA) sk = fmaf(st[e], ks[c * PER + e], sk);
+            const float q = qs[c * PER + e], k = DELTA ? ks[c * PER + e] : 0.0f;
+#pragma unroll
+            for (int u = 0; u < CP; ++u) {
+                sq[u] = fmaf(st[e][u], q, sq[u]);
+                if (DELTA) sk[u] = fmaf(st[e][u], k, sk[u]);
+            }
         }
-        sq += shfl_xor_f(sq, 16);
-        sq += shfl_xor_f(sq, 32);
-        if (DELTA) { sk += shfl_xor_f(sk, 16); sk += shfl_xor_f(sk, 32); }
-        if (lane < 16u) { part[0][wave][j] = sq; if (DELTA) part[1][wave][j] = sk; }
+#pragma unroll
+        for (int u = 0; u < CP; ++u) {
+            sq[u] += shfl_xor_f(sq[u], 16);
+            sq[u] += shfl_xor_f(sq[u], 32);
+            if (DELTA) { sk[u] += shfl_xor_f(sk[u], 16); sk[u] += shfl_xor_f(sk[u], 32); }
+            if (lane < 16u) { part[0][wave][CP * j + u] = sq[u]; if (DELTA) part[1][wave][CP * j + u] = sk[u]; }
+        }
         const float sum_qk = (red[2][0] + red[2][1]) + (red[2][2] + red[2][3]);
         float qn = 1.0f, kn = 1.0f;
         if (DELTA) {
             qn = p.q_scale / sqrtf((red[0][0] + red[0][1]) + (red[0][2] + red[0][3]) + 1e-6f);
             kn = 1.0f / sqrtf((red[1][0] + red[1][1]) + (red[1][2] + red[1][3]) + 1e-6f);
         }
-        const float v = vs[j];
         __syncthreads();
-        sq = (part[0][0][j] + part[0][1][j]) + (part[0][2][j] + part[0][3][j]);
-        if (DELTA) sk = (part[1][0][j] + part[1][1][j]) + (part[1][2][j] + part[1][3][j]);
-        const float u = DELTA ? beta * (v - decay * (sk * kn)) : beta * v, ku = kn * u;
-        if (tid < 16u) p.out[(size_t)(base + t) * p.out_stride + head * p.dv + c0 + j] = fmaf(decay, sq * qn, sum_qk * qn * ku) + skip * v;
+        float ku[CP], o[CP];
 #pragma unroll
-        for (int e = 0; e < PER; ++e) st[e] = fmaf(decay, st[e], ks[c * PER + e] * ku);
+        for (int u = 0; u < CP; ++u) {
+            const uint32_t d = CP * j + u;
+            const float v = vs[d], q_old = (part[0][0][d] + part[0][1][d]) + (part[0][2][d] + part[0][3][d]);
+            const float k_old = DELTA ? (part[1][0][d] + part[1][1][d]) + (part[1][2][d] + part[1][3][d]) : 0.0f;
+            ku[u] = kn * (DELTA ? beta * (v - decay * (k_old * kn)) : beta * v);
+            o[u] = fmaf(decay, q_old * qn, sum_qk * qn * ku[u]) + skip * v;
+        }
+        if (tid < 16u) {
+            float* out = p.out + (size_t)(base + t) * p.out_stride + head * p.dv + c0 + CP * j;
+#pragma unroll
+            for (int u = 0; u < CP; ++u) out[u] = o[u];
+        }
+#pragma unroll
+        for (int e = 0; e < PER; ++e) {
+            const float k = ks[c * PER + e];
+#pragma unroll
+            for (int u = 0; u < CP; ++u) st[e][u] = fmaf(decay, st[e][u], k * ku[u]);
+        }
         __syncthreads();                             // this row's LDS is free
     }
 #pragma unroll
     for (int e = 0; e < PER; ++e)
-        if (c * PER + e < dk) S[(size_t)(c * PER + e) * p.dv] = st[e];
+        if (c * PER + e < dk) {
+            float* at = S + (size_t)(c * PER + e) * p.dv;
+            if constexpr (CP == 4) *reinterpret_cast<sc_f4*>(at) = *reinterpret_cast<sc_f4*>(st[e]);
+            else at[0] = st[e][0];
+        }
 }
 
 // ---- chunked form: filter, silu, unit vectors ----------------------------------------------------------------
@@ -202,36 +233,23 @@ __global__ __launch_bounds__(256) void scan_history_kernel(ScanParams p) {
 }
 
 // ---- chunked form: what needs no state ---------------------------------------------------------------------
+// Block (chunk, group of `per` heads of one key head).  Wave w makes the tiles (ti, w), ti >= w, of q k^T (and k k^T) once;
+// W, and for the delta rule L, follow from them head by head.
+//   (I + L) X = R for X = [Kt | U0], sixteen rows at a time: the four diagonal blocks of I + L are inverted by forward
+//   substitution (a lane per column), X_b = inv_b (R_b - sum_{m < b} L_bm X_m) runs on the matrix cores, a wave per
+//   sixteen columns, its X in the accumulators, where it stands as the next product's B operand.
 template <bool DELTA>
-__global__ __launch_bounds__(256) void scan_prep_kernel(ScanParams p) {
+__global__ __launch_bounds__(256) void scan_prep_kernel(ScanParams p, uint32_t per) {
     extern __shared__ __attribute__((aligned(16))) float sc_lds[];
     __shared__ double X[64];
     __shared__ float beta[64], bg[64];
-    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, i = lane & 15u, g = lane >> 4;
-    const uint32_t chunk = blockIdx.x, head = blockIdx.y, dk = p.dk, dv = p.dv, ld = dk + 4u, t0 = chunk * SCAN_CHUNK;
+    __shared__ __attribute__((aligned(16))) float inv[DELTA ? 4 : 1][16][20];
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = __builtin_amdgcn_readfirstlane(tid >> 6), i = lane & 15u, g = lane >> 4;
+    const uint32_t chunk = blockIdx.x, ratio = p.heads / p.key_heads, groups = (ratio + per - 1u) / per;
+    const uint32_t key_head = blockIdx.y / groups, h0 = (blockIdx.y % groups) * per, h1 = min(h0 + per, ratio);
+    const uint32_t dk = p.dk, dv = p.dv, ld = dk + 4u, t0 = chunk * SCAN_CHUNK;
+    const sc_f4 zero = sc_f4{0.0f, 0.0f, 0.0f, 0.0f};
     float *ks = sc_lds, *qs = ks + 64u * ld, *L = qs;        // [64][ld], [64][ld] and then [64][68] (delta)
-    const uint32_t key_head = head / (p.heads / p.key_heads);
-    const size_t cell = (size_t)chunk * p.heads + head;
-    float* gates = p.gates + cell * 192u;
-    if (wave == 0) {                                 // rows past the end: no decay, u = 0
-        const bool live = t0 + lane < p.n_rows;
-        const float* row = p.proj + (size_t)min(t0 + lane, p.n_rows - 1u) * p.proj_stride;
-        const float step = scan_softplus(row[p.a_at + head] + bf16_to_f32(p.dt_bias[head]));
-        double x = live ? (double)(expf(bf16_to_f32(p.a_log[head])) * step) : 0.0;
-        const float b = live ? (DELTA ? scan_sigmoid(row[p.b_at + head]) : step) : 0.0f;
-#pragma unroll
-        for (int off = 1; off < 64; off *= 2) {
-            const double y = __shfl_up(x, off, 64);
-            x += (int)lane >= off ? y : 0.0;
-        }
-        X[lane] = x;
-        beta[lane] = b;
-        const float G = expf(-(float)x);
-        bg[lane] = b * G;
-        gates[lane] = G;
-        gates[64u + lane] = expf(-(float)(__shfl(x, 63, 64) - x));
-        gates[128u + lane] = b;
-    }
     for (uint32_t e = tid; e < 64u * (dk / 4u); e += 256u) {
         const uint32_t t = e / (dk / 4u), d = (e % (dk / 4u)) * 4u;
         const float* row = p.mixed + (size_t)min(t0 + t, p.n_rows - 1u) * p.channels + key_head * dk + d;
@@ -239,64 +257,116 @@ __global__ __launch_bounds__(256) void scan_prep_kernel(ScanParams p) {
         *reinterpret_cast<sc_f4*>(ks + t * ld + d) = *reinterpret_cast<const sc_f4*>(row + p.key_heads * dk);
     }
     __syncthreads();
-    // the ten tiles on and below the diagonal of W and L, a column of tiles per wave
-    float* W = p.w + cell * 4096u;
-    sc_f4 low[4];
+    sc_f4 kk[4], qk[4];
+    const uint32_t col = 16u * wave + i;
 #pragma unroll
     for (uint32_t ti = 0; ti < 4u; ++ti) {
-        const uint32_t tm = wave;
-        sc_f4 kk = sc_f4{0.0f, 0.0f, 0.0f, 0.0f}, qk = kk;
-        if (tm <= ti) {
-            const float *ka = ks + (16u * ti + i) * ld + 4u * g, *qa = qs + (16u * ti + i) * ld + 4u * g, *kb = ks + (16u * tm + i) * ld + 4u * g;
-            for (uint32_t d = 0; d < dk; d += 16u) {
-                const sc_f4 a = *reinterpret_cast<const sc_f4*>(ka + d), q = *reinterpret_cast<const sc_f4*>(qa + d), b = *reinterpret_cast<const sc_f4*>(kb + d);
+        kk[ti] = qk[ti] = zero;
+        if (ti < wave) continue;                     // uniform
+        const float *ka = ks + (16u * ti + i) * ld + 4u * g, *qa = qs + (16u * ti + i) * ld + 4u * g, *kb = ks + col * ld + 4u * g;
+        for (uint32_t d = 0; d < dk; d += 16u) {
+            const sc_f4 a = *reinterpret_cast<const sc_f4*>(ka + d), q = *reinterpret_cast<const sc_f4*>(qa + d), b = *reinterpret_cast<const sc_f4*>(kb + d);
 #pragma unroll
-                for (int r = 0; r < 4; ++r) {
-                    if (DELTA) kk = __builtin_amdgcn_mfma_f32_16x16x4f32(a[r], b[r], kk, 0, 0, 0);
-                    qk = __builtin_amdgcn_mfma_f32_16x16x4f32(q[r], b[r], qk, 0, 0, 0);
+            for (int r = 0; r < 4; ++r) {
+                if (DELTA) kk[ti] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[r], b[r], kk[ti], 0, 0, 0);
+                qk[ti] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[r], b[r], qk[ti], 0, 0, 0);
+            }
+        }
+    }
+    for (uint32_t h = h0; h < h1; ++h) {
+        const uint32_t head = key_head * ratio + h;
+        const size_t cell = (size_t)chunk * p.heads + head;
+        float* gates = p.gates + cell * 192u;
+        if (wave == 0) {                             // rows past the end: no decay, u = 0
+            const bool live = t0 + lane < p.n_rows;
+            const float* row = p.proj + (size_t)min(t0 + lane, p.n_rows - 1u) * p.proj_stride;
+            const float step = scan_softplus(row[p.a_at + head] + bf16_to_f32(p.dt_bias[head]));
+            double x = live ? (double)(expf(bf16_to_f32(p.a_log[head])) * step) : 0.0;
+            const float b = live ? (DELTA ? scan_sigmoid(row[p.b_at + head]) : step) : 0.0f;
+#pragma unroll
+            for (int off = 1; off < 64; off *= 2) {
+                const double y = __shfl_up(x, off, 64);
+                x += (int)lane >= off ? y : 0.0;
+            }
+            X[lane] = x;
+            beta[lane] = b;
+            const float G = expf(-(float)x);
+            bg[lane] = b * G;
+            gates[lane] = G;
+            gates[64u + lane] = expf(-(float)(__shfl(x, 63, 64) - x));
+            gates[128u + lane] = b;
+        }
+        __syncthreads();                             // and, the first time, everyone is done with q
+        float* W = p.w + cell * 4096u;
+#pragma unroll
+        for (uint32_t ti = 0; ti < 4u; ++ti)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const uint32_t row = 16u * ti + 4u * g + r;
+                const float f = col <= row ? expf(-(float)(X[row] - X[col])) : 0.0f;
+                W[row * 64u + col] = col <= row ? f * qk[ti][r] : 0.0f;
+                if (DELTA) L[row * 68u + col] = col < row ? beta[row] * f * kk[ti][r] : 0.0f;
+            }
+        if (DELTA) {
+            __syncthreads();
+            if (wave == 0) {                         // lane group g: the diagonal block g, column i of its inverse
+                const float* D = L + (16u * g) * 68u + 16u * g;
+                float x[16];
+#pragma unroll
+                for (int r = 0; r < 16; ++r) {
+                    float a = (uint32_t)r == i ? 1.0f : 0.0f;
+#pragma unroll
+                    for (int m = 0; m < r; m += 4) {
+                        const sc_f4 l = *reinterpret_cast<const sc_f4*>(D + r * 68 + m);
+#pragma unroll
+                        for (int u = 0; u < 4; ++u)
+                            if (m + u < r) a = fmaf(-l[u], x[m + u], a);
+                    }
+                    x[r] = a;
+                }
+#pragma unroll
+                for (int r = 0; r < 16; ++r) inv[g][r][i] = x[r];
+            }
+            __syncthreads();
+            for (uint32_t tile = wave; tile < (dk + dv) / 16u; tile += 4u) {
+                const bool keys = tile < dk / 16u;   // uniform
+                const uint32_t c = keys ? 16u * tile + i : 16u * tile - dk + i;
+                float* out = keys ? p.kt + cell * 64u * dk + c : p.u0 + cell * 64u * dv + c;
+                const uint32_t out_ld = keys ? dk : dv;
+                const float* v = p.mixed + 2u * p.key_heads * dk + head * dv + c;
+                sc_f4 R[4], x[4];
+#pragma unroll
+                for (int b = 0; b < 4; ++b)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) {
+                        const uint32_t row = 16u * b + 4u * g + r;
+                        R[b][r] = keys ? bg[row] * ks[row * ld + c] : beta[row] * v[(size_t)min(t0 + row, p.n_rows - 1u) * p.channels];
+                    }
+#pragma unroll
+                for (int b = 0; b < 4; ++b) {
+                    sc_f4 a0 = zero, a1 = zero;
+#pragma unroll
+                    for (int m = 0; m < b; ++m) {
+                        const sc_f4 l = *reinterpret_cast<const sc_f4*>(L + (16u * b + i) * 68u + 16u * m + 4u * g);
+                        a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(l[0], x[m][0], a0, 0, 0, 0);
+                        a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(l[1], x[m][1], a1, 0, 0, 0);
+                        a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(l[2], x[m][2], a0, 0, 0, 0);
+                        a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(l[3], x[m][3], a1, 0, 0, 0);
+                    }
+                    const sc_f4 rest = R[b] - (a0 + a1), d = *reinterpret_cast<const sc_f4*>(&inv[b][i][4u * g]);
+                    a0 = zero;
+                    a1 = zero;
+                    a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(d[0], rest[0], a0, 0, 0, 0);
+                    a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(d[1], rest[1], a1, 0, 0, 0);
+                    a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(d[2], rest[2], a0, 0, 0, 0);
+                    a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(d[3], rest[3], a1, 0, 0, 0);
+                    x[b] = a0 + a1;
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) out[(size_t)(16u * b + 4u * g + r) * out_ld] = x[b][r];
                 }
             }
         }
-        const uint32_t col = 16u * tm + i;
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const uint32_t row = 16u * ti + 4u * g + r;
-            const float ratio = col <= row ? expf(-(float)(X[row] - X[col])) : 0.0f;
-            W[row * 64u + col] = col <= row ? ratio * qk[r] : 0.0f;
-            low[ti][r] = col < row ? beta[row] * ratio * kk[r] : 0.0f;
-        }
-    }
-    if (!DELTA) return;
-    __syncthreads();                                 // everyone is done with q
-#pragma unroll
-    for (int ti = 0; ti < 4; ++ti)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) L[(16u * ti + 4u * g + r) * 68u + 16u * wave + i] = low[ti][r];
-    __syncthreads();
-    for (uint32_t c = tid; c < dk + dv; c += 256u) {
-        float x[64];
-        float* out = c < dk ? p.kt + cell * 64u * dk + c : p.u0 + cell * 64u * dv + (c - dk);
-        const uint32_t out_ld = c < dk ? dk : dv;
-        const float* v = p.mixed + 2u * p.key_heads * dk + head * dv + (c < dk ? 0u : c - dk);
-#pragma unroll
-        for (int r = 0; r < 64; ++r)
-            x[r] = c < dk ? bg[r] * ks[r * ld + c] : beta[r] * v[(size_t)min(t0 + r, p.n_rows - 1u) * p.channels];
-#pragma unroll
-        for (int r = 1; r < 64; ++r) {
-            float a0 = 0.0f, a1 = 0.0f;
-#pragma unroll
-            for (int m = 0; m < r; m += 4) {
-                const sc_f4 l = *reinterpret_cast<const sc_f4*>(L + r * 68 + m);         // zero from the diagonal on
-                a0 = fmaf(l[0], x[m], a0);
-                if (m + 1 < r) a1 = fmaf(l[1], x[m + 1], a1);
-                if (m + 2 < r) a0 = fmaf(l[2], x[m + 2], a0);
-                if (m + 3 < r) a1 = fmaf(l[3], x[m + 3], a1);
-            }
-            x[r] -= a0 + a1;
-            if (r % 4 == 3) __builtin_amdgcn_sched_barrier(0);           // else every row of L is fetched at once
-        }
-#pragma unroll
-        for (int r = 0; r < 64; ++r) out[(size_t)r * out_ld] = x[r];
+        __syncthreads();                             // X, beta and L are free
     }
 }
 
@@ -310,8 +380,9 @@ __device__ __forceinline__ void scan_barrier() {
 // Waves 4 .. 7 make the outputs of the rows 16 (w - 4) .. + 15.  Per chunk two phases, a barrier behind each:
 //   first:  U = U0 - Kt S (SSD: dt V) into LDS;      o = G S^T q
 //   second: S = G_63 S + k^T c U, S into LDS;        o += W U, stored
-// Each wave requests its operands of a phase one phase ahead.  KT: state tiles (16 KT >= dk, KT a multiple of 4).
-template <bool DELTA, int KT>
+// Each wave requests its operands PF chunks ahead, in PF sets of registers that take turns.  KT: state tiles (16 KT >= dk, KT
+// a multiple of 4).
+template <bool DELTA, int KT, int PF>
 __global__ __launch_bounds__(512) void scan_chain_kernel(ScanParams p, uint32_t chunks) {
     constexpr int TW = KT / 4;
     __shared__ __attribute__((aligned(16))) sc_f4 ss[KT][64], us[4][64], cu[4][64];
@@ -322,36 +393,78 @@ __global__ __launch_bounds__(512) void scan_chain_kernel(ScanParams p, uint32_t 
     float* state = p.state + (((size_t)p.rows.slot * p.heads + head) * dk) * dv + col;
     auto cell_of = [&](uint32_t n) { return (size_t)n * p.heads + head; };
     if (wave < 4u) {
-        sc_f4 S[TW], kA[DELTA ? KT : 1], u0, c4;
-        float kcol[TW][4][4], g63;
-        auto first_operands = [&](uint32_t n) {      // of phase one of chunk n
+        struct Operands {
+            sc_f4 kA[DELTA ? KT : 1], u0, c4;        // first phase
+            float kcol[TW][4][4], g63;               // second
+        };
+        sc_f4 S[TW];
+        auto fetch_first = [&](uint32_t n, Operands& o) {
+            n = min(n, chunks - 1u);
             const size_t cell = cell_of(n);
-            const uint32_t t0 = n * SCAN_CHUNK + 16u * w;
             if (DELTA) {
 #pragma unroll
-                for (int t = 0; t < KT; ++t) kA[t] = *reinterpret_cast<const sc_f4*>(p.kt + (cell * 64u + 16u * w + i) * dk + min(16u * t, dk - 16u) + 4u * g);
+                for (int t = 0; t < KT; ++t) o.kA[t] = *reinterpret_cast<const sc_f4*>(p.kt + (cell * 64u + 16u * w + i) * dk + min(16u * t, dk - 16u) + 4u * g);
 #pragma unroll
-                for (int r = 0; r < 4; ++r) u0[r] = p.u0[(cell * 64u + 16u * w + 4u * g + r) * dv + col];
+                for (int r = 0; r < 4; ++r) o.u0[r] = p.u0[(cell * 64u + 16u * w + 4u * g + r) * dv + col];
             } else {
-                const sc_f4 b = *reinterpret_cast<const sc_f4*>(p.gates + cell * 192u + 128u + 16u * w + 4u * g);
+                o.kA[0] = *reinterpret_cast<const sc_f4*>(p.gates + cell * 192u + 128u + 16u * w + 4u * g);
 #pragma unroll
-                for (int r = 0; r < 4; ++r) u0[r] = b[r] * p.mixed[(size_t)min(t0 + 4u * g + r, p.n_rows - 1u) * p.channels + v_at];
+                for (int r = 0; r < 4; ++r) o.u0[r] = p.mixed[(size_t)min(n * SCAN_CHUNK + 16u * w + 4u * g + r, p.n_rows - 1u) * p.channels + v_at];
             }
-            c4 = *reinterpret_cast<const sc_f4*>(p.gates + cell * 192u + 64u + 16u * w + 4u * g);
+            o.c4 = *reinterpret_cast<const sc_f4*>(p.gates + cell * 192u + 64u + 16u * w + 4u * g);
         };
-        auto second_operands = [&](uint32_t n) {
-            g63 = p.gates[cell_of(n) * 192u + 63u];
+        auto fetch_second = [&](uint32_t n, Operands& o) {
+            n = min(n, chunks - 1u);
+            o.g63 = p.gates[cell_of(n) * 192u + 63u];
 #pragma unroll
             for (int s = 0; s < 4; ++s)
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
                     const float* k = p.mixed + (size_t)min(n * SCAN_CHUNK + 16u * s + 4u * g + r, p.n_rows - 1u) * p.channels + (p.key_heads + key_head) * dk + i;
 #pragma unroll
-                    for (int t = 0; t < TW; ++t) kcol[t][s][r] = k[min(16u * (w * TW + t), dk - 16u)];
+                    for (int t = 0; t < TW; ++t) o.kcol[t][s][r] = k[min(16u * (w * TW + t), dk - 16u)];
                 }
         };
-        first_operands(0);
-        second_operands(0);
+        auto chunk = [&](uint32_t n, Operands& o) {
+            sc_f4 u;
+            if (DELTA) {
+                sc_f4 a0 = zero, a1 = zero;
+#pragma unroll
+                for (int t = 0; t < KT; ++t) {
+                    if ((uint32_t)t < kt) {          // uniform
+                        const sc_f4 b = ss[t][lane];
+                        a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(o.kA[t][0], b[0], a0, 0, 0, 0);
+                        a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(o.kA[t][1], b[1], a1, 0, 0, 0);
+                        a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(o.kA[t][2], b[2], a0, 0, 0, 0);
+                        a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(o.kA[t][3], b[3], a1, 0, 0, 0);
+                    }
+                }
+                u = o.u0 - (a0 + a1);
+            } else {
+                u = o.kA[0] * o.u0;
+            }
+            us[w][lane] = u;
+            cu[w][lane] = u * o.c4;
+            fetch_first(n + PF, o);
+            scan_barrier();
+#pragma unroll
+            for (int t = 0; t < TW; ++t) S[t] *= o.g63;
+#pragma unroll
+            for (int s = 0; s < 4; ++s) {
+                const sc_f4 b = cu[s][lane];
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+#pragma unroll
+                    for (int t = 0; t < TW; ++t) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.kcol[t][s][r], b[r], S[t], 0, 0, 0);
+            }
+#pragma unroll
+            for (int t = 0; t < TW; ++t) ss[w * TW + t][lane] = S[t];
+            fetch_second(n + PF, o);
+            scan_barrier();
+        };
+        Operands o[PF];
+#pragma unroll
+        for (int f = 0; f < PF; ++f) { fetch_first(f, o[f]); fetch_second(f, o[f]); }
 #pragma unroll
         for (int t = 0; t < TW; ++t) {
             const uint32_t tile = w * TW + t;
@@ -360,41 +473,10 @@ __global__ __launch_bounds__(512) void scan_chain_kernel(ScanParams p, uint32_t 
             ss[tile][lane] = S[t];
         }
         scan_barrier();
-        for (uint32_t n = 0; n < chunks; ++n) {
-            const uint32_t next = min(n + 1u, chunks - 1u);
-            sc_f4 u = u0;
-            if (DELTA) {
-                sc_f4 a0 = zero, a1 = zero;
+        for (uint32_t n = 0; n < chunks; n += PF) {
 #pragma unroll
-                for (int t = 0; t < KT; ++t) {
-                    if ((uint32_t)t < kt) {          // uniform
-                        const sc_f4 b = ss[t][lane];
-                        a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(kA[t][0], b[0], a0, 0, 0, 0);
-                        a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(kA[t][1], b[1], a1, 0, 0, 0);
-                        a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(kA[t][2], b[2], a0, 0, 0, 0);
-                        a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(kA[t][3], b[3], a1, 0, 0, 0);
-                    }
-                }
-                u -= a0 + a1;
-            }
-            us[w][lane] = u;
-            cu[w][lane] = u * c4;
-            first_operands(next);
-            scan_barrier();
-#pragma unroll
-            for (int t = 0; t < TW; ++t) S[t] *= g63;
-#pragma unroll
-            for (int s = 0; s < 4; ++s) {
-                const sc_f4 b = cu[s][lane];
-#pragma unroll
-                for (int r = 0; r < 4; ++r)
-#pragma unroll
-                    for (int t = 0; t < TW; ++t) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(kcol[t][s][r], b[r], S[t], 0, 0, 0);
-            }
-#pragma unroll
-            for (int t = 0; t < TW; ++t) ss[w * TW + t][lane] = S[t];
-            second_operands(next);
-            scan_barrier();
+            for (int f = 0; f < PF; ++f)
+                if (n + f < chunks) chunk(n + f, o[f]);
         }
 #pragma unroll
         for (int t = 0; t < TW; ++t) {
@@ -405,57 +487,65 @@ __global__ __launch_bounds__(512) void scan_chain_kernel(ScanParams p, uint32_t 
         }
         return;
     }
-    sc_f4 qA[KT], wA[4], G4;
-    float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+    struct Operands {
+        sc_f4 qA[KT], G4;                            // first phase
+        sc_f4 wA[4];                                 // second
+        float v[4];
+    };
     const float skip = DELTA ? 0.0f : bf16_to_f32(p.skip[head]);
-    auto first_operands = [&](uint32_t n) {
+    auto fetch_first = [&](uint32_t n, Operands& o) {
+        n = min(n, chunks - 1u);
         const float* q = p.mixed + (size_t)min(n * SCAN_CHUNK + 16u * w + i, p.n_rows - 1u) * p.channels + key_head * dk + 4u * g;
 #pragma unroll
-        for (int t = 0; t < KT; ++t) qA[t] = *reinterpret_cast<const sc_f4*>(q + min(16u * t, dk - 16u));
-        G4 = *reinterpret_cast<const sc_f4*>(p.gates + cell_of(n) * 192u + 16u * w + 4u * g);
+        for (int t = 0; t < KT; ++t) o.qA[t] = *reinterpret_cast<const sc_f4*>(q + min(16u * t, dk - 16u));
+        o.G4 = *reinterpret_cast<const sc_f4*>(p.gates + cell_of(n) * 192u + 16u * w + 4u * g);
     };
-    auto second_operands = [&](uint32_t n) {
+    auto fetch_second = [&](uint32_t n, Operands& o) {
+        n = min(n, chunks - 1u);
 #pragma unroll
-        for (int t = 0; t < 4; ++t) wA[t] = *reinterpret_cast<const sc_f4*>(p.w + cell_of(n) * 4096u + (16u * w + i) * 64u + 16u * t + 4u * g);
-        if (!DELTA) {
+        for (int t = 0; t < 4; ++t) o.wA[t] = *reinterpret_cast<const sc_f4*>(p.w + cell_of(n) * 4096u + (16u * w + i) * 64u + 16u * t + 4u * g);
 #pragma unroll
-            for (int r = 0; r < 4; ++r) v[r] = p.mixed[(size_t)min(n * SCAN_CHUNK + 16u * w + 4u * g + r, p.n_rows - 1u) * p.channels + v_at];
-        }
+        for (int r = 0; r < 4; ++r) o.v[r] = DELTA ? 0.0f : p.mixed[(size_t)min(n * SCAN_CHUNK + 16u * w + 4u * g + r, p.n_rows - 1u) * p.channels + v_at];
     };
-    first_operands(0);
-    second_operands(0);
-    scan_barrier();
-    for (uint32_t n = 0; n < chunks; ++n) {
-        const uint32_t next = min(n + 1u, chunks - 1u);
+    auto chunk = [&](uint32_t n, Operands& op) {
         sc_f4 o = zero, o1 = zero;
 #pragma unroll
         for (int t = 0; t < KT; ++t) {
             if ((uint32_t)t < kt) {                  // uniform
                 const sc_f4 b = ss[t][lane];
-                o = __builtin_amdgcn_mfma_f32_16x16x4f32(qA[t][0], b[0], o, 0, 0, 0);
-                o1 = __builtin_amdgcn_mfma_f32_16x16x4f32(qA[t][1], b[1], o1, 0, 0, 0);
-                o = __builtin_amdgcn_mfma_f32_16x16x4f32(qA[t][2], b[2], o, 0, 0, 0);
-                o1 = __builtin_amdgcn_mfma_f32_16x16x4f32(qA[t][3], b[3], o1, 0, 0, 0);
+                o = __builtin_amdgcn_mfma_f32_16x16x4f32(op.qA[t][0], b[0], o, 0, 0, 0);
+                o1 = __builtin_amdgcn_mfma_f32_16x16x4f32(op.qA[t][1], b[1], o1, 0, 0, 0);
+                o = __builtin_amdgcn_mfma_f32_16x16x4f32(op.qA[t][2], b[2], o, 0, 0, 0);
+                o1 = __builtin_amdgcn_mfma_f32_16x16x4f32(op.qA[t][3], b[3], o1, 0, 0, 0);
             }
         }
-        o = (o + o1) * G4;
-        first_operands(next);
+        o = (o + o1) * op.G4;
+        fetch_first(n + PF, op);
         scan_barrier();
 #pragma unroll
         for (int t = 0; t < 4; ++t) {
             if ((uint32_t)t <= w) {                  // uniform
                 const sc_f4 b = us[t][lane];
 #pragma unroll
-                for (int r = 0; r < 4; ++r) o = __builtin_amdgcn_mfma_f32_16x16x4f32(wA[t][r], b[r], o, 0, 0, 0);
+                for (int r = 0; r < 4; ++r) o = __builtin_amdgcn_mfma_f32_16x16x4f32(op.wA[t][r], b[r], o, 0, 0, 0);
             }
         }
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const uint32_t t = n * SCAN_CHUNK + 16u * w + 4u * g + r;
-            if (t < p.n_rows) p.out[(size_t)t * p.out_stride + head * dv + col] = o[r] + skip * v[r];
+            if (t < p.n_rows) p.out[(size_t)t * p.out_stride + head * dv + col] = o[r] + skip * op.v[r];
         }
-        second_operands(next);
+        fetch_second(n + PF, op);
         scan_barrier();
+    };
+    Operands o[PF];
+#pragma unroll
+    for (int f = 0; f < PF; ++f) { fetch_first(f, o[f]); fetch_second(f, o[f]); }
+    scan_barrier();
+    for (uint32_t n = 0; n < chunks; n += PF) {
+#pragma unroll
+        for (int f = 0; f < PF; ++f)
+            if (n + f < chunks) chunk(n + f, o[f]);
     }
 }
 
@@ -468,53 +558,81 @@ struct GatedNormParams {
     float out_scale, eps;
 };
 
-// THREADS per (part, row): a wave (four of them in a block) or a block.  Elements of a part are read twice, the second
-// time from the caches, unless they fit into KEEP registers per thread.
-template <int ACT, bool FIRST, int THREADS>
-__global__ __launch_bounds__(256) void gated_norm_kernel(GatedNormParams p) {
-    constexpr int KEEP = 8;
-    __shared__ float red[4];
-    const uint32_t tid = threadIdx.x % THREADS, part = THREADS == 64 ? blockIdx.y * 4u + threadIdx.x / 64u : blockIdx.y, row = blockIdx.x;
-    if (THREADS == 64 && part >= p.parts) return;
+// LANES threads (a piece of a wave, a wave, or several) per (part, row), 256 or LANES threads per block.  VEC: four
+// neighbouring elements at a time, KEEP of them in registers; else element by element, those past the registers read
+// twice.
+template <int ACT, bool FIRST, int LANES, int KEEP, bool VEC>
+__global__ __launch_bounds__(LANES > 256 ? LANES : 256) void gated_norm_kernel(GatedNormParams p) {
+    constexpr uint32_t PER_BLOCK = LANES < 256 ? 256 / LANES : 1, E = VEC ? 4 : 1;
+    __shared__ float red[LANES > 64 ? LANES / 64 : 1];
+    const uint32_t tid = threadIdx.x % LANES, part = blockIdx.y * PER_BLOCK + threadIdx.x / LANES, row = blockIdx.x;
+    if (LANES <= 64 && part >= p.parts) return;
     const uint32_t n = p.heads * p.dv_count / p.parts, e0 = part * n;
     const float *x = p.x + (size_t)row * p.x_stride, *gate = p.gate + (size_t)row * p.gate_stride;
-    auto place = [&](uint32_t e) { return p.dv == p.dv_count ? e : e / p.dv_count * p.dv + e % p.dv_count; };
-    float xs[KEEP], zs[KEEP], ss = 0.0f;
+    auto place = [&](uint32_t e) { return VEC || p.dv == p.dv_count ? e : e / p.dv_count * p.dv + e % p.dv_count; };
+    float xs[KEEP][E], zs[KEEP][E], ss = 0.0f;
 #pragma unroll
     for (int u = 0; u < KEEP; ++u) {
-        const uint32_t at = place(e0 + min(tid + THREADS * u, n - 1u));
-        xs[u] = x[at];
-        zs[u] = gate[at];
+        const uint32_t at = place(e0 + min((tid + LANES * u) * E, n - E));
+        if constexpr (VEC) {
+            *reinterpret_cast<sc_f4*>(xs[u]) = *reinterpret_cast<const sc_f4*>(x + at);
+            *reinterpret_cast<sc_f4*>(zs[u]) = *reinterpret_cast<const sc_f4*>(gate + at);
+        } else {
+            xs[u][0] = x[at];
+            zs[u][0] = gate[at];
+        }
     }
 #pragma unroll
-    for (int u = 0; u < KEEP; ++u) {
-        if (FIRST) xs[u] *= silu(zs[u]);
-        if (tid + THREADS * u < n) ss = fmaf(xs[u], xs[u], ss);
-    }
-    for (uint32_t e = tid + THREADS * KEEP; e < n; e += THREADS) {
-        const uint32_t at = place(e0 + e);
-        const float v = FIRST ? x[at] * silu(gate[at]) : x[at];
-        ss = fmaf(v, v, ss);
-    }
-    ss = wave_sum_bcast(ss);
-    if (THREADS == 256) {
-        if ((tid & 63u) == 0) red[tid >> 6] = ss;
-        __syncthreads();
-        ss = (red[0] + red[1]) + (red[2] + red[3]);
+    for (int u = 0; u < KEEP; ++u)
+#pragma unroll
+        for (uint32_t e = 0; e < E; ++e) {
+            if (FIRST) xs[u][e] *= silu(zs[u][e]);
+            if ((tid + LANES * u) * E < n) ss = fmaf(xs[u][e], xs[u][e], ss);
+        }
+    if (!VEC)
+        for (uint32_t e = tid + LANES * KEEP; e < n; e += LANES) {
+            const uint32_t at = place(e0 + e);
+            const float v = FIRST ? x[at] * silu(gate[at]) : x[at];
+            ss = fmaf(v, v, ss);
+        }
+    if (LANES >= 64) {
+        ss = wave_sum_bcast(ss);
+        if (LANES > 64) {
+            if ((tid & 63u) == 0) red[tid >> 6] = ss;
+            __syncthreads();
+            ss = 0.0f;
+#pragma unroll
+            for (int u = 0; u < LANES / 64; ++u) ss += red[u];
+        }
+    } else {
+#pragma unroll
+        for (int off = LANES / 2; off >= 1; off >>= 1) ss += shfl_xor_f(ss, off);
     }
     const float inv = p.out_scale / sqrtf(ss / (float)n + p.eps);
     act_t<ACT>* out = static_cast<act_t<ACT>*>(p.out) + (size_t)row * p.out_stride;
-    auto put = [&](uint32_t at, float v, float z) {
-        out[at] = f32_to_act<ACT>(FIRST ? v * inv * bf16_to_f32(p.weight[at]) : v * inv * bf16_to_f32(p.weight[at % p.dv]) * silu(z));
+    auto value = [&](uint32_t at, float v, float z) {
+        return FIRST ? v * inv * bf16_to_f32(p.weight[at]) : v * inv * bf16_to_f32(p.weight[at % p.dv]) * silu(z);
     };
 #pragma unroll
-    for (int u = 0; u < KEEP; ++u)
-        if (tid + THREADS * u < n) put(place(e0 + tid + THREADS * u), xs[u], zs[u]);
-    for (uint32_t e = tid + THREADS * KEEP; e < n; e += THREADS) {
-        const uint32_t at = place(e0 + e);
-        const float z = gate[at];
-        put(at, FIRST ? x[at] * silu(z) : x[at], z);
+    for (int u = 0; u < KEEP; ++u) {
+        if ((tid + LANES * u) * E >= n) break;
+        const uint32_t at = place(e0 + (tid + LANES * u) * E);
+        if constexpr (VEC) {
+            float v[4];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = value(at + e, xs[u][e], zs[u][e]);
+            if constexpr (ACT == ACT_FP32) *reinterpret_cast<sc_f4*>(out + at) = sc_f4{v[0], v[1], v[2], v[3]};
+            else *reinterpret_cast<uint2*>(out + at) = make_uint2(f32_to_bf16(v[0]) | ((uint32_t)f32_to_bf16(v[1]) << 16), f32_to_bf16(v[2]) | ((uint32_t)f32_to_bf16(v[3]) << 16));
+        } else {
+            out[at] = f32_to_act<ACT>(value(at, xs[u][0], zs[u][0]));
+        }
     }
+    if (!VEC)
+        for (uint32_t e = tid + LANES * KEEP; e < n; e += LANES) {
+            const uint32_t at = place(e0 + e);
+            const float z = gate[at];
+            out[at] = f32_to_act<ACT>(value(at, FIRST ? x[at] * silu(z) : x[at], z));
+        }
 }
 
 }  // namespace nvmai

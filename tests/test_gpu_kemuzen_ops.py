@@ -429,8 +429,27 @@ def test_scan_with_decays_from_none_to_total(kind):
         assert s.state_error(slot) < 1e-5
 
 
+@pytest.mark.parametrize("kind", [0, 1])
+@pytest.mark.parametrize("shape,n", [((16, 8, 128, 128, 4), 12), ((32, 2, 40, 64, 3), 9), ((2, 2, 16, 32, 4), 3)])
+def test_scan_of_a_batch(kind, shape, n):
+    """One token of many sequences at different places, small and large launches."""
+    import nvmai_amd as nv
+    s = Scan(kind, *shape, slots=n + 1)
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device="cuda")
+    starts = [1 + 5 * j % 37 for j in range(n)]
+    rows = [s.rows(40 + j, starts[j] + 3) for j in range(n)]
+    want = [s.want(r) for r in rows]
+    for j in range(n):
+        s.run(rows[j][:starts[j]], nv.row_map(n - j, 0))
+    for t in range(3):
+        say("scan batch", kind, shape, t)
+        got = s.run(np.stack([rows[j][starts[j] + t] for j in range(n)]),
+                    nv.row_map(slots=i32([n - j for j in range(n)]), positions=i32([x + t for x in starts])))
+        close(got, np.stack([want[j][starts[j] + t] for j in range(n)]), 1e-5, "token %d" % t)
+
+
 @pytest.mark.parametrize("dtype", TYPES)
-@pytest.mark.parametrize("heads,dv,parts", [(4, 40, 4), (6, 20, 4), (6, 20, 1), (3, 16, 3), (64, 64, 2), (40, 72, 1), (1, 1, 1), (1, 700, 1)])
+@pytest.mark.parametrize("heads,dv,parts", [(1, 4096, 1), (9, 512, 1), (3, 128, 3), (2, 256, 2), (4, 40, 4), (6, 20, 4), (6, 20, 1), (3, 16, 3), (64, 64, 2), (40, 72, 1), (1, 1, 1), (1, 700, 1)])
 def test_gated_norm(dtype, heads, dv, parts):
     import nvmai_amd as nv
     ctx, rows, vp = context(dtype), 5, up(dv, 16)
