@@ -921,7 +921,8 @@ int nvmai_hip_window_attention(nvmai_hip_ctx* ctx, nvmai_stream stream, const nv
  * [q: key_heads * key_dim | k: the same | v: heads * value_dim]; a_at, b_at: columns of one number per head.  history
  * [slots, history_rows, channels] floats holds the filter's inputs, position p in row p % history_rows
  * (>= taps + 31; positions before 0 read as zero, whatever it holds).  conv [channels, taps], a_log, dt_bias, skip: BF16.  state
- * [slots, heads, key_dim, value_dim], updated in place.  out: floats [rows, heads * value_dim].
+ * [slots, heads, key_dim, value_dim], updated in place.  out: floats, row t of head h at t * out_stride + h * out_head_stride
+ * (head by head, [heads, rows, value_dim], is the faster of the orders for a prompt).
  * Rows by arrays: one row each of distinct slots.  key_dim, value_dim: multiples of 16, at most 512 (the chunked form 256).
  * form: AUTO, NVMAI_SCAN_RECURRENT, NVMAI_SCAN_CHUNKED (consecutive rows of one slot; takes workspace). */
 enum { NVMAI_SCAN_DELTA = 0, NVMAI_SCAN_SSD = 1 };
@@ -934,15 +935,16 @@ typedef struct {
 } nvmai_scan_config;
 int nvmai_hip_scan(nvmai_hip_ctx* ctx, nvmai_stream stream, const nvmai_scan_config* config, const float* proj, uint32_t proj_stride,
                    const uint16_t* conv, const uint16_t* conv_bias, const uint16_t* a_log, const uint16_t* dt_bias, const uint16_t* skip,
-                   float* history, float* state, const nvmai_row_map* map, float* out, uint32_t out_stride, uint32_t rows, int form);
+                   float* history, float* state, const nvmai_row_map* map, float* out, uint32_t out_stride, uint64_t out_head_stride,
+                   uint32_t rows, int form);
 
-/* The gated norm behind a recurrence.  x, gate: floats, heads of value_dim columns of which value_count are real; the
+/* The gated norm behind a recurrence.  x (rows and heads at strides of their own), gate: floats, heads of value_dim columns of which value_count are real; the
  * heads * value_count real ones in order make `parts` equal parts, each normed by its own root mean square:
  *   gate_first: out = RMS(x * silu(gate)) * weight * out_scale, weight [heads * value_dim]
  *   else        out = RMS(x) * weight * silu(gate) * out_scale, weight [value_dim], shared by the heads
- * out: activations, columns laid out as x's; padding columns are not written. */
-int nvmai_hip_gated_norm(nvmai_hip_ctx* ctx, nvmai_stream stream, const float* x, uint32_t x_stride, const float* gate,
-                         uint32_t gate_stride, const uint16_t* weight, void* out, uint32_t out_stride, uint32_t rows, uint32_t heads,
+ * out: activations, columns laid out as gate's; padding columns are not written. */
+int nvmai_hip_gated_norm(nvmai_hip_ctx* ctx, nvmai_stream stream, const float* x, uint32_t x_stride, uint64_t x_head_stride,
+                         const float* gate, uint32_t gate_stride, const uint16_t* weight, void* out, uint32_t out_stride, uint32_t rows, uint32_t heads,
                          uint32_t value_dim, uint32_t value_count, uint32_t parts, int gate_first, float out_scale, float eps);
 
 #ifdef __cplusplus

@@ -219,8 +219,8 @@ SIGNATURES = {
                                   C.POINTER(RowMap), u32],
     "nvmai_hip_window_attention": [vp, vp, C.POINTER(WindowConfig), vp, u32, vp, u32, C.POINTER(KvRingView), C.POINTER(RowMap), u32,
                                    C.c_float, vp, u32, u32, C.c_int],
-    "nvmai_hip_scan": [vp, vp, C.POINTER(ScanConfig), vp, u32, vp, vp, vp, vp, vp, vp, vp, C.POINTER(RowMap), vp, u32, u32, C.c_int],
-    "nvmai_hip_gated_norm": [vp, vp, vp, u32, vp, u32, vp, vp, u32, u32, u32, u32, u32, u32, C.c_int, C.c_float, C.c_float],
+    "nvmai_hip_scan": [vp, vp, C.POINTER(ScanConfig), vp, u32, vp, vp, vp, vp, vp, vp, vp, C.POINTER(RowMap), vp, u32, u64, u32, C.c_int],
+    "nvmai_hip_gated_norm": [vp, vp, vp, u32, u64, vp, u32, vp, vp, u32, u32, u32, u32, u32, u32, C.c_int, C.c_float, C.c_float],
     "nvmai_hip_argmax_rows": [vp, vp, vp, u32, u32, u32, vp],
     "nvmai_hip_gla": [vp, vp, C.POINTER(GlaConfig), vp, vp, vp, vp, vp, u32, vp, vp, vp, vp, vp, u32, vp, u32, u32, u32, C.c_int],
     "nvmai_hip_latent_epilogue": [vp, vp, C.POINTER(LatentConfig), vp, u32, u32, u32, vp, u32, u32, vp, vp, u32,

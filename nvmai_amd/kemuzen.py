@@ -351,7 +351,8 @@ class KemuzenDecoder(DenseDecoder):
 
     def _scan(self, ctx, i, proj, rows_at, heads, vdim_p):
         w = self.w.layers[i]
-        y = self._buf("scan", proj.shape[0], heads * vdim_p, torch.float32)
+        T = proj.shape[0]
+        y = self._buf("scan", T, heads * vdim_p, torch.float32).view(heads, T, vdim_p)         # head by head
         return self.scans[i, ctx].encode(proj, w["conv"], w["conv_bias"], w["a_log"], w["dt_bias"], w["skip"], *self.states[i], rows_at, y)
 
     def _mix(self, ctx, i, h, rows_at):
@@ -362,13 +363,13 @@ class KemuzenDecoder(DenseDecoder):
             self._window(ctx, i, m, proj, rows_at, out)
         elif m.kind == "delta":
             y = self._scan(ctx, i, proj, rows_at, m.heads, m.vdim_p)
-            ops.gated_norm(ctx, y, proj[:, at["g"]:], w["norm"], out, m.heads, m.vdim_p, m.vdim, m.heads, False, self.cfg.eps)
+            ops.gated_norm(ctx, y, proj[:, at["g"]:], w["norm"], out, m.vdim, m.heads, False, self.cfg.eps)
         else:
             a, r = m.left, m.right
             self._window(ctx, i, a, proj, rows_at, out, proj[:, at["gate"]:], m.left_scale)
             y = self._scan(ctx, i, proj, rows_at, r.heads, r.vdim_p)
-            ops.gated_norm(ctx, y, proj[:, at["z"]:], w["norm"], out[:, a.heads * a.vdim_p:], r.heads, r.vdim_p, r.vdim, r.norm_groups, True,
-                           self.cfg.eps, m.right_scale)
+            ops.gated_norm(ctx, y, proj[:, at["z"]:], w["norm"], out[:, a.heads * a.vdim_p:], r.vdim, r.norm_groups, True, self.cfg.eps,
+                           m.right_scale)
         return ops.dense_linear(ctx, w["o"], out, y_f32=self._buf("delta", T, self.cfg.width_p, torch.float32), bias=w.get("o_bias"))
 
     # -- the layers -------------------------------------------------------------------------------------

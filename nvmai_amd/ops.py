@@ -1286,15 +1286,17 @@ class HeadScan:
         return torch.zeros((slots, c.history_rows, self.channels), **f32), torch.zeros((slots, c.heads, c.key_dim, c.value_dim), **f32)
 
     def encode(self, proj, conv, conv_bias, a_log, dt_bias, skip, history, state, rows_at, out, form=FORM_AUTO):
+        """out: floats [heads, rows, value_dim], any strides of heads and rows."""
         check(lib.nvmai_hip_scan(self.ctx.handle, _stream(), C.byref(self.cfg), _ptr(proj), proj.stride(0), _ptr(conv), _ptr(conv_bias),
                                  _ptr(a_log), _ptr(dt_bias), _ptr(skip), _ptr(history), _ptr(state), C.byref(rows_at), _ptr(out),
-                                 out.stride(0), proj.shape[0], form), "scan")
+                                 out.stride(1), out.stride(0), proj.shape[0], form), "scan")
         return out
 
 
-def gated_norm(ctx, x, gate, weight, out, heads, value_dim, value_count, parts, gate_first, eps, out_scale=1.0):
-    """RMS norm over `parts` equal parts of the heads' real columns, with a SiLU gate before (gate_first) or after it."""
-    check(lib.nvmai_hip_gated_norm(ctx.handle, _stream(), _ptr(x), x.stride(0), _ptr(gate), gate.stride(0), _ptr(weight), _ptr(out),
-                                   out.stride(0), x.shape[0], heads, value_dim, value_count, parts, int(gate_first), out_scale, eps),
-          "gated_norm")
+def gated_norm(ctx, x, gate, weight, out, value_count, parts, gate_first, eps, out_scale=1.0):
+    """x [heads, rows, value_dim], any strides of heads and rows.  RMS norm over `parts` equal parts of the heads' real
+    columns, with a SiLU gate before (gate_first) or after it."""
+    heads, rows, value_dim = x.shape
+    check(lib.nvmai_hip_gated_norm(ctx.handle, _stream(), _ptr(x), x.stride(1), x.stride(0), _ptr(gate), gate.stride(0), _ptr(weight), _ptr(out),
+                                   out.stride(0), rows, heads, value_dim, value_count, parts, int(gate_first), out_scale, eps), "gated_norm")
     return out

@@ -340,11 +340,14 @@ class Scan:
         c = len(self.real)
         proj[:, self.real] = rows[:, :c]
         proj[:, self.a_at:self.a_at + 2 * self.H] = rows[:, c:]
+        by_heads = len(rows) % 2 == 0                # the output head by head or row by row
         out = torch.full((len(rows), self.H * self.vp + 4), 9.0, device="cuda")
+        view = out.flatten()[:len(rows) * self.H * self.vp].view(self.H, len(rows), self.vp) if by_heads else \
+            out[:, :self.H * self.vp].unflatten(1, (self.H, self.vp)).transpose(0, 1)
         self.op.encode(torch.from_numpy(proj).cuda(), self.conv_p, self.bias_p, self.a_log, self.dt_bias, self.skip, self.history, self.state,
-                       rows_at, out, form)
-        assert (out[:, self.H * self.vp:] == 9.0).all()
-        o = f64(out)[:, :self.H * self.vp].reshape(len(rows), self.H, self.vp)
+                       rows_at, view, form)
+        assert (out.flatten()[len(rows) * self.H * self.vp:] if by_heads else out[:, self.H * self.vp:] == 9.0).all()
+        o = f64(view).transpose(1, 0, 2)
         assert not o[:, :, self.dv:].any()
         return o[:, :, :self.dv]
 
@@ -461,7 +464,8 @@ def test_gated_norm(dtype, heads, dv, parts):
         wr = f64(w)[:, :dv].reshape(-1) if first else np.tile(f64(w)[:dv], heads)
         say("gated_norm", dtype, heads, dv, parts, first)
         out = torch.full((rows, heads * vp + 8), 9.0, dtype=ctx.dtype, device="cuda")
-        nv.gated_norm(ctx, x.reshape(rows, -1), z.reshape(rows, -1), w, out, heads, vp, dv, parts, first, 1e-5, 1.5)
+        by_heads = x.transpose(0, 1).contiguous() if first else x.transpose(0, 1)
+        nv.gated_norm(ctx, by_heads, z.reshape(rows, -1), w, out, dv, parts, first, 1e-5, 1.5)
         n = xr * K.silu(zr) if first else xr
         n = K.rms(n.reshape(rows, parts, -1), 1e-5).reshape(rows, -1) * wr * 1.5
         want = n if first else n * K.silu(zr)
