@@ -403,6 +403,8 @@ int dense_launch(nvmai_hip_ctx* ctx, hipStream_t s, const DenseLinearParams& p) 
         dense_gemm_kernel<EPI, 128, 128><<<tiles(p.n, 128) * tiles(p.rows, 128), 256, 0, s>>>(p, tiles(p.n, 128), tiles(p.rows, 128));
     else if (tiles(p.n, 64) * tiles(p.rows, 128) >= cus)
         dense_gemm_kernel<EPI, 64, 128><<<tiles(p.n, 64) * tiles(p.rows, 128), 256, 0, s>>>(p, tiles(p.n, 64), tiles(p.rows, 128));
+    else if (tiles(p.n, 64) * tiles(p.rows, 64) <= cus)      // one tile per compute unit waits for each of its loads: halve them
+        dense_gemm_kernel<EPI, 32, 64><<<tiles(p.n, 32) * tiles(p.rows, 64), 256, 0, s>>>(p, tiles(p.n, 32), tiles(p.rows, 64));
     else
         dense_gemm_kernel<EPI, 64, 64><<<tiles(p.n, 64) * tiles(p.rows, 64), 256, 0, s>>>(p, tiles(p.n, 64), tiles(p.rows, 64));
     return launch_status();

@@ -49,13 +49,18 @@ void epilogue(const WindowEpilogueParams& p, hipStream_t s) {
     }
 }
 
+template <int DK, int DV, bool BOUND>
+int launch_flash_as(const WindowParams& p, hipStream_t s) {
+    const size_t lds = 2 * ((size_t)64 * DK * 2 + (size_t)DV * 128);
+    const int rc = raise_lds(reinterpret_cast<const void*>(window_flash_kernel<DK, DV, BOUND>), lds);
+    if (rc) return rc;
+    window_flash_kernel<DK, DV, BOUND><<<(p.n_rows + 127) / 128 * p.heads, 256, lds, s>>>(p);
+    return launch_status();
+}
+
 template <int DK, int DV>
 int launch_flash(const WindowParams& p, hipStream_t s) {
-    const size_t lds = 2 * ((size_t)64 * DK * 2 + (size_t)DV * 128);
-    const int rc = raise_lds(reinterpret_cast<const void*>(window_flash_kernel<DK, DV>), lds);
-    if (rc) return rc;
-    window_flash_kernel<DK, DV><<<(p.n_rows + 127) / 128 * p.heads, 256, lds, s>>>(p);
-    return launch_status();
+    return p.capped && !p.alibi && p.b <= WA_BOUND ? launch_flash_as<DK, DV, true>(p, s) : launch_flash_as<DK, DV, false>(p, s);
 }
 
 template <int ACT, int CT>

@@ -387,14 +387,18 @@ __global__ __launch_bounds__(256) void window_plain_kernel(WindowParams p) {
 // form.  LDS pieces of 16 bytes are exchanged within a row so that the lanes a read serves at once fall into different
 // banks.  DK, DV: sizes padded with zeros (a lane whose column does not exist loads from past the end of the
 // buffer, which reads as zero).
+// BOUND: the scores are capped and the cap b (in powers of two) is at most WA_BOUND, so weights relative to b / 2 instead of
+// the running maximum stay between 2^(-3 b / 2) and 2^(b / 2): no maximum, and b tanh(z) - b / 2 = b / 2 - 2 b / (1 + e^(2 z)) is
+// one exponential, one reciprocal and one multiply-add.
 template <int W>                         // row width in pieces
 __device__ __forceinline__ uint32_t wa_swizzle(uint32_t key) {
     return W >= 8 ? (key & 3u) | ((key >> 1) & 4u) : (key >> 3) & (W - 1u);
 }
 
 constexpr uint32_t WA_OUT_OF_BOUNDS = 0x80000000u;
+constexpr float WA_BOUND = 80.0f;
 
-template <int DK, int DV>
+template <int DK, int DV, bool BOUND>
 __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void window_flash_kernel(WindowParams p) {
     constexpr int KS = DK / 32, VS = DV / 16;
     constexpr int LK = DK / 32, LV = DV / 32;        // 1 KB loads per wave and tile
@@ -497,6 +501,30 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void window_flash_kern
 #pragma unroll
         for (int b = 0; b < 2; ++b) {
             const uint32_t pos = start + min(wt0 + 16u * b + i, p.n_rows - 1u);
+            uint32_t w[8];
+            if (BOUND) {
+                const float z2 = 2.0f * WA_LOG2E * p.a, half = 0.5f * p.b, slide = -2.0f * p.b;
+#pragma unroll
+                for (int t = 0; t < 4; ++t) {
+                    float e[4];
+#pragma unroll
+                    for (int j = 0; j < 4; ++j)
+                        e[j] = __builtin_amdgcn_exp2f(fmaf(slide, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(z2 * s[b][t][j])), half));
+                    if (masked) {
+#pragma unroll
+                        for (int j = 0; j < 4; ++j) {
+                            const uint32_t key = k0 + 32u * (t >> 1) + 8u * g + 4u * (t & 1) + j;
+                            e[j] = wa_visible(pos, key, p.window, p.keep) ? e[j] : 0.0f;
+                        }
+                    }
+                    l[b] += (e[0] + e[1]) + (e[2] + e[3]);
+                    w[2 * t] = wa_pack2(e[0], e[1]);
+                    w[2 * t + 1] = wa_pack2(e[2], e[3]);
+                }
+                pf[b][0] = make_uint4(w[0], w[1], w[2], w[3]);
+                pf[b][1] = make_uint4(w[4], w[5], w[6], w[7]);
+                continue;
+            }
 #pragma unroll
             for (int t = 0; t < 4; ++t) s[b][t] *= p.a;
             if (p.capped) {
@@ -534,7 +562,6 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void window_flash_kern
                 for (int t = 0; t < VS; ++t) acc[b][t] *= alpha;
             }
             // a query without a key so far has m = WA_NONE, and exp2(2 WA_NONE - WA_NONE) = 0
-            uint32_t w[8];
 #pragma unroll
             for (int t = 0; t < 4; ++t) {
                 float e[4];

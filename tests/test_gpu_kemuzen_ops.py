@@ -216,6 +216,21 @@ def test_window_attention_forms_and_masks(dtype, shape):
                 close(w.run(data, nv.row_map(0, 0), form), want, bar(dtype), "form %d mask %s" % (form, (size, keep)))
 
 
+@pytest.mark.parametrize("softcap", [2.0, 30.0, 50.0, 70.0])
+def test_window_attention_under_a_cap_with_scores_at_both_ends(softcap):
+    """Scores far past the cap on either side, and rows that see nothing but the lowest ones."""
+    import nvmai_amd as nv
+    w = Window("bfloat16", 4, 2, 64, 64, 48, 5, softcap, scale=1.0)
+    data = w.rows(4, 200)
+    data[0][50:60] = 40.0                            # queries and keys along one direction: after the norms q . k = +- 64 and more
+    data[1][:100] = -1.0
+    data[1][100:] += 0.5
+    want = w.want(data)
+    for form in (nv.WINDOW_FLASH, nv.WINDOW_SPLIT, nv.WINDOW_PLAIN):
+        say("window cap", softcap, form)
+        close(w.run(data, nv.row_map(0, 0), form), want, bar("bfloat16"), "form %d" % form)
+
+
 @pytest.mark.parametrize("dtype", TYPES)
 @pytest.mark.parametrize("size,keep", [(17, 3), (40, 6), (5, 70), (64, 0), (31, 33)])
 def test_window_ring_wraps_and_kept_tokens_stay(dtype, size, keep):
