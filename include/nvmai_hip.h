@@ -884,8 +884,9 @@ typedef struct {
     int32_t type;
 } nvmai_kv_ring;
 
-/* Position i sees j <= i with i - j < window (0: every j) or j < keep_first (<= pinned).
- *   score = scale * q . k;  softcap > 0: score = softcap * tanh(score / softcap);  alibi: score -= 2^(-8 (head + 1) / heads) (i - j)
+/* The token at t looks at the window positions that end with t (0: all up to t) and at the first keep_first (<= pinned).
+ * Its score for the one at s is z = scale * q . k, bent to softcap * tanh(z / softcap) where softcap > 0, less (alibi) the
+ * distance t - s times 2^(-8 (head + 1) / heads).
  * key_count is the real head size behind key_dim: the mean of the norms. */
 typedef struct {
     uint32_t heads, key_count, window, keep_first;

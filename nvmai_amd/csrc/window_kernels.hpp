@@ -1,8 +1,9 @@
 // Windowed grouped-query attention over a cache of normed keys and transposed values.  gfx950, wave64.
 //
-//   visible(i, j) = j <= i and (i - j < window or j < keep)
-//   score(h, i, j) = scale q(h, i) . k(h / (heads / kv_heads), j), then softcap tanh(score / softcap), then - slope_h (i - j)
-//   out(h, i) = out_scale sigmoid(gate(h, i)) sum_j softmax_j(score) v_j
+// The token at t looks at s <= t where t - s < window, and at s < keep.  With z = scale q_t . k_s (k of the
+// head's group), its score for s is cap(z) - slope (t - s): cap(z) = c tanh(z / c), or z where there is no cap; the slope of a
+// head is a power of two of its index, or 0.  The softmax weights' sum over the values is multiplied by out_scale and, where
+// there is a gate, by the sigmoid of one number per head and token.
 //
 // Keys and values of a slot lie in a ring (position p in row p % ring, ring a multiple of 64, so an aligned tile of
 // positions is a run of rows) behind `pinned` rows that hold the first positions for good: position p < pinned is in

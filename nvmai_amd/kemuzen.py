@@ -3,9 +3,9 @@ gated delta rule, or by windowed attention and a state-space recurrence side by 
 outputs only, and every layer ends with an input of its own per token.  Configuration, weights and step driver; what the
 driver shares with the other dense models is in dense_model.py.
 
-A layer is  x <- x + norm1(mixer(x)),  x <- x + norm2(ff(x)) when it has a feed-forward,  and  x <- x + norm(W_p (gelu(W_g x) * e))
-with e the layer's part of the token's side vector; the residual x is 32-bit and starts as the scaled embedding plus a
-sinusoid of the position.  Every size and constant comes from config.json or from a tensor's shape, layer by layer.
+With N the sublayers' norms, a layer adds N(M x), then N(F x) where it has a feed-forward F, then N(W_p (gelu(W_g x) . e)) to the
+residual x, each from x as the one before left it; e is the layer's part of the token's side vector.  The residual is
+32-bit and starts as the scaled embedding plus a sinusoid of the position.  Every size and constant comes from config.json or from a tensor's shape, layer by layer.
 
 Weights are laid out for one launch per projection group (a mixer's projections of its input are rows of one matrix, both
 mixers' of a parallel layer; its two output projections are columns of one) and padded with zeros so that the kernels see

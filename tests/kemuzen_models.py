@@ -52,7 +52,7 @@ MODELS = {
                               attention(6, 2, 20, 24, 5, 1, scale=0.4, ff=40, kv_from=0)], side=12),
     "aligned": config(256, 128, [parallel((4, 4, 64, 64, 33), (4, 64, 64, 4, 4, 1), (1.0, 0.5), ff=256), attention(8, 2, 32, 64, 32, 64, ff=64),
                                  delta(2, 1, 64, 128, 4, ff=128), attention(4, 4, 128, 64, 64, 4)], side=64, scale=1.0),
-    "wide": config(64, 96, [attention(34, 2, 160, 144, 100, 9, ff=64), parallel((17, 1, 40, 16, 21), (3, 48, 160, 1, 4, 3), (0.9, 0.8)),
+    "wide": config(64, 96, [attention(34, 2, 160, 144, 100, 9, ff=64), parallel((17, 1, 40, 16, 21), (3, 48, 160, 1, 4, 3), (1.1, 0.6)),
                             delta(2, 2, 144, 160, 2)], side=8, cap=30.0),
     # the smallest of everything, filters of one tap, no kept tokens
     "ones": config(40, 2, [attention(1, 1, 1, 1, 1, 0, ff=1), delta(1, 1, 1, 1, 1), parallel((1, 1, 3, 1, 2), (1, 2, 1, 1, 1, 1), (1.0, 1.0), ff=3),

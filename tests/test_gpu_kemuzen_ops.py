@@ -130,8 +130,8 @@ def test_softcap_of_rows():
     import nvmai_amd as nv
     x = randn(1, 3, 301, std=40.0)
     y = x[:, :300].clone()
-    nv.softcap_rows(context("float32"), x[:, :300], 15.0)
-    close(f64(x)[:, :300], K.softcap(f64(y), 15.0), 1e-6, "softcap")
+    nv.softcap_rows(context("float32"), x[:, :300], 9.0)
+    close(f64(x)[:, :300], K.softcap(f64(y), 9.0), 1e-6, "softcap")
 
 
 # ---- windowed attention ---------------------------------------------------------------------------------------
@@ -198,7 +198,7 @@ def bar(dtype):
 
 
 SHAPES = [(6, 2, 20, 24), (4, 4, 64, 64), (8, 1, 96, 128), (34, 2, 128, 48), (3, 3, 160, 144), (1, 1, 1, 1)]
-MASKS = [(17, 3), (64, 64), (1, 0), (33, 70), (40, 6), (None, 0)]
+MASKS = [(17, 3), (64, 64), (1, 0), (33, 70), (44, 7), (None, 0)]
 
 
 @pytest.mark.parametrize("dtype", TYPES)
@@ -232,7 +232,7 @@ def test_window_attention_under_a_cap_with_scores_at_both_ends(softcap):
 
 
 @pytest.mark.parametrize("dtype", TYPES)
-@pytest.mark.parametrize("size,keep", [(17, 3), (40, 6), (5, 70), (64, 0), (31, 33)])
+@pytest.mark.parametrize("size,keep", [(17, 3), (44, 7), (5, 70), (64, 0), (31, 33)])
 def test_window_ring_wraps_and_kept_tokens_stay(dtype, size, keep):
     """Portions of unequal sizes through a ring just large enough, in both slots of a cache, then tokens one by one in a batch."""
     import nvmai_amd as nv
@@ -257,7 +257,7 @@ def test_window_ring_wraps_and_kept_tokens_stay(dtype, size, keep):
 
 
 @pytest.mark.parametrize("dtype", TYPES)
-@pytest.mark.parametrize("size,keep", [(40, 6), (64, 3), (127, 1), (300, 65)])
+@pytest.mark.parametrize("size,keep", [(44, 7), (64, 3), (127, 1), (300, 65)])
 def test_single_keys_at_the_edges_of_a_window(dtype, size, keep):
     """One key that outweighs all others, put just inside and just outside the window and the kept tokens: its value shows
     or does not."""
@@ -303,23 +303,23 @@ def test_a_layer_uses_another_layers_cache():
 
 def test_few_rows_in_32_bits_over_a_bf16_cache():
     import nvmai_amd as nv
-    w = Window("bfloat16", 8, 2, 96, 80, 40, 6, 8.0, gate=True)
+    w = Window("bfloat16", 8, 2, 96, 80, 44, 7, 8.0, gate=True)
     data = w.rows(1, 130)
     want = w.want(data)
     w.run([x[:128] for x in data], nv.row_map(0, 0))
     few = nv.Context(0, nv.ACT_FP32)
-    w.ctx, w.op = few, nv.WindowAttention(few, 8, 96, w.m["scale"], 40, w.eps, 6, 8.0)
+    w.ctx, w.op = few, nv.WindowAttention(few, 8, 96, w.m["scale"], 44, w.eps, 7, 8.0)
     for form in (nv.WINDOW_SPLIT, nv.WINDOW_PLAIN):
         close(w.run([x[128:] for x in data], nv.row_map(0, 128), form), want[128:], 1e-2, "two rows")
 
 
 def test_window_attention_refuses_what_does_not_fit():
     import nvmai_amd as nv
-    w = Window("bfloat16", 4, 2, 32, 32, 40, 6, capacity=64)
+    w = Window("bfloat16", 4, 2, 32, 32, 44, 7, capacity=64)
     with pytest.raises(nv.NvmaiError):
-        w.run(w.rows(1, 64), nv.row_map(0, 64))      # 40 + 63 positions in a ring of 64
+        w.run(w.rows(1, 64), nv.row_map(0, 64))      # 44 + 63 positions in a ring of 64
     with pytest.raises(nv.NvmaiError):
-        nv.WindowAttention(w.ctx, 3, 32, 1.0, 40, 1e-5, 6).encode_epilogue(torch.zeros((1, w.cols), device="cuda"), 0, 0, 0, w.qnp, w.knp,
+        nv.WindowAttention(w.ctx, 3, 32, 1.0, 44, 1e-5, 7).encode_epilogue(torch.zeros((1, w.cols), device="cuda"), 0, 0, 0, w.qnp, w.knp,
                                                                              torch.zeros((1, 96), dtype=torch.bfloat16, device="cuda"), w.cache, nv.row_map(0, 0))
 
 
