@@ -211,6 +211,11 @@ __global__ __launch_bounds__(256) void scan_filter_kernel(ScanParams p) {
     }
     const bool key = seg < 2u * p.key_heads;
     const uint32_t dim = key ? p.dk : p.dv, at = key ? seg * p.dk : 2u * p.key_heads * p.dk + (seg - 2u * p.key_heads) * p.dv;
+    float* out = key ? p.q_of(seg, t0) : p.v_of(seg - 2u * p.key_heads, t0);
+    if (t0 >= p.n_rows) {                            // a run behind the last row: there is no row of proj to read
+        for (uint32_t e = lane; e < SCAN_RUN * dim; e += 64u) out[e] = 0.0f;
+        return;
+    }
     const float factor = seg < p.key_heads ? p.q_scale : 1.0f;
     const uint32_t slot = p.rows.slot, first = p.rows.position;
     constexpr int HIST = TAPS > 0 ? TAPS - 1 : 0, IN = TAPS > 0 ? SCAN_RUN + HIST : 1;
@@ -230,7 +235,6 @@ __global__ __launch_bounds__(256) void scan_filter_kernel(ScanParams p) {
             for (int s = 0; s < HIST; ++s) in[e][s] = scan_input(p, slot, 0, first, (int32_t)t0 + s - HIST, ch[e]);
         }
     }
-    float* out = key ? p.q_of(seg, t0) : p.v_of(seg - 2u * p.key_heads, t0);
 #pragma unroll
     for (uint32_t t = 0; t < SCAN_RUN; ++t) {
         const bool live = t0 + t < p.n_rows;         // uniform

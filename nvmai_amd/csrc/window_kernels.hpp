@@ -7,9 +7,10 @@
 //
 // Keys and values of a slot lie in a ring (position p in row p % ring, ring a multiple of 64, so an aligned tile of
 // positions is a run of rows) behind `pinned` rows that hold the first positions for good: position p < pinned is in
-// row p as well.  A range of tiles is then "the kept tiles, from the pinned rows" followed by "the window's tiles, from
-// the ring", and one test per (query, key) decides what is seen in either.  Values are stored transposed: 16 bytes of a
-// row are eight positions of one channel, an A operand of the second product as they lie.
+// row p as well and is read there (the ring may have passed over it while it is still seen).  What a token looks at is a
+// range of kept tiles followed by the window's tiles, and one test per (query, key) decides what is seen in either.
+// Values are stored transposed: 16 bytes of a row are eight positions of one channel, an A operand of the second product
+// as they lie.
 //   * split: decoding and short portions, sixteen heads of one kv head per block, waves and blocks share the tiles;
 //   * flash: prompts, 128 queries of one head per block, tiles of 64 keys through LDS;
 //   * plain: any sizes and types, a thread per key.
